@@ -84,8 +84,27 @@ class ShardKVCache(list):
             self.offsets[r] = 0
         self.sync_pos()
 
+    def reserve(self, rows, n: int) -> None:
+        """Room for ``n`` more tokens in each of ``rows`` (every row is allocated at ``max_seq``)."""
+        for r in rows:
+            if self.offsets[r] + n > self.max_seq:
+                raise ValueError(f"KV cache overflow: {self.offsets[r]}+{n} > {self.max_seq}")
+
+    def release(self, row: int) -> None:
+        """The row's sequence is finished: nothing to give back here, the next one resets the row."""
+
     def nbytes(self) -> int:
         return sum(t.numel() * 2 for t in self.k) * 2
+
+    # -- one row's contents as [n, Hkv, D] tensors (prefix cache, wire)
+    def read_nhd(self, layer: int, row: int, start: int, n: int) -> tuple[torch.Tensor, torch.Tensor]:
+        from . import ops
+        return (ops.kv_export_nhd(self.k[layer][row], start, n), ops.kv_export_nhd(self.v[layer][row], start, n))
+
+    def write_nhd(self, layer: int, row: int, start: int, k: torch.Tensor, v: torch.Tensor) -> None:
+        from . import ops
+        ops.kv_import_nhd(k, self.k[layer][row], start)
+        ops.kv_import_nhd(v, self.v[layer][row], start)
 
     def copy_row(self, src: int, dst: int) -> None:
         """Move one sequence's cache to another batch row (slot compaction)."""

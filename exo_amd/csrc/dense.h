@@ -1,0 +1,88 @@
+// Element types of the unquantised kernels: bf16 (served) and float (the 32-bit mode).  Both move
+// in 16-byte vectors and both multiply on the matrix cores with the same operand and result
+// layouts, so every kernel is written once over the element type:
+//   bf16   8 elements per vector, one v_mfma_f32_{16x16x32,32x32x16}_bf16 per vector pair
+//   float  4 elements per vector, four v_mfma_f32_{16x16x4,32x32x2}_f32 (element i of every
+//          lane's vector in the i-th: the K order inside a vector pair does not matter as long
+//          as both operands use the same one)
+// An operand row of 64 bytes is one 16x16 step (4 lane groups of 16 bytes), 32 bytes one 32x32
+// step (2 lane halves).
+#pragma once
+#include "common.h"
+
+template <typename T>
+struct Elem;
+template <>
+struct Elem<bf16_t> {
+  static constexpr int kVec = 8;
+  static __device__ __forceinline__ float load(bf16_t v) { return bf2f(v); }
+  static __device__ __forceinline__ bf16_t make(float f) { return f2bf(f); }
+  static __device__ __forceinline__ floatx4 mma16(const uint4& a, const uint4& b, floatx4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a),
+                                                   __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
+  }
+  static __device__ __forceinline__ floatx16 mma32(const uint4& a, const uint4& b, floatx16 c) {
+    return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, a),
+                                                   __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
+  }
+};
+template <>
+struct Elem<float> {
+  static constexpr int kVec = 4;
+  static __device__ __forceinline__ float load(float v) { return v; }
+  static __device__ __forceinline__ float make(float f) { return f; }
+  static __device__ __forceinline__ floatx4 mma16(const uint4& a, const uint4& b, floatx4 c) {
+    const floatx4 x = __builtin_bit_cast(floatx4, a), y = __builtin_bit_cast(floatx4, b);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) c = __builtin_amdgcn_mfma_f32_16x16x4f32(x[i], y[i], c, 0, 0, 0);
+    return c;
+  }
+  static __device__ __forceinline__ floatx16 mma32(const uint4& a, const uint4& b, floatx16 c) {
+    const floatx4 x = __builtin_bit_cast(floatx4, a), y = __builtin_bit_cast(floatx4, b);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) c = __builtin_amdgcn_mfma_f32_32x32x2f32(x[i], y[i], c, 0, 0, 0);
+    return c;
+  }
+};
+
+// the vector's elements as floats
+template <typename T>
+__device__ __forceinline__ void unpack_vec(const uint4& v, float (&f)[Elem<T>::kVec]);
+template <>
+__device__ __forceinline__ void unpack_vec<bf16_t>(const uint4& v, float (&f)[8]) {
+  const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    f[2 * i] = bf_lo(w[i]);
+    f[2 * i + 1] = bf_hi(w[i]);
+  }
+}
+template <>
+__device__ __forceinline__ void unpack_vec<float>(const uint4& v, float (&f)[4]) {
+  const floatx4 x = __builtin_bit_cast(floatx4, v);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) f[i] = x[i];
+}
+
+// gated unit of an expert: g capped at `limit`, u kept within +-limit,
+// g * sigmoid(alpha * g) * (u + shift)
+struct GluConst {
+  float limit, alpha, shift;
+};
+__device__ __forceinline__ float clamped_glu(float g, float u, const GluConst& c) {
+  g = fminf(g, c.limit);
+  u = fminf(fmaxf(u, -c.limit), c.limit);
+  return g / (1.f + expf(-c.alpha * g)) * (u + c.shift);
+}
+
+// range-checked buffer over `bytes` bytes: reads past the end return zero and move nothing
+__device__ __forceinline__ __amdgpu_buffer_rsrc_t buf_of(const void* base, uint32_t bytes) {
+  return __builtin_amdgcn_make_buffer_rsrc(const_cast<void*>(base), 0, bytes, 0x00020000);
+}
+__device__ __forceinline__ uint4 buf_load16(__amdgpu_buffer_rsrc_t r, uint32_t voff, uint32_t soff) {
+  return __builtin_bit_cast(uint4, __builtin_amdgcn_raw_buffer_load_b128(r, voff, soff, 0));
+}
+constexpr uint32_t kPastEnd = 0x7FFFFFF0u;  // an offset beyond every buffer used here
+
+// host: call f<T>() for the element type code of the C ABI (0 bf16, 1 float32)
+#define EXO_BY_TYPE(dtype, CALL_BF16, CALL_F32) ((dtype) == 0 ? (CALL_BF16) : (CALL_F32))

@@ -1,0 +1,683 @@
+// Attention over a paged KV pool, for batches that mix portions of prompts with single decoded
+// tokens.  Options, each a parameter of the layer: unit-RMS queries and keys, a per-head linear
+// distance penalty, a sliding window with kept first tokens, value size other than key size, keys
+// and values of another layer.  Scores, penalty, softmax and sums are float32; where the weights
+// enter a bf16 matrix product they go in as two bf16 terms (high and remainder), so that they keep
+// 16 bits.
+//
+// Pool layout (page = 64 positions of one sequence, all kv heads):
+//   keys    [page][G][64][ldk]   a position's key, already normalised
+//   values  [page][G][ldv][64]   TRANSPOSED: a value column's 64 positions in one run
+// With the values transposed both operands of both products are rows of memory in matrix-core
+// operand order; nothing is transposed on the way.  ldk, ldv are multiples of 32 and the padding is
+// zero, so any key / value size is taken.
+//
+// paged_rows_kernel: one query position per workgroup row (decode; also the 32-bit mode's prompts).
+//   The up to 16 query heads of a kv head are the 16 columns of 16x16 products:
+//     S^T[key][head] = K . Q^T,   O^T[d][head] += V^T . P^T
+//   Each wave walks tiles of 32 keys, dealt out round robin over the waves of all splits; only the
+//   tiles that hold a visible key are dealt (kept first tokens, then the window).  Splits meet
+//   through device-scope partials and an arrival counter.  FUSE: the launch also normalises and
+//   stores the row's own key and value (the workgroup that owns the last tile does).
+// paged_prompt_kernel: 32 query positions of one head per wave, four such units of one kv head and
+//   one sequence per workgroup sharing page-sized key tiles through LDS (two buffers, the next tile
+//   in registers meanwhile); 32x32 products, transposed like above so that running maximum, sum and
+//   rescale factor are per-lane scalars.
+#include "../../include/exo_mi355x.h"
+#include "dense.h"
+
+namespace {
+
+constexpr int kPage = 64;
+constexpr int kCounters = 16384;  // arrival counters at the start of the workspace
+constexpr float kLog2e = 1.4426950408889634f;
+
+struct Params {
+  const void* qkv;      // T [R][ldq]: q heads, then (own keys) k heads, v heads
+  void* kpool;
+  void* vpool;
+  const int32_t* table; // [slots][max_pages]
+  const int32_t* slot;  // [R]
+  const int32_t* pos;   // [R]
+  const int32_t* list;  // rows: row indices (null: all); prompt: blocks of {row, slot, pos, n}
+  const float* slopes;  // [H], or null
+  void* out;            // T [R][ldo]
+  float* ws;
+  int* counters;
+  float scale, eps;
+  int n, H, G, D, E, ldq, ldk, ldv, ldo, max_pages, size, keep, unit, nsplit, gsz, hgroups;
+};
+
+__device__ __forceinline__ void st_dev(float* p, float v) {
+  __hip_atomic_store(p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+}
+__device__ __forceinline__ float ld_dev(const float* p) {
+  return __hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+}
+
+// key tiles of `tile` positions that hold a key visible to a query in [first, last]: the kept
+// ones [0, sink), then [w0, w1]
+struct Tiles {
+  int sink, w0, n;
+  __device__ __forceinline__ int at(int j) const { return j < sink ? j : w0 + (j - sink); }
+};
+__device__ __forceinline__ Tiles tiles_of(int first, int last, int size, int keep, int tile) {
+  Tiles t;
+  t.sink = (min(keep, last + 1) + tile - 1) / tile;
+  const int lo = max(0, first - size + 1);
+  t.w0 = max(lo / tile, t.sink);
+  t.n = t.sink + max(0, last / tile + 1 - t.w0);
+  return t;
+}
+
+// one wave: src[0..D) / rms -> dst (element type T, float32 arithmetic)
+template <typename T>
+__device__ __forceinline__ void unit_row(const T* __restrict__ src, T* dst, int D, int unit, float eps, int lane) {
+  float ss = 0.f;
+  for (int d = lane; d < D; d += 64) {
+    const float v = Elem<T>::load(src[d]);
+    ss += v * v;
+  }
+  const float inv = unit ? 1.f / sqrtf(wave_sum(ss) / D + eps) : 1.f;
+  for (int d = lane; d < D; d += 64) dst[d] = Elem<T>::make(Elem<T>::load(src[d]) * inv);
+}
+
+// key and value of one (row, kv head) into the pool, by one wave each
+template <typename T>
+__device__ __forceinline__ void put_key(const Params& p, int row, int g, int page, int at, int lane) {
+  const T* src = reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + p.H * p.D + g * p.D;
+  T* dst = reinterpret_cast<T*>(p.kpool) + (((size_t)page * p.G + g) * kPage + at) * p.ldk;
+  unit_row<T>(src, dst, p.D, p.unit, p.eps, lane);
+}
+template <typename T>
+__device__ __forceinline__ void put_value(const Params& p, int row, int g, int page, int at, int lane) {
+  const T* src = reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + (p.H + p.G) * p.D + g * p.E;
+  T* dst = reinterpret_cast<T*>(p.vpool) + ((size_t)page * p.G + g) * p.ldv * kPage + at;
+  for (int d = lane; d < p.E; d += 64) dst[(size_t)d * kPage] = src[d];
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void paged_append_kernel(const Params p) {
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x >> 6);
+  const int row = blockIdx.x, unit = blockIdx.y * 4 + wave;  // units: keys of G heads, values of G heads
+  if (unit >= 2 * p.G) return;
+  const int pos = p.pos[row];
+  const int page = p.table[(size_t)p.slot[row] * p.max_pages + pos / kPage];
+  if (unit < p.G)
+    put_key<T>(p, row, unit, page, pos % kPage, lane);
+  else
+    put_value<T>(p, row, unit - p.G, page, pos % kPage, lane);
+}
+
+template <typename T>
+struct PTerms;  // softmax weights of 32 keys as B operands
+template <>
+struct PTerms<bf16_t> {
+  uint4 hi, lo;
+  __device__ __forceinline__ void set(const float (&a)[4], const float (&b)[4]) {
+    float ra[4], rb[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) ra[i] = a[i] - bf2f(f2bf(a[i])), rb[i] = b[i] - bf2f(f2bf(b[i]));
+    hi = uint4{pack_bf2(a[0], a[1]), pack_bf2(a[2], a[3]), pack_bf2(b[0], b[1]), pack_bf2(b[2], b[3])};
+    lo = uint4{pack_bf2(ra[0], ra[1]), pack_bf2(ra[2], ra[3]), pack_bf2(rb[0], rb[1]), pack_bf2(rb[2], rb[3])};
+  }
+};
+template <>
+struct PTerms<float> {
+  uint4 hi, lo;
+  __device__ __forceinline__ void set(const float (&a)[4], const float (&b)[4]) {
+    hi = __builtin_bit_cast(uint4, floatx4{a[0], a[1], a[2], a[3]});
+    lo = __builtin_bit_cast(uint4, floatx4{b[0], b[1], b[2], b[3]});
+  }
+};
+// a value column's entries of this lane's keys: 4g.. and 16 + 4g.. of the 32-key tile at v
+template <typename T>
+struct VTerms;
+template <>
+struct VTerms<bf16_t> {
+  uint2 a, b;
+  __device__ __forceinline__ void load(const bf16_t* v, int g) {
+    a = *reinterpret_cast<const uint2*>(v + 4 * g);
+    b = *reinterpret_cast<const uint2*>(v + 16 + 4 * g);
+  }
+  __device__ __forceinline__ floatx4 mma(const PTerms<bf16_t>& p, floatx4 c) const {
+    const uint4 x{a.x, a.y, b.x, b.y};
+    return Elem<bf16_t>::mma16(x, p.lo, Elem<bf16_t>::mma16(x, p.hi, c));
+  }
+};
+template <>
+struct VTerms<float> {
+  uint4 a, b;
+  __device__ __forceinline__ void load(const float* v, int g) {
+    a = *reinterpret_cast<const uint4*>(v + 4 * g);
+    b = *reinterpret_cast<const uint4*>(v + 16 + 4 * g);
+  }
+  __device__ __forceinline__ floatx4 mma(const PTerms<float>& p, floatx4 c) const {
+    return Elem<float>::mma16(b, p.lo, Elem<float>::mma16(a, p.hi, c));
+  }
+};
+
+constexpr int kRowWaves = 4;
+
+template <typename T, int DMAX, bool FUSE>
+__global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params p) {
+  constexpr int KST = DMAX * (int)sizeof(T) / 64;  // 64-byte steps over a key
+  constexpr int VT = DMAX / 16;                    // 16-row tiles of O^T
+  constexpr int QS = DMAX + 16 / (int)sizeof(T);   // LDS row stride of q
+  extern __shared__ __attribute__((aligned(16))) char lds_raw[];
+  T* qs = reinterpret_cast<T*>(lds_raw);                          // [16][QS]
+  float* os = reinterpret_cast<float*>(lds_raw);                  // later: [waves][gsz][ldv]
+  __shared__ float ms[kRowWaves][16], ls[kRowWaves][16];
+  __shared__ int s_last;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int split = blockIdx.x, kvh = blockIdx.y / p.hgroups, hg = blockIdx.y % p.hgroups;
+  const int row = p.list ? p.list[blockIdx.z] : (int)blockIdx.z;
+  const int group = p.H / p.G;
+  const int h0 = kvh * group + hg * p.gsz, gs = min(p.gsz, (kvh + 1) * group - h0);
+  const int pos = p.pos[row];
+  const int32_t* table = p.table + (size_t)p.slot[row] * p.max_pages;
+  const Tiles tl = tiles_of(pos, pos, p.size, p.keep, 32);
+
+  // ---- queries (and the row's own key and value) through float32 norms
+  for (int h = wave; h < 16; h += kRowWaves) {
+    T* dst = qs + h * QS;
+    if (h < gs) unit_row<T>(reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + (h0 + h) * p.D, dst, p.D, p.unit, p.eps, lane);
+    for (int d = (h < gs ? p.D : 0) + lane; d < QS; d += 64) dst[d] = Elem<T>::make(0.f);
+  }
+  if (FUSE && split == ((tl.n - 1) % (p.nsplit * kRowWaves)) / kRowWaves) {
+    const int page = table[pos / kPage];
+    if (wave == kRowWaves - 1) put_key<T>(p, row, kvh, page, pos % kPage, lane);
+    if (wave == kRowWaves - 2) put_value<T>(p, row, kvh, page, pos % kPage, lane);
+    wait_own_stores_done();
+  }
+  __syncthreads();
+  uint4 q[KST];
+#pragma unroll
+  for (int s = 0; s < KST; ++s)
+    q[s] = *reinterpret_cast<const uint4*>(reinterpret_cast<const char*>(qs + r * QS) + s * 64 + g * 16);
+
+  const float sc = p.scale * kLog2e;
+  const float slope = p.slopes && r < gs ? p.slopes[h0 + r] * kLog2e : 0.f;
+  const int ksteps = p.ldk * (int)sizeof(T) / 64, vtiles = p.ldv / 16;
+  floatx4 o[VT];
+#pragma unroll
+  for (int t = 0; t < VT; ++t) o[t] = floatx4{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+
+  for (int j = split * kRowWaves + wave; j < tl.n; j += p.nsplit * kRowWaves) {
+    const int key0 = tl.at(j) * 32;
+    const size_t head = (size_t)table[key0 / kPage] * p.G + kvh;
+    const T* kp = reinterpret_cast<const T*>(p.kpool) + (head * kPage + (key0 % kPage)) * p.ldk;
+    const T* vp = reinterpret_cast<const T*>(p.vpool) + head * p.ldv * kPage + (key0 % kPage);
+    uint4 ka[KST], kb[KST];
+#pragma unroll
+    for (int s = 0; s < KST; ++s)
+      if (s < ksteps) {
+        ka[s] = *reinterpret_cast<const uint4*>(reinterpret_cast<const char*>(kp + (size_t)r * p.ldk) + s * 64 + g * 16);
+        kb[s] = *reinterpret_cast<const uint4*>(reinterpret_cast<const char*>(kp + (size_t)(16 + r) * p.ldk) + s * 64 + g * 16);
+      }
+    VTerms<T> v[VT];
+#pragma unroll
+    for (int t = 0; t < VT; ++t)
+      if (t < vtiles) v[t].load(vp + (size_t)(t * 16 + r) * kPage, g);
+    floatx4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < KST; ++s)
+      if (s < ksteps) {
+        s0 = Elem<T>::mma16(ka[s], q[s], s0);
+        s1 = Elem<T>::mma16(kb[s], q[s], s1);
+      }
+    float x0[4], x1[4], mx = -INFINITY;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int ja = key0 + 4 * g + e, jb = ja + 16;
+      const bool va = ja <= pos && (pos - ja < p.size || ja < p.keep);
+      const bool vb = jb <= pos && (pos - jb < p.size || jb < p.keep);
+      x0[e] = va ? s0[e] * sc - slope * (float)(pos - ja) : -INFINITY;
+      x1[e] = vb ? s1[e] * sc - slope * (float)(pos - jb) : -INFINITY;
+      mx = fmaxf(mx, fmaxf(x0[e], x1[e]));
+    }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float mn = fmaxf(m, mx);  // finite: a dealt tile holds a visible key
+    const float a = __builtin_amdgcn_exp2f(m - mn);
+    float sum = 0.f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      x0[e] = __builtin_amdgcn_exp2f(x0[e] - mn);
+      x1[e] = __builtin_amdgcn_exp2f(x1[e] - mn);
+      sum += x0[e] + x1[e];
+    }
+    sum += __shfl_xor(sum, 16, 64);
+    sum += __shfl_xor(sum, 32, 64);
+    l = l * a + sum;
+    m = mn;
+    PTerms<T> pt;
+    pt.set(x0, x1);
+#pragma unroll
+    for (int t = 0; t < VT; ++t)
+      if (t < vtiles) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[t][e] *= a;
+        o[t] = v[t].mma(pt, o[t]);
+      }
+  }
+
+  // ---- the waves of the workgroup
+  if (g == 0) ms[wave][r] = m, ls[wave][r] = l;
+  __syncthreads();  // (also: q in LDS is no longer read)
+  float mw = ms[0][r];
+#pragma unroll
+  for (int w = 1; w < kRowWaves; ++w) mw = fmaxf(mw, ms[w][r]);
+  const float f = m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m - mw);
+  if (r < gs) {
+#pragma unroll
+    for (int t = 0; t < VT; ++t)
+      if (t < vtiles) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) os[((size_t)wave * p.gsz + r) * p.ldv + t * 16 + 4 * g + e] = o[t][e] * f;
+      }
+  }
+  __syncthreads();
+  T* out = reinterpret_cast<T*>(p.out) + (size_t)row * p.ldo;
+  const size_t wsrow = (size_t)blockIdx.z * p.H;
+  for (int i = threadIdx.x; i < gs * p.E; i += 64 * kRowWaves) {
+    const int h = i / p.E, d = i % p.E;
+    float acc = 0.f, lw = 0.f, mm = -INFINITY;
+#pragma unroll
+    for (int w = 0; w < kRowWaves; ++w) mm = fmaxf(mm, ms[w][h]);
+#pragma unroll
+    for (int w = 0; w < kRowWaves; ++w) {
+      acc += os[((size_t)w * p.gsz + h) * p.ldv + d];
+      lw += ms[w][h] == -INFINITY ? 0.f : ls[w][h] * __builtin_amdgcn_exp2f(ms[w][h] - mm);
+    }
+    if (p.nsplit == 1) {
+      out[(h0 + h) * p.E + d] = Elem<T>::make(acc / lw);
+    } else {
+      float* dst = p.ws + ((wsrow + h0 + h) * p.nsplit + split) * (p.E + 2);
+      st_dev(dst + d, acc);
+      if (d == 0) {
+        st_dev(dst + p.E, mm);
+        st_dev(dst + p.E + 1, lw);
+      }
+    }
+  }
+  if (p.nsplit == 1) return;
+
+  // ---- the splits: the last workgroup to arrive merges them (values at device scope, every
+  // wave's stores complete before the barrier, then one counter increment; it returns to zero)
+  wait_own_stores_done();
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    int* cnt = p.counters + (size_t)blockIdx.z * gridDim.y + blockIdx.y;
+    const int old = __hip_atomic_fetch_add(cnt, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    s_last = old == p.nsplit - 1;
+    if (s_last) __hip_atomic_store(cnt, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  __syncthreads();
+  if (!s_last) return;
+  for (int i = threadIdx.x; i < gs * p.E; i += 64 * kRowWaves) {
+    const int h = i / p.E, d = i % p.E;
+    const float* src = p.ws + (wsrow + h0 + h) * p.nsplit * (p.E + 2);
+    float mm = -INFINITY;
+    for (int s = 0; s < p.nsplit; ++s) mm = fmaxf(mm, ld_dev(src + (size_t)s * (p.E + 2) + p.E));
+    float acc = 0.f, lw = 0.f;
+    for (int s = 0; s < p.nsplit; ++s) {
+      const float* q1 = src + (size_t)s * (p.E + 2);
+      const float ms1 = ld_dev(q1 + p.E);
+      const float w1 = ms1 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(ms1 - mm);
+      acc += ld_dev(q1 + d) * w1;
+      lw += ld_dev(q1 + p.E + 1) * w1;
+    }
+    out[(h0 + h) * p.E + d] = Elem<T>::make(acc / lw);
+  }
+}
+
+// ------------------------------------------------------------------------------ prompts
+constexpr int kPadK = 8;
+
+template <int D>
+constexpr int prompt_lds() {
+  return 2 * (kPage * (D + kPadK) + D * (kPage + kPadK)) * 2;
+}
+
+// HW: query heads per workgroup (4, 2, 1); its other factor is token tiles of 32
+template <int D, int HW>
+__global__ __launch_bounds__(256, D > 128 ? 1 : 2) void paged_prompt_kernel(const Params p) {
+  constexpr int STEPS = D / 16, DT = D / 32, KS = D + kPadK, VS = kPage + kPadK;
+  constexpr int VEC = D / 8, LOADS = kPage * VEC / 256;
+  constexpr int BUF = kPage * KS + D * VS;
+  constexpr int TT = 4 / HW;  // token tiles per workgroup
+  extern __shared__ __attribute__((aligned(16))) bf16_t lds[];  // [2][BUF]
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int n = lane & 31, kq = lane >> 5;
+  const int group = p.H / p.G, hgroups = (group + HW - 1) / HW;
+  const int kvh = blockIdx.y / hgroups, hg = blockIdx.y % hgroups;
+  const int4 blk = reinterpret_cast<const int4*>(p.list)[gridDim.x - 1 - blockIdx.x];  // row, slot, pos, n
+  const int hi = hg * HW + wave % HW, tt = wave / HW;
+  const bool active = hi < group && tt * 32 < blk.w;
+  const int hq = kvh * group + min(hi, group - 1);
+  const int t_lane = min(tt * 32 + n, blk.w - 1);  // this lane's token of the block
+  const int row = blk.x + t_lane, qpos = blk.z + t_lane;
+  const int wfirst = blk.z + min(tt * 32, blk.w - 1), wlast = blk.z + min(tt * 32 + 31, blk.w - 1);
+  const int32_t* table = p.table + (size_t)blk.y * p.max_pages;
+  const Tiles tl = tiles_of(blk.z, blk.z + blk.w - 1, p.size, p.keep, kPage);
+
+  // Q^T operand: lane (query n, half kq) holds d = 16 step + 8 kq .. + 8, normalised in float32
+  uint4 q[STEPS];
+  {
+    const bf16_t* qp = reinterpret_cast<const bf16_t*>(p.qkv) + (size_t)row * p.ldq + (size_t)hq * p.D;
+    float ss = 0.f;
+    const bool vec = p.D % 8 == 0 && p.ldq % 8 == 0;
+#pragma unroll
+    for (int s = 0; s < STEPS; ++s) {
+      const int d0 = 16 * s + 8 * kq;
+      uint32_t w[4];
+      if (vec) {
+        const uint4 v = d0 < p.D ? *reinterpret_cast<const uint4*>(qp + d0) : uint4{0, 0, 0, 0};
+        w[0] = v.x, w[1] = v.y, w[2] = v.z, w[3] = v.w;
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const uint32_t a = d0 + 2 * i < p.D ? qp[d0 + 2 * i] : 0, b = d0 + 2 * i + 1 < p.D ? qp[d0 + 2 * i + 1] : 0;
+          w[i] = a | b << 16;
+        }
+      }
+      q[s] = uint4{w[0], w[1], w[2], w[3]};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) ss += bf_lo(w[i]) * bf_lo(w[i]) + bf_hi(w[i]) * bf_hi(w[i]);
+    }
+    ss += __shfl_xor(ss, 32, 64);
+    if (p.unit) {
+      const float inv = 1.f / sqrtf(ss / p.D + p.eps);
+#pragma unroll
+      for (int s = 0; s < STEPS; ++s)
+        q[s] = uint4{pack_bf2(bf_lo(q[s].x) * inv, bf_hi(q[s].x) * inv), pack_bf2(bf_lo(q[s].y) * inv, bf_hi(q[s].y) * inv),
+                     pack_bf2(bf_lo(q[s].z) * inv, bf_hi(q[s].z) * inv), pack_bf2(bf_lo(q[s].w) * inv, bf_hi(q[s].w) * inv)};
+    }
+  }
+
+  uint4 kreg[LOADS], vreg[LOADS];
+  const uint32_t kbytes = kPage * (uint32_t)p.ldk * 2, vbytes = (uint32_t)p.ldv * kPage * 2;
+  auto load_tile = [&](int j) {
+    const size_t head = (size_t)table[tl.at(j)] * p.G + kvh;
+    const __amdgpu_buffer_rsrc_t rk = buf_of(reinterpret_cast<const bf16_t*>(p.kpool) + head * kPage * p.ldk, kbytes);
+    const __amdgpu_buffer_rsrc_t rv = buf_of(reinterpret_cast<const bf16_t*>(p.vpool) + head * p.ldv * kPage, vbytes);
+#pragma unroll
+    for (int i = 0; i < LOADS; ++i) {
+      const int vi = tid + i * 256, kr = vi / VEC, kc = vi % VEC;
+      kreg[i] = buf_load16(rk, kc * 8 < p.ldk ? (kr * p.ldk + kc * 8) * 2 : kPastEnd, 0);
+      vreg[i] = buf_load16(rv, vi * 16, 0);  // rows of 64 positions; rows past ldv read as zero
+    }
+  };
+  auto store_tile = [&](int b) {
+    bf16_t* kl = lds + b * BUF;
+    bf16_t* vl = kl + kPage * KS;
+#pragma unroll
+    for (int i = 0; i < LOADS; ++i) {
+      const int vi = tid + i * 256;
+      *reinterpret_cast<uint4*>(&kl[(vi / VEC) * KS + (vi % VEC) * 8]) = kreg[i];
+      *reinterpret_cast<uint4*>(&vl[(vi >> 3) * VS + (vi & 7) * 8]) = vreg[i];
+    }
+  };
+  // A-operand row n of a 32-key sub-tile holds this key, so that result registers 8s..8s+7 of
+  // lane half kq are keys 16s + 8kq .. + 8 (the B operand order of the second product)
+  const int jr = n >> 3;
+  const int key_of_row = 16 * (jr >> 1) + 8 * ((n >> 2) & 1) + 4 * (jr & 1) + (n & 3);
+  const float sc = p.scale * kLog2e;
+  const float slope = p.slopes ? p.slopes[hq] * kLog2e : 0.f;
+
+  floatx16 o[DT];
+#pragma unroll
+  for (int t = 0; t < DT; ++t)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) o[t][e] = 0.f;
+  float m = -INFINITY, l = 0.f;
+
+  load_tile(0);
+  store_tile(0);
+  __builtin_amdgcn_s_waitcnt(0x0F70);  // vmcnt(0): no wait for the queries inside the loop
+  if (tl.n > 1) load_tile(1);
+  for (int j = 0; j < tl.n; ++j) {
+    __syncthreads();  // tile j is complete in its buffer, the other buffer is no longer read
+    if (j + 1 < tl.n) {
+      store_tile((j + 1) & 1);
+      if (j + 2 < tl.n) load_tile(j + 2);
+    }
+    const int key0 = tl.at(j) * kPage, key1 = key0 + kPage - 1;
+    // wave-uniform: nothing of the tile is visible to the wave's queries
+    if (!active || key0 > wlast || (wfirst - key1 >= p.size && key0 >= p.keep)) continue;
+    const bf16_t* kl = lds + (j & 1) * BUF;
+    const bf16_t* vl = kl + kPage * KS;
+    floatx16 s[2];
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks) {
+#pragma unroll
+      for (int e = 0; e < 16; ++e) s[ks][e] = 0.f;
+      const bf16_t* kr = &kl[(ks * 32 + key_of_row) * KS + kq * 8];
+#pragma unroll
+      for (int st = 0; st < STEPS; ++st)
+        s[ks] = Elem<bf16_t>::mma32(*reinterpret_cast<const uint4*>(kr + st * 16), q[st], s[ks]);
+    }
+    const bool partial = key1 > wfirst || (wlast - key0 >= p.size && key1 >= p.keep);
+    const int rel = qpos - key0 - 8 * kq;  // distance to the lane's first key
+    const float base = -slope * (float)rel;
+    float mx = -INFINITY;
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) {
+        const int k = ks * 32 + 16 * (e >> 3) + (e & 7);
+        float x = fmaf(s[ks][e], sc, fmaf(slope, (float)k, base));
+        if (partial && (k > rel || (rel - k >= p.size && key0 + 8 * kq + k >= p.keep))) x = -INFINITY;
+        s[ks][e] = x;
+        mx = fmaxf(mx, x);
+      }
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float mn = fmaxf(m, mx), mr = mn == -INFINITY ? 0.f : mn;  // (a query may see none of the tile)
+    const float al = __builtin_amdgcn_exp2f(m - mr);
+    float sum = 0.f;
+    uint4 ph[2][2], pl[2][2];
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks)
+#pragma unroll
+      for (int st = 0; st < 2; ++st) {
+        float a[8], b[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          a[e] = __builtin_amdgcn_exp2f(s[ks][8 * st + e] - mr);
+          sum += a[e];
+        }
+        ph[ks][st] = uint4{pack_bf2(a[0], a[1]), pack_bf2(a[2], a[3]), pack_bf2(a[4], a[5]), pack_bf2(a[6], a[7])};
+        const uint32_t w[4] = {ph[ks][st].x, ph[ks][st].y, ph[ks][st].z, ph[ks][st].w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) b[2 * e] = a[2 * e] - bf_lo(w[e]), b[2 * e + 1] = a[2 * e + 1] - bf_hi(w[e]);
+        pl[ks][st] = uint4{pack_bf2(b[0], b[1]), pack_bf2(b[2], b[3]), pack_bf2(b[4], b[5]), pack_bf2(b[6], b[7])};
+      }
+    sum += __shfl_xor(sum, 32, 64);
+    l = l * al + sum;
+    m = mn;
+#pragma unroll
+    for (int t = 0; t < DT; ++t) {
+#pragma unroll
+      for (int e = 0; e < 16; ++e) o[t][e] *= al;
+      const bf16_t* vr = &vl[(t * 32 + n) * VS + kq * 8];
+#pragma unroll
+      for (int ks = 0; ks < 2; ++ks)
+#pragma unroll
+        for (int st = 0; st < 2; ++st) {
+          const uint4 a = *reinterpret_cast<const uint4*>(vr + ks * 32 + st * 16);
+          o[t] = Elem<bf16_t>::mma32(a, ph[ks][st], o[t]);
+          o[t] = Elem<bf16_t>::mma32(a, pl[ks][st], o[t]);
+        }
+    }
+  }
+  if (!active || tt * 32 + n >= blk.w) return;
+  const float inv = 1.f / l;
+  bf16_t* op = reinterpret_cast<bf16_t*>(p.out) + (size_t)row * p.ldo + (size_t)hq * p.E;
+  const bool pairs = p.E % 4 == 0;
+#pragma unroll
+  for (int t = 0; t < DT; ++t)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = t * 32 + 8 * i + 4 * kq;
+      if (pairs) {
+        if (d < p.E)
+          *reinterpret_cast<uint2*>(op + d) = uint2{pack_bf2(o[t][4 * i] * inv, o[t][4 * i + 1] * inv),
+                                                    pack_bf2(o[t][4 * i + 2] * inv, o[t][4 * i + 3] * inv)};
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (d + e < p.E) op[d + e] = f2bf(o[t][4 * i + e] * inv);
+      }
+    }
+}
+
+Params params_of(const exo_paged_attn* a) {
+  Params p{};
+  p.qkv = a->qkv, p.kpool = a->k_pool, p.vpool = a->v_pool, p.table = a->table, p.slot = a->slot, p.pos = a->pos;
+  p.list = a->list, p.slopes = a->slopes, p.out = a->out;
+  p.scale = a->scale, p.eps = a->eps, p.n = a->n, p.H = a->heads, p.G = a->kv_heads, p.D = a->dim, p.E = a->vdim;
+  p.ldq = a->ldq, p.ldk = a->ldk, p.ldv = a->ldv, p.ldo = a->ldo, p.max_pages = a->max_pages;
+  p.size = a->window > 0 ? a->window : 0x3FFFFFFF;
+  p.keep = a->keep_first, p.unit = a->unit_qk;
+  p.nsplit = 1;
+  return p;
+}
+
+int check(const exo_paged_attn* a, const char* what) {
+  EXO_REQUIRE(a && (a->dtype == 0 || a->dtype == 1), "%s: bad dtype", what);
+  EXO_REQUIRE(a->n > 0 && a->n <= 65535 && a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0,
+              "%s: bad counts (n=%d heads=%d kv_heads=%d)", what, a->n, a->heads, a->kv_heads);
+  EXO_REQUIRE(a->dim > 0 && a->vdim > 0 && a->dim <= 256 && a->vdim <= 256, "%s: head sizes %d / %d not in 1..256", what,
+              a->dim, a->vdim);
+  EXO_REQUIRE(a->ldk % 32 == 0 && a->ldk >= a->dim && a->ldk <= 256 && a->ldv % 32 == 0 && a->ldv >= a->vdim && a->ldv <= 256,
+              "%s: pool strides %d / %d do not fit head sizes %d / %d", what, a->ldk, a->ldv, a->dim, a->vdim);
+  EXO_REQUIRE(a->qkv && a->k_pool && a->v_pool && a->table && a->max_pages > 0, "%s: null pointer", what);
+  EXO_REQUIRE(a->keep_first >= 0 && a->window >= 0, "%s: negative window", what);
+  return EXO_OK;
+}
+
+template <typename T, int DMAX, bool FUSE>
+int launch_rows(const Params& p, hipStream_t st) {
+  constexpr int qbytes = 16 * (DMAX + 16 / (int)sizeof(T)) * (int)sizeof(T);
+  const int obytes = kRowWaves * p.gsz * p.ldv * 4;
+  const int lds = qbytes > obytes ? qbytes : obytes;  // at most 64 KiB (16 heads x 256 values x 4 waves)
+  exo_note_variant("paged_rows<%s,%d,%s> splits=%d rows=%d", sizeof(T) == 2 ? "bf16" : "f32", DMAX, FUSE ? "fused" : "plain",
+                   p.nsplit, p.n);
+  static bool done = false;
+  const auto fn = paged_rows_kernel<T, DMAX, FUSE>;
+  if (!done) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, 80 * 1024);
+    if (e != hipSuccess) {
+      exo_set_error("exo_paged_attn_rows: cannot raise the dynamic LDS limit: %s", hipGetErrorString(e));
+      return EXO_ERR_HIP;
+    }
+    done = true;
+  }
+  fn<<<dim3(p.nsplit, p.G * p.hgroups, p.n), 64 * kRowWaves, lds, st>>>(p);
+  return EXO_OK;
+}
+
+template <typename T, int DMAX>
+int launch_rows_f(const Params& p, bool fuse, hipStream_t st) {
+  return fuse ? launch_rows<T, DMAX, true>(p, st) : launch_rows<T, DMAX, false>(p, st);
+}
+template <typename T>
+int launch_rows_d(const Params& p, int d, bool fuse, hipStream_t st) {
+  return d <= 64 ? launch_rows_f<T, 64>(p, fuse, st) : d <= 128 ? launch_rows_f<T, 128>(p, fuse, st) : launch_rows_f<T, 256>(p, fuse, st);
+}
+
+template <int D, int HW>
+int launch_prompt(const Params& p, hipStream_t st) {
+  constexpr int lds = prompt_lds<D>();
+  static bool done = false;
+  const auto fn = paged_prompt_kernel<D, HW>;
+  if (!done && lds > 64 * 1024) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    if (e != hipSuccess) {
+      exo_set_error("exo_paged_attn_prompt: cannot raise the dynamic LDS limit: %s", hipGetErrorString(e));
+      return EXO_ERR_HIP;
+    }
+  }
+  done = true;
+  const int group = p.H / p.G;
+  const dim3 grid(p.n, p.G * ((group + HW - 1) / HW));
+  exo_note_variant("paged_prompt<%d,%d> grid=%dx%d", D, HW, (int)grid.x, (int)grid.y);
+  fn<<<grid, 256, lds, st>>>(p);
+  return EXO_OK;
+}
+template <int D>
+int launch_prompt_h(const Params& p, hipStream_t st) {
+  const int group = p.H / p.G;
+  return group >= 3 ? launch_prompt<D, 4>(p, st) : group == 2 ? launch_prompt<D, 2>(p, st) : launch_prompt<D, 1>(p, st);
+}
+
+}  // namespace
+
+extern "C" int exo_paged_append(const exo_paged_attn* a, exo_stream_t stream) {
+  const int rc = check(a, "exo_paged_append");
+  if (rc) return rc;
+  EXO_REQUIRE(a->slot && a->pos && a->ldq >= (a->heads + a->kv_heads) * a->dim + a->kv_heads * a->vdim,
+              "exo_paged_append: rows of %d elements do not hold q, k and v", a->ldq);
+  const Params p = params_of(a);
+  const dim3 grid(p.n, (2 * p.G + 3) / 4);
+  if (a->dtype == 0)
+    paged_append_kernel<bf16_t><<<grid, 256, 0, (hipStream_t)stream>>>(p);
+  else
+    paged_append_kernel<float><<<grid, 256, 0, (hipStream_t)stream>>>(p);
+  EXO_CHECK_LAUNCH("exo_paged_append");
+  return EXO_OK;
+}
+
+extern "C" int64_t exo_paged_attn_workspace(int n, int heads, int vdim, int nsplit) {
+  return ((int64_t)n * heads * nsplit * (vdim + 2) + kCounters) * 4;
+}
+
+extern "C" int exo_paged_attn_rows(const exo_paged_attn* a, int nsplit, int append, void* workspace,
+                                   int64_t workspace_bytes, exo_stream_t stream) {
+  const int rc = check(a, "exo_paged_attn_rows");
+  if (rc) return rc;
+  EXO_REQUIRE(a->slot && a->pos && a->out && a->ldo >= a->heads * a->vdim && a->ldq >= a->heads * a->dim,
+              "exo_paged_attn_rows: bad rows or output");
+  EXO_REQUIRE(!append || a->ldq >= (a->heads + a->kv_heads) * a->dim + a->kv_heads * a->vdim,
+              "exo_paged_attn_rows: rows of %d elements do not hold q, k and v", a->ldq);
+  EXO_REQUIRE(nsplit >= 1 && nsplit <= 256 &&
+                  (nsplit == 1 || (workspace && (int64_t)a->n * a->heads <= kCounters && workspace_bytes >= exo_paged_attn_workspace(a->n, a->heads, a->vdim, nsplit))),
+              "exo_paged_attn_rows: workspace too small for %d splits", nsplit);
+  Params p = params_of(a);
+  p.nsplit = nsplit;
+  const int group = p.H / p.G;
+  p.hgroups = (group + 15) / 16;
+  p.gsz = (group + p.hgroups - 1) / p.hgroups;
+  p.counters = reinterpret_cast<int*>(workspace);
+  p.ws = nsplit > 1 ? reinterpret_cast<float*>(workspace) + kCounters : nullptr;
+  const int d = p.ldk > p.ldv ? p.ldk : p.ldv;
+  const hipStream_t st = (hipStream_t)stream;
+  const int rc2 = a->dtype == 0 ? launch_rows_d<bf16_t>(p, d, append != 0, st) : launch_rows_d<float>(p, d, append != 0, st);
+  if (rc2) return rc2;
+  EXO_CHECK_LAUNCH("exo_paged_attn_rows");
+  return EXO_OK;
+}
+
+extern "C" int exo_paged_prompt_block(int heads, int kv_heads) {
+  const int group = kv_heads > 0 ? heads / kv_heads : 0;
+  return group >= 3 ? 32 : group == 2 ? 64 : 128;
+}
+
+extern "C" int exo_paged_attn_prompt(const exo_paged_attn* a, exo_stream_t stream) {
+  const int rc = check(a, "exo_paged_attn_prompt");
+  if (rc) return rc;
+  EXO_REQUIRE(a->dtype == 0, "exo_paged_attn_prompt: bf16 only");
+  EXO_REQUIRE(a->list && a->out && a->ldo >= a->heads * a->vdim && a->ldq >= a->heads * a->dim && a->ldo % 4 == 0 &&
+                  a->ldk % 8 == 0,
+              "exo_paged_attn_prompt: bad rows or output");
+  const Params p = params_of(a);
+  const int d = p.ldk > p.ldv ? p.ldk : p.ldv;
+  const hipStream_t st = (hipStream_t)stream;
+  const int rc2 = d <= 64 ? launch_prompt_h<64>(p, st) : d <= 128 ? launch_prompt_h<128>(p, st) : launch_prompt_h<256>(p, st);
+  if (rc2) return rc2;
+  EXO_CHECK_LAUNCH("exo_paged_attn_prompt");
+  return EXO_OK;
+}

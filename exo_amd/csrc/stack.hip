@@ -1,0 +1,470 @@
+// Small operators of a layer-list decoder with a float32 residual stream: embedding rows,
+// normalisation of a sublayer's OUTPUT before it is added, routing with a choice correction and
+// identity experts, and the expert products of a decode step.  Element type bf16 or float
+// (dense.h); every norm, router and sum here is float32.
+#include "../../include/exo_mi355x.h"
+#include "dense.h"
+
+namespace {
+
+constexpr int kRowThreads = 256;
+
+// sum over a workgroup of kRowThreads threads, in every thread
+__device__ __forceinline__ float block_sum(float v, float* tmp) {
+  v = wave_sum(v);
+  const int wave = threadIdx.x >> 6;
+  __syncthreads();  // (tmp may still be read from an earlier call)
+  if ((threadIdx.x & 63) == 0) tmp[wave] = v;
+  __syncthreads();
+  float s = 0.f;
+#pragma unroll
+  for (int w = 0; w < kRowThreads / 64; ++w) s += tmp[w];
+  return s;
+}
+
+// ------------------------------------------------------------------------------ embedding
+template <typename T>
+__global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const T* __restrict__ table, float* __restrict__ x,
+                                  T* __restrict__ xb, int V, int H, int ldt, int ldx) {
+  const int row = blockIdx.x;
+  const int id = min(max(ids[row], 0), V - 1);
+  for (int c = threadIdx.x; c < H; c += blockDim.x) {
+    const T v = table[(size_t)id * ldt + c];
+    x[(size_t)row * H + c] = Elem<T>::load(v);
+    xb[(size_t)row * ldx + c] = v;
+  }
+}
+
+// ------------------------------------------------------------------------------ norms
+// y = x / rms(x) * gain, rows given by an index list (null: row i)
+template <typename T>
+__global__ __launch_bounds__(kRowThreads) void norm_rows_kernel(const float* __restrict__ x,
+                                                                const int32_t* __restrict__ rows,
+                                                                const float* __restrict__ gain, T* __restrict__ y,
+                                                                int H, int ldy, float eps) {
+  __shared__ float tmp[kRowThreads / 64];
+  const float* xr = x + (size_t)(rows ? rows[blockIdx.x] : (int)blockIdx.x) * H;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < H; c += kRowThreads) ss += xr[c] * xr[c];
+  const float inv = 1.f / sqrtf(block_sum(ss, tmp) / H + eps);
+  for (int c = threadIdx.x; c < H; c += kRowThreads)
+    y[(size_t)blockIdx.x * ldy + c] = Elem<T>::make(xr[c] * inv * gain[c]);
+}
+
+struct MoeSum {        // the feed-forward's output as a sum over a token's experts
+  const void* y;       // T [R][top][ldy] expert outputs (null: `branch` holds the sum already)
+  const int32_t* idx;  // [R][top]
+  const float* wt;     // [R][top]
+  const void* shared;  // T [R][lds] output of the shared expert, or null
+  const float* logits; // router logits; column E + identity is the shared expert's gate
+  int top, experts, ldy, lds, ldl, gate_col;
+};
+
+// x += gain * v / rms(v), v = the branch row (or the weighted sum over the experts); xb = x
+template <typename T>
+__global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const float* __restrict__ branch, int ldb,
+                                                                    const MoeSum m, const float* __restrict__ gain,
+                                                                    float* __restrict__ x, T* __restrict__ xb, int H,
+                                                                    int ldx, float eps) {
+  extern __shared__ float v[];  // [H]
+  __shared__ float tmp[kRowThreads / 64];
+  const int row = blockIdx.x;
+  float* xr = x + (size_t)row * H;
+  float ss = 0.f;
+  if (m.y) {
+    const T* y = reinterpret_cast<const T*>(m.y) + (size_t)row * m.top * m.ldy;
+    const T* sh = m.shared ? reinterpret_cast<const T*>(m.shared) + (size_t)row * m.lds : nullptr;
+    float pass = 0.f, sg = 0.f;  // weight of the input itself; gate of the shared expert
+    for (int j = 0; j < m.top; ++j)
+      if (m.idx[row * m.top + j] >= m.experts) pass += m.wt[row * m.top + j];
+    if (sh) sg = 1.f / (1.f + expf(-m.logits[(size_t)row * m.ldl + m.gate_col]));
+    for (int c = threadIdx.x; c < H; c += kRowThreads) {
+      float s = pass * xr[c];
+      for (int j = 0; j < m.top; ++j)
+        if (m.idx[row * m.top + j] < m.experts) s += m.wt[row * m.top + j] * Elem<T>::load(y[(size_t)j * m.ldy + c]);
+      if (sh) s += sg * Elem<T>::load(sh[c]);
+      v[c] = s;
+      ss += s * s;
+    }
+  } else {
+    for (int c = threadIdx.x; c < H; c += kRowThreads) {
+      const float s = branch[(size_t)row * ldb + c];
+      v[c] = s;
+      ss += s * s;
+    }
+  }
+  const float inv = 1.f / sqrtf(block_sum(ss, tmp) / H + eps);
+  for (int c = threadIdx.x; c < H; c += kRowThreads) {
+    const float s = xr[c] + v[c] * inv * gain[c];
+    xr[c] = s;
+    xb[(size_t)row * ldx + c] = Elem<T>::make(s);
+  }
+}
+
+// ------------------------------------------------------------------------------ routing
+// One wave per token: softmax over all N outputs, the `top` largest of score + correction (equals:
+// the lower index), weight = score * scale.
+constexpr int kRouteRegs = 8;  // N <= 512
+__device__ __forceinline__ void route_choose(const float* __restrict__ logits, const float* __restrict__ corr, int N,
+                                             int top, float scale, int lane, int& my_id, float& my_wt) {
+  float s[kRouteRegs], c[kRouteRegs];
+  float mx = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < kRouteRegs; ++i) {
+    const int e = min(lane + 64 * i, N - 1);
+    s[i] = logits[e];
+    c[i] = corr[e];
+  }
+#pragma unroll
+  for (int i = 0; i < kRouteRegs; ++i) {
+    if (lane + 64 * i >= N) s[i] = -INFINITY;
+    mx = fmaxf(mx, s[i]);
+  }
+  mx = wave_max(mx);
+  float sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < kRouteRegs; ++i) {
+    s[i] = expf(s[i] - mx);
+    sum += s[i];
+  }
+  sum = wave_sum(sum);
+#pragma unroll
+  for (int i = 0; i < kRouteRegs; ++i) {
+    s[i] = s[i] / sum;
+    c[i] = lane + 64 * i < N ? s[i] + c[i] : -INFINITY;
+  }
+  my_id = 0;
+  my_wt = 0.f;
+  for (int j = 0; j < top; ++j) {
+    float best = c[0];
+    int bi = 0;
+#pragma unroll
+    for (int i = 1; i < kRouteRegs; ++i)
+      if (c[i] > best) best = c[i], bi = i;
+    int be = lane + 64 * bi;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ov = __shfl_xor(best, o, 64);
+      const int oe = __shfl_xor(be, o, 64);
+      if (ov > best || (ov == best && oe < be)) best = ov, be = oe;
+    }
+    const int owner = be & 63, reg = be >> 6;
+    float sv = 0.f;
+#pragma unroll
+    for (int i = 0; i < kRouteRegs; ++i)
+      if (i == reg) {
+        sv = s[i];
+        if (lane == owner) c[i] = -INFINITY;
+      }
+    sv = __shfl(sv, owner, 64);
+    if (lane == j) my_id = be, my_wt = sv * scale;
+  }
+}
+
+__global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ logits, const float* __restrict__ corr,
+                                                       int32_t* __restrict__ idx, float* __restrict__ wt, int N, int ldl,
+                                                       int top, float scale) {
+  const int row = blockIdx.x, lane = threadIdx.x;
+  int id;
+  float w;
+  route_choose(logits + (size_t)row * ldl, corr, N, top, scale, lane, id, w);
+  if (lane < top) {
+    idx[(size_t)row * top + lane] = id;
+    wt[(size_t)row * top + lane] = w;
+  }
+}
+
+// ------------------------------------------------------------------------------ experts, decode
+// A decode step's (token, expert) pairs, weights streamed once per pair: 16 output rows per
+// workgroup, K over its waves, as dense_gemv_kernel.
+struct MoeRows {
+  const void* x;       // T [R][ldx]
+  const void *gate, *up, *down;     // experts: [E][ff][ldx], [E][H][lda]
+  const void *sgate, *sup, *sdown;  // the shared expert, or null
+  void* act;           // T [R][top][lda]
+  void* sact;          // T [R][ldsa]
+  float* out;          // [R][H]
+  const float* xres;   // [R][H] the sublayer's input (identity experts)
+  int32_t* idx;        // [R][top]
+  float* wt;
+  const float* logits; // [R][ldl]
+  int R, top, experts, ff, sff, H, ldx, lda, ldsa, ldl, gate_col;
+  GluConst glu, sglu;
+};
+
+constexpr int kBatch = 4;
+constexpr int kGuWaves = 4;
+
+template <typename T>
+__global__ __launch_bounds__(64 * kGuWaves) void moe_glu_rows_kernel(const MoeRows p) {
+  __shared__ float red[kGuWaves][2][256];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int tiles = (p.ff + 15) / 16, pairs = p.R * p.top;
+  int b = blockIdx.x, rows, N, ldo, tok0;
+  const char *wg, *wu;
+  T* out;
+  GluConst glu;
+  const uint32_t row_b = (uint32_t)p.ldx * sizeof(T);
+  if (b < pairs * tiles) {
+    const int pair = b / tiles;
+    const int e = p.idx[pair];
+    if (e >= p.experts) return;  // whole workgroup: the input itself, nothing to multiply
+    b -= pair * tiles;
+    const size_t off = (size_t)e * p.ff * row_b;
+    wg = reinterpret_cast<const char*>(p.gate) + off;
+    wu = reinterpret_cast<const char*>(p.up) + off;
+    tok0 = pair / p.top;
+    rows = 1;
+    N = p.ff;
+    out = reinterpret_cast<T*>(p.act) + (size_t)pair * p.lda;
+    ldo = p.lda;
+    glu = p.glu;
+  } else {
+    b -= pairs * tiles;
+    wg = reinterpret_cast<const char*>(p.sgate);
+    wu = reinterpret_cast<const char*>(p.sup);
+    tok0 = 0;
+    rows = p.R;
+    N = p.sff;
+    out = reinterpret_cast<T*>(p.sact);
+    ldo = p.ldsa;
+    glu = p.sglu;
+  }
+  const int n0 = b * 16, nrows = min(16, N - n0);
+  const __amdgpu_buffer_rsrc_t rg = buf_of(wg + (size_t)n0 * row_b, (uint32_t)nrows * row_b);
+  const __amdgpu_buffer_rsrc_t ru = buf_of(wu + (size_t)n0 * row_b, (uint32_t)nrows * row_b);
+  const __amdgpu_buffer_rsrc_t rx =
+      buf_of(reinterpret_cast<const char*>(p.x) + (size_t)tok0 * row_b, (uint32_t)rows * row_b);
+  const int steps = (int)(row_b >> 6), per = (steps + kGuWaves - 1) / kGuWaves;
+  const int s0 = min(steps, wave * per), s1 = min(steps, s0 + per);
+  const uint32_t off = r * row_b + g * 16;
+  floatx4 ag = {0.f, 0.f, 0.f, 0.f}, au = {0.f, 0.f, 0.f, 0.f};
+  for (int s = s0; s < s1; s += kBatch) {
+    uint4 gv[kBatch], uv[kBatch], xv[kBatch];
+#pragma unroll
+    for (int i = 0; i < kBatch; ++i) {
+      const uint32_t o = s + i < s1 ? off + (s + i) * 64 : kPastEnd;
+      gv[i] = buf_load16(rg, o, 0);
+      uv[i] = buf_load16(ru, o, 0);
+      xv[i] = buf_load16(rx, o, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < kBatch; ++i) {
+      ag = Elem<T>::mma16(gv[i], xv[i], ag);
+      au = Elem<T>::mma16(uv[i], xv[i], au);
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    red[wave][0][r * 16 + 4 * g + e] = ag[e];
+    red[wave][1][r * 16 + 4 * g + e] = au[e];
+  }
+  __syncthreads();
+  for (int o = threadIdx.x; o < 16 * rows; o += 64 * kGuWaves) {
+    const int m = o >> 4, n = o & 15;
+    if (n >= nrows) continue;
+    float gs = 0.f, us = 0.f;
+#pragma unroll
+    for (int w = 0; w < kGuWaves; ++w) gs += red[w][0][o], us += red[w][1][o];
+    out[(size_t)m * ldo + n0 + n] = Elem<T>::make(clamped_glu(gs, us, glu));
+  }
+}
+
+constexpr int kDnWaves = 8;
+
+// out[t] = sum of weight * (down @ act) over the token's experts, + gate * shared, + weight * input
+template <typename T>
+__global__ __launch_bounds__(64 * kDnWaves) void moe_down_rows_kernel(const MoeRows p) {
+  __shared__ float red[kDnWaves][16];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int t = blockIdx.y, n0 = blockIdx.x * 16, nrows = min(16, p.H - n0);
+  const uint32_t arow = (uint32_t)p.lda * sizeof(T), srow = (uint32_t)p.ldsa * sizeof(T);
+  const int es = (int)(arow >> 6), ss = p.sdown ? (int)(srow >> 6) : 0;  // steps per expert, shared
+  const int units = p.top * es + ss, per = (units + kDnWaves - 1) / kDnWaves;
+  int u = min(units, wave * per);
+  const int u1 = min(units, u + per);
+  float tot[4] = {0.f, 0.f, 0.f, 0.f};
+  while (u < u1) {  // the part of one expert's K range that falls into this wave's share
+    const int slot = min(u / es, p.top);
+    const bool sh = slot == p.top;
+    const int base = slot * es, lim = sh ? ss : es;
+    const int s0 = u - base, s1 = min(lim, u1 - base);
+    u = base + s1;
+    float wt;
+    const char *w, *a;
+    uint32_t rowb;
+    if (sh) {
+      wt = 1.f / (1.f + expf(-p.logits[(size_t)t * p.ldl + p.gate_col]));
+      w = reinterpret_cast<const char*>(p.sdown);
+      a = reinterpret_cast<const char*>(p.sact) + (size_t)t * srow;
+      rowb = srow;
+    } else {
+      const int e = p.idx[t * p.top + slot];
+      if (e >= p.experts) continue;
+      wt = p.wt[t * p.top + slot];
+      w = reinterpret_cast<const char*>(p.down) + (size_t)e * p.H * arow;
+      a = reinterpret_cast<const char*>(p.act) + (size_t)(t * p.top + slot) * arow;
+      rowb = arow;
+    }
+    const __amdgpu_buffer_rsrc_t rw = buf_of(w + (size_t)n0 * rowb, (uint32_t)nrows * rowb);
+    const __amdgpu_buffer_rsrc_t rx = buf_of(a, rowb);
+    floatx4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int s = s0; s < s1; s += kBatch) {
+      uint4 wv[kBatch], xv[kBatch];
+#pragma unroll
+      for (int i = 0; i < kBatch; ++i) {
+        const bool ok = s + i < s1;
+        wv[i] = buf_load16(rw, ok ? r * rowb + g * 16 + (s + i) * 64 : kPastEnd, 0);
+        xv[i] = buf_load16(rx, ok ? g * 16 + (s + i) * 64 : kPastEnd, 0);  // every column: the one row
+      }
+#pragma unroll
+      for (int i = 0; i < kBatch; ++i) acc = Elem<T>::mma16(wv[i], xv[i], acc);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) tot[e] = fmaf(wt, acc[e], tot[e]);
+  }
+  if (r == 0) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) red[wave][4 * g + e] = tot[e];
+  }
+  __syncthreads();
+  if (threadIdx.x < (unsigned)nrows) {
+    const int n = threadIdx.x;
+    float v = 0.f;
+#pragma unroll
+    for (int w = 0; w < kDnWaves; ++w) v += red[w][n];
+    float pass = 0.f;
+    for (int j = 0; j < p.top; ++j)
+      if (p.idx[t * p.top + j] >= p.experts) pass += p.wt[t * p.top + j];
+    if (pass != 0.f) v += pass * p.xres[(size_t)t * p.H + n0 + n];
+    p.out[(size_t)t * p.H + n0 + n] = v;
+  }
+}
+
+}  // namespace
+
+#define EXO_TYPE_OK(what) EXO_REQUIRE(dtype == 0 || dtype == 1, what ": dtype must be 0 (bf16) or 1 (float32)")
+#define EXO_LAUNCH_T(kernel, grid, block, lds, ...)                                  \
+  do {                                                                               \
+    if (dtype == 0)                                                                  \
+      kernel<bf16_t><<<grid, block, lds, (hipStream_t)stream>>>(__VA_ARGS__);        \
+    else                                                                             \
+      kernel<float><<<grid, block, lds, (hipStream_t)stream>>>(__VA_ARGS__);         \
+  } while (0)
+
+extern "C" int exo_embed_rows(const int32_t* ids, const void* table, float* x, void* xb, int n, int V, int H, int ldt,
+                              int ldx, int dtype, exo_stream_t stream) {
+  EXO_TYPE_OK("exo_embed_rows");
+  EXO_REQUIRE(ids && table && x && xb && n >= 0 && V > 0 && H > 0 && ldt >= H && ldx >= H, "exo_embed_rows: bad argument");
+  if (n == 0) return EXO_OK;
+  if (dtype == 0)
+    embed_rows_kernel<bf16_t><<<n, 256, 0, (hipStream_t)stream>>>(ids, (const bf16_t*)table, x, (bf16_t*)xb, V, H, ldt, ldx);
+  else
+    embed_rows_kernel<float><<<n, 256, 0, (hipStream_t)stream>>>(ids, (const float*)table, x, (float*)xb, V, H, ldt, ldx);
+  EXO_CHECK_LAUNCH("exo_embed_rows");
+  return EXO_OK;
+}
+
+extern "C" int exo_norm_rows(const float* x, const int32_t* rows, const float* gain, void* y, int n, int H, int ldy,
+                             float eps, int dtype, exo_stream_t stream) {
+  EXO_TYPE_OK("exo_norm_rows");
+  EXO_REQUIRE(x && gain && y && n >= 0 && H > 0 && ldy >= H, "exo_norm_rows: bad argument");
+  if (n == 0) return EXO_OK;
+  if (dtype == 0)
+    norm_rows_kernel<bf16_t><<<n, kRowThreads, 0, (hipStream_t)stream>>>(x, rows, gain, (bf16_t*)y, H, ldy, eps);
+  else
+    norm_rows_kernel<float><<<n, kRowThreads, 0, (hipStream_t)stream>>>(x, rows, gain, (float*)y, H, ldy, eps);
+  EXO_CHECK_LAUNCH("exo_norm_rows");
+  return EXO_OK;
+}
+
+static int post_norm(const float* branch, int ldb, const MoeSum& m, const float* gain, float* x, void* xb, int n, int H,
+                     int ldx, float eps, int dtype, exo_stream_t stream) {
+  EXO_REQUIRE(gain && x && xb && n >= 0 && H > 0 && H <= 16000 && ldx >= H, "exo_post_norm_add: bad argument (H=%d)", H);
+  if (n == 0) return EXO_OK;
+  const size_t lds = (size_t)H * 4;
+  if (dtype == 0)
+    post_norm_add_kernel<bf16_t><<<n, kRowThreads, lds, (hipStream_t)stream>>>(branch, ldb, m, gain, x, (bf16_t*)xb, H, ldx, eps);
+  else
+    post_norm_add_kernel<float><<<n, kRowThreads, lds, (hipStream_t)stream>>>(branch, ldb, m, gain, x, (float*)xb, H, ldx, eps);
+  EXO_CHECK_LAUNCH("exo_post_norm_add");
+  return EXO_OK;
+}
+
+extern "C" int exo_post_norm_add(const float* branch, int ldb, const float* gain, float* x, void* xb, int n, int H,
+                                 int ldx, float eps, int dtype, exo_stream_t stream) {
+  EXO_TYPE_OK("exo_post_norm_add");
+  EXO_REQUIRE(branch && ldb >= H, "exo_post_norm_add: bad branch");
+  return post_norm(branch, ldb, MoeSum{}, gain, x, xb, n, H, ldx, eps, dtype, stream);
+}
+
+extern "C" int exo_moe_sum_post_norm(const void* y, const int32_t* idx, const float* wt, const void* shared,
+                                     const float* logits, int top, int experts, int ldy, int lds, int ldl, int gate_col,
+                                     const float* gain, float* x, void* xb, int n, int H, int ldx, float eps, int dtype,
+                                     exo_stream_t stream) {
+  EXO_TYPE_OK("exo_moe_sum_post_norm");
+  EXO_REQUIRE(y && idx && wt && top > 0 && experts > 0 && ldy >= H && (!shared || (logits && lds >= H && gate_col < ldl)),
+              "exo_moe_sum_post_norm: bad argument");
+  return post_norm(nullptr, 0, MoeSum{y, idx, wt, shared, logits, top, experts, ldy, lds, ldl, gate_col}, gain, x, xb, n,
+                   H, ldx, eps, dtype, stream);
+}
+
+extern "C" int exo_moe_route(const float* logits, const float* correction, int32_t* idx, float* wt, int rows, int n,
+                             int ldl, int top, float scale, exo_stream_t stream) {
+  EXO_REQUIRE(logits && correction && idx && wt, "exo_moe_route: null pointer");
+  EXO_REQUIRE(rows >= 0 && n > 0 && n <= 64 * kRouteRegs && ldl >= n && top > 0 && top <= 64 && top <= n,
+              "exo_moe_route: need 0 < n <= %d and 0 < top <= min(64, n); got n=%d top=%d", 64 * kRouteRegs, n, top);
+  if (rows == 0) return EXO_OK;
+  moe_route_kernel<<<rows, 64, 0, (hipStream_t)stream>>>(logits, correction, idx, wt, n, ldl, top, scale);
+  EXO_CHECK_LAUNCH("exo_moe_route");
+  return EXO_OK;
+}
+
+static MoeRows moe_rows_of(const exo_moe_rows* a) {
+  MoeRows p{};
+  p.x = a->x, p.gate = a->gate, p.up = a->up, p.down = a->down;
+  p.sgate = a->shared_gate, p.sup = a->shared_up, p.sdown = a->shared_down;
+  p.act = a->act, p.sact = a->shared_act, p.out = a->out, p.xres = a->x_res;
+  p.idx = a->idx, p.wt = a->wt, p.logits = a->logits;
+  p.R = a->rows, p.top = a->top, p.experts = a->experts, p.ff = a->ff, p.sff = a->shared_ff, p.H = a->H;
+  p.ldx = a->ldx, p.lda = a->lda, p.ldsa = a->ldsa, p.ldl = a->ldl, p.gate_col = a->gate_col;
+  p.glu = GluConst{a->limit, a->alpha, a->shift};
+  p.sglu = GluConst{a->shared_limit, a->shared_alpha, a->shared_shift};
+  return p;
+}
+static int moe_rows_check(const exo_moe_rows* a) {
+  EXO_REQUIRE(a && (a->dtype == 0 || a->dtype == 1), "exo_moe_rows: bad dtype");
+  EXO_REQUIRE(a->rows > 0 && a->rows <= 16 && a->top > 0 && a->experts > 0 && a->ff > 0 && a->H > 0,
+              "exo_moe_rows: need 1..16 rows and positive sizes (rows=%d)", a->rows);
+  EXO_REQUIRE(a->ldx % 64 == 0 && a->lda % 64 == 0 && a->ldx >= a->H && a->lda >= a->ff,
+              "exo_moe_rows: row strides must be multiples of 64 (ldx=%d lda=%d)", a->ldx, a->lda);
+  EXO_REQUIRE(a->x && a->gate && a->up && a->down && a->act && a->out && a->x_res && a->idx && a->wt,
+              "exo_moe_rows: null pointer");
+  EXO_REQUIRE(!a->shared_gate || (a->shared_up && a->shared_down && a->shared_act && a->logits && a->shared_ff > 0 &&
+                                  a->ldsa % 64 == 0 && a->ldsa >= a->shared_ff && a->gate_col < a->ldl),
+              "exo_moe_rows: incomplete shared expert");
+  return EXO_OK;
+}
+
+extern "C" int exo_moe_glu_rows(const exo_moe_rows* a, exo_stream_t stream) {
+  const int rc = moe_rows_check(a);
+  if (rc) return rc;
+  const int dtype = a->dtype;
+  const MoeRows p = moe_rows_of(a);
+  const int grid = p.R * p.top * exo_ceil_div(p.ff, 16) + (p.sgate ? exo_ceil_div(p.sff, 16) : 0);
+  EXO_LAUNCH_T(moe_glu_rows_kernel, grid, 64 * kGuWaves, 0, p);
+  EXO_CHECK_LAUNCH("exo_moe_glu_rows");
+  return EXO_OK;
+}
+
+extern "C" int exo_moe_down_rows(const exo_moe_rows* a, exo_stream_t stream) {
+  const int rc = moe_rows_check(a);
+  if (rc) return rc;
+  const int dtype = a->dtype;
+  const MoeRows p = moe_rows_of(a);
+  EXO_LAUNCH_T(moe_down_rows_kernel, dim3(exo_ceil_div(p.H, 16), p.R), 64 * kDnWaves, 0, p);
+  EXO_CHECK_LAUNCH("exo_moe_down_rows");
+  return EXO_OK;
+}

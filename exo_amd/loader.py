@@ -19,6 +19,7 @@ from pathlib import Path
 import torch
 
 from .config import ModelConfig
+from .stack_config import StackConfig
 
 
 def layer_index_of(key: str) -> int | None:
@@ -48,7 +49,9 @@ def _checkpoint_files(model_dir: Path) -> dict[str, Path]:
     return out
 
 
-def wanted(key: str, cfg: ModelConfig, start_layer: int, end_layer: int) -> bool:
+def wanted(key: str, cfg: ModelConfig | StackConfig, start_layer: int, end_layer: int) -> bool:
+    if isinstance(cfg, StackConfig):
+        return cfg.wants(key, start_layer, end_layer)
     li = layer_index_of(key)
     if li is not None:
         return start_layer <= li < end_layer
@@ -61,7 +64,7 @@ def wanted(key: str, cfg: ModelConfig, start_layer: int, end_layer: int) -> bool
 
 
 def load_shard_weights(
-    model_dir: str | Path, cfg: ModelConfig, start_layer: int, end_layer: int, device
+    model_dir: str | Path, cfg: ModelConfig | StackConfig, start_layer: int, end_layer: int, device
 ) -> Generator[tuple[int, int], None, dict[str, torch.Tensor]]:
     """Generator: yields (layers_loaded, total_layers) after each local layer is
     resident (the reference's ModelLoadingResponse cadence, runner.py:263-269) and
@@ -75,8 +78,10 @@ def load_shard_weights(
         raise ValueError(f"checkpoint at {model_dir} holds no tensor of layers "
                          f"[{start_layer},{end_layer})")
 
+    layer_of = cfg.layer_of if isinstance(cfg, StackConfig) else layer_index_of
+
     def order(k: str):
-        li = layer_index_of(k)
+        li = layer_of(k)
         return (0, 0, k) if li is None else (1, li, k)
 
     keys.sort(key=order)
@@ -86,7 +91,7 @@ def load_shard_weights(
     done_layer = None
     try:
         for k in keys:
-            li = layer_index_of(k)
+            li = layer_of(k)
             if li is not None and done_layer is not None and li != done_layer:
                 yield (done_layer - start_layer + 1, total)
             if li is not None:

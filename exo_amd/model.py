@@ -151,7 +151,98 @@ class _Buffers:
         self.argmax_ws = ops.argmax_workspace(B, device)
 
 
-class ShardModel:
+class DecoderShard:
+    """What every model class of this engine shares: the layer range it owns and the
+    single-token step captured into HIP graphs.  A subclass provides ``_buffers(B, T)``
+    (``tokens``, ``h``, ``logits``, ``next_token``, ...), ``_run(B, T, cache, bf, logits_mode,
+    rows)`` - the launches of a forward - and ``_keys_hint(cache, rows)``, the context regime its
+    launches are laid out for."""
+
+    cfg: ModelConfig
+    start_layer: int
+    end_layer: int
+    _graphs: dict[tuple, tuple]
+
+    @property
+    def is_first(self) -> bool:
+        return self.start_layer == 0
+
+    @property
+    def is_last(self) -> bool:
+        return self.end_layer == self.cfg.num_hidden_layers
+
+    def _sampling_logits(self, logits: torch.Tensor, bf) -> torch.Tensor:
+        """The bf16 logits that the sampling kernels read."""
+        return logits
+
+    # ------------------------------------------------------------------ graph decode
+    def decode_step(self, cache: ShardKVCache, B: int, use_graph: bool = True,
+                    feedback: bool = False, sampler=None, mode: int = 0, row0: int = 0) -> _Buffers:
+        """One single-token step for cache rows [row0, row0+B): reads ``bufs.tokens`` (first shard)
+        or ``bufs.h``, leaves logits / next_token / lse / logprob (last shard) or the
+        hidden state in the returned buffers, advances the device positions.  The kernel
+        sequence is captured once per B into a HIP graph and replayed.  ``feedback``
+        (last shard): the graph also writes the chosen token into ``tokens``, so steps
+        can be chained without the host.  ``sampler`` (a DeviceSampler, last shard): the step
+        ends in the device sampling kernels with the stages ``mode`` names instead of the
+        plain argmax; results are then in the sampler's ``token`` / ``logprob`` / ``top_*``."""
+        bf = self._buffers(B, 1)
+        rsl = slice(row0, row0 + B)
+        if row0 < 0 or row0 + B > cache.batch:
+            raise ValueError(f"rows [{row0}, {row0 + B}) outside the cache's {cache.batch} rows")
+        cache.reserve(range(row0, row0 + B), 1)
+        if sampler is not None and not self.is_last:
+            raise ValueError("sampling needs the shard that holds the lm_head")
+        if sampler is not None and row0 != 0:
+            raise ValueError("the sampling state is indexed by cache row: row0 must be 0 with a sampler")
+
+        def body():
+            out = self._run(B, 1, cache, bf, "all", rsl if row0 else None)
+            if self.is_last and sampler is not None:
+                sampler.sample(self._sampling_logits(out, bf), B, mode, feedback=bf.tokens if feedback else None,
+                               pos_inc=cache.pos[rsl])
+            elif self.is_last:
+                ops.argmax_logsumexp(self._sampling_logits(out, bf), bf.next_token, bf.lse, bf.logprob, bf.argmax_ws,
+                                     cache.pos[rsl])
+                if feedback:
+                    bf.tokens.copy_(bf.next_token)
+            else:
+                cache.pos[rsl] += 1
+
+        if not use_graph:
+            body()
+        else:
+            key = (B, feedback, sampler is not None, mode, row0, self._keys_hint(cache, rsl))
+            hit = self._graphs.get(key)
+            if hit is None or hit[1] is not cache or hit[2] is not sampler:
+                # warm up outside capture (lazy module loads, attribute settings), then
+                # restore what the warm-up changed: the positions it advanced, the hidden
+                # state a later shard adds its residuals into in place, the input tokens
+                # the feedback overwrote, the sampler's counters and history ring
+                saved = cache.pos.clone()
+                saved_in = bf.tokens.clone() if self.is_first else bf.h.clone()
+                saved_sampler = sampler.snapshot() if sampler is not None else None
+                s = torch.cuda.Stream()
+                s.wait_stream(torch.cuda.current_stream())
+                with torch.cuda.stream(s):
+                    body()
+                torch.cuda.current_stream().wait_stream(s)
+                torch.cuda.synchronize()
+                cache.pos.copy_(saved)
+                (bf.tokens if self.is_first else bf.h).copy_(saved_in)
+                if sampler is not None:
+                    sampler.restore(saved_sampler)
+                g = torch.cuda.CUDAGraph()
+                with capture_graph(g):
+                    body()
+                cache.pos.copy_(saved)
+                self._graphs[key] = (g, cache, sampler)
+            self._graphs[key][0].replay()
+        cache.advance_host(1, range(row0, row0 + B))
+        return bf
+
+
+class ShardModel(DecoderShard):
     def __init__(self, cfg: ModelConfig, weights: dict[str, torch.Tensor], start_layer: int = 0,
                  end_layer: int | None = None, device="cuda:0"):
         self.cfg = cfg
@@ -178,15 +269,6 @@ class ShardModel:
         self._graphs: dict[int, tuple] = {}
         self._rope_tab: torch.Tensor | None = None
         self._retired_rope_tabs: list[torch.Tensor] = []
-
-    # ------------------------------------------------------------------ properties
-    @property
-    def is_first(self) -> bool:
-        return self.start_layer == 0
-
-    @property
-    def is_last(self) -> bool:
-        return self.end_layer == self.cfg.num_hidden_layers
 
     def _rope_table(self, n: int) -> torch.Tensor:
         """(cos, sin) table covering n positions, built once on the device."""
@@ -357,70 +439,3 @@ class ShardModel:
         if self.is_last and logits != "none":
             return out.view(B, -1, self.cfg.vocab_size).clone()
         return out.view(B, T, -1).clone()
-
-    # ------------------------------------------------------------------ graph decode
-    def decode_step(self, cache: ShardKVCache, B: int, use_graph: bool = True,
-                    feedback: bool = False, sampler=None, mode: int = 0, row0: int = 0) -> _Buffers:
-        """One single-token step for cache rows [row0, row0+B): reads ``bufs.tokens`` (first shard)
-        or ``bufs.h``, leaves logits / next_token / lse / logprob (last shard) or the
-        hidden state in the returned buffers, advances the device positions.  The kernel
-        sequence is captured once per B into a HIP graph and replayed.  ``feedback``
-        (last shard): the graph also writes the chosen token into ``tokens``, so steps
-        can be chained without the host.  ``sampler`` (a DeviceSampler, last shard): the step
-        ends in the device sampling kernels with the stages ``mode`` names instead of the
-        plain argmax; results are then in the sampler's ``token`` / ``logprob`` / ``top_*``."""
-        bf = self._buffers(B, 1)
-        rsl = slice(row0, row0 + B)
-        if row0 < 0 or row0 + B > cache.batch:
-            raise ValueError(f"rows [{row0}, {row0 + B}) outside the cache's {cache.batch} rows")
-        if max(cache.offsets[rsl]) + 1 > cache.max_seq:
-            raise ValueError("KV cache overflow")
-        if sampler is not None and not self.is_last:
-            raise ValueError("sampling needs the shard that holds the lm_head")
-        if sampler is not None and row0 != 0:
-            raise ValueError("the sampling state is indexed by cache row: row0 must be 0 with a sampler")
-
-        def body():
-            out = self._run(B, 1, cache, bf, "all", rsl if row0 else None)
-            if self.is_last and sampler is not None:
-                sampler.sample(out, B, mode, feedback=bf.tokens if feedback else None,
-                               pos_inc=cache.pos[rsl])
-            elif self.is_last:
-                ops.argmax_logsumexp(out, bf.next_token, bf.lse, bf.logprob, bf.argmax_ws,
-                                     cache.pos[rsl])
-                if feedback:
-                    bf.tokens.copy_(bf.next_token)
-            else:
-                cache.pos[rsl] += 1
-
-        if not use_graph:
-            body()
-        else:
-            key = (B, feedback, sampler is not None, mode, row0, self._keys_hint(cache, rsl))
-            hit = self._graphs.get(key)
-            if hit is None or hit[1] is not cache or hit[2] is not sampler:
-                # warm up outside capture (lazy module loads, attribute settings), then
-                # restore what the warm-up changed: the positions it advanced, the hidden
-                # state a later shard adds its residuals into in place, the input tokens
-                # the feedback overwrote, the sampler's counters and history ring
-                saved = cache.pos.clone()
-                saved_in = bf.tokens.clone() if self.is_first else bf.h.clone()
-                saved_sampler = sampler.snapshot() if sampler is not None else None
-                s = torch.cuda.Stream()
-                s.wait_stream(torch.cuda.current_stream())
-                with torch.cuda.stream(s):
-                    body()
-                torch.cuda.current_stream().wait_stream(s)
-                torch.cuda.synchronize()
-                cache.pos.copy_(saved)
-                (bf.tokens if self.is_first else bf.h).copy_(saved_in)
-                if sampler is not None:
-                    sampler.restore(saved_sampler)
-                g = torch.cuda.CUDAGraph()
-                with capture_graph(g):
-                    body()
-                cache.pos.copy_(saved)
-                self._graphs[key] = (g, cache, sampler)
-            self._graphs[key][0].replay()
-        cache.advance_host(1, range(row0, row0 + B))
-        return bf

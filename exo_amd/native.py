@@ -16,6 +16,27 @@ _i = C.c_int
 _i64 = C.c_int64
 _f = C.c_float
 
+
+class MoeRows(C.Structure):
+    """struct exo_moe_rows: the experts of a decode step."""
+
+    _fields_ = [(n, _vp) for n in ("x", "gate", "up", "down", "shared_gate", "shared_up", "shared_down", "act",
+                                   "shared_act", "out", "x_res", "idx", "wt", "logits", "correction")] + \
+               [(n, _i) for n in ("rows", "top", "experts", "ff", "shared_ff", "H", "ldx", "lda", "ldsa", "ldl",
+                                  "gate_col", "dtype")] + \
+               [(n, _f) for n in ("limit", "alpha", "shift", "shared_limit", "shared_alpha", "shared_shift")]
+
+
+class PagedAttn(C.Structure):
+    """struct exo_paged_attn: one attention layer over a paged pool."""
+
+    _fields_ = [(n, _vp) for n in ("qkv", "k_pool", "v_pool", "table", "slot", "pos", "list", "slopes", "out")] + \
+               [("scale", _f), ("eps", _f)] + \
+               [(n, _i) for n in ("n", "heads", "kv_heads", "dim", "vdim", "ldq", "ldk", "ldv", "ldo", "max_pages",
+                                  "window", "keep_first", "unit_qk", "dtype")]
+
+
+
 # name -> (restype, argtypes); mirrors include/exo_mi355x.h one to one
 SIGNATURES: dict[str, tuple] = {
     "exo_abi_version": (_i, []),
@@ -64,6 +85,22 @@ SIGNATURES: dict[str, tuple] = {
     "exo_moe_combine": (_i, [_vp, _vp, _vp, _vp, _i, _i, _i, _vp]),
     "exo_argmax_workspace": (_i64, [_i]),
     "exo_argmax_logsumexp": (_i, [_vp] * 6 + [_i, _i, _vp]),
+    "exo_embed_rows": (_i, [_vp] * 4 + [_i] * 6 + [_vp]),
+    "exo_norm_rows": (_i, [_vp] * 4 + [_i] * 3 + [_f, _i, _vp]),
+    "exo_post_norm_add": (_i, [_vp, _i] + [_vp] * 3 + [_i] * 3 + [_f, _i, _vp]),
+    "exo_moe_sum_post_norm": (_i, [_vp] * 5 + [_i] * 6 + [_vp] * 3 + [_i] * 3 + [_f, _i, _vp]),
+    "exo_moe_route": (_i, [_vp] * 4 + [_i] * 4 + [_f, _vp]),
+    "exo_dense_gemv": (_i, [_vp] * 4 + [_i] * 7 + [_vp]),
+    "exo_dense_gemm": (_i, [_vp] * 4 + [_i, _vp, _i64] + [_i] * 6 + [_vp]),
+    "exo_dense_glu_gemm": (_i, [_vp] * 4 + [_f] * 3 + [_i] * 6 + [_vp]),
+    "exo_dense_grouped_gemm": (_i, [_vp] * 5 + [_f] * 3 + [_i] * 9 + [_vp]),
+    "exo_moe_glu_rows": (_i, [C.POINTER(MoeRows), _vp]),
+    "exo_moe_down_rows": (_i, [C.POINTER(MoeRows), _vp]),
+    "exo_paged_append": (_i, [C.POINTER(PagedAttn), _vp]),
+    "exo_paged_attn_workspace": (_i64, [_i] * 4),
+    "exo_paged_attn_rows": (_i, [C.POINTER(PagedAttn), _i, _i, _vp, _i64, _vp]),
+    "exo_paged_prompt_block": (_i, [_i, _i]),
+    "exo_paged_attn_prompt": (_i, [C.POINTER(PagedAttn), _vp]),
     "exo_sample_workspace": (_i64, [_i]),
     "exo_sample": (_i, [_vp] * 13 + [_i64, _i, _i, _i, _i, _vp]),
 }

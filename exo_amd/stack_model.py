@@ -1,0 +1,422 @@
+"""The forward of layer-list decoders (``stack_config``) over a paged KV pool.
+
+One step function serves everything: ``step(cache, entries)`` takes, per sequence, the cache row
+and its next tokens - a portion of a prompt, a single decoded token, or both kinds side by side in
+one batch - runs them together and returns logits at the places asked for.  ``__call__`` and
+``decode_step`` (the graph-captured single-token step) are the protocol of ``ShardModel`` on top of
+the same launches, so the engines, ``prefill`` and ``generate`` drive either model class.
+
+Precision: the residual stream, norms, routing and attention weights are float32; matrix operands
+and the cache have the model's element type - bf16 as served, or float32 throughout
+(``dtype=torch.float32``).
+
+Launches of a layer (rows R of the step):
+  R <= 16   q|k|v GEMV, attention (with norm and cache append inside when every row is a single
+            token), o GEMV, norm + residual, router GEMV, routing, gated experts + shared expert in
+            one launch, weighted down-projections in one launch, norm + residual
+  R > 16    the same with GEMMs, the experts grouped by expert, their weighted sum inside the
+            norm + residual launch; portions of prompts take the tiled attention, single tokens
+            beside them the split one
+"""
+
+from __future__ import annotations
+
+import numpy as np
+import torch
+
+from . import dense_ops as D
+from . import ops
+from .dense_ops import pad64, padded
+from .model import DecoderShard
+from .paged_cache import PagedKVCache
+from .stack_config import AttentionSpec, LayerSpec, StackConfig
+
+
+class _Layer:
+    """One layer's tensors on the device: projections concatenated, experts stacked, rows padded."""
+
+    def __init__(self, spec: LayerSpec, w: dict, i: int, H: int, dtype, device):
+        self.index, self.spec = i, spec
+        p, m, f = f"l{i}.", spec.mixer, spec.mlp
+
+        def get(name: str, *shape: int) -> torch.Tensor:
+            t = w[p + name]
+            if tuple(t.shape) != shape:
+                raise ValueError(f"{p}{name}: shape {tuple(t.shape)}, config says {shape}")
+            return t.to(device)
+
+        def mat(*parts) -> torch.Tensor:
+            return padded(torch.cat([get(*x) for x in parts]), dtype, device)
+
+        def gain(name: str) -> torch.Tensor:
+            return (1.0 + get(name, H).float()).contiguous()
+
+        outs = [("q", m.heads * m.dim)]
+        if m.kv_from is None:
+            outs += [("k", m.kv_heads * m.dim), ("v", m.kv_heads * m.vdim)]
+        self.qkv = mat(*((f"mix.{n}", rows, H) for n, rows in outs))
+        self.o = mat(("mix.o", H, m.heads * m.vdim))
+        self.qkv_b = self.o_b = None
+        if m.bias:
+            self.qkv_b = torch.cat([get(f"mix.{n}.b", rows) for n, rows in outs]).float().contiguous()
+            self.o_b = get("mix.o.b", H).float().contiguous()
+        self.slopes = None if m.slopes is None else torch.tensor(m.slopes, dtype=torch.float32, device=device)
+        self.norm1 = gain("norm1")
+        self.norm2 = self.router = None
+        if f is None:
+            return
+        self.norm2 = gain("norm2")
+        r, ff = f.router, f.expert.ff
+
+        def stack(name: str, n: int, k: int) -> torch.Tensor:
+            out = torch.zeros(r.experts, n, pad64(k), dtype=dtype, device=device)
+            for e in range(r.experts):
+                out[e, :, :k].copy_(get(f"mlp.e{e}.{name}", n, k))
+            return out
+
+        self.gate, self.up, self.down = stack("gate", ff, H), stack("up", ff, H), stack("down", H, ff)
+        self.correction = get("mlp.correction", r.outputs).float().contiguous()
+        # the shared expert's gate is one more output of the router product
+        rows = [("mlp.router", r.outputs, H)]
+        self.s_gate = self.s_up = self.s_down = None
+        if f.shared is not None:
+            rows.append(("mlp.shared.sg", 1, H))
+            self.s_gate, self.s_up = mat(("mlp.shared.gate", f.shared.ff, H)), mat(("mlp.shared.up", f.shared.ff, H))
+            self.s_down = mat(("mlp.shared.down", H, f.shared.ff))
+        self.router = mat(*rows)
+
+    def tensors(self) -> list[torch.Tensor]:
+        return [t for t in vars(self).values() if isinstance(t, torch.Tensor)]
+
+
+class _Buffers:
+    """Activations of up to ``rows`` rows.  The columns between a logical size and its row stride
+    are zero for good: no kernel writes them."""
+
+    def __init__(self, model: "StackModel", rows: int, seqs: int):
+        self.model, self.cap = model, rows
+        H, dev, t = model.cfg.hidden_size, model.device, model.dtype
+        self._z = lambda *s, dtype=t: torch.zeros(*s, dtype=dtype, device=dev)  # noqa: E731
+        self._named: dict[tuple, torch.Tensor] = {}
+        self.tokens = self._z(rows, dtype=torch.int32)
+        self.h = self._z(rows, H, dtype=torch.float32)       # the residual stream
+        self.xb = self._z(rows, pad64(H))                    # its copy as matrix operand
+        self.xn = self._z(rows, pad64(H))                    # rows entering the head
+        self.branch = self._z(rows, H, dtype=torch.float32)  # a sublayer's output
+        self.experts: dict[int, D.ExpertRows] = {}
+        # outputs of a single-token step (last shard)
+        self.logits = self.logits16 = None
+        self.next_token = self._z(seqs, dtype=torch.int32)
+        self.lse = self._z(seqs, dtype=torch.float32)
+        self.logprob = self._z(seqs, dtype=torch.float32)
+        self.argmax_ws = ops.argmax_workspace(seqs, dev)
+
+    def _get(self, name: str, *shape: int, dtype=None) -> torch.Tensor:
+        key = (name, *shape)
+        if key not in self._named:
+            self._named[key] = self._z(*shape, dtype=self.model.dtype if dtype is None else dtype)
+        return self._named[key]
+
+    def qkv(self, n: int) -> torch.Tensor:
+        return self._get("qkv", self.cap, -(-n // 8) * 8)
+
+    def attn(self, n: int) -> torch.Tensor:
+        return self._get("attn", self.cap, pad64(n))
+
+    def router_logits(self, n: int) -> torch.Tensor:
+        return self._get("router", self.cap, n, dtype=torch.float32)
+
+    def idx(self, top: int) -> torch.Tensor:
+        return self._get("idx", self.cap, top, dtype=torch.int32)
+
+    def wt(self, top: int) -> torch.Tensor:
+        return self._get("wt", self.cap, top, dtype=torch.float32)
+
+    def act(self, top: int, ff: int) -> torch.Tensor:
+        return self._get(f"act{ff}", self.cap, top, pad64(ff))
+
+    def shared_act(self, ff: int) -> torch.Tensor:
+        return self._get(f"shared{ff}", self.cap, pad64(ff))
+
+    def expert_out(self, top: int) -> torch.Tensor:
+        return self._get("expert_out", self.cap, top, self.model.cfg.hidden_size)
+
+    def shared_out(self) -> torch.Tensor:
+        return self._get("shared_out", self.cap, self.model.cfg.hidden_size)
+
+
+class _Batch:
+    """What attention needs to know about the rows of a step, on the device."""
+
+    def __init__(self, rows: int, slot, pos, keys: int, single=None, n_single: int | None = None, blocks=None,
+                 want=None, n_want: int | None = None):
+        self.rows, self.slot, self.pos, self.keys = rows, slot, pos, keys
+        self.single, self.n_single = single, rows if n_single is None else n_single  # rows alone (None: all)
+        self.blocks = blocks or {}                                                   # tokens -> (list, count)
+        self.want, self.n_want = want, rows if n_want is None else n_want            # rows with logits
+
+    @property
+    def decode(self) -> bool:
+        """Every row is a single token of a sequence of its own."""
+        return self.n_single == self.rows and not self.blocks and self.single is None
+
+
+class StackModel(DecoderShard):
+    def __init__(self, cfg: StackConfig, weights: dict[str, torch.Tensor], start_layer: int = 0,
+                 end_layer: int | None = None, device="cuda:0", dtype=torch.bfloat16):
+        if dtype not in (torch.bfloat16, torch.float32):
+            raise ValueError(f"element type {dtype} not supported (bfloat16, float32)")
+        self.cfg, self.dtype, self.device = cfg, dtype, torch.device(device)
+        self.start_layer = start_layer
+        self.end_layer = cfg.num_hidden_layers if end_layer is None else end_layer
+        if not (0 <= self.start_layer < self.end_layer <= cfg.num_hidden_layers):
+            raise ValueError(f"bad layer range [{start_layer},{end_layer}) of {cfg.num_hidden_layers}")
+        H = cfg.hidden_size
+        self.layers = [_Layer(cfg.layers[i], weights, i, H, dtype, self.device)
+                       for i in range(self.start_layer, self.end_layer)]
+        # layer -> index of the pool's layer that holds its keys and values
+        self.kv_index: dict[int, int] = {}
+        self.kv_shapes: list[tuple[int, int, int]] = []
+        for L in self.layers:
+            m = L.spec.mixer
+            if m.kv_from is None:
+                self.kv_index[L.index] = len(self.kv_shapes)
+                self.kv_shapes.append((m.kv_heads, m.dim, m.vdim))
+            elif m.kv_from not in self.kv_index:
+                raise ValueError(f"layer {L.index} uses the keys of layer {m.kv_from}, which is outside the shard "
+                                 f"[{self.start_layer},{self.end_layer})")
+            else:
+                self.kv_index[L.index] = self.kv_index[m.kv_from]
+        self.embed = self.norm = self.head = None
+        if self.is_first:
+            self.embed = padded(weights["embed"].to(self.device), dtype, self.device)
+        if self.is_last:
+            self.norm = (1.0 + weights["final.norm"].to(self.device).float()).contiguous()
+            self.head = padded(weights["head"].to(self.device), dtype, self.device)
+        self._bufs: dict[tuple, _Buffers] = {}
+        self._graphs: dict[tuple, tuple] = {}
+        self._attn: tuple | None = None  # (cache, per-layer argument blocks)
+        self._row_ids: dict[tuple[int, int], torch.Tensor] = {}
+        self.layer_hook = None  # called with (layer index, residual rows) after every layer (eager steps)
+
+    # ------------------------------------------------------------------ engine protocol
+    mixed_steps = True  # portions of prompts and decoded tokens share a step
+
+    def weight_bytes(self) -> int:
+        ts = [t for L in self.layers for t in L.tensors()] + ([self.head] if self.is_last else [])
+        return sum(t.numel() * t.element_size() for t in ts)
+
+    def make_cache(self, batch: int = 1, max_seq: int = 4096, pool_tokens: int | None = None) -> PagedKVCache:
+        return PagedKVCache(self.kv_shapes, batch, max_seq, self.device, self.dtype, pool_tokens)
+
+    def _buffers(self, B: int, T: int) -> _Buffers:
+        """Activations of B x T rows: single-token steps (T = 1) have a set per batch size - a
+        captured step points at it -, everything else shares one that grows in powers of two."""
+        if T == 1:
+            key, rows = (B, 1), B
+        else:
+            key, rows = ("rows",), B * T
+        bf = self._bufs.get(key)
+        if bf is None or bf.cap < rows:
+            cap = rows if T == 1 else max(64, 1 << (rows - 1).bit_length())
+            self._bufs[key] = bf = None  # (drop the old set before the larger one is allocated)
+            self._bufs[key] = bf = _Buffers(self, cap, B)
+        return bf
+
+    @staticmethod
+    def _keys_hint(cache: PagedKVCache, rsl: slice) -> int:
+        """Upper bound (a power of two) of the keys the longest row holds after the step: launches
+        are laid out for it, and a captured step stays valid below it."""
+        return max(256, 1 << max(cache.offsets[rsl]).bit_length())
+
+    def _sampling_logits(self, logits: torch.Tensor, bf: _Buffers) -> torch.Tensor:
+        if logits.dtype == torch.bfloat16:
+            return logits
+        if bf.logits16 is None:
+            bf.logits16 = torch.empty_like(logits, dtype=torch.bfloat16)
+        bf.logits16.copy_(logits)
+        return bf.logits16
+
+    def _attention(self, cache: PagedKVCache) -> list[D.PagedAttention]:
+        if self._attn is None or self._attn[0] is not cache:
+            self._attn = (cache, [D.PagedAttention(L.spec.mixer, L.slopes, self.kv_index[L.index], cache, self.cfg.eps)
+                                  for L in self.layers])
+        return self._attn[1]
+
+    # ------------------------------------------------------------------ the launches
+    def _mixer(self, L: _Layer, att: D.PagedAttention, bf: _Buffers, b: _Batch) -> None:
+        """bf.branch <- attention of bf.xb"""
+        m: AttentionSpec = L.spec.mixer
+        n, own = b.rows, m.kv_from is None
+        qkv, out = bf.qkv(L.qkv.shape[0]), bf.attn(m.heads * m.vdim)
+        D.linear(bf.xb, L.qkv, qkv, n, bias=L.qkv_b)
+        if b.decode:
+            att.rows(qkv, out, b.slot, b.pos, n, b.keys, append=own)
+        else:
+            if own:
+                att.append(qkv, b.slot, b.pos, n)
+            if b.blocks:
+                att.prompt(qkv, out, *b.blocks[att.prompt_block(m)])
+            if b.n_single:
+                att.rows(qkv, out, b.slot, b.pos, b.n_single, b.keys, append=False, lst=b.single)
+        D.linear(out, L.o, bf.branch, n, bias=L.o_b)
+
+    def _mlp(self, L: _Layer, bf: _Buffers, n: int) -> None:
+        """residual += norm2(experts of bf.xb)"""
+        f, H = L.spec.mlp, self.cfg.hidden_size
+        r, eps = f.router, self.cfg.eps
+        logits, idx, wt = bf.router_logits(L.router.shape[0]), bf.idx(r.top), bf.wt(r.top)
+        D.linear(bf.xb, L.router, logits, n)
+        D.moe_route(logits, L.correction, r.scale, idx, wt, n)
+        if n <= D.GEMV_MAX_ROWS:
+            ex = bf.experts.get(L.index)
+            if ex is None:
+                ex = bf.experts[L.index] = D.ExpertRows(f, L, bf, H)
+            ex.glu(n)
+            ex.down(n)
+            D.post_norm_add(bf.branch, L.norm2, eps, bf.h, bf.xb, n)
+            return
+        act, out = bf.act(r.top, f.expert.ff), bf.expert_out(r.top)
+        ws = ops.moe_group(idx[:n], r.experts, check_indices=False)  # identity ids are past the end: left out
+        D.grouped_gemm(bf.xb, L.gate, ws, act, n, r.top, up=L.up, spec=f.expert)
+        D.grouped_gemm(act, L.down, ws, out, n, r.top, x_per_pair=True)
+        shared = None
+        if f.shared is not None:
+            sact, shared = bf.shared_act(f.shared.ff), bf.shared_out()
+            D.glu_gemm(bf.xb, L.s_gate, L.s_up, sact, n, f.shared)
+            D.linear(sact, L.s_down, shared, n)
+        D.moe_sum_post_norm(out, idx, wt, shared, logits, r.experts, r.outputs, L.norm2, eps, bf.h, bf.xb, n)
+
+    def _forward(self, cache: PagedKVCache, bf: _Buffers, b: _Batch, logits: bool) -> torch.Tensor:
+        """Launch the shard over the rows of ``b``: input bf.tokens (first shard) or bf.h; returns the
+        logits [n_want, V] of the wanted rows, or the residual."""
+        n, H, eps = b.rows, self.cfg.hidden_size, self.cfg.eps
+        if self.is_first:
+            D.embed_rows(bf.tokens[:n], self.embed, bf.h, bf.xb, H)
+        else:
+            bf.xb[:n, :H].copy_(bf.h[:n])
+        for L, att in zip(self.layers, self._attention(cache)):
+            self._mixer(L, att, bf, b)
+            D.post_norm_add(bf.branch, L.norm1, eps, bf.h, bf.xb, n)
+            if L.spec.mlp is not None:
+                self._mlp(L, bf, n)
+            if self.layer_hook is not None:
+                self.layer_hook(L.index, bf.h[:n])
+        if not self.is_last or not logits:
+            return bf.h[:n]
+        D.norm_rows(bf.h, self.norm, eps, bf.xn, b.n_want, rows=b.want)
+        if bf.logits is None or bf.logits.shape[0] != b.n_want:
+            bf.logits = torch.empty(b.n_want, self.cfg.vocab_size, dtype=self.dtype, device=self.device)
+            bf.logits16 = None
+        D.linear(bf.xn, self.head, bf.logits, b.n_want)
+        return bf.logits
+
+    def _run(self, B: int, T: int, cache: PagedKVCache, bf: _Buffers, logits_mode: str, rows: slice | None = None):
+        """The single-token step of cache rows ``rows`` (default the first B): positions are read on
+        the device, so a captured launch sequence can be replayed."""
+        assert T == 1
+        rsl = rows if rows is not None else slice(0, B)
+        key = (rsl.start, B)
+        if key not in self._row_ids:
+            self._row_ids[key] = torch.arange(rsl.start, rsl.start + B, dtype=torch.int32, device=self.device)
+        b = _Batch(B, self._row_ids[key], cache.pos[rsl], self._keys_hint(cache, rsl))
+        return self._forward(cache, bf, b, logits_mode != "none")
+
+    # ------------------------------------------------------------------ steps
+    def _batch(self, cache: PagedKVCache, counts: list[tuple[int, int]], want: list[int]) -> _Batch:
+        """``counts``: (cache row, tokens) per entry, in batch order; ``want``: batch rows with logits."""
+        n = sum(c for _, c in counts)
+        slot, pos, single = np.empty(n, np.int32), np.empty(n, np.int32), []
+        sizes = {D.PagedAttention.prompt_block(L.spec.mixer) for L in self.layers}
+        blocks: dict[int, list] = {s: [] for s in sizes}
+        at, keys = 0, 1
+        tiled = self.dtype == torch.bfloat16  # the 32-bit mode runs every position by itself
+        for row, c in counts:
+            p0 = cache.offsets[row]
+            slot[at : at + c] = row
+            pos[at : at + c] = np.arange(p0, p0 + c)
+            keys = max(keys, p0 + c)
+            if c == 1 or not tiled:
+                single.extend(range(at, at + c))
+            else:
+                for s in sizes:
+                    blocks[s] += [(at + o, row, p0 + o, min(s, c - o)) for o in range(0, c, s)]
+            at += c
+        parts = [slot, pos, np.asarray(single, np.int32), np.asarray(want, np.int32)]
+        have = [s for s in sizes if blocks[s]]
+        parts += [np.asarray(blocks[s], np.int32).reshape(-1) for s in have]
+        starts, total = [], 0
+        for p in parts:  # 16-byte aligned pieces of one upload
+            starts.append(total)
+            total += -(-p.size // 4) * 4
+        flat = np.zeros(total, np.int32)
+        for s0, p in zip(starts, parts):
+            flat[s0 : s0 + p.size] = p
+        dev = torch.from_numpy(flat).to(self.device)
+        t = [dev[s0 : s0 + p.size] for s0, p in zip(starts, parts)]
+        one_each = all(c == 1 for _, c in counts)
+        return _Batch(n, t[0], t[1], keys, single=None if one_each else t[2], n_single=len(single),
+                      blocks={s: (t[4 + i], len(blocks[s])) for i, s in enumerate(have)},
+                      want=t[3], n_want=len(want))
+
+    def step(self, cache: PagedKVCache, entries: list[tuple[int, list[int], list[int]]]) -> torch.Tensor | None:
+        """One batch: ``entries`` are (cache row, its next tokens, places among them whose logits are
+        asked for), each row at most once.  Appends the tokens to the rows' sequences and returns
+        the logits [wanted, V] in entry order (None if nothing is wanted).  The result is valid until
+        the next step."""
+        if not (self.is_first and self.is_last):
+            raise ValueError("step() needs a shard that holds the whole model")
+        if len({e[0] for e in entries}) != len(entries) or any(not e[1] for e in entries):
+            raise ValueError("a step takes each row once, with at least one token")
+        V = self.cfg.vocab_size
+        tokens = [int(t) for _, toks, _ in entries for t in toks]
+        if tokens and not 0 <= min(tokens) <= max(tokens) < V:
+            raise ValueError(f"token ids outside [0, {V})")
+        want, at = [], 0
+        for _, toks, places in entries:
+            if any(not 0 <= w < len(toks) for w in places):
+                raise ValueError(f"places {places} outside a portion of {len(toks)} tokens")
+            want += [at + w for w in places]
+            at += len(toks)
+        return self._step(cache, [(r, len(t)) for r, t, _ in entries], want, tokens=tokens)
+
+    def _step(self, cache, counts, want, tokens=None, hidden=None) -> torch.Tensor | None:
+        n = sum(c for _, c in counts)
+        if n == 0:
+            return None
+        cache.reserve_each(counts)
+        bf = self._buffers(1, max(n, 2))
+        if tokens is not None:
+            bf.tokens[:n].copy_(torch.tensor(tokens, dtype=torch.int32))
+        else:
+            bf.h[:n].copy_(hidden)
+        b = self._batch(cache, counts, want)
+        out = self._forward(cache, bf, b, bool(want))
+        for row, c in counts:
+            cache.advance_host(c, [row])
+        cache.sync_pos()
+        return out if want or not self.is_last else None
+
+    def __call__(self, tokens: torch.Tensor | None, cache: PagedKVCache,
+                 input_embeddings: torch.Tensor | None = None, logits: str = "all",
+                 rows: slice | None = None) -> torch.Tensor:
+        """``ShardModel.__call__``: tokens int [B,T] (first shard) or input_embeddings float32 [B,T,H];
+        appends T entries to the cache rows; logits [B,T,V] ("all"), [B,1,V] ("last") on the last
+        shard, else the residual [B,T,H] (float32)."""
+        src = tokens if self.is_first else input_embeddings
+        assert src is not None
+        B, T = src.shape[:2]
+        r0 = rows.start if rows is not None else 0
+        if (rows is not None and rows.stop - rows.start != B) or r0 + B > cache.batch:
+            raise ValueError(f"batch {B} does not match cache rows {rows} (cache batch {cache.batch})")
+        want: list[int] = []
+        if self.is_last and logits != "none":
+            want = list(range(B * T)) if logits == "all" else [b * T + T - 1 for b in range(B)]
+        counts = [(r0 + b, T) for b in range(B)]
+        if self.is_first:
+            out = self._step(cache, counts, want, tokens=tokens.reshape(-1).tolist())
+        else:
+            out = self._step(cache, counts, want, hidden=input_embeddings.reshape(B * T, -1))
+        if want:
+            return out.view(B, -1, self.cfg.vocab_size).clone()
+        return self._bufs[("rows",)].h[: B * T].view(B, T, -1).clone()

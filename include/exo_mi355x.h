@@ -431,6 +431,89 @@ int exo_sample(const uint16_t* logits, const exo_sampler_params* params, int32_t
                void* workspace, int64_t workspace_bytes, int rows, int V, int hist_cap, int mode,
                exo_stream_t stream);
 
+/* ---- layer-list decoders with unquantised weights (no operator of the reference: its model
+ * library has no such design).  dtype: 0 bf16, 1 float32 (weights, activations and cache; every
+ * kernel accumulates in float32, and norms, routers, softmax and the residual are float32 in
+ * both).  Row strides (ld*) of matrix operands are multiples of 64 elements and the columns past
+ * the logical size are zero. ---- */
+
+/* x[i] = xb[i] = table[ids[i]]: the float32 residual and its copy in the element type. */
+int exo_embed_rows(const int32_t* ids, const void* table, float* x, void* xb, int n, int V, int H,
+                   int ldt, int ldx, int dtype, exo_stream_t stream);
+/* y[i] = x[rows[i]] / rms * gain (rows null: row i); x float32 [.., H]. */
+int exo_norm_rows(const float* x, const int32_t* rows, const float* gain, void* y, int n, int H,
+                  int ldy, float eps, int dtype, exo_stream_t stream);
+/* Norm of a sublayer's output, then the residual sum: x += gain * branch / rms(branch), xb = x. */
+int exo_post_norm_add(const float* branch, int ldb, const float* gain, float* x, void* xb, int n,
+                      int H, int ldx, float eps, int dtype, exo_stream_t stream);
+/* The same with the branch formed from a token's experts: sum of wt * y over the chosen experts
+ * (idx >= experts: the input x itself), plus sigmoid(logits[gate_col]) * shared. */
+int exo_moe_sum_post_norm(const void* y, const int32_t* idx, const float* wt, const void* shared,
+                          const float* logits, int top, int experts, int ldy, int lds, int ldl,
+                          int gate_col, const float* gain, float* x, void* xb, int n, int H,
+                          int ldx, float eps, int dtype, exo_stream_t stream);
+/* softmax over n logits; the `top` largest of score + correction; weight = score * scale. */
+int exo_moe_route(const float* logits, const float* correction, int32_t* idx, float* wt, int rows,
+                  int n, int ldl, int top, float scale, exo_stream_t stream);
+
+/* y[M,N] = x[M,K] @ w[N,K]^T (+ bias), y in the element type or (y_f32) float32. */
+int exo_dense_gemv(const void* x, const void* w, const float* bias, void* y, int y_f32, int M,
+                   int N, int ldx, int ldw, int ldy, int dtype, exo_stream_t stream); /* M <= 16 */
+int exo_dense_gemm(const void* x, const void* w, const float* bias, void* y, int y_f32,
+                   float* workspace, int64_t workspace_floats, int M, int N, int ldx, int ldw,
+                   int ldy, int dtype, exo_stream_t stream);
+/* g = min(x @ w^T, limit), u = clamp(x @ w_up^T, +-limit): y = g sigmoid(alpha g) (u + shift). */
+int exo_dense_glu_gemm(const void* x, const void* w, const void* w_up, void* y, float limit,
+                       float alpha, float shift, int M, int N, int ldx, int ldw, int ldy,
+                       int dtype, exo_stream_t stream);
+/* Experts of a prompt by (token, slot) pair through exo_moe_group's workspace; w_up null: the
+ * plain product.  x_per_pair: x has a row per pair, else per token. */
+int exo_dense_grouped_gemm(const void* x, const void* w, const void* w_up, const void* group_ws,
+                           void* y, float limit, float alpha, float shift, int T, int topk,
+                           int x_per_pair, int E, int N, int ldx, int ldw, int ldy, int dtype,
+                           exo_stream_t stream);
+
+/* Experts of a decode step (up to 16 rows): gated products, then the weighted sum. */
+typedef struct {
+  const void *x, *gate, *up, *down, *shared_gate, *shared_up, *shared_down;
+  void *act, *shared_act;
+  float* out;
+  const float* x_res;
+  int32_t* idx;
+  float* wt;
+  const float *logits, *correction;
+  int rows, top, experts, ff, shared_ff, H, ldx, lda, ldsa, ldl, gate_col, dtype;
+  float limit, alpha, shift, shared_limit, shared_alpha, shared_shift;
+} exo_moe_rows;
+int exo_moe_glu_rows(const exo_moe_rows* args, exo_stream_t stream);
+int exo_moe_down_rows(const exo_moe_rows* args, exo_stream_t stream);
+
+/* Attention over a paged KV pool: keys [page][kv_heads][64][ldk], values transposed
+ * [page][kv_heads][ldv][64]; table [slots][max_pages]; row i of qkv belongs to slot[i] at
+ * position pos[i].  window 0: causal; else a key is seen if fewer than `window` positions back or
+ * among the first keep_first positions.  slopes: per-head distance penalty, or null. */
+typedef struct {
+  const void* qkv;
+  void *k_pool, *v_pool;
+  const int32_t *table, *slot, *pos, *list;
+  const float* slopes;
+  void* out;
+  float scale, eps;
+  int n, heads, kv_heads, dim, vdim, ldq, ldk, ldv, ldo, max_pages, window, keep_first, unit_qk, dtype;
+} exo_paged_attn;
+/* keys (normalised if unit_qk) and values of all n rows into the pool */
+int exo_paged_append(const exo_paged_attn* args, exo_stream_t stream);
+/* one query position per row (list: the rows, null: all n); append: also stores the row's own key
+ * and value.  nsplit > 1: n * heads <= 16384, and the workspace starts with 16384 arrival counters that
+ * the caller zeroes once (every launch leaves them zero). */
+int64_t exo_paged_attn_workspace(int n, int heads, int vdim, int nsplit);
+int exo_paged_attn_rows(const exo_paged_attn* args, int nsplit, int append, void* workspace,
+                        int64_t workspace_bytes, exo_stream_t stream);
+/* portions of prompts, bf16: list holds n blocks {first row, slot, first position, tokens}, each of
+ * at most exo_paged_prompt_block(heads, kv_heads) tokens of one sequence */
+int exo_paged_prompt_block(int heads, int kv_heads);
+int exo_paged_attn_prompt(const exo_paged_attn* args, exo_stream_t stream);
+
 #ifdef __cplusplus
 }
 #endif
