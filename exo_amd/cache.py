@@ -106,6 +106,18 @@ class ShardKVCache(list):
         ops.kv_import_nhd(k, self.k[layer][row], start)
         ops.kv_import_nhd(v, self.v[layer][row], start)
 
+    def snapshot(self, row: int) -> list[torch.Tensor]:
+        """Detached copy of the row's positions, per layer [2, Hkv, n, D]."""
+        n = self.offsets[row]
+        return [torch.stack((k[row, :, :n], v[row, :, :n])) for k, v in zip(self.k, self.v)]
+
+    def restore(self, row: int, layers: list[torch.Tensor], length: int) -> None:
+        for kv, k, v in zip(layers, self.k, self.v):
+            k[row, :, :length].copy_(kv[0, :, :length])
+            v[row, :, :length].copy_(kv[1, :, :length])
+        self.offsets[row] = length
+        self.sync_pos()
+
     def copy_row(self, src: int, dst: int) -> None:
         """Move one sequence's cache to another batch row (slot compaction)."""
         n = self.offsets[src]

@@ -30,7 +30,6 @@ from typing import BinaryIO
 import msgpack
 import torch
 
-from . import ops
 from .cache import ShardKVCache
 
 DTYPES = ("bfloat16", "float16", "float32")
@@ -314,9 +313,11 @@ def send_kv_cache(stream: BinaryIO, cache: ShardKVCache, *, row: int = 0, dtype:
     if offset <= start_pos:
         return 0
     n = offset - start_pos
-    for layer_idx, (k, v) in enumerate(zip(cache.k, cache.v)):
-        k_nhd = ops.kv_export_nhd(k[row], start_pos, n)
-        v_nhd = ops.kv_export_nhd(v[row], start_pos, n)
+    for layer_idx in range(len(cache.k)):
+        k_nhd, v_nhd = cache.read_nhd(layer_idx, row, start_pos, n)
+        if k_nhd.dtype != torch.bfloat16 or k_nhd.shape != v_nhd.shape:
+            raise ValueError(f"layer {layer_idx}: the wire carries bfloat16 keys and values of one size, not "
+                             f"{k_nhd.dtype} {tuple(k_nhd.shape)} / {tuple(v_nhd.shape)}")
         write_kv_chunk(stream, layer_idx=layer_idx, num_tokens=n, n_heads=k_nhd.shape[1],
                        head_dim=k_nhd.shape[2], dtype=dtype, keys=tensor_to_bytes(k_nhd),
                        values=tensor_to_bytes(v_nhd))
@@ -435,6 +436,8 @@ def ingest_into_cache(result: PrefillResult, cache: ShardKVCache, *, row: int = 
     if final_offset > cache.max_seq:
         raise ValueError(f"{final_offset} positions do not fit the cache ({cache.max_seq})")
     dev = cache.k[0].device
+    cache.offsets[row] = start_pos
+    cache.reserve([row], received)
     for i in range(len(cache)):
         pos = start_pos
         for c in result.kv_chunks.get(i, []):
@@ -442,8 +445,7 @@ def ingest_into_cache(result: PrefillResult, cache: ShardKVCache, *, row: int = 
                 raise ValueError(f"layer {i}: wire dtype {c.dtype} into a bfloat16 cache")
             k = bytes_to_tensor(c.keys, c.shape, c.dtype, dev)
             v = bytes_to_tensor(c.values, c.shape, c.dtype, dev)
-            ops.kv_import_nhd(k, cache.k[i][row], pos)
-            ops.kv_import_nhd(v, cache.v[i][row], pos)
+            cache.write_nhd(i, row, pos, k, v)
             pos += c.num_tokens
     cache.offsets[row] = final_offset
     cache.sync_pos()

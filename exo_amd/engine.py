@@ -28,15 +28,16 @@ from typing import Any
 import torch
 
 from .cache import ShardKVCache
-from .config import ModelConfig
 from .generate import (
-    DEFAULT_TOP_LOGPROBS, MAX_TOKENS, PrefillCancelled, TokenStream, extract_top_logprobs,
+    DEFAULT_TOP_LOGPROBS, MAX_TOKENS, PREFILL_STEP_SIZE, PrefillCancelled, TokenStream, extract_top_logprobs,
     GenerateState, generate, make_sampler, prefill, processors_for,
 )
 from .loader import load_shard_weights
-from .model import ShardModel
+from .model import DecoderShard
+from .paged_cache import PAGE, pages_for
 from .prefix_cache import KVPrefixCache, save_prefix_cache
 from .sampling import TOP_LOGPROBS, DeviceSampler, SamplerSettings
+from .registry import build_model, load_config
 from .tokenizer import load_tokenizer
 logger = logging.getLogger("exo_amd")
 
@@ -107,10 +108,23 @@ class _Seq:
     sampler: Callable | None = None
     processors: list | None = None
     tokens: list[int] = field(default_factory=list)  # what the logits processors see
+    filling: "_Filling | None" = None  # prompt not yet in the cache (mixed steps)
 
     @property
     def on_device(self) -> bool:
         return self.sampler is None
+
+
+@dataclass
+class _Filling:
+    """The part of a prompt that mixed steps still have to feed."""
+
+    pending: list[int]                 # tokens up to, but not including, the last prompt token
+    done: int
+    total: int
+    progress: Callable[[int, int], None]
+    on_filled: Callable[[float, int], None]  # (cache row is complete) rate, row
+    t0: float | None = None
 
 
 @dataclass
@@ -137,15 +151,29 @@ class ShardBatchGenerator:
     of the one it returns, so the device never idles on the host's detokenising and
     bookkeeping; the results travel through pinned host buffers guarded by an event.  When
     the set of rows changes (a request finishes, is cancelled or joins), the chain restarts
-    from the host's tokens after the step in flight has been read."""
+    from the host's tokens after the step in flight has been read.
 
-    def __init__(self, model: ShardModel, tokenizer, max_batch: int = EXO_MAX_CONCURRENT_REQUESTS,
-                 max_seq: int = 8192, kv_prefix_cache: KVPrefixCache | None = None):
+    A model with a mixed step (``mixed_steps``: a paged pool and a step function that takes portions
+    of prompts beside single tokens) does not prefill in ``submit``: the request joins ``filling``,
+    and while any is there a step is one batch of the next token of every active row and up to
+    PREFILL_STEP_SIZE prompt tokens, oldest request first.  Active rows stay in front of the filling
+    ones in the pool; moving a row only moves its pages' ownership."""
+
+    def __init__(self, model: DecoderShard, tokenizer, max_batch: int = EXO_MAX_CONCURRENT_REQUESTS,
+                 max_seq: int = 8192, kv_prefix_cache: KVPrefixCache | None = None,
+                 pool_tokens: int | None = None):
         if not (model.is_first and model.is_last):
             raise ValueError("the batch generator needs a shard that holds the whole model")
         self.model, self.tokenizer = model, tokenizer
         self.max_batch, self.max_seq = max_batch, max_seq
-        self.cache: ShardKVCache = model.make_cache(max_batch, max_seq)
+        self.mixed = getattr(model, "mixed_steps", False)
+        if pool_tokens is not None and not self.mixed:
+            raise ValueError("pool_tokens needs a model with a paged pool")
+        self.cache: ShardKVCache = model.make_cache(max_batch, max_seq, **(
+            {"pool_tokens": pool_tokens} if self.mixed else {}))
+        if self.mixed:  # (one request never needs more than the whole pool)
+            self.max_seq = min(max_seq, self.cache.n_pages * PAGE)
+        self.filling: list[_Seq] = []  # by pool row, behind the active rows
         self.kv_prefix_cache = kv_prefix_cache
         self.rows: list[_Seq] = []
         self._next_uid = 0
@@ -163,7 +191,19 @@ class ShardBatchGenerator:
 
     @property
     def has_work(self) -> bool:
-        return bool(self.rows)
+        return bool(self.rows or self.filling)
+
+    def can_admit(self, prompt_tokens: int, max_output_tokens: int | None) -> bool:
+        """Whether the pool holds the request to its end beside those already here (a row cache
+        always does: its rows are allocated at full length)."""
+        if len(self.rows) + len(self.filling) >= self.max_batch:
+            return False
+        if not self.mixed:
+            return True
+        def need(prompt: int, out: int | None) -> int:
+            return pages_for(min(prompt + (out or MAX_TOKENS) + 2, self.max_seq))
+        held = sum(need(len(q.prompt_tokens), q.params.max_output_tokens) for q in self.rows + self.filling)
+        return held + need(prompt_tokens, max_output_tokens) <= self.cache.n_pages
 
     def _eos(self) -> list[int]:
         return list(getattr(self.tokenizer, "eos_token_ids", []) or [])
@@ -172,7 +212,7 @@ class ShardBatchGenerator:
                on_prefill_progress: Callable[[int, int], None] | None = None,
                distributed_prompt_progress_callback: Callable[[], None] | None = None,
                on_generation_token: Callable[[], None] | None = None) -> int:
-        if len(self.rows) >= self.max_batch:
+        if len(self.rows) + len(self.filling) >= self.max_batch:
             raise RuntimeError("no free batch row")
         toks = prompt if not isinstance(prompt, str) else self.tokenizer.encode(prompt)
         toks = [int(t) for t in toks]
@@ -184,7 +224,7 @@ class ShardBatchGenerator:
             if max_tokens <= 0:
                 raise ValueError(f"prompt of {len(toks)} tokens exceeds the cache ({self.max_seq})")
         settings = SamplerSettings.from_task(task_params, self._eos(), zero_seed_is_default=False)
-        row = len(self.rows)
+        row = len(self.rows) + len(self.filling)
         # prefix cache lookup (batch_generate.py:164-181): bench requests opt in
         use_prefix = self.kv_prefix_cache is not None and (
             not task_params.bench or task_params.use_prefix_cache)
@@ -202,26 +242,34 @@ class ShardBatchGenerator:
             if on_prefill_progress is not None:
                 on_prefill_progress(done, total)
 
-        try:
-            tps, n = self._prefill_row(task_params, toks, remaining, prefix_hit_length, row, progress,
-                                       on_prefill_progress)
-        except PrefillCancelled:
-            self.cache.reset(rows=range(row, row + 1))
-            raise
+        def save(tps: float, row: int) -> None:
+            if use_prefix:
+                try:
+                    save_prefix_cache(self.kv_prefix_cache, toks, self.cache, row, prefix_hit_length,
+                                      matched_index, prefill_tps=tps)
+                except Exception:  # a failed save never fails the request (batch_generate.py:534)
+                    logger.warning("failed to save prefix cache", exc_info=True)
+
+        tps = 0.0
+        remote = len(remaining) > REMOTE_PREFILL_MIN_TOKENS and task_params.prefill_endpoint is not None
+        here = not self.mixed or remote  # the prompt is in the cache when submit returns
+        if here:
+            try:
+                tps, n = self._prefill_row(task_params, toks, remaining, prefix_hit_length, row, progress,
+                                           on_prefill_progress)
+            except PrefillCancelled:
+                self.cache.reset(rows=range(row, row + 1))
+                raise
         prefix_cache_hit = "none"
         if matched_index is not None and prefix_hit_length > 0:
             prefix_cache_hit = "exact" if is_exact_hit else "partial"
             if is_exact_hit:
                 tps = self.kv_prefix_cache.prefill_tps[matched_index]
-        if use_prefix:
-            try:
-                save_prefix_cache(self.kv_prefix_cache, toks, self.cache, row, prefix_hit_length,
-                                  matched_index, prefill_tps=tps)
-            except Exception:  # a failed save never fails the request (batch_generate.py:534)
-                logger.warning("failed to save prefix cache", exc_info=True)
-        if len(remaining) >= 2:
-            self.model(torch.tensor([[remaining[-2]]], dtype=torch.int32), self.cache,
-                       logits="none", rows=slice(row, row + 1))
+        if here:
+            save(tps, row)
+            if len(remaining) >= 2:
+                self.model(torch.tensor([[remaining[-2]]], dtype=torch.int32), self.cache,
+                           logits="none", rows=slice(row, row + 1))
         k_top = task_params.top_logprobs or DEFAULT_TOP_LOGPROBS
         seq = _Seq(
             uid=self._next_uid, params=task_params, prompt_tokens=toks, settings=settings,
@@ -231,18 +279,34 @@ class ShardBatchGenerator:
             # the generator is handed the last two prompt tokens (batch_generate.py:282,301):
             # they are all the logits processors see of the prompt
             tokens=list(toks[-2:]))
-        if settings.on_device() and k_top <= TOP_LOGPROBS:
-            self.sampler.set_row(row, settings, seq.tokens)
-        else:
+        if not (settings.on_device() and k_top <= TOP_LOGPROBS):
             gen = torch.Generator(device=self.model.device)
             gen.manual_seed(settings.seed)
             seq.processors = processors_for(task_params, self._eos())
             seq.sampler = make_sampler(settings.temperature, settings.top_p, settings.min_p,
                                        settings.top_k, gen)
         self._next_uid += 1
-        self.rows.append(seq)
-        self._pending_input.append(toks[-1])
+        pending = [] if here else list(remaining[:-1])
+        self.filling.append(seq)  # (pool row: the one prepared above)
+        if pending:
+            seq.filling = _Filling(pending, 0, len(pending), progress, save)
+        else:
+            self._activate(seq)
         return seq.uid
+
+    def _activate(self, seq: _Seq) -> None:
+        """The sequence's prompt is in the cache up to its last token: it joins the active rows."""
+        row = len(self.rows)
+        at = self.filling.index(seq)
+        if at:  # its pool row changes places with the first filling one
+            self.cache.swap_rows(row + at, row)
+            self.filling[at] = self.filling[0]
+        del self.filling[0]
+        seq.filling = None
+        if seq.on_device:
+            self.sampler.set_row(row, seq.settings, seq.tokens)
+        self.rows.append(seq)
+        self._pending_input.append(seq.prompt_tokens[-1])
 
     def _prefill_row(self, task_params, toks, remaining, prefix_hit_length, row, progress,
                      on_prefill_progress) -> tuple[float, int]:
@@ -294,6 +358,10 @@ class ShardBatchGenerator:
         want_top = any(s.want_top for s in self.rows)
         self.model.decode_step(self.cache, B, feedback=True, sampler=self.sampler,
                                mode=self.sampler.mode(B, want_top))
+        return self._read_back(B, want_top)
+
+    def _read_back(self, B: int, want_top: bool) -> _Flight:
+        """Enqueue the copy of a step's sampling results into a pinned host buffer set."""
         slot, self._slot = self._slot, self._slot ^ 1
         h, d = self._host[slot], self.sampler
         h["token"][:B].copy_(d.token[:B], non_blocking=True)
@@ -305,7 +373,69 @@ class ShardBatchGenerator:
         ev.record()
         return _Flight(rows=list(self.rows), slot=slot, event=ev, want_top=want_top)
 
+    def _mixed_step(self) -> list[tuple[int, GenerationResponse]]:
+        """One batch: the next token of every active row and portions of the filling prompts."""
+        B, budget = len(self.rows), PREFILL_STEP_SIZE
+        entries: list = [(r, [t], [0]) for r, t in enumerate(self._pending_input)]
+        portions: list[tuple[_Seq, int]] = []
+        for seq in sorted(self.filling, key=lambda q: q.uid):
+            f = seq.filling
+            if budget > 0:
+                f.t0 = time.perf_counter() if f.t0 is None else f.t0
+                portions.append((seq, min(budget, len(f.pending))))
+                budget -= portions[-1][1]
+        where = {id(q): B + i for i, q in enumerate(self.filling)}
+        entries += [(where[id(q)], q.filling.pending[:m], []) for q, m in portions]
+        logits = self.model.step(self.cache, entries)
+        out: list[tuple[int, GenerationResponse]] = []
+        if B:
+            on_device = all(q.on_device for q in self.rows)
+            if on_device:
+                want_top = any(q.want_top for q in self.rows)
+                bufs = self.model._bufs[("rows",)]
+                if self._sampler_stale:
+                    for r, q in enumerate(self.rows):
+                        self.sampler.set_row(r, q.settings, q.tokens, draws=q.stream.n_gen)
+                    self._sampler_stale = False
+                self.sampler.sample(self.model._sampling_logits(logits, bufs), B, self.sampler.mode(B, want_top))
+                flight = self._read_back(B, want_top)
+        for q, m in portions:
+            f = q.filling
+            del f.pending[:m]
+            f.done += m
+            if not f.pending:
+                torch.cuda.synchronize()
+                if q.stream.prefix_cache_hit != "exact":  # (an exact hit reports the stored entry's rate)
+                    q.stream.prefill_tps = f.total / max(time.perf_counter() - f.t0, 1e-9)
+                f.on_filled(q.stream.prefill_tps, where[id(q)])
+        if B:
+            # responses may end rows: collected while the filling rows are still where they were
+            out = self._collect(flight) if on_device else self._sample_on_host(logits.float(), None)
+        for q, _ in portions:
+            try:
+                q.filling.progress(q.filling.done, q.filling.total)
+            except PrefillCancelled:
+                self._drop_filling(q)
+                continue
+            if not q.filling.pending:
+                self._activate(q)
+        return out
+
+    def _drop_filling(self, seq: _Seq) -> None:
+        """A request leaves before its prompt is in the cache."""
+        at, base, last = self.filling.index(seq), len(self.rows), len(self.filling) - 1
+        self.cache.release(base + at)
+        if at != last:
+            self.cache.copy_row(base + last, base + at)
+            self.filling[at] = self.filling[last]
+        self.filling.pop()
+
     def step(self) -> list[tuple[int, GenerationResponse]]:
+        if self.filling:
+            if self._flight is not None:  # drain the device-side chain first
+                cur, self._flight = self._flight, None
+                return self._collect(cur)
+            return self._mixed_step()
         if not self.rows:
             self._flight = None
             return []
@@ -364,16 +494,22 @@ class ShardBatchGenerator:
         """A step with the processors and samplers of every row run on the host with torch:
         taken only while a row's settings are outside what the sampling kernels accept."""
         B = len(self.rows)
-        self._sampler_stale = True
         bufs = self.model._buffers(B, 1)
         bufs.tokens.copy_(torch.tensor(self._pending_input, dtype=torch.int32))
         bufs = self.model.decode_step(self.cache, B)
         greedy_tokens = bufs.next_token.tolist()  # synchronises
+        return self._sample_on_host(bufs.logits.float(), greedy_tokens)
+
+    def _sample_on_host(self, all_logits: torch.Tensor, greedy_tokens: list[int] | None,
+                        ) -> list[tuple[int, GenerationResponse]]:
+        self._sampler_stale = True
+        if greedy_tokens is None:
+            greedy_tokens = torch.argmax(all_logits, dim=-1).tolist()
         now = time.perf_counter()
         out: list[tuple[int, GenerationResponse]] = []
         finished: list[int] = []
         for r, seq in enumerate(self.rows):
-            logits = bufs.logits[r : r + 1].float()
+            logits = all_logits[r : r + 1]
             if seq.on_device:  # its settings on the host all the same, for this step
                 procs = processors_for(seq.params, self._eos())
                 if seq.settings.temperature == 0 and not procs:
@@ -418,14 +554,21 @@ class ShardBatchGenerator:
                 self._pending_input[r] = self._pending_input[last]
             self.rows.pop()
             self._pending_input.pop()
+            self.cache.release(last)
+            if self.filling:  # the active rows end one earlier: the last filling row takes the place
+                self.cache.copy_row(last + len(self.filling), last)
+                self.filling.insert(0, self.filling.pop())
 
     def cancel(self, uids: list[int]) -> None:
+        for q in [q for q in self.filling if q.uid in set(uids)]:
+            self._drop_filling(q)
         self._drop_rows([r for r, s in enumerate(self.rows) if s.uid in set(uids)])
         if not self.rows:
             self._flight = None
 
     def close(self) -> None:
         self.rows.clear()
+        self.filling.clear()
         self._pending_input.clear()
         self._flight = None
         self.cache = None  # type: ignore[assignment]
@@ -456,7 +599,7 @@ def _prompt_of(tokenizer, params: TextGenerationTaskParams):
 
 @dataclass(eq=False)
 class BatchGenerator(Engine):
-    model: ShardModel
+    model: DecoderShard
     tokenizer: Any
     model_id: str
     device_rank: int = 0
@@ -465,6 +608,7 @@ class BatchGenerator(Engine):
     check_for_cancel_every: int = 50
     max_seq: int = 8192
     kv_prefix_cache: KVPrefixCache | None = None
+    pool_tokens: int | None = None  # paged pools: tokens all requests hold together (default: no limit)
     gen_factory: Any = None  # tests inject a fake inner generator (like the reference's FakeExoBatchGenerator)
     _cancelled_tasks: set = field(default_factory=set, init=False)
     _all_tasks: dict = field(default_factory=dict, init=False)
@@ -477,7 +621,7 @@ class BatchGenerator(Engine):
             self._gen = self.gen_factory()
         else:
             self._gen = ShardBatchGenerator(self.model, self.tokenizer, EXO_MAX_CONCURRENT_REQUESTS,
-                                            self.max_seq, self.kv_prefix_cache)
+                                            self.max_seq, self.kv_prefix_cache, self.pool_tokens)
 
     def warmup(self) -> None:
         """generate.py:399-462: a short greedy generation on a fixed prompt; sets how
@@ -511,7 +655,10 @@ class BatchGenerator(Engine):
 
     def step(self):
         while self._queue and len(self._active_tasks) < EXO_MAX_CONCURRENT_REQUESTS:
-            task = self._queue.popleft()
+            task = self._queue[0]
+            if not self._fits(task):
+                break  # waits for pages (or a row) that running requests will give back
+            self._queue.popleft()
             try:
                 uid = self._start_task(task)
             except PrefillCancelled:
@@ -559,6 +706,13 @@ class BatchGenerator(Engine):
                 results.append((tid, CancelledResponse()))
         self._cancelled_tasks.clear()
         return results
+
+    def _fits(self, task: GenerationTask) -> bool:
+        if self.pool_tokens is None:
+            return True
+        prompt = _prompt_of(self.tokenizer, task.task_params)
+        n = len(self.tokenizer.encode(prompt)) if isinstance(prompt, str) else len(prompt)
+        return self._gen.can_admit(n, task.task_params.max_output_tokens)
 
     def _send_error(self, task: GenerationTask, e: Exception) -> None:
         if self.device_rank == 0 and self.event_sender is not None:
@@ -620,7 +774,7 @@ class SequentialGenerator(Engine):
     FinishedResponse and starts the next queued request.  Cancellation is looked at every
     ``check_for_cancel_every`` tokens and between prefill chunks."""
 
-    model: ShardModel
+    model: DecoderShard
     tokenizer: Any
     model_id: str
     device_rank: int = 0
@@ -773,7 +927,7 @@ class Mi355xBuilder(Builder):
     cancel_receiver: Any = None
     device: str = "cuda:0"
     max_seq: int = 8192
-    inference_model: ShardModel | None = None
+    inference_model: DecoderShard | None = None
     tokenizer: Any = None
 
     def connect(self, bound_instance: BoundInstance) -> None:
@@ -787,7 +941,7 @@ class Mi355xBuilder(Builder):
             raise RuntimeError("immediate_exception requested by shard metadata")
         path = Path(bound_instance.model_path) if bound_instance.model_path else build_model_path(
             shard.model_id)
-        cfg = ModelConfig.from_path(path)
+        cfg = load_config(path)
         if shard.n_layers != cfg.num_hidden_layers:
             raise ValueError(f"shard says {shard.n_layers} layers, checkpoint has {cfg.num_hidden_layers}")
         it = load_shard_weights(path, cfg, shard.start_layer, shard.end_layer, self.device)
@@ -797,7 +951,7 @@ class Mi355xBuilder(Builder):
                 yield ModelLoadingResponse(layers_loaded=done, total=total)
         except StopIteration as stop:
             weights = stop.value
-        self.inference_model = ShardModel(cfg, weights, shard.start_layer, shard.end_layer, self.device)
+        self.inference_model = build_model(cfg, weights, shard.start_layer, shard.end_layer, self.device)
         self.tokenizer = load_tokenizer(path, cfg.vocab_size)
 
     def build(self) -> Engine:

@@ -18,7 +18,7 @@ import torch
 
 from . import ops
 from .cache import ShardKVCache, cache_length
-from .model import ShardModel
+from .model import DecoderShard
 from .types import GenerationResponse, GenerationStats, TextGenerationTaskParams, TopLogprobItem, Usage
 
 MAX_TOKENS = 32168  # src/exo/worker/engines/mlx/constants.py:7
@@ -166,7 +166,7 @@ def extract_top_logprobs(logprobs: torch.Tensor, tokenizer, top_logprobs: int,
 # ---------------------------------------------------------------------- prefill
 
 
-def prefill(model: ShardModel, prompt_tokens, cache: ShardKVCache,
+def prefill(model: DecoderShard, prompt_tokens, cache: ShardKVCache,
             on_prefill_progress: Callable[[int, int], None] | None = None,
             step: int = PREFILL_STEP_SIZE, faithful_extra_steps: bool = True,
             row: int = 0, graph_steps: bool = False) -> tuple[float, int]:
@@ -304,14 +304,14 @@ class GenerateState:
     graphs ``generate()`` captures are bound to them, so a caller that keeps the state (the
     sequential engine) captures once instead of once per request."""
 
-    def __init__(self, model: ShardModel, max_seq: int):
+    def __init__(self, model: DecoderShard, max_seq: int):
         from .sampling import DeviceSampler
         self.max_seq = max_seq
         self.cache = model.make_cache(1, max_seq)
         self.sampler = DeviceSampler(1, model.cfg.vocab_size, model.device)
 
 
-def generate(model: ShardModel, tokenizer, task: TextGenerationTaskParams, prompt_tokens: list[int],
+def generate(model: DecoderShard, tokenizer, task: TextGenerationTaskParams, prompt_tokens: list[int],
              on_prefill_progress: Callable[[int, int], None] | None = None,
              on_generation_token: Callable[[], None] | None = None,
              max_seq: int | None = None, eos_token_ids: list[int] | None = None,

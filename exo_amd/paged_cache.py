@@ -116,6 +116,14 @@ class PagedKVCache(list):
         self.offsets[dst], self.offsets[src] = self.offsets[src], 0
         self.sync_pos()
 
+    def swap_rows(self, a: int, b: int) -> None:
+        if a == b:
+            return
+        self.pages[a], self.pages[b] = self.pages[b], self.pages[a]
+        self.offsets[a], self.offsets[b] = self.offsets[b], self.offsets[a]
+        self.table[[a, b]] = self.table[[b, a]]
+        self.sync_pos()
+
     def nbytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in self.k + self.v)
 
@@ -142,3 +150,15 @@ class PagedKVCache(list):
         page = self._row_pages(row, 0, start + n)[at // PAGE]
         self.k[layer][page, :, at % PAGE, :d] = k.to(self.k[layer].dtype)
         self.v[layer][page, :, :e, at % PAGE] = v.to(self.v[layer].dtype)
+
+    def snapshot(self, row: int) -> list[tuple[torch.Tensor, torch.Tensor]]:
+        """Detached copy of the row's positions, per layer (keys, values)."""
+        return [self.read_nhd(i, row, 0, self.offsets[row]) for i in range(len(self.k))]
+
+    def restore(self, row: int, layers: list[tuple[torch.Tensor, torch.Tensor]], length: int) -> None:
+        self.reset(rows=[row])
+        self.reserve([row], length)
+        for i, (k, v) in enumerate(layers):
+            self.write_nhd(i, row, 0, k[:length], v[:length])
+        self.offsets[row] = length
+        self.sync_pos()

@@ -15,9 +15,10 @@ the reference's snapshot machinery for SSM / rotating caches has no counterpart 
   the Mac's memory is unified; here the KV lives in HBM, so the pressure signal is the
   device's used fraction.
 
-Stored layout: per layer one bf16 tensor ``[2, Hkv, n, D]`` (keys, values) holding just
-the ``n`` valid positions, contiguous, so an entry costs exactly its tokens and a restore
-is ``2 * L`` strided device copies into the pool row.
+Stored layout: what the cache's ``snapshot`` returns per layer, holding just the ``n`` valid
+positions, contiguous, so an entry costs exactly its tokens: one bf16 tensor ``[2, Hkv, n, D]``
+(keys, values) from a row cache, whose restore is ``2 * L`` strided device copies; keys
+``[n, G, D]`` and values ``[n, G, E]`` from a paged pool.
 """
 
 from __future__ import annotations
@@ -30,6 +31,7 @@ import numpy as np
 import torch
 
 from .cache import ShardKVCache
+from .paged_cache import PagedKVCache
 
 
 def _default_memory_threshold(total_bytes: int) -> float:
@@ -74,7 +76,7 @@ def get_prefix_length(prompt, cached_prompt) -> int:
 class StoredKV:
     """One entry: the first ``length`` positions of every local layer."""
 
-    layers: list[torch.Tensor]  # per layer [2, Hkv, length, D] bf16
+    layers: list  # per layer [2, Hkv, length, D], or a (keys, values) pair of a paged pool
     length: int
 
     @property
@@ -82,16 +84,15 @@ class StoredKV:
         return self.length
 
     def nbytes(self) -> int:
-        return sum(t.numel() * t.element_size() for t in self.layers)
+        ts = [t for x in self.layers for t in (x if isinstance(x, tuple) else (x,))]
+        return sum(t.numel() * t.element_size() for t in ts)
 
 
-def snapshot_row(cache: ShardKVCache, row: int) -> StoredKV:
-    n = cache.offsets[row]
-    layers = [torch.stack((k[row, :, :n], v[row, :, :n])) for k, v in zip(cache.k, cache.v)]
-    return StoredKV(layers, n)
+def snapshot_row(cache: ShardKVCache | PagedKVCache, row: int) -> StoredKV:
+    return StoredKV(cache.snapshot(row), cache.offsets[row])
 
 
-def restore_row(stored: StoredKV, cache: ShardKVCache, row: int, length: int) -> None:
+def restore_row(stored: StoredKV, cache: ShardKVCache | PagedKVCache, row: int, length: int) -> None:
     """Write the first ``length`` stored positions into pool row ``row`` and set its fill
     level (the reference deep-copies the entry and trims the copy, cache.py:377-387)."""
     if length > stored.length:
@@ -100,11 +101,7 @@ def restore_row(stored: StoredKV, cache: ShardKVCache, row: int, length: int) ->
         raise ValueError(f"restore of {length} positions into a cache of {cache.max_seq}")
     if len(stored.layers) != len(cache.k):
         raise ValueError("stored entry and cache differ in layer count")
-    for kv, k, v in zip(stored.layers, cache.k, cache.v):
-        k[row, :, :length].copy_(kv[0, :, :length])
-        v[row, :, :length].copy_(kv[1, :, :length])
-    cache.offsets[row] = length
-    cache.sync_pos()
+    cache.restore(row, stored.layers, length)
 
 
 def cache_length(entry) -> int:
