@@ -54,8 +54,8 @@ def host(t):
 
 def close(got, want, tol, what):
     want = np.asarray(want, np.float64)
-    err = np.abs(np.asarray(got, np.float64) - want).max() / np.sqrt(np.mean(want**2))
-    assert err < tol, f"{what}: {err:.2e} of the RMS"
+    err = (np.abs(np.asarray(got, np.float64) - want) / np.maximum(np.abs(want), np.sqrt(np.mean(want**2)))).max()
+    assert err < tol, f"{what}: {err:.2e} of the larger of value and RMS"
 
 
 # ------------------------------------------------------------------ products
@@ -171,11 +171,14 @@ def attn_case(spec, T, seed=0, far=()):
     return np.concatenate([q.reshape(T, -1), k.reshape(T, -1), v.reshape(T, -1)], 1), (q, k, v)
 
 
-def attn_oracle(spec, qkv, eps):
+def attn_oracle(spec, qkv, eps, dtype=F32):
+    """``dtype`` bf16: normalised queries and keys rounded once, as the kernels hold them."""
     q, k, v = (a.astype(np.float64) for a in qkv)
     sl = np.zeros(spec.heads) if spec.slopes is None else np.asarray(spec.slopes)
     if spec.unit_qk:
         q, k = O.rms_unit(q, eps), O.rms_unit(k, eps)
+        if dtype == BF:
+            q, k = (bf16_round(a.astype(np.float32)).astype(np.float64) for a in (q, k))
     return O.attend(q, k, v, spec.scale, sl, O.visible(len(q), spec.window, spec.keep_first))
 
 
@@ -236,16 +239,17 @@ def test_attention_shapes(device, dtype, shape):
         say("attention", dtype, shape, window, keep)
         T, eps = 210, 0.3  # an eps that shows
         rows_np, qkv = attn_case(spec, T, seed=i, far=[(200, 2), (150, 86), (90, 0)])
-        want = attn_oracle(spec, qkv, eps)
+        want = attn_oracle(spec, qkv, eps, dtype)
         for cuts in ([T], [3, 2, 64, 64, 1, 30, 1, 500], [150] + [1] * 60):
             got = run_portions(spec, rows_np, cuts, dtype, eps, start_pages=2, fused=cuts[0] != 3)
-            close(got, want, 4e-2 if dtype == BF else 5e-5, f"{shape} {window} {keep} {cuts[:3]}")
+            close(got, want, 1.2e-2 if dtype == BF else 5e-5, f"{shape} {window} {keep} {cuts[:3]}")
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_attention_edges(device, dtype):
     """One key that carries the whole weight if it is seen, on both sides of every edge: the window,
-    the kept first positions, page and tile borders; in a prompt and decoded."""
+    the kept first positions, page and tile borders; in a prompt and decoded.  (Scores reach 128, so a
+    query element that rounds the other way in bf16 moves a few per cent; a wrong key moves all.)"""
     for window, keep in [(64, 20), (63, 0), (65, 33), (97, 64), (32, 1), (5, 63)]:
         spec = make_spec(4, 2, 64, 32, window, keep, scale=2.0, slopes=False)
         T = 330
@@ -254,13 +258,13 @@ def test_attention_edges(device, dtype):
             q = [i for d in (-1, 0, 1) for i in (key + window + d, 250 + d, 319 + d) if key < i < T] + [T - 1]
             say("edges", dtype, window, keep, "key", key)
             rows_np, qkv = attn_case(spec, T, seed=key, far=[(i, key) for i in q])
-            want = attn_oracle(spec, qkv, 1e-6)
+            want = attn_oracle(spec, qkv, 1e-6, dtype)
             seen = [np.abs(want[i] - qkv[2][key][[0, 0, 1, 1]]).max() < 0.3 for i in q]
             vis = O.visible(T, window, keep)
             assert seen == [bool(vis[i, key]) for i in q]  # the planted key decides these rows
-            close(run_portions(spec, rows_np, [T], dtype, 1e-6), want, 4e-2 if dtype == BF else 5e-5, "prompt")
+            close(run_portions(spec, rows_np, [T], dtype, 1e-6), want, 6e-2 if dtype == BF else 5e-5, "prompt")
             cuts = [min(q) - 1, 2, 2] + [1] * T if min(q) > 1 else [1] * T
-            close(run_portions(spec, rows_np, cuts, dtype, 1e-6), want, 4e-2 if dtype == BF else 5e-5, "decoded")
+            close(run_portions(spec, rows_np, cuts, dtype, 1e-6), want, 6e-2 if dtype == BF else 5e-5, "decoded")
 
 
 def test_attention_keeps_many_small_weights(device):
@@ -269,7 +273,7 @@ def test_attention_keeps_many_small_weights(device):
     spec = make_spec(4, 4, 64, 64, None, 0, scale=0.02)
     T = 512
     rows_np, qkv = attn_case(spec, T, seed=3)
-    want = attn_oracle(spec, qkv, 1e-6)
+    want = attn_oracle(spec, qkv, 1e-6, BF)
     for cuts in ([T], [T - 6] + [1] * 6):
         got = run_portions(spec, rows_np, cuts, BF, 1e-6)
         assert U.rel_rms(got[-6:].reshape(6, -1), want[-6:].reshape(6, -1)).max() < 4e-3
@@ -281,10 +285,10 @@ def test_decode_attention_splits_agree_and_replay(device):
     spec = make_spec(8, 2, 64, 64, None, 0)
     T = 1500
     rows_np, qkv = attn_case(spec, T, seed=9, far=[(T - 1, 3)])
-    want = attn_oracle(spec, tuple(a for a in qkv), 1e-6)[-3:]
+    want = attn_oracle(spec, qkv, 1e-6, BF)[-3:]
     got = run_portions(spec, rows_np, [T - 3, 1, 1, 1], BF, 1e-6)[-3:]
     assert "splits" in native.last_variant() and "splits=1 " not in native.last_variant()
-    close(got, want, 4e-2, "splits")
+    close(got, want, 1.2e-2, "splits")
     assert np.array_equal(got, run_portions(spec, rows_np, [T - 3, 1, 1, 1], BF, 1e-6)[-3:])
 
 
