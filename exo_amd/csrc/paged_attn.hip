@@ -179,19 +179,48 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
   const int32_t* table = p.table + (size_t)p.slot[row] * p.max_pages;
   const Tiles tl = tiles_of(pos, pos, p.size, p.keep, 32);
 
+  const int ksteps = p.ldk * (int)sizeof(T) / 64, vtiles = p.ldv / 16;
+  struct Tile {
+    uint4 ka[KST], kb[KST];
+    VTerms<T> v[VT];
+  };
+  auto load_tile = [&](Tile& t, int key0) {
+    const size_t head = (size_t)table[key0 / kPage] * p.G + kvh;
+    const char* kp = reinterpret_cast<const char*>(reinterpret_cast<const T*>(p.kpool) +
+                                                   (head * kPage + (key0 % kPage) + r) * p.ldk) + g * 16;
+    const T* vp = reinterpret_cast<const T*>(p.vpool) + (head * p.ldv + r) * kPage + (key0 % kPage);
+#pragma unroll
+    for (int s = 0; s < KST; ++s)
+      if (s < ksteps) {
+        t.ka[s] = *reinterpret_cast<const uint4*>(kp + s * 64);
+        t.kb[s] = *reinterpret_cast<const uint4*>(kp + (size_t)16 * p.ldk * sizeof(T) + s * 64);
+      }
+#pragma unroll
+    for (int i = 0; i < VT; ++i)
+      if (i < vtiles) t.v[i].load(vp + (size_t)i * 16 * kPage, g);
+  };
+  // A wave's first tile is requested before the queries are normalised - unless it is the one
+  // that the row's own key goes into below.
+  const int stride = p.nsplit * kRowWaves;
+  int j = split * kRowWaves + wave;
+  Tile tile;
+  const bool early = j < tl.n && !(FUSE && j == tl.n - 1);
+  if (early) load_tile(tile, tl.at(j) * 32);
+
   // ---- queries (and the row's own key and value) through float32 norms
   for (int h = wave; h < 16; h += kRowWaves) {
     T* dst = qs + h * QS;
     if (h < gs) unit_row<T>(reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + (h0 + h) * p.D, dst, p.D, p.unit, p.eps, lane);
     for (int d = (h < gs ? p.D : 0) + lane; d < QS; d += 64) dst[d] = Elem<T>::make(0.f);
   }
-  if (FUSE && split == ((tl.n - 1) % (p.nsplit * kRowWaves)) / kRowWaves) {
+  if (FUSE && split == ((tl.n - 1) % stride) / kRowWaves) {
     const int page = table[pos / kPage];
     if (wave == kRowWaves - 1) put_key<T>(p, row, kvh, page, pos % kPage, lane);
     if (wave == kRowWaves - 2) put_value<T>(p, row, kvh, page, pos % kPage, lane);
     wait_own_stores_done();
   }
   __syncthreads();
+  if (!early && j < tl.n) load_tile(tile, tl.at(j) * 32);
   uint4 q[KST];
 #pragma unroll
   for (int s = 0; s < KST; ++s)
@@ -199,34 +228,19 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
 
   const float sc = p.scale * kLog2e;
   const float slope = p.slopes && r < gs ? p.slopes[h0 + r] * kLog2e : 0.f;
-  const int ksteps = p.ldk * (int)sizeof(T) / 64, vtiles = p.ldv / 16;
   floatx4 o[VT];
 #pragma unroll
   for (int t = 0; t < VT; ++t) o[t] = floatx4{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
 
-  for (int j = split * kRowWaves + wave; j < tl.n; j += p.nsplit * kRowWaves) {
+  while (j < tl.n) {
     const int key0 = tl.at(j) * 32;
-    const size_t head = (size_t)table[key0 / kPage] * p.G + kvh;
-    const T* kp = reinterpret_cast<const T*>(p.kpool) + (head * kPage + (key0 % kPage)) * p.ldk;
-    const T* vp = reinterpret_cast<const T*>(p.vpool) + head * p.ldv * kPage + (key0 % kPage);
-    uint4 ka[KST], kb[KST];
-#pragma unroll
-    for (int s = 0; s < KST; ++s)
-      if (s < ksteps) {
-        ka[s] = *reinterpret_cast<const uint4*>(reinterpret_cast<const char*>(kp + (size_t)r * p.ldk) + s * 64 + g * 16);
-        kb[s] = *reinterpret_cast<const uint4*>(reinterpret_cast<const char*>(kp + (size_t)(16 + r) * p.ldk) + s * 64 + g * 16);
-      }
-    VTerms<T> v[VT];
-#pragma unroll
-    for (int t = 0; t < VT; ++t)
-      if (t < vtiles) v[t].load(vp + (size_t)(t * 16 + r) * kPage, g);
     floatx4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int s = 0; s < KST; ++s)
       if (s < ksteps) {
-        s0 = Elem<T>::mma16(ka[s], q[s], s0);
-        s1 = Elem<T>::mma16(kb[s], q[s], s1);
+        s0 = Elem<T>::mma16(tile.ka[s], q[s], s0);
+        s1 = Elem<T>::mma16(tile.kb[s], q[s], s1);
       }
     float x0[4], x1[4], mx = -INFINITY;
 #pragma unroll
@@ -260,8 +274,10 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
       if (t < vtiles) {
 #pragma unroll
         for (int e = 0; e < 4; ++e) o[t][e] *= a;
-        o[t] = v[t].mma(pt, o[t]);
+        o[t] = tile.v[t].mma(pt, o[t]);
       }
+    j += stride;
+    if (j < tl.n) load_tile(tile, tl.at(j) * 32);
   }
 
   // ---- the waves of the workgroup
@@ -317,20 +333,31 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
   }
   __syncthreads();
   if (!s_last) return;
+  // every split's factor first (all of them requested at once), then the values in batches
+  float* fac = os;  // [gs][nsplit]
+  for (int h = wave; h < gs; h += kRowWaves) {
+    const float* src = p.ws + (wsrow + h0 + h) * p.nsplit * (p.E + 2) + p.E;
+    const bool on = lane < p.nsplit;  // (at most 64 splits)
+    const float m1 = on ? ld_dev(src + (size_t)lane * (p.E + 2)) : -INFINITY;
+    const float l1 = on ? ld_dev(src + (size_t)lane * (p.E + 2) + 1) : 0.f;
+    const float w1 = m1 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m1 - wave_max(m1));
+    const float inv = 1.f / wave_sum(l1 * w1);
+    if (on) fac[h * p.nsplit + lane] = w1 * inv;
+  }
+  __syncthreads();
   for (int i = threadIdx.x; i < gs * p.E; i += 64 * kRowWaves) {
     const int h = i / p.E, d = i % p.E;
-    const float* src = p.ws + (wsrow + h0 + h) * p.nsplit * (p.E + 2);
-    float mm = -INFINITY;
-    for (int s = 0; s < p.nsplit; ++s) mm = fmaxf(mm, ld_dev(src + (size_t)s * (p.E + 2) + p.E));
-    float acc = 0.f, lw = 0.f;
-    for (int s = 0; s < p.nsplit; ++s) {
-      const float* q1 = src + (size_t)s * (p.E + 2);
-      const float ms1 = ld_dev(q1 + p.E);
-      const float w1 = ms1 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(ms1 - mm);
-      acc += ld_dev(q1 + d) * w1;
-      lw += ld_dev(q1 + p.E + 1) * w1;
+    const float* src = p.ws + (wsrow + h0 + h) * p.nsplit * (p.E + 2) + d;
+    float acc = 0.f;
+    for (int s0 = 0; s0 < p.nsplit; s0 += 16) {
+      float v[16];
+#pragma unroll
+      for (int s = 0; s < 16; ++s) v[s] = ld_dev(src + (size_t)min(s0 + s, p.nsplit - 1) * (p.E + 2));
+#pragma unroll
+      for (int s = 0; s < 16; ++s)
+        if (s0 + s < p.nsplit) acc += v[s] * fac[h * p.nsplit + s0 + s];
     }
-    out[(h0 + h) * p.E + d] = Elem<T>::make(acc / lw);
+    out[(h0 + h) * p.E + d] = Elem<T>::make(acc);
   }
 }
 
@@ -562,7 +589,7 @@ int check(const exo_paged_attn* a, const char* what) {
 template <typename T, int DMAX, bool FUSE>
 int launch_rows(const Params& p, hipStream_t st) {
   constexpr int qbytes = 16 * (DMAX + 16 / (int)sizeof(T)) * (int)sizeof(T);
-  const int obytes = kRowWaves * p.gsz * p.ldv * 4;
+  const int obytes = kRowWaves * p.gsz * (p.ldv > 16 ? p.ldv : 16) * 4;  // (the merge's factors: gsz * 64)
   const int lds = qbytes > obytes ? qbytes : obytes;  // at most 64 KiB (16 heads x 256 values x 4 waves)
   exo_note_variant("paged_rows<%s,%d,%s> splits=%d rows=%d", sizeof(T) == 2 ? "bf16" : "f32", DMAX, FUSE ? "fused" : "plain",
                    p.nsplit, p.n);
@@ -643,14 +670,19 @@ extern "C" int exo_paged_attn_rows(const exo_paged_attn* a, int nsplit, int appe
               "exo_paged_attn_rows: bad rows or output");
   EXO_REQUIRE(!append || a->ldq >= (a->heads + a->kv_heads) * a->dim + a->kv_heads * a->vdim,
               "exo_paged_attn_rows: rows of %d elements do not hold q, k and v", a->ldq);
-  EXO_REQUIRE(nsplit >= 1 && nsplit <= 256 &&
+  EXO_REQUIRE(nsplit >= 1 && nsplit <= 64 &&
                   (nsplit == 1 || (workspace && (int64_t)a->n * a->heads <= kCounters && workspace_bytes >= exo_paged_attn_workspace(a->n, a->heads, a->vdim, nsplit))),
               "exo_paged_attn_rows: workspace too small for %d splits", nsplit);
   Params p = params_of(a);
   p.nsplit = nsplit;
   const int group = p.H / p.G;
+  // few (sequence, kv head) pairs: fewer query heads per workgroup, whose keys then come from the
+  // L2 again, but whose merge is shorter
   p.hgroups = (group + 15) / 16;
+  while (nsplit > 1 && p.hgroups < group && p.hgroups < 16 && (int64_t)a->n * p.G * p.hgroups * nsplit * 2 <= 256) p.hgroups *= 2;
+  if (p.hgroups > group) p.hgroups = group;
   p.gsz = (group + p.hgroups - 1) / p.hgroups;
+  p.hgroups = (group + p.gsz - 1) / p.gsz;  // (none without a head)
   p.counters = reinterpret_cast<int*>(workspace);
   p.ws = nsplit > 1 ? reinterpret_cast<float*>(workspace) + kCounters : nullptr;
   const int d = p.ldk > p.ldv ? p.ldk : p.ldv;

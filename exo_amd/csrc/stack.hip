@@ -4,6 +4,7 @@
 // (dense.h); every norm, router and sum here is float32.
 #include "../../include/exo_mi355x.h"
 #include "dense.h"
+#include "route.h"
 
 namespace {
 
@@ -60,76 +61,125 @@ struct MoeSum {        // the feed-forward's output as a sum over a token's expe
   int top, experts, ldy, lds, ldl, gate_col;
 };
 
-// x += gain * v / rms(v), v = the branch row (or the weighted sum over the experts); xb = x
+// x += gain * v / rms(v), v = the branch row (or the weighted sum over the experts); xb = x.
+// Four columns per thread and pass (VEC: rows of four columns are aligned), v in registers.
+constexpr int kCols = 4, kPasses = 16;  // H <= 16384
+
 template <typename T>
+__device__ __forceinline__ void load_cols(const T* p, float (&f)[kCols], bool vec, int left) {
+  if (vec) {
+    if (sizeof(T) == 2) {
+      const uint2 v = *reinterpret_cast<const uint2*>(p);
+      f[0] = bf_lo(v.x), f[1] = bf_hi(v.x), f[2] = bf_lo(v.y), f[3] = bf_hi(v.y);
+    } else {
+      const floatx4 v = *reinterpret_cast<const floatx4*>(p);
+#pragma unroll
+      for (int i = 0; i < kCols; ++i) f[i] = v[i];
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < kCols; ++i) f[i] = i < left ? Elem<T>::load(p[i]) : 0.f;
+  }
+}
+
+template <typename T, int PASSES>
 __global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const float* __restrict__ branch, int ldb,
                                                                     const MoeSum m, const float* __restrict__ gain,
                                                                     float* __restrict__ x, T* __restrict__ xb, int H,
                                                                     int ldx, float eps) {
-  extern __shared__ float v[];  // [H]
   __shared__ float tmp[kRowThreads / 64];
   const int row = blockIdx.x;
   float* xr = x + (size_t)row * H;
-  float ss = 0.f;
+  const bool vec = H % kCols == 0 && (m.y ? m.ldy % kCols == 0 && m.lds % kCols == 0 : ldb % kCols == 0);
+  float v[PASSES][kCols], xv[PASSES][kCols];
+  float pass = 0.f, sg = 0.f;  // weight of the input itself; gate of the shared expert
+  const T *y = nullptr, *sh = nullptr;
   if (m.y) {
-    const T* y = reinterpret_cast<const T*>(m.y) + (size_t)row * m.top * m.ldy;
-    const T* sh = m.shared ? reinterpret_cast<const T*>(m.shared) + (size_t)row * m.lds : nullptr;
-    float pass = 0.f, sg = 0.f;  // weight of the input itself; gate of the shared expert
+    y = reinterpret_cast<const T*>(m.y) + (size_t)row * m.top * m.ldy;
+    if (m.shared) {
+      sh = reinterpret_cast<const T*>(m.shared) + (size_t)row * m.lds;
+      sg = 1.f / (1.f + expf(-m.logits[(size_t)row * m.ldl + m.gate_col]));
+    }
     for (int j = 0; j < m.top; ++j)
       if (m.idx[row * m.top + j] >= m.experts) pass += m.wt[row * m.top + j];
-    if (sh) sg = 1.f / (1.f + expf(-m.logits[(size_t)row * m.ldl + m.gate_col]));
-    for (int c = threadIdx.x; c < H; c += kRowThreads) {
-      float s = pass * xr[c];
-      for (int j = 0; j < m.top; ++j)
-        if (m.idx[row * m.top + j] < m.experts) s += m.wt[row * m.top + j] * Elem<T>::load(y[(size_t)j * m.ldy + c]);
-      if (sh) s += sg * Elem<T>::load(sh[c]);
-      v[c] = s;
-      ss += s * s;
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < PASSES; ++i) {
+    const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
+    if (left <= 0) break;
+    load_cols<float>(xr + c, xv[i], vec, left);
+    if (m.y) {
+#pragma unroll
+      for (int e = 0; e < kCols; ++e) v[i][e] = pass * xv[i][e];
+      for (int j = 0; j < m.top; ++j) {
+        if (m.idx[row * m.top + j] >= m.experts) continue;
+        const float w = m.wt[row * m.top + j];
+        float f[kCols];
+        load_cols<T>(y + (size_t)j * m.ldy + c, f, vec, left);
+#pragma unroll
+        for (int e = 0; e < kCols; ++e) v[i][e] = fmaf(w, f[e], v[i][e]);
+      }
+      if (sh) {
+        float f[kCols];
+        load_cols<T>(sh + c, f, vec, left);
+#pragma unroll
+        for (int e = 0; e < kCols; ++e) v[i][e] = fmaf(sg, f[e], v[i][e]);
+      }
+    } else {
+      load_cols<float>(branch + (size_t)row * ldb + c, v[i], vec, left);
     }
-  } else {
-    for (int c = threadIdx.x; c < H; c += kRowThreads) {
-      const float s = branch[(size_t)row * ldb + c];
-      v[c] = s;
-      ss += s * s;
-    }
+#pragma unroll
+    for (int e = 0; e < kCols; ++e) ss += e < left ? v[i][e] * v[i][e] : 0.f;
   }
   const float inv = 1.f / sqrtf(block_sum(ss, tmp) / H + eps);
-  for (int c = threadIdx.x; c < H; c += kRowThreads) {
-    const float s = xr[c] + v[c] * inv * gain[c];
-    xr[c] = s;
-    xb[(size_t)row * ldx + c] = Elem<T>::make(s);
+#pragma unroll
+  for (int i = 0; i < PASSES; ++i) {
+    const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
+    if (left <= 0) break;
+    float gn[kCols];
+    load_cols<float>(gain + c, gn, H % kCols == 0, left);
+#pragma unroll
+    for (int e = 0; e < kCols; ++e)
+      if (e < left) {
+        const float s = xv[i][e] + v[i][e] * inv * gn[e];
+        xr[c + e] = s;
+        xb[(size_t)row * ldx + c + e] = Elem<T>::make(s);
+      }
   }
 }
 
 // ------------------------------------------------------------------------------ routing
-// One wave per token: softmax over all N outputs, the `top` largest of score + correction (equals:
-// the lower index), weight = score * scale.
-constexpr int kRouteRegs = 8;  // N <= 512
+// One wave per token: softmax over all N <= 64 NR outputs, the `top` largest of score + correction
+// (equals: the lower index), weight = score * scale.  On return lane j < top holds the j-th choice.
+// Reductions on the DPP path; the winner's lane comes from a ballot, so a choice costs about a
+// hundred cycles.
+template <int NR>
 __device__ __forceinline__ void route_choose(const float* __restrict__ logits, const float* __restrict__ corr, int N,
                                              int top, float scale, int lane, int& my_id, float& my_wt) {
-  float s[kRouteRegs], c[kRouteRegs];
+  float s[NR], c[NR];
   float mx = -INFINITY;
 #pragma unroll
-  for (int i = 0; i < kRouteRegs; ++i) {
+  for (int i = 0; i < NR; ++i) {  // unconditional: all requests go out before the first wait
     const int e = min(lane + 64 * i, N - 1);
     s[i] = logits[e];
     c[i] = corr[e];
   }
 #pragma unroll
-  for (int i = 0; i < kRouteRegs; ++i) {
+  for (int i = 0; i < NR; ++i) {
     if (lane + 64 * i >= N) s[i] = -INFINITY;
     mx = fmaxf(mx, s[i]);
   }
-  mx = wave_max(mx);
+  mx = wave_max_f32_uniform(mx);
   float sum = 0.f;
 #pragma unroll
-  for (int i = 0; i < kRouteRegs; ++i) {
+  for (int i = 0; i < NR; ++i) {
     s[i] = expf(s[i] - mx);
     sum += s[i];
   }
-  sum = wave_sum(sum);
+  sum = wave_sum_uniform(sum);
 #pragma unroll
-  for (int i = 0; i < kRouteRegs; ++i) {
+  for (int i = 0; i < NR; ++i) {
     s[i] = s[i] / sum;
     c[i] = lane + 64 * i < N ? s[i] + c[i] : -INFINITY;
   }
@@ -137,37 +187,32 @@ __device__ __forceinline__ void route_choose(const float* __restrict__ logits, c
   my_wt = 0.f;
   for (int j = 0; j < top; ++j) {
     float best = c[0];
-    int bi = 0;
 #pragma unroll
-    for (int i = 1; i < kRouteRegs; ++i)
-      if (c[i] > best) best = c[i], bi = i;
-    int be = lane + 64 * bi;
+    for (int i = 1; i < NR; ++i) best = fmaxf(best, c[i]);
+    best = wave_max_f32_uniform(best);
+    bool found = false;
 #pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ov = __shfl_xor(best, o, 64);
-      const int oe = __shfl_xor(be, o, 64);
-      if (ov > best || (ov == best && oe < be)) best = ov, be = oe;
-    }
-    const int owner = be & 63, reg = be >> 6;
-    float sv = 0.f;
-#pragma unroll
-    for (int i = 0; i < kRouteRegs; ++i)
-      if (i == reg) {
-        sv = s[i];
+    for (int i = 0; i < NR; ++i) {
+      const uint64_t who = __ballot(c[i] == best);
+      if (!found && who) {
+        found = true;
+        const int owner = __builtin_ctzll(who);
+        const float sv = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, s[i]), owner));
         if (lane == owner) c[i] = -INFINITY;
+        if (lane == j) my_id = owner + 64 * i, my_wt = sv * scale;
       }
-    sv = __shfl(sv, owner, 64);
-    if (lane == j) my_id = be, my_wt = sv * scale;
+    }
   }
 }
 
+template <int NR>
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ logits, const float* __restrict__ corr,
                                                        int32_t* __restrict__ idx, float* __restrict__ wt, int N, int ldl,
                                                        int top, float scale) {
   const int row = blockIdx.x, lane = threadIdx.x;
   int id;
   float w;
-  route_choose(logits + (size_t)row * ldl, corr, N, top, scale, lane, id, w);
+  route_choose<NR>(logits + (size_t)row * ldl, corr, N, top, scale, lane, id, w);
   if (lane < top) {
     idx[(size_t)row * top + lane] = id;
     wt[(size_t)row * top + lane] = w;
@@ -188,6 +233,9 @@ struct MoeRows {
   int32_t* idx;        // [R][top]
   float* wt;
   const float* logits; // [R][ldl]
+  const float* corr;   // routing inside the gated launch (null: idx and wt are given)
+  float rscale;
+  int outputs;
   int R, top, experts, ff, sff, H, ldx, lda, ldsa, ldl, gate_col;
   GluConst glu, sglu;
 };
@@ -195,7 +243,9 @@ struct MoeRows {
 constexpr int kBatch = 4;
 constexpr int kGuWaves = 4;
 
-template <typename T>
+// NR > 0: every wave chooses its token's experts itself from the router's logits (no barrier, one
+// launch fewer); the first tile of a token's first pair leaves idx and wt for the launch behind.
+template <typename T, int NR>
 __global__ __launch_bounds__(64 * kGuWaves) void moe_glu_rows_kernel(const MoeRows p) {
   __shared__ float red[kGuWaves][2][256];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x >> 6);
@@ -208,9 +258,22 @@ __global__ __launch_bounds__(64 * kGuWaves) void moe_glu_rows_kernel(const MoeRo
   const uint32_t row_b = (uint32_t)p.ldx * sizeof(T);
   if (b < pairs * tiles) {
     const int pair = b / tiles;
-    const int e = p.idx[pair];
-    if (e >= p.experts) return;  // whole workgroup: the input itself, nothing to multiply
+    const int t = pair / p.top, slot = pair - t * p.top;
     b -= pair * tiles;
+    int e;
+    if constexpr (NR > 0) {
+      int id;
+      float w;
+      route_choose<NR>(p.logits + (size_t)t * p.ldl, p.corr, p.outputs, p.top, p.rscale, lane, id, w);
+      if (b == 0 && slot == 0 && wave == 0 && lane < p.top) {
+        p.idx[pair + lane] = id;
+        p.wt[pair + lane] = w;
+      }
+      e = __builtin_amdgcn_readlane(id, slot);
+    } else {
+      e = __builtin_amdgcn_readfirstlane(p.idx[pair]);
+    }
+    if (e >= p.experts) return;  // whole workgroup: the input itself, nothing to multiply
     const size_t off = (size_t)e * p.ff * row_b;
     wg = reinterpret_cast<const char*>(p.gate) + off;
     wu = reinterpret_cast<const char*>(p.up) + off;
@@ -271,7 +334,7 @@ __global__ __launch_bounds__(64 * kGuWaves) void moe_glu_rows_kernel(const MoeRo
   }
 }
 
-constexpr int kDnWaves = 8;
+constexpr int kDnWaves = 16, kDnBatch = 8;
 
 // out[t] = sum of weight * (down @ act) over the token's experts, + gate * shared, + weight * input
 template <typename T>
@@ -285,6 +348,9 @@ __global__ __launch_bounds__(64 * kDnWaves) void moe_down_rows_kernel(const MoeR
   const int units = p.top * es + ss, per = (units + kDnWaves - 1) / kDnWaves;
   int u = min(units, wave * per);
   const int u1 = min(units, u + per);
+  // the token's choice in lanes 0 .. top - 1
+  const int my_id = p.idx[t * p.top + min(lane, p.top - 1)];
+  const float my_wt = p.wt[t * p.top + min(lane, p.top - 1)];
   float tot[4] = {0.f, 0.f, 0.f, 0.f};
   while (u < u1) {  // the part of one expert's K range that falls into this wave's share
     const int slot = min(u / es, p.top);
@@ -301,9 +367,9 @@ __global__ __launch_bounds__(64 * kDnWaves) void moe_down_rows_kernel(const MoeR
       a = reinterpret_cast<const char*>(p.sact) + (size_t)t * srow;
       rowb = srow;
     } else {
-      const int e = p.idx[t * p.top + slot];
+      const int e = __builtin_amdgcn_readlane(my_id, slot);
       if (e >= p.experts) continue;
-      wt = p.wt[t * p.top + slot];
+      wt = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, my_wt), slot));
       w = reinterpret_cast<const char*>(p.down) + (size_t)e * p.H * arow;
       a = reinterpret_cast<const char*>(p.act) + (size_t)(t * p.top + slot) * arow;
       rowb = arow;
@@ -311,16 +377,16 @@ __global__ __launch_bounds__(64 * kDnWaves) void moe_down_rows_kernel(const MoeR
     const __amdgpu_buffer_rsrc_t rw = buf_of(w + (size_t)n0 * rowb, (uint32_t)nrows * rowb);
     const __amdgpu_buffer_rsrc_t rx = buf_of(a, rowb);
     floatx4 acc = {0.f, 0.f, 0.f, 0.f};
-    for (int s = s0; s < s1; s += kBatch) {
-      uint4 wv[kBatch], xv[kBatch];
+    for (int s = s0; s < s1; s += kDnBatch) {
+      uint4 wv[kDnBatch], xv[kDnBatch];
 #pragma unroll
-      for (int i = 0; i < kBatch; ++i) {
+      for (int i = 0; i < kDnBatch; ++i) {
         const bool ok = s + i < s1;
         wv[i] = buf_load16(rw, ok ? r * rowb + g * 16 + (s + i) * 64 : kPastEnd, 0);
         xv[i] = buf_load16(rx, ok ? g * 16 + (s + i) * 64 : kPastEnd, 0);  // every column: the one row
       }
 #pragma unroll
-      for (int i = 0; i < kBatch; ++i) acc = Elem<T>::mma16(wv[i], xv[i], acc);
+      for (int i = 0; i < kDnBatch; ++i) acc = Elem<T>::mma16(wv[i], xv[i], acc);
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e) tot[e] = fmaf(wt, acc[e], tot[e]);
@@ -329,15 +395,13 @@ __global__ __launch_bounds__(64 * kDnWaves) void moe_down_rows_kernel(const MoeR
 #pragma unroll
     for (int e = 0; e < 4; ++e) red[wave][4 * g + e] = tot[e];
   }
+  const float pass = wave_sum_uniform(lane < p.top && my_id >= p.experts ? my_wt : 0.f);  // the input's own weight
   __syncthreads();
   if (threadIdx.x < (unsigned)nrows) {
     const int n = threadIdx.x;
     float v = 0.f;
 #pragma unroll
     for (int w = 0; w < kDnWaves; ++w) v += red[w][n];
-    float pass = 0.f;
-    for (int j = 0; j < p.top; ++j)
-      if (p.idx[t * p.top + j] >= p.experts) pass += p.wt[t * p.top + j];
     if (pass != 0.f) v += pass * p.xres[(size_t)t * p.H + n0 + n];
     p.out[(size_t)t * p.H + n0 + n] = v;
   }
@@ -382,13 +446,22 @@ extern "C" int exo_norm_rows(const float* x, const int32_t* rows, const float* g
 
 static int post_norm(const float* branch, int ldb, const MoeSum& m, const float* gain, float* x, void* xb, int n, int H,
                      int ldx, float eps, int dtype, exo_stream_t stream) {
-  EXO_REQUIRE(gain && x && xb && n >= 0 && H > 0 && H <= 16000 && ldx >= H, "exo_post_norm_add: bad argument (H=%d)", H);
+  EXO_REQUIRE(gain && x && xb && n >= 0 && H > 0 && H <= 16384 && ldx >= H, "exo_post_norm_add: bad argument (H=%d)", H);
   if (n == 0) return EXO_OK;
-  const size_t lds = (size_t)H * 4;
-  if (dtype == 0)
-    post_norm_add_kernel<bf16_t><<<n, kRowThreads, lds, (hipStream_t)stream>>>(branch, ldb, m, gain, x, (bf16_t*)xb, H, ldx, eps);
-  else
-    post_norm_add_kernel<float><<<n, kRowThreads, lds, (hipStream_t)stream>>>(branch, ldb, m, gain, x, (float*)xb, H, ldx, eps);
+#define EXO_POST(P)                                                                                              \
+  do {                                                                                                           \
+    if (dtype == 0)                                                                                              \
+      post_norm_add_kernel<bf16_t, P><<<n, kRowThreads, 0, (hipStream_t)stream>>>(branch, ldb, m, gain, x, (bf16_t*)xb, H, ldx, eps); \
+    else                                                                                                         \
+      post_norm_add_kernel<float, P><<<n, kRowThreads, 0, (hipStream_t)stream>>>(branch, ldb, m, gain, x, (float*)xb, H, ldx, eps);   \
+  } while (0)
+  const int passes = exo_ceil_div(H, kRowThreads * kCols);
+  if (passes <= 1) EXO_POST(1);
+  else if (passes <= 2) EXO_POST(2);
+  else if (passes <= 4) EXO_POST(4);
+  else if (passes <= 8) EXO_POST(8);
+  else EXO_POST(16);
+#undef EXO_POST
   EXO_CHECK_LAUNCH("exo_post_norm_add");
   return EXO_OK;
 }
@@ -414,10 +487,11 @@ extern "C" int exo_moe_sum_post_norm(const void* y, const int32_t* idx, const fl
 extern "C" int exo_moe_route(const float* logits, const float* correction, int32_t* idx, float* wt, int rows, int n,
                              int ldl, int top, float scale, exo_stream_t stream) {
   EXO_REQUIRE(logits && correction && idx && wt, "exo_moe_route: null pointer");
-  EXO_REQUIRE(rows >= 0 && n > 0 && n <= 64 * kRouteRegs && ldl >= n && top > 0 && top <= 64 && top <= n,
-              "exo_moe_route: need 0 < n <= %d and 0 < top <= min(64, n); got n=%d top=%d", 64 * kRouteRegs, n, top);
+  EXO_REQUIRE(rows >= 0 && n > 0 && n <= 512 && ldl >= n && top > 0 && top <= 64 && top <= n,
+              "exo_moe_route: need 0 < n <= %d and 0 < top <= min(64, n); got n=%d top=%d", 512, n, top);
   if (rows == 0) return EXO_OK;
-  moe_route_kernel<<<rows, 64, 0, (hipStream_t)stream>>>(logits, correction, idx, wt, n, ldl, top, scale);
+  const auto fn = n <= 64 ? moe_route_kernel<1> : n <= 128 ? moe_route_kernel<2> : n <= 256 ? moe_route_kernel<4> : moe_route_kernel<8>;
+  fn<<<rows, 64, 0, (hipStream_t)stream>>>(logits, correction, idx, wt, n, ldl, top, scale);
   EXO_CHECK_LAUNCH("exo_moe_route");
   return EXO_OK;
 }
@@ -427,7 +501,8 @@ static MoeRows moe_rows_of(const exo_moe_rows* a) {
   p.x = a->x, p.gate = a->gate, p.up = a->up, p.down = a->down;
   p.sgate = a->shared_gate, p.sup = a->shared_up, p.sdown = a->shared_down;
   p.act = a->act, p.sact = a->shared_act, p.out = a->out, p.xres = a->x_res;
-  p.idx = a->idx, p.wt = a->wt, p.logits = a->logits;
+  p.idx = a->idx, p.wt = a->wt, p.logits = a->logits, p.corr = a->correction, p.rscale = a->router_scale;
+  p.outputs = a->outputs;
   p.R = a->rows, p.top = a->top, p.experts = a->experts, p.ff = a->ff, p.sff = a->shared_ff, p.H = a->H;
   p.ldx = a->ldx, p.lda = a->lda, p.ldsa = a->ldsa, p.ldl = a->ldl, p.gate_col = a->gate_col;
   p.glu = GluConst{a->limit, a->alpha, a->shift};
@@ -436,8 +511,10 @@ static MoeRows moe_rows_of(const exo_moe_rows* a) {
 }
 static int moe_rows_check(const exo_moe_rows* a) {
   EXO_REQUIRE(a && (a->dtype == 0 || a->dtype == 1), "exo_moe_rows: bad dtype");
-  EXO_REQUIRE(a->rows > 0 && a->rows <= 16 && a->top > 0 && a->experts > 0 && a->ff > 0 && a->H > 0,
-              "exo_moe_rows: need 1..16 rows and positive sizes (rows=%d)", a->rows);
+  EXO_REQUIRE(a->rows > 0 && a->rows <= 16 && a->top > 0 && a->experts > 0 && a->ff > 0 && a->H > 0 && a->top <= 64,
+              "exo_moe_rows: need 1..16 rows, top <= 64 and positive sizes (rows=%d top=%d)", a->rows, a->top);
+  EXO_REQUIRE(!a->correction || (a->logits && a->outputs >= a->top && a->outputs <= 512 && a->ldl >= a->outputs),
+              "exo_moe_rows: bad router (%d outputs)", a->outputs);
   EXO_REQUIRE(a->ldx % 64 == 0 && a->lda % 64 == 0 && a->ldx >= a->H && a->lda >= a->ff,
               "exo_moe_rows: row strides must be multiples of 64 (ldx=%d lda=%d)", a->ldx, a->lda);
   EXO_REQUIRE(a->x && a->gate && a->up && a->down && a->act && a->out && a->x_res && a->idx && a->wt,
@@ -454,7 +531,20 @@ extern "C" int exo_moe_glu_rows(const exo_moe_rows* a, exo_stream_t stream) {
   const int dtype = a->dtype;
   const MoeRows p = moe_rows_of(a);
   const int grid = p.R * p.top * exo_ceil_div(p.ff, 16) + (p.sgate ? exo_ceil_div(p.sff, 16) : 0);
-  EXO_LAUNCH_T(moe_glu_rows_kernel, grid, 64 * kGuWaves, 0, p);
+  const int n = p.corr ? p.outputs : 0;
+#define EXO_GLU(NR)                                                                                   \
+  do {                                                                                                \
+    if (dtype == 0)                                                                                   \
+      moe_glu_rows_kernel<bf16_t, NR><<<grid, 64 * kGuWaves, 0, (hipStream_t)stream>>>(p);            \
+    else                                                                                              \
+      moe_glu_rows_kernel<float, NR><<<grid, 64 * kGuWaves, 0, (hipStream_t)stream>>>(p);             \
+  } while (0)
+  if (n == 0) EXO_GLU(0);
+  else if (n <= 64) EXO_GLU(1);
+  else if (n <= 128) EXO_GLU(2);
+  else if (n <= 256) EXO_GLU(4);
+  else EXO_GLU(8);
+#undef EXO_GLU
   EXO_CHECK_LAUNCH("exo_moe_glu_rows");
   return EXO_OK;
 }

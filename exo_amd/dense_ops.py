@@ -112,7 +112,7 @@ def grouped_gemm(x, w, group_ws, out, T: int, topk: int, up=None, spec=None, x_p
 
 class ExpertRows:
     """The experts of a decode step (up to 16 rows): argument block built once per layer and
-    buffer set, launched as gated products and as weighted down-projections."""
+    buffer set, launched as gated products (which also route) and as weighted down-projections."""
 
     def __init__(self, moe, w, bf, H: int):
         """``moe``: MoeSpec; ``w``: the layer's tensors; ``bf``: the activation buffers."""
@@ -125,7 +125,7 @@ class ExpertRows:
             x_res=p(bf.h), idx=p(bf.idx(r.top)), wt=p(bf.wt(r.top)), logits=p(bf.router_logits(w.router.shape[0])),
             correction=p(w.correction),
             top=r.top, experts=r.experts, ff=e.ff, shared_ff=s.ff if s else 0, H=H, ldx=bf.xb.shape[1],
-            lda=pad64(e.ff), ldsa=pad64(s.ff) if s else 0, ldl=w.router.shape[0], gate_col=r.outputs,
+            lda=pad64(e.ff), ldsa=pad64(s.ff) if s else 0, ldl=w.router.shape[0], gate_col=r.outputs, outputs=r.outputs, router_scale=r.scale,
             dtype=_code(bf.xb), limit=e.limit, alpha=e.alpha, shift=e.shift,
             shared_limit=s.limit if s else 0.0, shared_alpha=s.alpha if s else 0.0, shared_shift=s.shift if s else 0.0)
 
@@ -190,7 +190,9 @@ class PagedAttention:
         s = self.spec
         tiles = -(-self.visible(keys) // 32) + 2
         wgs = n * s.kv_heads * (-(-(s.heads // s.kv_heads) // 16))
-        nsplit = max(1, min(-(-tiles // 4), 512 // wgs, 64))
+        nsplit = max(1, min(-(-tiles // 4), 256 // wgs, 16))
+        if nsplit > 8:
+            nsplit -= nsplit % 8  # (the head groups of one split then share an XCD's L2)
         if n * s.heads > 16384:
             nsplit = 1
         ws = attn_workspace(n, s.heads, s.vdim, nsplit, qkv.device) if nsplit > 1 else None

@@ -23,8 +23,8 @@ class MoeRows(C.Structure):
     _fields_ = [(n, _vp) for n in ("x", "gate", "up", "down", "shared_gate", "shared_up", "shared_down", "act",
                                    "shared_act", "out", "x_res", "idx", "wt", "logits", "correction")] + \
                [(n, _i) for n in ("rows", "top", "experts", "ff", "shared_ff", "H", "ldx", "lda", "ldsa", "ldl",
-                                  "gate_col", "dtype")] + \
-               [(n, _f) for n in ("limit", "alpha", "shift", "shared_limit", "shared_alpha", "shared_shift")]
+                                  "gate_col", "outputs", "dtype")] + \
+               [(n, _f) for n in ("router_scale", "limit", "alpha", "shift", "shared_limit", "shared_alpha", "shared_shift")]
 
 
 class PagedAttn(C.Structure):

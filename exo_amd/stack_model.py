@@ -267,7 +267,6 @@ class StackModel(DecoderShard):
         r, eps = f.router, self.cfg.eps
         logits, idx, wt = bf.router_logits(L.router.shape[0]), bf.idx(r.top), bf.wt(r.top)
         D.linear(bf.xb, L.router, logits, n)
-        D.moe_route(logits, L.correction, r.scale, idx, wt, n)
         if n <= D.GEMV_MAX_ROWS:
             ex = bf.experts.get(L.index)
             if ex is None:
@@ -276,6 +275,7 @@ class StackModel(DecoderShard):
             ex.down(n)
             D.post_norm_add(bf.branch, L.norm2, eps, bf.h, bf.xb, n)
             return
+        D.moe_route(logits, L.correction, r.scale, idx, wt, n)
         act, out = bf.act(r.top, f.expert.ff), bf.expert_out(r.top)
         ws = ops.moe_group(idx[:n], r.experts, check_indices=False)  # identity ids are past the end: left out
         D.grouped_gemm(bf.xb, L.gate, ws, act, n, r.top, up=L.up, spec=f.expert)

@@ -473,7 +473,9 @@ int exo_dense_grouped_gemm(const void* x, const void* w, const void* w_up, const
                            int x_per_pair, int E, int N, int ldx, int ldw, int ldy, int dtype,
                            exo_stream_t stream);
 
-/* Experts of a decode step (up to 16 rows): gated products, then the weighted sum. */
+/* Experts of a decode step (up to 16 rows): gated products, then the weighted sum.  correction
+ * non-null: the gated launch also routes (as exo_moe_route over `outputs` logits) and leaves idx
+ * and wt; null: they are given. */
 typedef struct {
   const void *x, *gate, *up, *down, *shared_gate, *shared_up, *shared_down;
   void *act, *shared_act;
@@ -482,8 +484,8 @@ typedef struct {
   int32_t* idx;
   float* wt;
   const float *logits, *correction;
-  int rows, top, experts, ff, shared_ff, H, ldx, lda, ldsa, ldl, gate_col, dtype;
-  float limit, alpha, shift, shared_limit, shared_alpha, shared_shift;
+  int rows, top, experts, ff, shared_ff, H, ldx, lda, ldsa, ldl, gate_col, outputs, dtype;
+  float router_scale, limit, alpha, shift, shared_limit, shared_alpha, shared_shift;
 } exo_moe_rows;
 int exo_moe_glu_rows(const exo_moe_rows* args, exo_stream_t stream);
 int exo_moe_down_rows(const exo_moe_rows* args, exo_stream_t stream);
