@@ -508,8 +508,16 @@ def gekazen_launches(torch, m, B, ctx):
     def mm(n, k, extra=0):
         return 2 * n * k + 2 * B * (n + k) + extra, 2 * B * n * k
     nq = Ls[0].qkv.shape[0]
-    fused = hasattr(m, "_fused_rows") and not prompt and m._fused_rows(B)
-    add("qkv + bias", lambda L: D.linear(bf.xb, L.qkv, qkv, B, bias=L.qkv_b), *mm(nq, H))
+    fused = not prompt and D.post_linear_fits(B, Ls[0].qkv, bf.xb, H)  # norm + residual inside the next product
+    other = torch.empty_like(bf.h)
+
+    def product(L, w, out, bias=None, xb=None):
+        if fused:
+            D.post_linear(bf.h, bf.branch, L.norm1, c.eps, other, xb, w, out, B, bias)
+        else:
+            D.linear(bf.xb, w, out, B, bias=bias)
+    pre = "norm, residual, " if fused else ""
+    add(pre + "qkv + bias", lambda L: product(L, L.qkv, qkv, L.qkv_b), *mm(nq, H))
     if prompt:
         add("append keys, values", lambda L: att[L.index].append(qkv, batch.slot, batch.pos, B), 2 * kvb, 0)
         add("attention", lambda L: att[L.index].prompt(qkv, out, *batch.blocks[att[0].prompt_block(a)]),
@@ -518,28 +526,31 @@ def gekazen_launches(torch, m, B, ctx):
         add("norm, append, attention", lambda L: att[L.index].rows(qkv, out, batch.slot, batch.pos, B, batch.keys, append=True),
             kvb, 2 * sum(vis) * a.heads * (a.dim + a.vdim))
     add("o + bias", lambda L: D.linear(out, L.o, bf.branch, B, bias=L.o_b), *mm(H, a.heads * a.vdim))
-    add("norm + residual", lambda L: D.post_norm_add(bf.branch, L.norm1, c.eps, bf.h, bf.xb, B), B * H * 14, 0)
+    if not fused:
+        add("norm + residual (twice a layer)" if not prompt else "norm + residual",
+            lambda L: D.post_norm_add(bf.branch, L.norm1, c.eps, bf.h, bf.xb, B), B * H * 14, 0)
     lg, idx, wt = bf.router_logits(Ls[0].router.shape[0]), bf.idx(r.top), bf.wt(r.top)
-    add("router", lambda L: D.linear(bf.xb, L.router, lg, B), *mm(Ls[0].router.shape[0], H))
-    add("routing", lambda L: D.moe_route(lg, L.correction, r.scale, idx, wt, B), B * r.outputs * 4, 0)
+    add(pre + "router", lambda L: product(L, L.router, lg, xb=bf.xb), *mm(Ls[0].router.shape[0], H))
+    if prompt:
+        add("routing", lambda L: D.moe_route(lg, L.correction, r.scale, idx, wt, B), B * r.outputs * 4, 0)
     per = 2 * e.ff * H
     sh = f.shared.ff * H * 2
     if not prompt:
-        for L in Ls:  # each layer's own choice, so that its experts are the ones it streams
-            pass
+        for L in Ls:
+            if (L.index, bf.cur) not in bf.experts:
+                bf.experts[L.index, bf.cur] = D.ExpertRows(f, L, bf, H, bf.h)
+        ex = [bf.experts[L.index, bf.cur] for L in Ls]
+        # every layer streams the experts it chose in the forward above
+        logits = [torch.full((B, lg.shape[1]), -30.0, device="cuda").scatter_(1, p.long().to("cuda"), 3.0) for p in picks]
+        set_logits = [(lambda t=t: lg[:B].copy_(t)) for t in logits]
         chosen = [p.to("cuda") for p in picks]
-
-        def with_picks(fn):
-            def go(L):
-                bf.idx(r.top).copy_(chosen[L.index - Ls[0].index])
-                fn(L)
-            return go
-        base = time_launches(torch, [(lambda L=L: bf.idx(r.top).copy_(chosen[L.index - Ls[0].index])) for L in Ls])
-        for name, fn, mats in (("experts: gate, up (+ shared)", lambda L: bf.experts[L.index].glu(B), 2),
-                               ("experts: down, weighted sum (+ shared)", lambda L: bf.experts[L.index].down(B), 1)):
-            us = time_launches(torch, [(lambda L=L, f=with_picks(fn): f(L)) for L in Ls]) - base
+        set_idx = [(lambda t=t: idx[:B].copy_(t)) for t in chosen]
+        both = lambda a, b: (lambda: (a(), b()))  # noqa: E731
+        for name, pre_fns, fns, mats in (
+                ("routing, experts: gate, up (+ shared)", set_logits, [(lambda x=x: x.glu(B)) for x in ex], 2),
+                ("experts: down, weighted sum (+ shared)", set_idx, [(lambda x=x: x.down(B)) for x in ex], 1)):
+            us = time_launches(torch, [both(a, b) for a, b in zip(pre_fns, fns)]) - time_launches(torch, pre_fns)
             rows.append(row_of(name, us, mats * (experts * per + sh), mats * 2 * (pairs * e.ff * H + B * f.shared.ff * H)))
-        add("norm + residual (2)", lambda L: D.post_norm_add(bf.branch, L.norm2, c.eps, bf.h, bf.xb, B), B * H * 14, 0)
     else:
         act, eo = bf.act(r.top, e.ff), bf.expert_out(r.top)
         bf.idx(r.top)[:B].copy_(picks[0].to("cuda"))

@@ -9,7 +9,7 @@
 //    tail: rows past N, x rows past M and steps past a wave's range read as zero.
 //  * dense_gemm_kernel, any number of rows: a (64 MI) x (64 NJ) tile per workgroup of four waves
 //    (2 x 2, each (32 MI) x (32 NJ) in 32x32 products), K steps of 128 bytes per row through two
-//    LDS buffers, the next step's vectors in registers meanwhile; one barrier per step.  A row's
+//    LDS buffers, the next three steps' vectors in registers meanwhile; one barrier per step.  A row's
 //    eight 16-byte chunks sit at slot chunk ^ (row % 8), so operand reads of 32 rows meet no bank
 //    twice.  PAIR: the weight tile holds rows of a gate and an up matrix, 32 and 32, so that a
 //    wave's column tiles are (gate, up) of the same outputs and the gated unit is its epilogue.
@@ -38,27 +38,32 @@ __device__ __forceinline__ void store_out(void* y, size_t i, float v, int y_f32)
     reinterpret_cast<T*>(y)[i] = Elem<T>::make(v);
 }
 
-// acc += the products of 16 weight rows (buffer rw, lane offset woff) with x (rx, xoff) over the
-// 64-byte steps [s0, s1)
-template <typename T>
-__device__ __forceinline__ floatx4 gemv_span(__amdgpu_buffer_rsrc_t rw, uint32_t woff,
-                                             __amdgpu_buffer_rsrc_t rx, uint32_t xoff, int s0, int s1,
-                                             floatx4 acc) {
-  for (int s = s0; s < s1; s += kBatch) {
-    uint4 wv[kBatch], xv[kBatch];
-#pragma unroll
-    for (int i = 0; i < kBatch; ++i) wv[i] = buf_load16(rw, s + i < s1 ? woff + (s + i) * 64 : kPastEnd, 0);
-#pragma unroll
-    for (int i = 0; i < kBatch; ++i) xv[i] = buf_load16(rx, s + i < s1 ? xoff + (s + i) * 64 : kPastEnd, 0);
-#pragma unroll
-    for (int i = 0; i < kBatch; ++i) acc = Elem<T>::mma16(wv[i], xv[i], acc);
-  }
-  return acc;
+// Norm of the previous sublayer's output and residual sum, in front of the product that reads the
+// residual: every workgroup forms x + gain * branch / rms(branch) for itself (in LDS, element type),
+// workgroup 0 also writes it out - to another buffer than it is read from, since the others may
+// still be reading.
+struct PostNorm {
+  const float* x;       // [M][H]
+  const float* branch;  // [M][H]
+  const float* gain;    // [H]
+  float* x_out;         // [M][H]
+  void* xb_out;         // T [M][ldx], or null
+  int H;
+  float eps;
+};
+constexpr int kPostPasses = 4;  // float4 per lane of a row's waves
+
+__host__ __device__ inline int post_waves_per_row(int M, int NW) {
+  int p = 1;
+  while (p < M) p *= 2;
+  return NW > p ? NW / p : 1;
 }
 
-template <typename T, int NW>
-__global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p) {
+template <typename T, int NW, bool POST>
+__global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p, const PostNorm q) {
   __shared__ float red[NW][256];
+  __shared__ float part[NW];
+  extern __shared__ __attribute__((aligned(16))) char xs[];  // POST: [M][ldx * sizeof(T) + 16]
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x >> 6);
   const int r = lane & 15, g = lane >> 4;
   const int n0 = blockIdx.x * 16, rows = min(16, p.N - n0);
@@ -68,8 +73,87 @@ __global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p)
   const __amdgpu_buffer_rsrc_t rw =
       buf_of(reinterpret_cast<const char*>(p.w) + (size_t)n0 * wrow, (uint32_t)rows * wrow);
   const __amdgpu_buffer_rsrc_t rx = buf_of(p.x, (uint32_t)p.M * xrow);
+  const uint32_t woff = r * wrow + g * 16;
+  uint4 wv[kBatch];
+  auto load_w = [&](int s) {
+#pragma unroll
+    for (int i = 0; i < kBatch; ++i) wv[i] = buf_load16(rw, s + i < s1 ? woff + (s + i) * 64 : kPastEnd, 0);
+  };
+  if (POST) {
+    // a row's columns over wpr waves; its inputs are requested ahead of the first weights
+    const int wpr = post_waves_per_row(p.M, NW), rpi = NW / wpr;  // rows per iteration
+    const uint32_t lrow = xrow + 16;
+    const bool vec = q.H % 4 == 0;
+    for (int m0 = 0; m0 < p.M; m0 += rpi) {
+      const int m = m0 + wave / wpr, c0 = ((wave % wpr) * 64 + lane) * 4, cs = wpr * 256;
+      floatx4 v[kPostPasses], x[kPostPasses], gn[kPostPasses];
+      float ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < kPostPasses; ++i) {
+        const int c = c0 + i * cs;
+        v[i] = x[i] = gn[i] = floatx4{0.f, 0.f, 0.f, 0.f};
+        if (m < p.M && c < q.H) {
+          const size_t o = (size_t)m * q.H + c;
+          if (vec) {
+            v[i] = *reinterpret_cast<const floatx4*>(q.branch + o);
+            x[i] = *reinterpret_cast<const floatx4*>(q.x + o);
+            gn[i] = *reinterpret_cast<const floatx4*>(q.gain + c);
+          } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (c + e < q.H) v[i][e] = q.branch[o + e], x[i][e] = q.x[o + e], gn[i][e] = q.gain[c + e];
+          }
+        }
+      }
+      if (m0 == 0) load_w(s0);
+#pragma unroll
+      for (int i = 0; i < kPostPasses; ++i)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss += v[i][e] * v[i][e];
+      ss = wave_sum(ss);
+      __syncthreads();  // (the sums of an earlier iteration have been read)
+      if (lane == 0) part[wave] = ss;
+      __syncthreads();
+      float tot = 0.f;
+      for (int w = 0; w < wpr; ++w) tot += part[wave / wpr * wpr + w];
+      const float inv = 1.f / sqrtf(tot / q.H + q.eps);
+#pragma unroll
+      for (int i = 0; i < kPostPasses; ++i) {
+        const int c = c0 + i * cs;
+        if (m >= p.M || c >= p.ldx) continue;
+        T out[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float y = x[i][e] + v[i][e] * inv * gn[i][e];  // zero past H
+          out[e] = Elem<T>::make(y);
+          if (blockIdx.x == 0 && c + e < q.H) {
+            q.x_out[(size_t)m * q.H + c + e] = y;
+            if (q.xb_out) reinterpret_cast<T*>(q.xb_out)[(size_t)m * p.ldx + c + e] = out[e];
+          }
+        }
+        T* dst = reinterpret_cast<T*>(xs + m * lrow) + c;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) dst[e] = out[e];
+      }
+    }
+    __syncthreads();
+  } else {
+    load_w(s0);
+  }
   floatx4 acc = {0.f, 0.f, 0.f, 0.f};
-  acc = gemv_span<T>(rw, r * wrow + g * 16, rx, r * xrow + g * 16, s0, s1, acc);
+  for (int s = s0; s < s1; s += kBatch) {
+    uint4 xv[kBatch];
+#pragma unroll
+    for (int i = 0; i < kBatch; ++i) {
+      if (POST)  // (steps past the range: any finite values, their weights are zero)
+        xv[i] = *reinterpret_cast<const uint4*>(xs + min(r, p.M - 1) * (xrow + 16) + g * 16 + min(s + i, s1 - 1) * 64);
+      else
+        xv[i] = buf_load16(rx, s + i < s1 ? r * xrow + g * 16 + (s + i) * 64 : kPastEnd, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < kBatch; ++i) acc = Elem<T>::mma16(wv[i], xv[i], acc);
+    if (s + kBatch < s1) load_w(s + kBatch);
+  }
 #pragma unroll
   for (int e = 0; e < 4; ++e) red[wave][r * 16 + 4 * g + e] = acc[e];  // [m][n]
   __syncthreads();
@@ -104,10 +188,11 @@ struct GemmParams {
 };
 
 template <typename T, int MI, int NJ, bool GROUPED, bool PAIR>
-__global__ __launch_bounds__(256) void dense_gemm_kernel(const GemmParams p) {
+__global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const GemmParams p) {
   constexpr int BM = 64 * MI, BW = 64 * NJ;      // tile rows of x, of weights
   constexpr int BN = PAIR ? BW / 2 : BW;         // output columns
   constexpr int XV = BM * 8 / 256, WV = BW * 8 / 256;
+  constexpr int PD = 3;
   extern __shared__ __attribute__((aligned(16))) char lds[];  // [2][(BM + BW) * 128]
   __shared__ int row_pair[GROUPED ? BM : 1];
   constexpr int BUF = (BM + BW) * 128;
@@ -167,26 +252,28 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const GemmParams p) {
     const int n = PAIR ? (i / NJ) * (16 * NJ) + ((i % NJ) >> 1) * 32 + (tr & 31) : tr;
     woff[i] = (uint32_t)n * wrow + c * 16;
   }
-  uint4 xr[XV], wr[WV];
-  auto load_regs = [&](int s) {
-    const uint32_t so = (uint32_t)(k0 + s) * 128;
+  // PD steps of tiles in flight in registers.  Requests past the last step re-read it: every load
+  // is unconditional, so the waits count exactly the loads in front of the ones they are for.
+  uint4 xr[PD][XV], wr[PD][WV];
+  auto load_regs = [&](uint4 (&x)[XV], uint4 (&w)[WV], int s) {
+    const uint32_t so = (uint32_t)(k0 + min(s, steps - 1)) * 128;
 #pragma unroll
-    for (int i = 0; i < XV; ++i) xr[i] = buf_load16(rx, xoff[i], so);
+    for (int i = 0; i < XV; ++i) x[i] = buf_load16(rx, xoff[i], so);
 #pragma unroll
-    for (int i = 0; i < WV; ++i) wr[i] = buf_load16(rw[PAIR ? (i % NJ) & 1 : 0], woff[i], so);
+    for (int i = 0; i < WV; ++i) w[i] = buf_load16(rw[PAIR ? (i % NJ) & 1 : 0], woff[i], so);
   };
-  auto store_lds = [&](int b) {
+  auto store_lds = [&](const uint4 (&x)[XV], const uint4 (&w)[WV], int b) {
     char* xl = lds + b * BUF;
     char* wl = xl + BM * 128;
 #pragma unroll
     for (int i = 0; i < XV; ++i) {
       const int id = tid + 256 * i, tr = id >> 3, c = id & 7;
-      *reinterpret_cast<uint4*>(xl + tr * 128 + ((c ^ (tr & 7)) << 4)) = xr[i];
+      *reinterpret_cast<uint4*>(xl + tr * 128 + ((c ^ (tr & 7)) << 4)) = x[i];
     }
 #pragma unroll
     for (int i = 0; i < WV; ++i) {
       const int id = tid + 256 * i, tr = id >> 3, c = id & 7;
-      *reinterpret_cast<uint4*>(wl + tr * 128 + ((c ^ (tr & 7)) << 4)) = wr[i];
+      *reinterpret_cast<uint4*>(wl + tr * 128 + ((c ^ (tr & 7)) << 4)) = w[i];
     }
   };
   const int frow = lane & 31, half = lane >> 5;
@@ -198,29 +285,34 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const GemmParams p) {
 #pragma unroll
       for (int e = 0; e < 16; ++e) acc[i][j][e] = 0.f;
 
-  load_regs(0);
-  store_lds(0);
-  if (steps > 1) load_regs(1);
-  for (int s = 0; s < steps; ++s) {
-    __syncthreads();  // step s is complete in its buffer, the other buffer is no longer read
-    if (s + 1 < steps) {
-      store_lds((s + 1) & 1);
-      if (s + 2 < steps) load_regs(s + 2);
-    }
-    const char* xl = lds + (s & 1) * BUF + (wm + frow) * 128;
-    const char* wl = lds + (s & 1) * BUF + (BM + wn + frow) * 128;
 #pragma unroll
-    for (int t = 0; t < 4; ++t) {
-      const int slot = ((2 * t + half) ^ (frow & 7)) << 4;
-      uint4 a[MI], b[NJ];
+  for (int u = 0; u < PD; ++u) load_regs(xr[u], wr[u], u);
+  store_lds(xr[0], wr[0], 0);
+  load_regs(xr[0], wr[0], PD);
+  for (int s0 = 0; s0 < steps; s0 += PD) {
 #pragma unroll
-      for (int i = 0; i < MI; ++i) a[i] = *reinterpret_cast<const uint4*>(xl + i * 4096 + slot);
+    for (int u = 0; u < PD; ++u) {
+      const int s = s0 + u;
+      if (s >= steps) break;
+      __syncthreads();  // step s is complete in its buffer, the other buffer is no longer read
+      const int v = (u + 1) % PD;
+      store_lds(xr[v], wr[v], (s + 1) & 1);
+      load_regs(xr[v], wr[v], s + 1 + PD);
+      const char* xl = lds + (s & 1) * BUF + (wm + frow) * 128;
+      const char* wl = lds + (s & 1) * BUF + (BM + wn + frow) * 128;
 #pragma unroll
-      for (int j = 0; j < NJ; ++j) b[j] = *reinterpret_cast<const uint4*>(wl + j * 4096 + slot);
+      for (int t = 0; t < 4; ++t) {
+        const int slot = ((2 * t + half) ^ (frow & 7)) << 4;
+        uint4 a[MI], b[NJ];
 #pragma unroll
-      for (int i = 0; i < MI; ++i)
+        for (int i = 0; i < MI; ++i) a[i] = *reinterpret_cast<const uint4*>(xl + i * 4096 + slot);
 #pragma unroll
-        for (int j = 0; j < NJ; ++j) acc[i][j] = Elem<T>::mma32(a[i], b[j], acc[i][j]);
+        for (int j = 0; j < NJ; ++j) b[j] = *reinterpret_cast<const uint4*>(wl + j * 4096 + slot);
+#pragma unroll
+        for (int i = 0; i < MI; ++i)
+#pragma unroll
+          for (int j = 0; j < NJ; ++j) acc[i][j] = Elem<T>::mma32(a[i], b[j], acc[i][j]);
+      }
     }
   }
 
@@ -322,16 +414,34 @@ int launch_plain(GemmParams p, int64_t ws_floats, hipStream_t st) {
   return EXO_OK;
 }
 
-template <typename T>
-int launch_gemv(const GemvParams& p, hipStream_t st) {
+int gemv_waves(int N) {
+  const int tiles = exo_ceil_div(N, 16);
+  return tiles >= 1024 ? 4 : tiles >= 256 ? 8 : 16;
+}
+// the columns of a row fit its waves' registers, the rows fit the LDS
+bool post_fits(int M, int N, int H, int ldx, int elem) {
+  return M <= 16 && ldx <= post_waves_per_row(M, gemv_waves(N)) * 256 * kPostPasses && H <= ldx &&
+         (int64_t)M * (ldx * elem + 16) <= 40 * 1024;
+}
+
+template <typename T, int NW>
+void launch_gemv_nw(const GemvParams& p, const PostNorm* q, hipStream_t st) {
   const int tiles = exo_ceil_div(p.N, 16);
-  exo_note_variant("dense_gemv<%s> M=%d tiles=%d", sizeof(T) == 2 ? "bf16" : "f32", p.M, tiles);
-  if (tiles >= 1024)
-    dense_gemv_kernel<T, 4><<<tiles, 256, 0, st>>>(p);
-  else if (tiles >= 256)
-    dense_gemv_kernel<T, 8><<<tiles, 512, 0, st>>>(p);
+  if (q)
+    dense_gemv_kernel<T, NW, true><<<tiles, 64 * NW, p.M * (p.ldx * (int)sizeof(T) + 16), st>>>(p, *q);
   else
-    dense_gemv_kernel<T, 16><<<tiles, 1024, 0, st>>>(p);
+    dense_gemv_kernel<T, NW, false><<<tiles, 64 * NW, 0, st>>>(p, PostNorm{});
+}
+template <typename T>
+int launch_gemv(const GemvParams& p, const PostNorm* q, hipStream_t st) {
+  const int nw = gemv_waves(p.N);
+  exo_note_variant("dense_gemv<%s,%d,%s> M=%d N=%d", sizeof(T) == 2 ? "bf16" : "f32", nw, q ? "post" : "plain", p.M, p.N);
+  if (nw == 4)
+    launch_gemv_nw<T, 4>(p, q, st);
+  else if (nw == 8)
+    launch_gemv_nw<T, 8>(p, q, st);
+  else
+    launch_gemv_nw<T, 16>(p, q, st);
   return EXO_OK;
 }
 
@@ -351,9 +461,28 @@ extern "C" int exo_dense_gemv(const void* x, const void* w, const float* bias, v
   EXO_DENSE_ARGS("exo_dense_gemv");
   EXO_REQUIRE(M <= 16 && ldy >= N, "exo_dense_gemv: M=%d must be <= 16 and ldy=%d >= N=%d", M, ldy, N);
   const GemvParams p{x, w, bias, y, M, N, ldx, ldw, ldy, y_f32};
-  const int rc = EXO_BY_TYPE(dtype, launch_gemv<bf16_t>(p, (hipStream_t)stream), launch_gemv<float>(p, (hipStream_t)stream));
+  const int rc = EXO_BY_TYPE(dtype, launch_gemv<bf16_t>(p, nullptr, (hipStream_t)stream),
+                             launch_gemv<float>(p, nullptr, (hipStream_t)stream));
   if (rc) return rc;
   EXO_CHECK_LAUNCH("exo_dense_gemv");
+  return EXO_OK;
+}
+
+extern "C" int exo_post_gemv_fits(int M, int N, int H, int ldx, int dtype) {
+  return M > 0 && N > 0 && H > 0 && post_fits(M, N, H, ldx, dtype == 0 ? 2 : 4);
+}
+
+extern "C" int exo_post_gemv(const float* x, const float* branch, const float* gain, float eps, float* x_out,
+                             void* xb_out, const void* w, const float* bias, void* y, int y_f32, int M, int N, int H,
+                             int ldx, int ldw, int ldy, int dtype, exo_stream_t stream) {
+  EXO_DENSE_ARGS("exo_post_gemv");
+  EXO_REQUIRE(branch && gain && x_out && x_out != x && ldy >= N, "exo_post_gemv: null pointer, x_out == x or bad ldy");
+  EXO_REQUIRE(post_fits(M, N, H, ldx, dtype == 0 ? 2 : 4), "exo_post_gemv: %d rows of %d columns do not fit one launch", M, H);
+  const GemvParams p{nullptr, w, bias, y, M, N, ldx, ldw, ldy, y_f32};
+  const PostNorm q{x, branch, gain, x_out, xb_out, H, eps};
+  const int rc = EXO_BY_TYPE(dtype, launch_gemv<bf16_t>(p, &q, (hipStream_t)stream), launch_gemv<float>(p, &q, (hipStream_t)stream));
+  if (rc) return rc;
+  EXO_CHECK_LAUNCH("exo_post_gemv");
   return EXO_OK;
 }
 

@@ -94,6 +94,22 @@ def linear(x, w, out, n: int, bias=None, force_gemm: bool = False) -> None:
                              w.shape[1], out.shape[1], _code(x), _stream()), "linear(gemm)")
 
 
+POST_MAX_ROWS = 4  # beyond, every workgroup repeating the norm costs more than a launch
+
+
+def post_linear_fits(n: int, w, xb, H: int) -> bool:
+    return n <= POST_MAX_ROWS and bool(native.load().exo_post_gemv_fits(n, w.shape[0], H, xb.shape[1], _code(xb)))
+
+
+def post_linear(x, branch, gain, eps: float, x_out, xb, w, out, n: int, bias=None) -> None:
+    """``post_norm_add`` and ``linear`` in one launch: x_out = x + norm(branch) (another buffer than
+    x), xb (may be None) its copy, out = x_out @ w^T (+ bias)."""
+    check(native.load().exo_post_gemv(
+        _ptr(x), _ptr(branch), _ptr(gain), eps, _ptr(x_out), _ptr(xb), _ptr(w), _ptr(bias), _ptr(out),
+        int(out.dtype == torch.float32), n, w.shape[0], gain.numel(), w.shape[1], w.shape[1], out.shape[1], _code(w),
+        _stream()), "post_linear")
+
+
 def glu_gemm(x, gate, up, out, n: int, spec) -> None:
     """out[:n] = clamped gated unit of x[:n] (any n)."""
     check(native.load().exo_dense_glu_gemm(
@@ -112,17 +128,18 @@ def grouped_gemm(x, w, group_ws, out, T: int, topk: int, up=None, spec=None, x_p
 
 class ExpertRows:
     """The experts of a decode step (up to 16 rows): argument block built once per layer and
-    buffer set, launched as gated products (which also route) and as weighted down-projections."""
+    residual buffer, launched as gated products (which also route) and as weighted down-projections."""
 
-    def __init__(self, moe, w, bf, H: int):
-        """``moe``: MoeSpec; ``w``: the layer's tensors; ``bf``: the activation buffers."""
+    def __init__(self, moe, w, bf, H: int, h):
+        """``moe``: MoeSpec; ``w``: the layer's tensors; ``bf``: the activation buffers; ``h``: the
+        residual that enters the feed-forward."""
         r, e, s = moe.router, moe.expert, moe.shared
         p = lambda t: None if t is None else t.data_ptr()  # noqa: E731
         self.args = native.MoeRows(
             x=p(bf.xb), gate=p(w.gate), up=p(w.up), down=p(w.down),
             shared_gate=p(w.s_gate), shared_up=p(w.s_up), shared_down=p(w.s_down),
             act=p(bf.act(r.top, e.ff)), shared_act=p(bf.shared_act(s.ff)) if s else None, out=p(bf.branch),
-            x_res=p(bf.h), idx=p(bf.idx(r.top)), wt=p(bf.wt(r.top)), logits=p(bf.router_logits(w.router.shape[0])),
+            x_res=p(h), idx=p(bf.idx(r.top)), wt=p(bf.wt(r.top)), logits=p(bf.router_logits(w.router.shape[0])),
             correction=p(w.correction),
             top=r.top, experts=r.experts, ff=e.ff, shared_ff=s.ff if s else 0, H=H, ldx=bf.xb.shape[1],
             lda=pad64(e.ff), ldsa=pad64(s.ff) if s else 0, ldl=w.router.shape[0], gate_col=r.outputs, outputs=r.outputs, router_scale=r.scale,

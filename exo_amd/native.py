@@ -91,6 +91,8 @@ SIGNATURES: dict[str, tuple] = {
     "exo_moe_sum_post_norm": (_i, [_vp] * 5 + [_i] * 6 + [_vp] * 3 + [_i] * 3 + [_f, _i, _vp]),
     "exo_moe_route": (_i, [_vp] * 4 + [_i] * 4 + [_f, _vp]),
     "exo_dense_gemv": (_i, [_vp] * 4 + [_i] * 7 + [_vp]),
+    "exo_post_gemv_fits": (_i, [_i] * 5),
+    "exo_post_gemv": (_i, [_vp, _vp, _vp, _f] + [_vp] * 5 + [_i] * 8 + [_vp]),
     "exo_dense_gemm": (_i, [_vp] * 4 + [_i, _vp, _i64] + [_i] * 6 + [_vp]),
     "exo_dense_glu_gemm": (_i, [_vp] * 4 + [_f] * 3 + [_i] * 6 + [_vp]),
     "exo_dense_grouped_gemm": (_i, [_vp] * 5 + [_f] * 3 + [_i] * 9 + [_vp]),

@@ -12,8 +12,10 @@ and the cache have the model's element type - bf16 as served, or float32 through
 
 Launches of a layer (rows R of the step):
   R <= 16   q|k|v GEMV, attention (with norm and cache append inside when every row is a single
-            token), o GEMV, norm + residual, router GEMV, routing, gated experts + shared expert in
-            one launch, weighted down-projections in one launch, norm + residual
+            token), o GEMV, router GEMV, gated experts + shared expert in one launch that also
+            routes, weighted down-projections in one launch.  The norm of a sublayer's output and
+            its residual sum run inside the next product that reads the residual (up to 4 rows) or
+            as a launch of their own
   R > 16    the same with GEMMs, the experts grouped by expert, their weighted sum inside the
             norm + residual launch; portions of prompts take the tiled attention, single tokens
             beside them the split one
@@ -99,17 +101,24 @@ class _Buffers:
         self._z = lambda *s, dtype=t: torch.zeros(*s, dtype=dtype, device=dev)  # noqa: E731
         self._named: dict[tuple, torch.Tensor] = {}
         self.tokens = self._z(rows, dtype=torch.int32)
-        self.h = self._z(rows, H, dtype=torch.float32)       # the residual stream
+        # the residual stream; two buffers, since a launch that also advances it reads one and
+        # writes the other (``h`` is the current one)
+        self.hs = [self._z(rows, H, dtype=torch.float32) for _ in range(2 if rows <= D.POST_MAX_ROWS else 1)]
+        self.cur = 0
         self.xb = self._z(rows, pad64(H))                    # its copy as matrix operand
         self.xn = self._z(rows, pad64(H))                    # rows entering the head
         self.branch = self._z(rows, H, dtype=torch.float32)  # a sublayer's output
-        self.experts: dict[int, D.ExpertRows] = {}
+        self.experts: dict[tuple[int, int], D.ExpertRows] = {}
         # outputs of a single-token step (last shard)
         self.logits = self.logits16 = None
         self.next_token = self._z(seqs, dtype=torch.int32)
         self.lse = self._z(seqs, dtype=torch.float32)
         self.logprob = self._z(seqs, dtype=torch.float32)
         self.argmax_ws = ops.argmax_workspace(seqs, dev)
+
+    @property
+    def h(self) -> torch.Tensor:
+        return self.hs[self.cur]
 
     def _get(self, name: str, *shape: int, dtype=None) -> torch.Tensor:
         key = (name, *shape)
@@ -244,12 +253,28 @@ class StackModel(DecoderShard):
         return self._attn[1]
 
     # ------------------------------------------------------------------ the launches
-    def _mixer(self, L: _Layer, att: D.PagedAttention, bf: _Buffers, b: _Batch) -> None:
-        """bf.branch <- attention of bf.xb"""
+    def _settle(self, bf: _Buffers, n: int, gain: torch.Tensor | None) -> None:
+        """residual += norm(branch), if a sublayer's output is still outstanding (``gain``)"""
+        if gain is not None:
+            D.post_norm_add(bf.branch, gain, self.cfg.eps, bf.h, bf.xb, n)
+
+    def _product(self, bf: _Buffers, n: int, gain: torch.Tensor | None, w, out, bias=None, keep_copy: bool = False) -> None:
+        """out <- residual @ w^T, after the outstanding norm and sum; ``keep_copy``: bf.xb is read
+        by later launches too"""
+        if gain is not None and len(bf.hs) > 1 and D.post_linear_fits(n, w, bf.xb, self.cfg.hidden_size):
+            x = bf.h
+            bf.cur ^= 1
+            D.post_linear(x, bf.branch, gain, self.cfg.eps, bf.h, bf.xb if keep_copy else None, w, out, n, bias)
+            return
+        self._settle(bf, n, gain)
+        D.linear(bf.xb, w, out, n, bias=bias)
+
+    def _mixer(self, L: _Layer, att: D.PagedAttention, bf: _Buffers, b: _Batch, gain: torch.Tensor | None) -> None:
+        """bf.branch <- attention of the residual"""
         m: AttentionSpec = L.spec.mixer
         n, own = b.rows, m.kv_from is None
         qkv, out = bf.qkv(L.qkv.shape[0]), bf.attn(m.heads * m.vdim)
-        D.linear(bf.xb, L.qkv, qkv, n, bias=L.qkv_b)
+        self._product(bf, n, gain, L.qkv, qkv, bias=L.qkv_b)
         if b.decode:
             att.rows(qkv, out, b.slot, b.pos, n, b.keys, append=own)
         else:
@@ -261,20 +286,20 @@ class StackModel(DecoderShard):
                 att.rows(qkv, out, b.slot, b.pos, b.n_single, b.keys, append=False, lst=b.single)
         D.linear(out, L.o, bf.branch, n, bias=L.o_b)
 
-    def _mlp(self, L: _Layer, bf: _Buffers, n: int) -> None:
-        """residual += norm2(experts of bf.xb)"""
+    def _mlp(self, L: _Layer, bf: _Buffers, n: int, gain: torch.Tensor | None) -> torch.Tensor | None:
+        """The experts of the residual: bf.branch (returns the gain of the norm still outstanding),
+        or already normed and added (returns None)"""
         f, H = L.spec.mlp, self.cfg.hidden_size
         r, eps = f.router, self.cfg.eps
         logits, idx, wt = bf.router_logits(L.router.shape[0]), bf.idx(r.top), bf.wt(r.top)
-        D.linear(bf.xb, L.router, logits, n)
+        self._product(bf, n, gain, L.router, logits, keep_copy=True)
         if n <= D.GEMV_MAX_ROWS:
-            ex = bf.experts.get(L.index)
-            if ex is None:
-                ex = bf.experts[L.index] = D.ExpertRows(f, L, bf, H)
-            ex.glu(n)
-            ex.down(n)
-            D.post_norm_add(bf.branch, L.norm2, eps, bf.h, bf.xb, n)
-            return
+            key = (L.index, bf.cur)
+            if key not in bf.experts:
+                bf.experts[key] = D.ExpertRows(f, L, bf, H, bf.h)
+            bf.experts[key].glu(n)
+            bf.experts[key].down(n)
+            return L.norm2
         D.moe_route(logits, L.correction, r.scale, idx, wt, n)
         act, out = bf.act(r.top, f.expert.ff), bf.expert_out(r.top)
         ws = ops.moe_group(idx[:n], r.experts, check_indices=False)  # identity ids are past the end: left out
@@ -286,29 +311,39 @@ class StackModel(DecoderShard):
             D.glu_gemm(bf.xb, L.s_gate, L.s_up, sact, n, f.shared)
             D.linear(sact, L.s_down, shared, n)
         D.moe_sum_post_norm(out, idx, wt, shared, logits, r.experts, r.outputs, L.norm2, eps, bf.h, bf.xb, n)
+        return None
 
     def _forward(self, cache: PagedKVCache, bf: _Buffers, b: _Batch, logits: bool) -> torch.Tensor:
-        """Launch the shard over the rows of ``b``: input bf.tokens (first shard) or bf.h; returns the
-        logits [n_want, V] of the wanted rows, or the residual."""
+        """Launch the shard over the rows of ``b``: input bf.tokens (first shard) or bf.hs[0]; returns
+        the logits [n_want, V] of the wanted rows, or the residual."""
         n, H, eps = b.rows, self.cfg.hidden_size, self.cfg.eps
+        bf.cur = 0
         if self.is_first:
             D.embed_rows(bf.tokens[:n], self.embed, bf.h, bf.xb, H)
         else:
             bf.xb[:n, :H].copy_(bf.h[:n])
+        gain = None  # of the norm that the latest sublayer's output still has to pass
         for L, att in zip(self.layers, self._attention(cache)):
-            self._mixer(L, att, bf, b)
-            D.post_norm_add(bf.branch, L.norm1, eps, bf.h, bf.xb, n)
+            self._mixer(L, att, bf, b, gain)
+            gain = L.norm1
             if L.spec.mlp is not None:
-                self._mlp(L, bf, n)
+                gain = self._mlp(L, bf, n, gain)
             if self.layer_hook is not None:
+                self._settle(bf, n, gain)
+                gain = None
                 self.layer_hook(L.index, bf.h[:n])
+        self._settle(bf, n, gain)
         if not self.is_last or not logits:
+            if bf.cur:  # callers find the residual where they put it
+                bf.hs[0][:n].copy_(bf.h[:n])
+                bf.cur = 0
             return bf.h[:n]
         D.norm_rows(bf.h, self.norm, eps, bf.xn, b.n_want, rows=b.want)
         if bf.logits is None or bf.logits.shape[0] != b.n_want:
             bf.logits = torch.empty(b.n_want, self.cfg.vocab_size, dtype=self.dtype, device=self.device)
             bf.logits16 = None
         D.linear(bf.xn, self.head, bf.logits, b.n_want)
+        bf.cur = 0
         return bf.logits
 
     def _run(self, B: int, T: int, cache: PagedKVCache, bf: _Buffers, logits_mode: str, rows: slice | None = None):

@@ -459,6 +459,13 @@ int exo_moe_route(const float* logits, const float* correction, int32_t* idx, fl
 /* y[M,N] = x[M,K] @ w[N,K]^T (+ bias), y in the element type or (y_f32) float32. */
 int exo_dense_gemv(const void* x, const void* w, const float* bias, void* y, int y_f32, int M,
                    int N, int ldx, int ldw, int ldy, int dtype, exo_stream_t stream); /* M <= 16 */
+/* exo_post_norm_add and the product in one launch (few rows: exo_post_gemv_fits): the residual
+ * x + gain * branch / rms(branch) goes to x_out (not x) and, in the element type, to xb_out (may be
+ * null), and is the product's input. */
+int exo_post_gemv_fits(int M, int N, int H, int ldx, int dtype);
+int exo_post_gemv(const float* x, const float* branch, const float* gain, float eps, float* x_out,
+                  void* xb_out, const void* w, const float* bias, void* y, int y_f32, int M, int N,
+                  int H, int ldx, int ldw, int ldy, int dtype, exo_stream_t stream);
 int exo_dense_gemm(const void* x, const void* w, const float* bias, void* y, int y_f32,
                    float* workspace, int64_t workspace_floats, int M, int N, int ldx, int ldw,
                    int ldy, int dtype, exo_stream_t stream);

@@ -113,6 +113,24 @@ def test_residual_norm(device, dtype, n, H):
     close(host(out[:, :H]), O.rms_norm_offset(x[[n - 1, 0]].astype(np.float64), w, eps), TOL[dtype], "norm of rows")
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("n,H,N", [(1, 70, 40), (1, 4096, 5000), (2, 1021, 17), (3, 300, 130), (4, 2048, 331), (4, 1000, 20000)])
+def test_residual_norm_inside_a_product(device, dtype, n, H, N):
+    say("post gemv", dtype, n, H, N)
+    x, y, g, w, b = rand((n, H), 1), rand((n, H), 2, 3e-3), rand((H,), 3), rand((N, H), 4, H**-0.5), rand((N,), 5)
+    W, xb = mat(w, dtype), torch.zeros(n, D.pad64(H), dtype=dtype, device="cuda")
+    if not D.post_linear_fits(n, W, xb, H):
+        assert dtype == F32 or N == 20000  # too many columns for the launch's registers or LDS
+        return
+    xt, xo, out = dev(x), torch.zeros(n, H, device="cuda"), torch.zeros(n, N, device="cuda")
+    D.post_linear(xt, dev(y), dev(1 + g), 1e-5, xo, xb, W, out, n, bias=dev(b))
+    want = x + O.rms_norm_offset(y.astype(np.float64), g, 1e-5)
+    close(host(xo), want, 1e-5, "residual")
+    close(host(xb[:, :H]), want, TOL[dtype], "its copy")
+    assert not host(xb[:, H:]).any() and np.array_equal(host(xt), x)
+    close(host(out), host(xb[:, :H]).astype(np.float64) @ w.T + b, 2e-5, "product")
+
+
 @pytest.mark.parametrize("n,top", [(1, 1), (7, 7), (12, 3), (64, 8), (65, 5), (300, 40), (512, 8)])
 def test_router(device, n, top):
     say("router", n, top)
@@ -151,7 +169,7 @@ def test_feed_forward(device, dtype, H, E, I, top, ff, sff, n):
     bf = model._buffers(1, max(n, 2))
     bf.h[:n].copy_(dev(x))
     bf.xb[:n, :H].copy_(dev(x))
-    model._mlp(model.layers[0], bf, n)
+    model._settle(bf, n, model._mlp(model.layers[0], bf, n, None))
     ww = O.to_float64(w)
     want = O.moe(x.astype(np.float64), ww, "l0.mlp.", m)
     want = x + O.rms_norm_offset(want, ww["l0.norm2"], cfg.eps)
