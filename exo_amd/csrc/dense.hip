@@ -9,7 +9,7 @@
 //    tail: rows past N, x rows past M and steps past a wave's range read as zero.
 //  * dense_gemm_kernel, any number of rows: a (64 MI) x (64 NJ) tile per workgroup of four waves
 //    (2 x 2, each (32 MI) x (32 NJ) in 32x32 products), K steps of 128 bytes per row through two
-//    LDS buffers, the next three steps' vectors in registers meanwhile; one barrier per step.  A row's
+//    LDS buffers, the next two steps' vectors in registers meanwhile; one barrier per step.  A row's
 //    eight 16-byte chunks sit at slot chunk ^ (row % 8), so operand reads of 32 rows meet no bank
 //    twice.  PAIR: the weight tile holds rows of a gate and an up matrix, 32 and 32, so that a
 //    wave's column tiles are (gate, up) of the same outputs and the gated unit is its epilogue.
@@ -192,7 +192,7 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const GemmParams p) 
   constexpr int BM = 64 * MI, BW = 64 * NJ;      // tile rows of x, of weights
   constexpr int BN = PAIR ? BW / 2 : BW;         // output columns
   constexpr int XV = BM * 8 / 256, WV = BW * 8 / 256;
-  constexpr int PD = 3;
+  constexpr int PD = 2;
   extern __shared__ __attribute__((aligned(16))) char lds[];  // [2][(BM + BW) * 128]
   __shared__ int row_pair[GROUPED ? BM : 1];
   constexpr int BUF = (BM + BW) * 128;
@@ -298,6 +298,7 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const GemmParams p) 
       const int v = (u + 1) % PD;
       store_lds(xr[v], wr[v], (s + 1) & 1);
       load_regs(xr[v], wr[v], s + 1 + PD);
+      __builtin_amdgcn_sched_barrier(0);  // (left alone, the requests sink behind the products)
       const char* xl = lds + (s & 1) * BUF + (wm + frow) * 128;
       const char* wl = lds + (s & 1) * BUF + (BM + wn + frow) * 128;
 #pragma unroll
@@ -396,7 +397,7 @@ int launch_plain(GemmParams p, int64_t ws_floats, hipStream_t st) {
   if (!PAIR && p.part) {  // few tiles: split K until the chip has about one workgroup per CU
     const int64_t tiles = tall ? t2 : t1;
     int ks = 1;
-    while (ks < 16 && tiles * ks * 2 <= 512 && steps / (ks * 2) >= 4) ks *= 2;
+    while (ks < 16 && tiles * ks * 2 <= 256 && steps / (ks * 2) >= 4) ks *= 2;
     while (ks > 1 && (int64_t)ks * p.M * p.N > ws_floats) ks /= 2;
     if (ks > 1) {
       p.ksteps = exo_ceil_div(steps, ks);

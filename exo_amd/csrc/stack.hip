@@ -139,13 +139,21 @@ __global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const float*
     if (left <= 0) break;
     float gn[kCols];
     load_cols<float>(gain + c, gn, H % kCols == 0, left);
+    float y[kCols];
 #pragma unroll
-    for (int e = 0; e < kCols; ++e)
-      if (e < left) {
-        const float s = xv[i][e] + v[i][e] * inv * gn[e];
-        xr[c + e] = s;
-        xb[(size_t)row * ldx + c + e] = Elem<T>::make(s);
-      }
+    for (int e = 0; e < kCols; ++e) y[e] = xv[i][e] + v[i][e] * inv * gn[e];
+    T* bo = xb + (size_t)row * ldx + c;
+    if (vec && ldx % kCols == 0) {
+      *reinterpret_cast<floatx4*>(xr + c) = floatx4{y[0], y[1], y[2], y[3]};
+      if (sizeof(T) == 2)
+        *reinterpret_cast<uint2*>(bo) = uint2{pack_bf2(y[0], y[1]), pack_bf2(y[2], y[3])};
+      else
+        *reinterpret_cast<floatx4*>(bo) = floatx4{y[0], y[1], y[2], y[3]};
+    } else {
+#pragma unroll
+      for (int e = 0; e < kCols; ++e)
+        if (e < left) xr[c + e] = y[e], bo[e] = Elem<T>::make(y[e]);
+    }
   }
 }
 
