@@ -96,17 +96,101 @@ __device__ __forceinline__ void put_value(const Params& p, int row, int g, int p
   for (int d = lane; d < p.E; d += 64) dst[(size_t)d * kPage] = src[d];
 }
 
+// A wave takes eight rows of one head: the keys' loads go out together, and the values of eight
+// consecutive positions of one page leave as one 16-byte (bf16) store per column - element by
+// element they would be eight stores that touch a line each.
+constexpr int kAppendRows = 8;
+
 template <typename T>
 __global__ __launch_bounds__(256) void paged_append_kernel(const Params p) {
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x >> 6);
-  const int row = blockIdx.x, unit = blockIdx.y * 4 + wave;  // units: keys of G heads, values of G heads
+  const int row0 = blockIdx.x * kAppendRows, unit = blockIdx.y * 4 + wave;  // units: keys of G heads, values of G heads
   if (unit >= 2 * p.G) return;
-  const int pos = p.pos[row];
-  const int page = p.table[(size_t)p.slot[row] * p.max_pages + pos / kPage];
-  if (unit < p.G)
-    put_key<T>(p, row, unit, page, pos % kPage, lane);
-  else
-    put_value<T>(p, row, unit - p.G, page, pos % kPage, lane);
+  const int n = min(kAppendRows, p.n - row0);
+  const int lr = row0 + min(lane, n - 1);  // lane i < n: row i's place
+  const int my_pos = p.pos[lr], my_slot = p.slot[lr];
+  const int my_page = p.table[(size_t)my_slot * p.max_pages + my_pos / kPage];
+  if (unit < p.G) {
+    const T* src = reinterpret_cast<const T*>(p.qkv) + (size_t)row0 * p.ldq + p.H * p.D + unit * p.D;
+    constexpr int VEC = Elem<T>::kVec;
+    if (p.D % VEC == 0 && p.ldq % VEC == 0) {  // 16 bytes per lane, several rows per pass
+      int lpr = 1;  // lanes per row
+      while (lpr * VEC < p.D) lpr *= 2;
+      const int c = lane % lpr;
+      for (int i0 = 0; i0 < n; i0 += 64 / lpr) {
+        const int i = i0 + lane / lpr, ic = min(i, n - 1);
+        const bool on = c * VEC < p.D;
+        const uint4 raw = on ? *reinterpret_cast<const uint4*>(src + (size_t)ic * p.ldq + c * VEC) : uint4{0, 0, 0, 0};
+        float f[VEC], ss = 0.f;
+        unpack_vec<T>(raw, f);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) ss += f[e] * f[e];
+        const float inv = p.unit ? 1.f / sqrtf(group_sum(ss, lpr) / p.D + p.eps) : 1.f;
+        const int page = __shfl(my_page, ic, 64), at = __shfl(my_pos, ic, 64) % kPage;
+        struct alignas(16) Vec {
+          T e[VEC];
+        } w;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) w.e[e] = Elem<T>::make(f[e] * inv);
+        if (on && i < n)
+          *reinterpret_cast<uint4*>(reinterpret_cast<T*>(p.kpool) + (((size_t)page * p.G + unit) * kPage + at) * p.ldk +
+                                    c * VEC) = __builtin_bit_cast(uint4, w);
+      }
+      return;
+    }
+    float v[kAppendRows][4];  // D <= 256
+#pragma unroll
+    for (int i = 0; i < kAppendRows; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int d = lane + 64 * j;
+        v[i][j] = d < p.D ? Elem<T>::load(src[(size_t)min(i, n - 1) * p.ldq + d]) : 0.f;
+      }
+#pragma unroll
+    for (int i = 0; i < kAppendRows; ++i) {
+      if (i >= n) break;
+      float ss = 0.f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) ss += v[i][j] * v[i][j];
+      const float inv = p.unit ? 1.f / sqrtf(wave_sum(ss) / p.D + p.eps) : 1.f;
+      const int page = __builtin_amdgcn_readlane(my_page, i), at = __builtin_amdgcn_readlane(my_pos, i) % kPage;
+      T* dst = reinterpret_cast<T*>(p.kpool) + (((size_t)page * p.G + unit) * kPage + at) * p.ldk;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (lane + 64 * j < p.D) dst[lane + 64 * j] = Elem<T>::make(v[i][j] * inv);
+    }
+    return;
+  }
+  const int g = unit - p.G;
+  const T* src = reinterpret_cast<const T*>(p.qkv) + (size_t)row0 * p.ldq + (p.H + p.G) * p.D + g * p.E;
+  const int pos0 = __builtin_amdgcn_readfirstlane(my_pos), page0 = __builtin_amdgcn_readfirstlane(my_page);
+  const bool run = n == kAppendRows && pos0 % kAppendRows == 0 &&
+                   __ballot(lane < kAppendRows && (my_page != page0 || my_pos != pos0 + lane)) == 0;
+  for (int d = lane; d < p.E; d += 64) {
+    T v[kAppendRows];
+#pragma unroll
+    for (int i = 0; i < kAppendRows; ++i) v[i] = src[(size_t)min(i, n - 1) * p.ldq + d];
+    if (run) {
+      T* dst = reinterpret_cast<T*>(p.vpool) + (((size_t)page0 * p.G + g) * p.ldv + d) * kPage + pos0 % kPage;
+      constexpr int per = 16 / (int)sizeof(T);
+#pragma unroll
+      for (int k = 0; k < kAppendRows; k += per) {
+        struct alignas(16) Vec {
+          T e[per];
+        } w;
+#pragma unroll
+        for (int i = 0; i < per; ++i) w.e[i] = v[k + i];
+        *reinterpret_cast<uint4*>(dst + k) = __builtin_bit_cast(uint4, w);
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < kAppendRows; ++i) {
+        if (i >= n) break;
+        const int page = __builtin_amdgcn_readlane(my_page, i), at = __builtin_amdgcn_readlane(my_pos, i) % kPage;
+        reinterpret_cast<T*>(p.vpool)[(((size_t)page * p.G + g) * p.ldv + d) * kPage + at] = v[i];
+      }
+    }
+  }
 }
 
 template <typename T>
@@ -649,7 +733,7 @@ extern "C" int exo_paged_append(const exo_paged_attn* a, exo_stream_t stream) {
   EXO_REQUIRE(a->slot && a->pos && a->ldq >= (a->heads + a->kv_heads) * a->dim + a->kv_heads * a->vdim,
               "exo_paged_append: rows of %d elements do not hold q, k and v", a->ldq);
   const Params p = params_of(a);
-  const dim3 grid(p.n, (2 * p.G + 3) / 4);
+  const dim3 grid((p.n + kAppendRows - 1) / kAppendRows, (2 * p.G + 3) / 4);
   if (a->dtype == 0)
     paged_append_kernel<bf16_t><<<grid, 256, 0, (hipStream_t)stream>>>(p);
   else
