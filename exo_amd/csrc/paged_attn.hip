@@ -424,7 +424,8 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
     const bool on = lane < p.nsplit;  // (at most 64 splits)
     const float m1 = on ? ld_dev(src + (size_t)lane * (p.E + 2)) : -INFINITY;
     const float l1 = on ? ld_dev(src + (size_t)lane * (p.E + 2) + 1) : 0.f;
-    const float w1 = m1 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m1 - wave_max(m1));
+    const float mm = wave_max(m1);  // (by all lanes: not inside the choice below)
+    const float w1 = m1 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m1 - mm);
     const float inv = 1.f / wave_sum(l1 * w1);
     if (on) fac[h * p.nsplit + lane] = w1 * inv;
   }

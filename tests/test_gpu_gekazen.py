@@ -310,6 +310,22 @@ def test_decode_attention_splits_agree_and_replay(device):
     assert np.array_equal(got, run_portions(spec, rows_np, [T - 3, 1, 1, 1], BF, 1e-6)[-3:])
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("window,keep", [(None, 0), (None, 39), (192, 39), (700, 5)])
+def test_decode_attention_over_few_and_many_splits(device, dtype, window, keep):
+    """Lengths at which one to eight splits hold tiles, the last one only some of its waves: near
+    keys (high slopes) and far ones, in single tokens and portions of seven."""
+    spec = make_spec(8, 2, 64, 48, window, keep)
+    T = 1100
+    rows_np, qkv = attn_case(spec, T, seed=17)
+    want = attn_oracle(spec, qkv, 1e-6, dtype)
+    for start in (120, 250, 380, 510, 640, 890, 1020):
+        say("splits", dtype, window, keep, start)
+        for cuts in ([start] + [1] * 50, [start] + [7] * 8):
+            got = run_portions(spec, rows_np[: start + 50], cuts, dtype, 1e-6)
+            close(got, want[: start + 50], 1.2e-2 if dtype == BF else 5e-5, f"from {start}")
+
+
 # ------------------------------------------------------------------ whole models
 
 
