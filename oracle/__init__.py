@@ -32,4 +32,7 @@ Pin status per function (what, other than the formula itself, checks it):
 * generation protocol (prefill / trim 2 / re-feed last two tokens)  pinned by the
   cache-length invariants the reference's tests state
   (src/exo/worker/tests/unittests/test_mlx/test_kv_prefix_cache.py:157,374).
+* ``gekazen`` (a design the reference does not have)  pinned - attention with mask and distance
+  penalty against ``torch.nn.functional.scaled_dot_product_attention``, norms, gated unit and
+  routing on hand-worked values, causality.
 """

@@ -244,7 +244,7 @@ def run_portions(spec, rows_np, cuts, dtype, eps, start_pages=0, fused=True):
     return np.concatenate(got)
 
 
-SHAPES = [(4, 4, 64, 64), (6, 2, 48, 80), (8, 2, 128, 128), (5, 1, 96, 32), (40, 2, 32, 32), (2, 2, 256, 192),
+SHAPES = [(5, 5, 64, 64), (6, 2, 48, 80), (8, 2, 128, 128), (5, 1, 96, 32), (40, 2, 32, 32), (2, 2, 256, 192),
           (3, 3, 36, 20), (4, 2, 24, 7), (7, 1, 64, 128)]
 WINDOWS = [(None, 0), (1, 0), (33, 0), (64, 5), (65, 64), (100, 70), (40, 500)]
 
@@ -288,7 +288,7 @@ def test_attention_edges(device, dtype):
 def test_attention_keeps_many_small_weights(device):
     """Five hundred near-equal keys whose values nearly cancel: weights rounded to 8 bits before the
     product with the values would show."""
-    spec = make_spec(4, 4, 64, 64, None, 0, scale=0.02)
+    spec = make_spec(3, 3, 64, 64, None, 0, scale=0.02)
     T = 512
     rows_np, qkv = attn_case(spec, T, seed=3)
     want = attn_oracle(spec, qkv, 1e-6, BF)
@@ -616,6 +616,40 @@ def test_engine_prefix_cache_and_sequential(built):
     got = drain(seq, [task(3, p, 12)])["t3"]
     greedy_agrees(built, p, got, F32)
     seq.close()
+
+
+def test_paged_rows_travel_over_the_wire(built):
+    """Keys and values of a paged row through the prefill wire format into another pool, whole and
+    behind a prefix; head sizes or an element type that the format cannot say are refused."""
+    import io
+
+    from exo_amd import disaggregated as W
+
+    cfg = U.config([U.layer(), U.layer(kv_from=0), U.layer(heads=4, kv_heads=4, window=50)])
+    w = U.weights(cfg, 4)
+    m = build_model(config_from_dict(cfg), U.torch_weights(w, "cuda"))
+    toks = [t % cfg["vocab"] for t in built.toks["b"]]
+    src, dst, ref = m.make_cache(2, 256), m.make_cache(2, 256), m.make_cache(1, 256)
+    m.step(src, [(1, toks[:130], [])])
+    m.step(dst, [(1, toks[:70], [])])
+    for start in (0, 70):
+        buf = io.BytesIO()
+        assert W.write_cache_to_wire(buf, src, row=1, request_id="r", model_id="m", start_pos=start) == 130 - start
+        buf.seek(0)
+        row = 1 if start else 0
+        assert W.ingest_into_cache(W.read_result(buf), dst, row=row, start_pos=start) == 130
+        for i in range(len(src)):
+            for a, b in zip(src.read_nhd(i, 1, 0, 130), dst.read_nhd(i, row, 0, 130)):
+                assert torch.equal(a, b)
+    m.step(ref, [(0, toks[:130], [])])
+    want = host(m.step(ref, [(0, toks[130:133], [0, 1, 2])])).copy()
+    got = host(m.step(dst, [(0, toks[130:133], [0, 1, 2])]))
+    assert np.array_equal(got, want)
+    for bad in (built.models[BF], build_model(config_from_dict(cfg), U.torch_weights(w, "cuda"), dtype=F32)):
+        c = bad.make_cache(1, 64)
+        bad.step(c, [(0, [1, 2, 3], [])])
+        with pytest.raises(ValueError, match="the wire carries"):
+            W.write_cache_to_wire(io.BytesIO(), c, row=0)
 
 
 def test_engine_samples_on_device_and_on_host(built):
