@@ -493,11 +493,11 @@ def gekazen_launches(torch, m, B, ctx):
     m.layer_hook = None
     a, f = c.layers[0].mixer, c.layers[0].mlp
     e, r = f.expert, f.router
-    att = dict(zip(range(len(Ls)), m._attention(cache)))
+    att = [bound[0] for bound in m._mixers(cache)]
     real = [int((p < r.experts).sum()) for p in picks]
     uniq = [len(set(p[p < r.experts].tolist())) for p in picks]
     pairs, experts = sum(real) / len(real), sum(uniq) / len(uniq)
-    qkv, out = bf.qkv(Ls[0].qkv.shape[0]), bf.attn(a.heads * a.vdim)
+    qkv, out = bf.cols("proj", -(-Ls[0].n_main // 8) * 8), bf.mixed("attn", a.heads * a.vdim)
     vis = [min(i + 1, (a.window or 1 << 30) + a.keep_first) for i in (range(B) if prompt else [ctx] * B)]
     kvb = 2 * a.kv_heads * (a.dim + a.vdim) * (B if prompt else sum(vis))
     rows = []
@@ -507,17 +507,17 @@ def gekazen_launches(torch, m, B, ctx):
 
     def mm(n, k, extra=0):
         return 2 * n * k + 2 * B * (n + k) + extra, 2 * B * n * k
-    nq = Ls[0].qkv.shape[0]
-    fused = not prompt and D.post_linear_fits(B, Ls[0].qkv, bf.xb, H)  # norm + residual inside the next product
+    nq = Ls[0].proj.shape[0]
+    fused = not prompt and D.post_linear_fits(B, Ls[0].proj, bf.xb, H)  # norm + residual inside the next product
     other = torch.empty_like(bf.h)
 
     def product(L, w, out, bias=None, xb=None):
         if fused:
-            D.post_linear(bf.h, bf.branch, L.norm1, c.eps, other, xb, w, out, B, bias)
+            D.post_linear(bf.h, D.Branches(bf.branch, L.norm1), c.eps, other, xb, w, out, B, bias)
         else:
             D.linear(bf.xb, w, out, B, bias=bias)
     pre = "norm, residual, " if fused else ""
-    add(pre + "qkv + bias", lambda L: product(L, L.qkv, qkv, L.qkv_b), *mm(nq, H))
+    add(pre + "qkv + bias", lambda L: product(L, L.proj, qkv, L.proj_b), *mm(nq, H))
     if prompt:
         add("append keys, values", lambda L: att[L.index].append(qkv, batch.slot, batch.pos, B), 2 * kvb, 0)
         add("attention", lambda L: att[L.index].prompt(qkv, out, *batch.blocks[att[0].prompt_block(a)]),
@@ -525,20 +525,20 @@ def gekazen_launches(torch, m, B, ctx):
     else:
         add("norm, append, attention", lambda L: att[L.index].rows(qkv, out, batch.slot, batch.pos, B, batch.keys, append=True),
             kvb, 2 * sum(vis) * a.heads * (a.dim + a.vdim))
-    add("o + bias", lambda L: D.linear(out, L.o, bf.branch, B, bias=L.o_b), *mm(H, a.heads * a.vdim))
+    add("o + bias", lambda L: D.linear(out, L.parts[0].o, bf.branch, B, bias=L.parts[0].o_b), *mm(H, a.heads * a.vdim))
     if not fused:
         add("norm + residual (twice a layer)" if not prompt else "norm + residual",
-            lambda L: D.post_norm_add(bf.branch, L.norm1, c.eps, bf.h, bf.xb, B), B * H * 14, 0)
-    lg, idx, wt = bf.router_logits(Ls[0].router.shape[0]), bf.idx(r.top), bf.wt(r.top)
-    add(pre + "router", lambda L: product(L, L.router, lg, xb=bf.xb), *mm(Ls[0].router.shape[0], H))
+            lambda L: D.post_norm_add(D.Branches(bf.branch, L.norm1), c.eps, bf.h, bf.xb, B), B * H * 14, 0)
+    lg, idx, wt = bf.router_logits(Ls[0].ff.router.shape[0]), bf.idx(r.top), bf.wt(r.top)
+    add(pre + "router", lambda L: product(L, L.ff.router, lg, xb=bf.xb), *mm(Ls[0].ff.router.shape[0], H))
     if prompt:
-        add("routing", lambda L: D.moe_route(lg, L.correction, r.scale, idx, wt, B), B * r.outputs * 4, 0)
+        add("routing", lambda L: D.moe_route(lg, L.ff.correction, r.scale, idx, wt, B), B * r.outputs * 4, 0)
     per = 2 * e.ff * H
     sh = f.shared.ff * H * 2
     if not prompt:
         for L in Ls:
             if (L.index, bf.cur) not in bf.experts:
-                bf.experts[L.index, bf.cur] = D.ExpertRows(f, L, bf, H, bf.h)
+                bf.experts[L.index, bf.cur] = D.ExpertRows(f, L.ff, bf, H, bf.h)
         ex = [bf.experts[L.index, bf.cur] for L in Ls]
         # every layer streams the experts it chose in the forward above
         logits = [torch.full((B, lg.shape[1]), -30.0, device="cuda").scatter_(1, p.long().to("cuda"), 3.0) for p in picks]
@@ -556,14 +556,14 @@ def gekazen_launches(torch, m, B, ctx):
         bf.idx(r.top)[:B].copy_(picks[0].to("cuda"))
         ws = ops.moe_group(idx[:B], r.experts, check_indices=False)
         add("group", lambda L: ops.moe_group(idx[:B], r.experts, check_indices=False), B * r.top * 8, 0)
-        add("experts: gate, up", lambda L: D.grouped_gemm(bf.xb, L.gate, ws, act, B, r.top, up=L.up, spec=e),
+        add("experts: gate, up", lambda L: D.grouped_gemm(bf.xb, L.ff.gate, ws, act, B, r.top, up=L.ff.up, spec=e),
             2 * experts * per + 2 * B * H + 2 * pairs * e.ff, 4 * pairs * e.ff * H)
-        add("experts: down", lambda L: D.grouped_gemm(act, L.down, ws, eo, B, r.top, x_per_pair=True),
+        add("experts: down", lambda L: D.grouped_gemm(act, L.ff.down, ws, eo, B, r.top, x_per_pair=True),
             experts * per + 2 * pairs * (H + e.ff), 2 * pairs * e.ff * H)
         sa, so = bf.shared_act(f.shared.ff), bf.shared_out()
-        add("shared: gate, up", lambda L: D.glu_gemm(bf.xb, L.s_gate, L.s_up, sa, B, f.shared),
+        add("shared: gate, up", lambda L: D.glu_gemm(bf.xb, L.ff.s_gate, L.ff.s_up, sa, B, f.shared),
             2 * sh + 2 * B * (H + f.shared.ff), 4 * B * f.shared.ff * H)
-        add("shared: down", lambda L: D.linear(sa, L.s_down, so, B), sh + 2 * B * (H + f.shared.ff), 2 * B * f.shared.ff * H)
+        add("shared: down", lambda L: D.linear(sa, L.ff.s_down, so, B), sh + 2 * B * (H + f.shared.ff), 2 * B * f.shared.ff * H)
         add("expert sum, norm + residual", lambda L: D.moe_sum_post_norm(eo, idx, wt, so, lg, r.experts, r.outputs, L.norm2,
                                                                      c.eps, bf.h, bf.xb, B), 2 * (pairs + B) * H + 10 * B * H, 0)
     return rows

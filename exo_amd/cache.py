@@ -37,7 +37,7 @@ class LayerKV:
         return max(self._owner.offsets, default=0)
 
     def is_trimmable(self) -> bool:
-        return True
+        return self._owner.trimmable
 
     def trim(self, n: int) -> int:
         """Entries are trimmed together (every layer holds the same tokens); the call on
@@ -61,6 +61,14 @@ class ShardKVCache(list):
         self.pos = torch.zeros(batch, dtype=torch.int32, device=device)
         self.offsets = [0] * batch
         self._last_trim = 0
+
+    trimmable = True  # a row can go back to an earlier position
+
+    def save_states(self, rows) -> None:
+        """Nothing here changes with a step but what lies behind the fill level."""
+
+    def load_states(self, rows, saved) -> None:
+        pass
 
     # -- fill level
     def advance_host(self, t: int, rows=None) -> None:

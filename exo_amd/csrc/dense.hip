@@ -6,7 +6,9 @@
 //    waves, weights straight from memory into the A operand of a 16x16 matrix product (16 rows x
 //    64 bytes per load instruction), x rows as the 16 columns of B.  One batch of kBatch loads per
 //    wave is in flight before anything is waited for.  Range-checked loads stand in for every
-//    tail: rows past N, x rows past M and steps past a wave's range read as zero.
+//    tail: rows past N, x rows past M and steps past a wave's range read as zero.  PAIR: a gate and
+//    an up matrix, the gated unit as epilogue.  DUAL: two products with nothing in common but the
+//    number of rows share the launch.
 //  * dense_gemm_kernel, any number of rows: a (64 MI) x (64 NJ) tile per workgroup of four waves
 //    (2 x 2, each (32 MI) x (32 NJ) in 32x32 products), K steps of 128 bytes per row through two
 //    LDS buffers, the next two steps' vectors in registers meanwhile; one barrier per step.  A row's
@@ -14,6 +16,8 @@
 //    twice.  PAIR: the weight tile holds rows of a gate and an up matrix, 32 and 32, so that a
 //    wave's column tiles are (gate, up) of the same outputs and the gated unit is its epilogue.
 //    GROUPED: the rows are one expert's (token, slot) pairs, from exo_moe_group's tile list.
+// Either may send its last output columns to a second, float32 buffer: inputs of 32-bit arithmetic
+// (step sizes, gates, decays) are rows of the same weight matrix as the bf16 projections.
 #include "../../include/exo_mi355x.h"
 #include "dense.h"
 
@@ -24,10 +28,13 @@ constexpr int kBatch = 8;
 
 struct GemvParams {
   const void* x;
-  const void* w;
+  const void* w;   // gate matrix in pair mode
+  const void* w2;  // up matrix
   const float* bias;
   void* y;
-  int M, N, ldx, ldw, ldy, y_f32;
+  float* y2;       // columns from n1 on
+  int M, N, n1, ldx, ldw, ldy, ldy2, y_f32;
+  GluConst glu;
 };
 
 template <typename T>
@@ -39,19 +46,24 @@ __device__ __forceinline__ void store_out(void* y, size_t i, float v, int y_f32)
 }
 
 // Norm of the previous sublayer's output and residual sum, in front of the product that reads the
-// residual: every workgroup forms x + gain * branch / rms(branch) for itself (in LDS, element type),
-// workgroup 0 also writes it out - to another buffer than it is read from, since the others may
-// still be reading.
+// residual: every workgroup forms y = x + mult * gain * v / rms(v) for itself and from it the product's
+// operand (in LDS, element type): y, or y / rms(y) * pre.  v is the branch, or half the sum of two
+// branches that are normed each with a gain of its own.  Workgroup 0 also writes y out - to another
+// buffer than x is read from, since the others may still be reading.
 struct PostNorm {
-  const float* x;       // [M][H]
-  const float* branch;  // [M][H]
-  const float* gain;    // [H]
-  float* x_out;         // [M][H]
-  void* xb_out;         // T [M][ldx], or null
+  const float* x;        // [M][H]
+  const float* branch;   // [M][H]
+  const float* branch2;  // [M][H], or null
+  const float* gain_a;   // [H] gains of two branches
+  const float* gain_b;
+  const float* gain;     // [H]
+  const float* pre;      // [H], or null
+  float* x_out;          // [M][H]
+  void* xb_out;          // T [M][ldx] the operand, or null
   int H;
-  float eps;
+  float eps, mult;
 };
-constexpr int kPostPasses = 4;  // float4 per lane of a row's waves
+constexpr int kPostPasses = 4;  // at most so many float4 per lane of a row's waves
 
 __host__ __device__ inline int post_waves_per_row(int M, int NW) {
   int p = 1;
@@ -59,25 +71,66 @@ __host__ __device__ inline int post_waves_per_row(int M, int NW) {
   return NW > p ? NW / p : 1;
 }
 
-template <typename T, int NW, bool POST>
-__global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p, const PostNorm q) {
-  __shared__ float red[NW][256];
-  __shared__ float part[NW];
+// sums over the wpr waves that share a row
+template <int NW>
+__device__ __forceinline__ void row_sums(float& a, float& b, float (&part)[2][NW], int wave, int wpr, int lane) {
+  a = wave_sum(a);
+  b = wave_sum(b);
+  __syncthreads();  // (earlier sums have been read)
+  if (lane == 0) part[0][wave] = a, part[1][wave] = b;
+  __syncthreads();
+  a = b = 0.f;
+  for (int w = 0; w < wpr; ++w) a += part[0][wave / wpr * wpr + w], b += part[1][wave / wpr * wpr + w];
+}
+
+// four columns from c on, zero past H
+__device__ __forceinline__ floatx4 row4(const float* p, int c, int H, bool on, bool vec) {
+  floatx4 v = {0.f, 0.f, 0.f, 0.f};
+  if (on && c < H) {
+    if (vec) {
+      v = *reinterpret_cast<const floatx4*>(p + c);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (c + e < H) v[e] = p[c + e];
+    }
+  }
+  return v;
+}
+
+// PP: float4 of a row per lane in front of the product (0: no norm there); TWO: of two branches
+template <typename T, int NW, int PP, bool TWO, bool PAIR, bool DUAL>
+__global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p0, const GemvParams p1, const PostNorm q) {
+  constexpr bool POST = PP > 0;
+  constexpr int NP = POST ? PP : 1, NU = TWO ? NP : 1;
+  constexpr int NM = PAIR ? 2 : 1;
+  constexpr int BATCH = PAIR ? kBatch / 2 : kBatch;
+  __shared__ float red[NM][NW][256];
+  __shared__ float part[2][NW];
   extern __shared__ __attribute__((aligned(16))) char xs[];  // POST: [M][ldx * sizeof(T) + 16]
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x >> 6);
   const int r = lane & 15, g = lane >> 4;
-  const int n0 = blockIdx.x * 16, rows = min(16, p.N - n0);
+  const int tiles0 = (p0.N + 15) / 16;
+  const bool second = DUAL && (int)blockIdx.x >= tiles0;
+  const GemvParams& p = second ? p1 : p0;
+  const int n0 = ((int)blockIdx.x - (second ? tiles0 : 0)) * 16, rows = min(16, p.N - n0);
   const uint32_t wrow = (uint32_t)p.ldw * sizeof(T), xrow = (uint32_t)p.ldx * sizeof(T);
   const int steps = (int)(wrow >> 6);
   const int per = (steps + NW - 1) / NW, s0 = min(steps, wave * per), s1 = min(steps, s0 + per);
   const __amdgpu_buffer_rsrc_t rw =
       buf_of(reinterpret_cast<const char*>(p.w) + (size_t)n0 * wrow, (uint32_t)rows * wrow);
+  const __amdgpu_buffer_rsrc_t ru =
+      buf_of(reinterpret_cast<const char*>(PAIR ? p.w2 : p.w) + (size_t)n0 * wrow, (uint32_t)rows * wrow);
   const __amdgpu_buffer_rsrc_t rx = buf_of(p.x, (uint32_t)p.M * xrow);
   const uint32_t woff = r * wrow + g * 16;
-  uint4 wv[kBatch];
+  uint4 wv[NM][BATCH];
   auto load_w = [&](int s) {
 #pragma unroll
-    for (int i = 0; i < kBatch; ++i) wv[i] = buf_load16(rw, s + i < s1 ? woff + (s + i) * 64 : kPastEnd, 0);
+    for (int i = 0; i < BATCH; ++i) {
+      const uint32_t o = s + i < s1 ? woff + (s + i) * 64 : kPastEnd;
+      wv[0][i] = buf_load16(rw, o, 0);
+      if (PAIR) wv[NM - 1][i] = buf_load16(ru, o, 0);
+    }
   };
   if (POST) {
     // a row's columns over wpr waves; its inputs are requested ahead of the first weights
@@ -86,48 +139,69 @@ __global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p,
     const bool vec = q.H % 4 == 0;
     for (int m0 = 0; m0 < p.M; m0 += rpi) {
       const int m = m0 + wave / wpr, c0 = ((wave % wpr) * 64 + lane) * 4, cs = wpr * 256;
-      floatx4 v[kPostPasses], x[kPostPasses], gn[kPostPasses];
-      float ss = 0.f;
+      const bool on = m < p.M;
+      const size_t o = (size_t)m * q.H;
+      floatx4 v[NP], x[NP], u[NU];
 #pragma unroll
-      for (int i = 0; i < kPostPasses; ++i) {
-        const int c = c0 + i * cs;
-        v[i] = x[i] = gn[i] = floatx4{0.f, 0.f, 0.f, 0.f};
-        if (m < p.M && c < q.H) {
-          const size_t o = (size_t)m * q.H + c;
-          if (vec) {
-            v[i] = *reinterpret_cast<const floatx4*>(q.branch + o);
-            x[i] = *reinterpret_cast<const floatx4*>(q.x + o);
-            gn[i] = *reinterpret_cast<const floatx4*>(q.gain + c);
-          } else {
-#pragma unroll
-            for (int e = 0; e < 4; ++e)
-              if (c + e < q.H) v[i][e] = q.branch[o + e], x[i][e] = q.x[o + e], gn[i][e] = q.gain[c + e];
-          }
-        }
+      for (int i = 0; i < NP; ++i) {
+        v[i] = row4(q.branch + o, c0 + i * cs, q.H, on, vec);
+        if (TWO) u[TWO ? i : 0] = row4(q.branch2 + o, c0 + i * cs, q.H, on, vec);
+        x[i] = row4(q.x + o, c0 + i * cs, q.H, on, vec);
       }
       if (m0 == 0) load_w(s0);
+      float ss = 0.f, su = 0.f;
+      if (TWO) {  // half the sum of the two normed branches
 #pragma unroll
-      for (int i = 0; i < kPostPasses; ++i)
+        for (int i = 0; i < NP; ++i)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) ss += v[i][e] * v[i][e], su += u[TWO ? i : 0][e] * u[TWO ? i : 0][e];
+        row_sums<NW>(ss, su, part, wave, wpr, lane);
+        const float ia = 0.5f / sqrtf(ss / q.H + q.eps), ib = 0.5f / sqrtf(su / q.H + q.eps);
+#pragma unroll
+        for (int i = 0; i < NP; ++i) {
+          const floatx4 ga = row4(q.gain_a, c0 + i * cs, q.H, on, vec), gb = row4(q.gain_b, c0 + i * cs, q.H, on, vec);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[i][e] = v[i][e] * ia * ga[e] + u[TWO ? i : 0][e] * ib * gb[e];
+        }
+        ss = su = 0.f;
+      }
+#pragma unroll
+      for (int i = 0; i < NP; ++i)
 #pragma unroll
         for (int e = 0; e < 4; ++e) ss += v[i][e] * v[i][e];
-      ss = wave_sum(ss);
-      __syncthreads();  // (the sums of an earlier iteration have been read)
-      if (lane == 0) part[wave] = ss;
-      __syncthreads();
-      float tot = 0.f;
-      for (int w = 0; w < wpr; ++w) tot += part[wave / wpr * wpr + w];
-      const float inv = 1.f / sqrtf(tot / q.H + q.eps);
+      row_sums<NW>(ss, su, part, wave, wpr, lane);
+      const float inv = q.mult / sqrtf(ss / q.H + q.eps);
+      ss = 0.f;
 #pragma unroll
-      for (int i = 0; i < kPostPasses; ++i) {
+      for (int i = 0; i < NP; ++i) {
+        const floatx4 gn = row4(q.gain, c0 + i * cs, q.H, on, vec);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          x[i][e] += v[i][e] * inv * gn[e];  // zero past H
+          ss += x[i][e] * x[i][e];
+        }
+      }
+      float pinv = 1.f;
+      if (q.pre) {
+        row_sums<NW>(ss, su, part, wave, wpr, lane);
+        pinv = 1.f / sqrtf(ss / q.H + q.eps);
+      }
+#pragma unroll
+      for (int i = 0; i < NP; ++i) {
         const int c = c0 + i * cs;
-        if (m >= p.M || c >= p.ldx) continue;
+        if (!on || c >= p.ldx) continue;
+        floatx4 y = x[i];
+        if (q.pre) {
+          const floatx4 gp = row4(q.pre, c, q.H, on, vec);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) y[e] = y[e] * pinv * gp[e];
+        }
         T out[4];
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          const float y = x[i][e] + v[i][e] * inv * gn[i][e];  // zero past H
-          out[e] = Elem<T>::make(y);
+          out[e] = Elem<T>::make(y[e]);
           if (blockIdx.x == 0 && c + e < q.H) {
-            q.x_out[(size_t)m * q.H + c + e] = y;
+            q.x_out[o + c + e] = x[i][e];
             if (q.xb_out) reinterpret_cast<T*>(q.xb_out)[(size_t)m * p.ldx + c + e] = out[e];
           }
         }
@@ -140,31 +214,47 @@ __global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p,
   } else {
     load_w(s0);
   }
-  floatx4 acc = {0.f, 0.f, 0.f, 0.f};
-  for (int s = s0; s < s1; s += kBatch) {
-    uint4 xv[kBatch];
+  floatx4 acc[NM];
 #pragma unroll
-    for (int i = 0; i < kBatch; ++i) {
+  for (int k = 0; k < NM; ++k) acc[k] = floatx4{0.f, 0.f, 0.f, 0.f};
+  for (int s = s0; s < s1; s += BATCH) {
+    uint4 xv[BATCH];
+#pragma unroll
+    for (int i = 0; i < BATCH; ++i) {
       if (POST)  // (steps past the range: any finite values, their weights are zero)
         xv[i] = *reinterpret_cast<const uint4*>(xs + min(r, p.M - 1) * (xrow + 16) + g * 16 + min(s + i, s1 - 1) * 64);
       else
         xv[i] = buf_load16(rx, s + i < s1 ? r * xrow + g * 16 + (s + i) * 64 : kPastEnd, 0);
     }
 #pragma unroll
-    for (int i = 0; i < kBatch; ++i) acc = Elem<T>::mma16(wv[i], xv[i], acc);
-    if (s + kBatch < s1) load_w(s + kBatch);
+    for (int i = 0; i < BATCH; ++i)
+#pragma unroll
+      for (int k = 0; k < NM; ++k) acc[k] = Elem<T>::mma16(wv[k][i], xv[i], acc[k]);
+    if (s + BATCH < s1) load_w(s + BATCH);
   }
 #pragma unroll
-  for (int e = 0; e < 4; ++e) red[wave][r * 16 + 4 * g + e] = acc[e];  // [m][n]
+  for (int k = 0; k < NM; ++k)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) red[k][wave][r * 16 + 4 * g + e] = acc[k][e];  // [m][n]
   __syncthreads();
   for (int o = threadIdx.x; o < 16 * p.M; o += 64 * NW) {
     const int m = o >> 4, n = o & 15;
     if (n >= rows) continue;
-    float v = 0.f;
+    float v = 0.f, u = 0.f;
 #pragma unroll
-    for (int w = 0; w < NW; ++w) v += red[w][o];
+    for (int w = 0; w < NW; ++w) {
+      v += red[0][w][o];
+      if (PAIR) u += red[NM - 1][w][o];
+    }
+    if (PAIR) {
+      store_out<T>(p.y, (size_t)m * p.ldy + n0 + n, clamped_glu(v, u, p.glu), p.y_f32);
+      continue;
+    }
     if (p.bias) v += p.bias[n0 + n];
-    store_out<T>(p.y, (size_t)m * p.ldy + n0 + n, v, p.y_f32);
+    if (n0 + n < p.n1)
+      store_out<T>(p.y, (size_t)m * p.ldy + n0 + n, v, p.y_f32);
+    else
+      p.y2[(size_t)m * p.ldy2 + n0 + n - p.n1] = v;
   }
 }
 
@@ -175,7 +265,8 @@ struct GemmParams {
   const void* w2;  // up matrix
   const float* bias;
   void* y;
-  int M, N, ldx, ldw, ldy, y_f32;
+  float* y2;       // columns from n1 on
+  int M, N, n1, ldx, ldw, ldy, ldy2, y_f32;
   GluConst glu;
   // grouped
   const int32_t* sorted;
@@ -342,7 +433,10 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const GemmParams p) 
             p.part[((size_t)blockIdx.z * p.M + row) * p.N + n] = acc[i][j][e];
           } else {
             const float v = acc[i][j][e] + (p.bias ? p.bias[n] : 0.f);
-            store_out<T>(p.y, row * p.ldy + n, v, p.y_f32);
+            if (GROUPED || n < p.n1)
+              store_out<T>(p.y, row * p.ldy + n, v, p.y_f32);
+            else
+              p.y2[row * p.ldy2 + n - p.n1] = v;
           }
         }
       }
@@ -356,7 +450,10 @@ __global__ __launch_bounds__(256) void dense_reduce_kernel(const GemmParams p) {
   if (n >= p.N) return;
   float v = p.bias ? p.bias[n] : 0.f;
   for (int z = 0; z < p.ksplit; ++z) v += p.part[((size_t)z * p.M + m) * p.N + n];
-  store_out<T>(p.y, (size_t)m * p.ldy + n, v, p.y_f32);
+  if (n < p.n1)
+    store_out<T>(p.y, (size_t)m * p.ldy + n, v, p.y_f32);
+  else
+    p.y2[(size_t)m * p.ldy2 + n - p.n1] = v;
 }
 
 int raise_lds(const void* fn, int bytes, bool* done) {
@@ -425,24 +522,48 @@ bool post_fits(int M, int N, int H, int ldx, int elem) {
          (int64_t)M * (ldx * elem + 16) <= 40 * 1024;
 }
 
-template <typename T, int NW>
-void launch_gemv_nw(const GemvParams& p, const PostNorm* q, hipStream_t st) {
-  const int tiles = exo_ceil_div(p.N, 16);
-  if (q)
-    dense_gemv_kernel<T, NW, true><<<tiles, 64 * NW, p.M * (p.ldx * (int)sizeof(T) + 16), st>>>(p, *q);
+template <typename T, int NW, int PP>
+void launch_gemv_post(const GemvParams& p, const PostNorm& q, hipStream_t st) {
+  const int tiles = exo_ceil_div(p.N, 16), lds = p.M * (p.ldx * (int)sizeof(T) + 16);
+  if (q.branch2 && p.w2)
+    dense_gemv_kernel<T, NW, PP, true, true, false><<<tiles, 64 * NW, lds, st>>>(p, p, q);
+  else if (q.branch2)
+    dense_gemv_kernel<T, NW, PP, true, false, false><<<tiles, 64 * NW, lds, st>>>(p, p, q);
+  else if (p.w2)
+    dense_gemv_kernel<T, NW, PP, false, true, false><<<tiles, 64 * NW, lds, st>>>(p, p, q);
   else
-    dense_gemv_kernel<T, NW, false><<<tiles, 64 * NW, 0, st>>>(p, PostNorm{});
+    dense_gemv_kernel<T, NW, PP, false, false, false><<<tiles, 64 * NW, lds, st>>>(p, p, q);
+}
+template <typename T, int NW>
+void launch_gemv_nw(const GemvParams& p, const GemvParams* p1, const PostNorm* q, hipStream_t st) {
+  const int tiles = exo_ceil_div(p.N, 16);
+  const PostNorm none{};
+  if (q) {
+    const int passes = exo_ceil_div(p.ldx, post_waves_per_row(p.M, NW) * 256);  // (post_fits: at most kPostPasses)
+    if (passes <= 1)
+      launch_gemv_post<T, NW, 1>(p, *q, st);
+    else if (passes <= 2)
+      launch_gemv_post<T, NW, 2>(p, *q, st);
+    else
+      launch_gemv_post<T, NW, kPostPasses>(p, *q, st);
+  } else if (p1)
+    dense_gemv_kernel<T, NW, 0, false, false, true><<<tiles + exo_ceil_div(p1->N, 16), 64 * NW, 0, st>>>(p, *p1, none);
+  else if (p.w2)
+    dense_gemv_kernel<T, NW, 0, false, true, false><<<tiles, 64 * NW, 0, st>>>(p, p, none);
+  else
+    dense_gemv_kernel<T, NW, 0, false, false, false><<<tiles, 64 * NW, 0, st>>>(p, p, none);
 }
 template <typename T>
-int launch_gemv(const GemvParams& p, const PostNorm* q, hipStream_t st) {
-  const int nw = gemv_waves(p.N);
-  exo_note_variant("dense_gemv<%s,%d,%s> M=%d N=%d", sizeof(T) == 2 ? "bf16" : "f32", nw, q ? "post" : "plain", p.M, p.N);
+int launch_gemv(const GemvParams& p, const GemvParams* p1, const PostNorm* q, hipStream_t st) {
+  const int nw = gemv_waves(p.N + (p1 ? p1->N : 0));
+  exo_note_variant("dense_gemv<%s,%d,%s,%s> M=%d N=%d", sizeof(T) == 2 ? "bf16" : "f32", nw, q ? "post" : "plain",
+                   p1 ? "dual" : p.w2 ? "pair" : "single", p.M, p.N);
   if (nw == 4)
-    launch_gemv_nw<T, 4>(p, q, st);
+    launch_gemv_nw<T, 4>(p, p1, q, st);
   else if (nw == 8)
-    launch_gemv_nw<T, 8>(p, q, st);
+    launch_gemv_nw<T, 8>(p, p1, q, st);
   else
-    launch_gemv_nw<T, 16>(p, q, st);
+    launch_gemv_nw<T, 16>(p, p1, q, st);
   return EXO_OK;
 }
 
@@ -457,63 +578,86 @@ int launch_gemv(const GemvParams& p, const PostNorm* q, hipStream_t st) {
 
 }  // namespace
 
-extern "C" int exo_dense_gemv(const void* x, const void* w, const float* bias, void* y, int y_f32, int M, int N,
-                              int ldx, int ldw, int ldy, int dtype, exo_stream_t stream) {
-  EXO_DENSE_ARGS("exo_dense_gemv");
-  EXO_REQUIRE(M <= 16 && ldy >= N, "exo_dense_gemv: M=%d must be <= 16 and ldy=%d >= N=%d", M, ldy, N);
-  const GemvParams p{x, w, bias, y, M, N, ldx, ldw, ldy, y_f32};
-  const int rc = EXO_BY_TYPE(dtype, launch_gemv<bf16_t>(p, nullptr, (hipStream_t)stream),
-                             launch_gemv<float>(p, nullptr, (hipStream_t)stream));
+// ---- the struct interface: one product (or gated pair), rows of any number
+static int linear_check(const exo_linear* a, const char* what) {
+  EXO_REQUIRE(a && (a->dtype == 0 || a->dtype == 1), "%s: dtype must be 0 (bf16) or 1 (float32)", what);
+  EXO_REQUIRE(a->w && a->y, "%s: null pointer", what);
+  EXO_REQUIRE(a->M > 0 && a->N > 0 && a->ldx > 0 && a->ldx == a->ldw && a->ldw % 64 == 0,
+              "%s: need M, N > 0 and equal row strides that are multiples of 64 (got M=%d N=%d %d/%d)", what, a->M, a->N,
+              a->ldx, a->ldw);
+  EXO_REQUIRE((((uintptr_t)a->x | (uintptr_t)a->w | (uintptr_t)a->w_up) & 15) == 0, "%s: operands must be 16-byte aligned", what);
+  EXO_REQUIRE((int64_t)a->ldw * 256 * 4 < (1ll << 31), "%s: row stride %d too large", what, a->ldw);
+  EXO_REQUIRE(a->n1 > 0 && a->n1 <= a->N && a->ldy >= a->n1 && (a->n1 == a->N || (a->y2 && a->ldy2 >= a->N - a->n1)),
+              "%s: outputs do not hold %d columns (%d in the first: %d, %d)", what, a->N, a->n1, a->ldy, a->ldy2);
+  EXO_REQUIRE(!a->w_up || (a->n1 == a->N && !a->bias), "%s: a gated pair has one output and no bias", what);
+  return EXO_OK;
+}
+static GemvParams gemv_of(const exo_linear* a) {
+  GemvParams p{};
+  p.x = a->x, p.w = a->w, p.w2 = a->w_up, p.bias = a->bias, p.y = a->y, p.y2 = a->y2;
+  p.M = a->M, p.N = a->N, p.n1 = a->n1, p.ldx = a->ldx, p.ldw = a->ldw, p.ldy = a->ldy, p.ldy2 = a->ldy2, p.y_f32 = a->y_f32;
+  p.glu = GluConst{a->limit, a->alpha, a->shift};
+  return p;
+}
+
+extern "C" int exo_linear_rows(const exo_linear* a, const exo_linear* b, exo_stream_t stream) {
+  int rc = linear_check(a, "exo_linear_rows");
   if (rc) return rc;
-  EXO_CHECK_LAUNCH("exo_dense_gemv");
+  EXO_REQUIRE(a->M <= 16 && a->x, "exo_linear_rows: M=%d must be <= 16, x not null", a->M);
+  GemvParams second{};
+  if (b) {
+    rc = linear_check(b, "exo_linear_rows");
+    if (rc) return rc;
+    EXO_REQUIRE(b->x && b->M == a->M && b->dtype == a->dtype && !a->w_up && !b->w_up,
+                "exo_linear_rows: two products of one launch need the same rows and no gated pair");
+    second = gemv_of(b);
+  }
+  const GemvParams p = gemv_of(a);
+  rc = EXO_BY_TYPE(a->dtype, launch_gemv<bf16_t>(p, b ? &second : nullptr, nullptr, (hipStream_t)stream),
+                   launch_gemv<float>(p, b ? &second : nullptr, nullptr, (hipStream_t)stream));
+  if (rc) return rc;
+  EXO_CHECK_LAUNCH("exo_linear_rows");
   return EXO_OK;
 }
 
-extern "C" int exo_post_gemv_fits(int M, int N, int H, int ldx, int dtype) {
+extern "C" int exo_post_linear_fits(int M, int N, int H, int ldx, int dtype) {
   return M > 0 && N > 0 && H > 0 && post_fits(M, N, H, ldx, dtype == 0 ? 2 : 4);
 }
 
-extern "C" int exo_post_gemv(const float* x, const float* branch, const float* gain, float eps, float* x_out,
-                             void* xb_out, const void* w, const float* bias, void* y, int y_f32, int M, int N, int H,
-                             int ldx, int ldw, int ldy, int dtype, exo_stream_t stream) {
-  EXO_DENSE_ARGS("exo_post_gemv");
-  EXO_REQUIRE(branch && gain && x_out && x_out != x && ldy >= N, "exo_post_gemv: null pointer, x_out == x or bad ldy");
-  EXO_REQUIRE(post_fits(M, N, H, ldx, dtype == 0 ? 2 : 4), "exo_post_gemv: %d rows of %d columns do not fit one launch", M, H);
-  const GemvParams p{nullptr, w, bias, y, M, N, ldx, ldw, ldy, y_f32};
-  const PostNorm q{x, branch, gain, x_out, xb_out, H, eps};
-  const int rc = EXO_BY_TYPE(dtype, launch_gemv<bf16_t>(p, &q, (hipStream_t)stream), launch_gemv<float>(p, &q, (hipStream_t)stream));
+extern "C" int exo_post_linear(const exo_post_norm* q, const exo_linear* a, exo_stream_t stream) {
+  int rc = linear_check(a, "exo_post_linear");
   if (rc) return rc;
-  EXO_CHECK_LAUNCH("exo_post_gemv");
+  EXO_REQUIRE(q && q->x && q->branch && q->gain && q->x_out && q->x_out != q->x, "exo_post_linear: null pointer or x_out == x");
+  EXO_REQUIRE(!q->branch2 || (q->gain_a && q->gain_b), "exo_post_linear: two branches need a gain each");
+  EXO_REQUIRE(post_fits(a->M, a->N, q->H, a->ldx, a->dtype == 0 ? 2 : 4), "exo_post_linear: %d rows of %d columns do not fit one launch",
+              a->M, q->H);
+  const GemvParams p = gemv_of(a);
+  const PostNorm n{q->x, q->branch, q->branch2, q->gain_a, q->gain_b, q->gain, q->pre, q->x_out, q->operand, q->H, q->eps, q->mult};
+  rc = EXO_BY_TYPE(a->dtype, launch_gemv<bf16_t>(p, nullptr, &n, (hipStream_t)stream),
+                   launch_gemv<float>(p, nullptr, &n, (hipStream_t)stream));
+  if (rc) return rc;
+  EXO_CHECK_LAUNCH("exo_post_linear");
   return EXO_OK;
 }
 
-extern "C" int exo_dense_gemm(const void* x, const void* w, const float* bias, void* y, int y_f32, float* workspace,
-                              int64_t workspace_floats, int M, int N, int ldx, int ldw, int ldy, int dtype,
-                              exo_stream_t stream) {
-  EXO_DENSE_ARGS("exo_dense_gemm");
-  EXO_REQUIRE(ldy >= N && M <= 65535 * 64, "exo_dense_gemm: bad ldy=%d or M=%d", ldy, M);
-  GemmParams p{};
-  p.x = x, p.w = w, p.bias = bias, p.y = y, p.M = M, p.N = N, p.ldx = ldx, p.ldw = ldw, p.ldy = ldy, p.y_f32 = y_f32;
-  p.part = workspace;
-  const int rc = EXO_BY_TYPE(dtype, (launch_plain<bf16_t, false>(p, workspace_floats, (hipStream_t)stream)),
-                             (launch_plain<float, false>(p, workspace_floats, (hipStream_t)stream)));
+extern "C" int exo_linear_gemm(const exo_linear* a, float* workspace, int64_t workspace_floats, exo_stream_t stream) {
+  int rc = linear_check(a, "exo_linear_gemm");
   if (rc) return rc;
-  EXO_CHECK_LAUNCH("exo_dense_gemm");
-  return EXO_OK;
-}
-
-extern "C" int exo_dense_glu_gemm(const void* x, const void* w, const void* w_up, void* y, float limit, float alpha,
-                                  float shift, int M, int N, int ldx, int ldw, int ldy, int dtype,
-                                  exo_stream_t stream) {
-  EXO_DENSE_ARGS("exo_dense_glu_gemm");
-  EXO_REQUIRE(w_up && ldy >= N && M <= 65535 * 64, "exo_dense_glu_gemm: bad w_up, ldy=%d or M=%d", ldy, M);
+  EXO_REQUIRE(a->x && a->M <= 65535 * 64, "exo_linear_gemm: null x or bad M=%d", a->M);
   GemmParams p{};
-  p.x = x, p.w = w, p.w2 = w_up, p.y = y, p.M = M, p.N = N, p.ldx = ldx, p.ldw = ldw, p.ldy = ldy;
-  p.glu = GluConst{limit, alpha, shift};
-  const int rc = EXO_BY_TYPE(dtype, (launch_plain<bf16_t, true>(p, 0, (hipStream_t)stream)),
-                             (launch_plain<float, true>(p, 0, (hipStream_t)stream)));
+  p.x = a->x, p.w = a->w, p.w2 = a->w_up, p.bias = a->bias, p.y = a->y, p.y2 = a->y2;
+  p.M = a->M, p.N = a->N, p.n1 = a->n1, p.ldx = a->ldx, p.ldw = a->ldw, p.ldy = a->ldy, p.ldy2 = a->ldy2, p.y_f32 = a->y_f32;
+  p.glu = GluConst{a->limit, a->alpha, a->shift};
+  p.part = a->w_up ? nullptr : workspace;
+  EXO_REQUIRE(!a->w_up || a->y_f32 == (a->dtype == 1), "exo_linear_gemm: a gated pair leaves in the element type");
+  if (a->w_up)
+    rc = EXO_BY_TYPE(a->dtype, (launch_plain<bf16_t, true>(p, 0, (hipStream_t)stream)),
+                     (launch_plain<float, true>(p, 0, (hipStream_t)stream)));
+  else
+    rc = EXO_BY_TYPE(a->dtype, (launch_plain<bf16_t, false>(p, workspace_floats, (hipStream_t)stream)),
+                     (launch_plain<float, false>(p, workspace_floats, (hipStream_t)stream)));
   if (rc) return rc;
-  EXO_CHECK_LAUNCH("exo_dense_glu_gemm");
+  EXO_CHECK_LAUNCH("exo_linear_gemm");
   return EXO_OK;
 }
 

@@ -1,5 +1,6 @@
 // Attention over a paged KV pool, for batches that mix portions of prompts with single decoded
-// tokens.  Options, each a parameter of the layer: unit-RMS queries and keys, a per-head linear
+// tokens.  Options, each a parameter of the layer: unit-RMS queries and keys (with a gain per
+// channel), a gate per head on the output (sigmoid of a given number), a per-head linear
 // distance penalty, a sliding window with kept first tokens, value size other than key size, keys
 // and values of another layer.  Scores, penalty, softmax and sums are float32; where the weights
 // enter a bf16 matrix product they go in as two bf16 terms (high and remainder), so that they keep
@@ -41,11 +42,14 @@ struct Params {
   const int32_t* pos;   // [R]
   const int32_t* list;  // rows: row indices (null: all); prompt: blocks of {row, slot, pos, n}
   const float* slopes;  // [H], or null
+  const float* qgain;   // [D], or null
+  const float* kgain;   // [D], or null
+  const float* gate;    // [R][ldg] a number per head, or null
   void* out;            // T [R][ldo]
   float* ws;
   int* counters;
   float scale, eps;
-  int n, H, G, D, E, ldq, ldk, ldv, ldo, max_pages, size, keep, unit, nsplit, gsz, hgroups;
+  int n, H, G, D, E, ldq, ldk, ldv, ldo, ldg, max_pages, size, keep, unit, nsplit, gsz, hgroups;
 };
 
 __device__ __forceinline__ void st_dev(float* p, float v) {
@@ -70,16 +74,22 @@ __device__ __forceinline__ Tiles tiles_of(int first, int last, int size, int kee
   return t;
 }
 
-// one wave: src[0..D) / rms -> dst (element type T, float32 arithmetic)
+// what a head's output is multiplied with
+__device__ __forceinline__ float head_gate(const Params& p, int row, int h) {
+  return p.gate ? 1.f / (1.f + expf(-p.gate[(size_t)row * p.ldg + h])) : 1.f;
+}
+
+// one wave: src[0..D) / rms * gain -> dst (element type T, float32 arithmetic)
 template <typename T>
-__device__ __forceinline__ void unit_row(const T* __restrict__ src, T* dst, int D, int unit, float eps, int lane) {
+__device__ __forceinline__ void unit_row(const T* __restrict__ src, T* dst, int D, int unit, float eps,
+                                         const float* __restrict__ gain, int lane) {
   float ss = 0.f;
   for (int d = lane; d < D; d += 64) {
     const float v = Elem<T>::load(src[d]);
     ss += v * v;
   }
   const float inv = unit ? 1.f / sqrtf(wave_sum(ss) / D + eps) : 1.f;
-  for (int d = lane; d < D; d += 64) dst[d] = Elem<T>::make(Elem<T>::load(src[d]) * inv);
+  for (int d = lane; d < D; d += 64) dst[d] = Elem<T>::make(Elem<T>::load(src[d]) * inv * (gain ? gain[d] : 1.f));
 }
 
 // key and value of one (row, kv head) into the pool, by one wave each
@@ -87,7 +97,7 @@ template <typename T>
 __device__ __forceinline__ void put_key(const Params& p, int row, int g, int page, int at, int lane) {
   const T* src = reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + p.H * p.D + g * p.D;
   T* dst = reinterpret_cast<T*>(p.kpool) + (((size_t)page * p.G + g) * kPage + at) * p.ldk;
-  unit_row<T>(src, dst, p.D, p.unit, p.eps, lane);
+  unit_row<T>(src, dst, p.D, p.unit, p.eps, p.kgain, lane);
 }
 template <typename T>
 __device__ __forceinline__ void put_value(const Params& p, int row, int g, int page, int at, int lane) {
@@ -131,7 +141,7 @@ __global__ __launch_bounds__(256) void paged_append_kernel(const Params p) {
           T e[VEC];
         } w;
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) w.e[e] = Elem<T>::make(f[e] * inv);
+        for (int e = 0; e < VEC; ++e) w.e[e] = Elem<T>::make(f[e] * inv * (p.kgain && on ? p.kgain[c * VEC + e] : 1.f));
         if (on && i < n)
           *reinterpret_cast<uint4*>(reinterpret_cast<T*>(p.kpool) + (((size_t)page * p.G + unit) * kPage + at) * p.ldk +
                                     c * VEC) = __builtin_bit_cast(uint4, w);
@@ -157,7 +167,7 @@ __global__ __launch_bounds__(256) void paged_append_kernel(const Params p) {
       T* dst = reinterpret_cast<T*>(p.kpool) + (((size_t)page * p.G + unit) * kPage + at) * p.ldk;
 #pragma unroll
       for (int j = 0; j < 4; ++j)
-        if (lane + 64 * j < p.D) dst[lane + 64 * j] = Elem<T>::make(v[i][j] * inv);
+        if (lane + 64 * j < p.D) dst[lane + 64 * j] = Elem<T>::make(v[i][j] * inv * (p.kgain ? p.kgain[lane + 64 * j] : 1.f));
     }
     return;
   }
@@ -294,7 +304,7 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
   // ---- queries (and the row's own key and value) through float32 norms
   for (int h = wave; h < 16; h += kRowWaves) {
     T* dst = qs + h * QS;
-    if (h < gs) unit_row<T>(reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + (h0 + h) * p.D, dst, p.D, p.unit, p.eps, lane);
+    if (h < gs) unit_row<T>(reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + (h0 + h) * p.D, dst, p.D, p.unit, p.eps, p.qgain, lane);
     for (int d = (h < gs ? p.D : 0) + lane; d < QS; d += 64) dst[d] = Elem<T>::make(0.f);
   }
   if (FUSE && split == ((tl.n - 1) % stride) / kRowWaves) {
@@ -393,7 +403,7 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
       lw += ms[w][h] == -INFINITY ? 0.f : ls[w][h] * __builtin_amdgcn_exp2f(ms[w][h] - mm);
     }
     if (p.nsplit == 1) {
-      out[(h0 + h) * p.E + d] = Elem<T>::make(acc / lw);
+      out[(h0 + h) * p.E + d] = Elem<T>::make(acc / lw * head_gate(p, row, h0 + h));
     } else {
       float* dst = p.ws + ((wsrow + h0 + h) * p.nsplit + split) * (p.E + 2);
       st_dev(dst + d, acc);
@@ -442,7 +452,7 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
       for (int s = 0; s < 16; ++s)
         if (s0 + s < p.nsplit) acc += v[s] * fac[h * p.nsplit + s0 + s];
     }
-    out[(h0 + h) * p.E + d] = Elem<T>::make(acc);
+    out[(h0 + h) * p.E + d] = Elem<T>::make(acc * head_gate(p, row, h0 + h));
   }
 }
 
@@ -504,9 +514,17 @@ __global__ __launch_bounds__(256, D > 128 ? 1 : 2) void paged_prompt_kernel(cons
     if (p.unit) {
       const float inv = 1.f / sqrtf(ss / p.D + p.eps);
 #pragma unroll
-      for (int s = 0; s < STEPS; ++s)
-        q[s] = uint4{pack_bf2(bf_lo(q[s].x) * inv, bf_hi(q[s].x) * inv), pack_bf2(bf_lo(q[s].y) * inv, bf_hi(q[s].y) * inv),
-                     pack_bf2(bf_lo(q[s].z) * inv, bf_hi(q[s].z) * inv), pack_bf2(bf_lo(q[s].w) * inv, bf_hi(q[s].w) * inv)};
+      for (int s = 0; s < STEPS; ++s) {
+        const uint32_t w[4] = {q[s].x, q[s].y, q[s].z, q[s].w};
+        uint32_t u[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int d = 16 * s + 8 * kq + 2 * i;  // (past D the queries are zero)
+          const float ga = p.qgain ? p.qgain[min(d, p.D - 1)] * inv : inv, gb = p.qgain ? p.qgain[min(d + 1, p.D - 1)] * inv : inv;
+          u[i] = pack_bf2(bf_lo(w[i]) * ga, bf_hi(w[i]) * gb);
+        }
+        q[s] = uint4{u[0], u[1], u[2], u[3]};
+      }
     }
   }
 
@@ -626,7 +644,7 @@ __global__ __launch_bounds__(256, D > 128 ? 1 : 2) void paged_prompt_kernel(cons
     }
   }
   if (!active || tt * 32 + n >= blk.w) return;
-  const float inv = 1.f / l;
+  const float inv = head_gate(p, row, hq) / l;
   bf16_t* op = reinterpret_cast<bf16_t*>(p.out) + (size_t)row * p.ldo + (size_t)hq * p.E;
   const bool pairs = p.E % 4 == 0;
 #pragma unroll
@@ -650,6 +668,7 @@ Params params_of(const exo_paged_attn* a) {
   Params p{};
   p.qkv = a->qkv, p.kpool = a->k_pool, p.vpool = a->v_pool, p.table = a->table, p.slot = a->slot, p.pos = a->pos;
   p.list = a->list, p.slopes = a->slopes, p.out = a->out;
+  p.qgain = a->q_gain, p.kgain = a->k_gain, p.gate = a->gate, p.ldg = a->ldg;
   p.scale = a->scale, p.eps = a->eps, p.n = a->n, p.H = a->heads, p.G = a->kv_heads, p.D = a->dim, p.E = a->vdim;
   p.ldq = a->ldq, p.ldk = a->ldk, p.ldv = a->ldv, p.ldo = a->ldo, p.max_pages = a->max_pages;
   p.size = a->window > 0 ? a->window : 0x3FFFFFFF;
@@ -667,6 +686,8 @@ int check(const exo_paged_attn* a, const char* what) {
   EXO_REQUIRE(a->ldk % 32 == 0 && a->ldk >= a->dim && a->ldk <= 256 && a->ldv % 32 == 0 && a->ldv >= a->vdim && a->ldv <= 256,
               "%s: pool strides %d / %d do not fit head sizes %d / %d", what, a->ldk, a->ldv, a->dim, a->vdim);
   EXO_REQUIRE(a->qkv && a->k_pool && a->v_pool && a->table && a->max_pages > 0, "%s: null pointer", what);
+  EXO_REQUIRE(!a->gate || a->ldg >= a->heads, "%s: %d gates per row for %d heads", what, a->ldg, a->heads);
+  EXO_REQUIRE(a->unit_qk || (!a->q_gain && !a->k_gain), "%s: a query / key gain belongs to the norm", what);
   EXO_REQUIRE(a->keep_first >= 0 && a->window >= 0, "%s: negative window", what);
   return EXO_OK;
 }

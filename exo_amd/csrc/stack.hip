@@ -1,5 +1,5 @@
 // Small operators of a layer-list decoder with a float32 residual stream: embedding rows,
-// normalisation of a sublayer's OUTPUT before it is added, routing with a choice correction and
+// normalisation of a sublayer's OUTPUT before it is added and of the sum as the next one's input, routing with a choice correction and
 // identity experts, and the expert products of a decode step.  Element type bf16 or float
 // (dense.h); every norm, router and sum here is float32.
 #include "../../include/exo_mi355x.h"
@@ -61,7 +61,8 @@ struct MoeSum {        // the feed-forward's output as a sum over a token's expe
   int top, experts, ldy, lds, ldl, gate_col;
 };
 
-// x += gain * v / rms(v), v = the branch row (or the weighted sum over the experts); xb = x.
+// x += mult * gain * v / rms(v), v = the branch row, half the sum of two branches normed each with a
+// gain of its own, or the weighted sum over the experts; xb = x, or x / rms(x) * pre.
 // Four columns per thread and pass (VEC: rows of four columns are aligned), v in registers.
 constexpr int kCols = 4, kPasses = 16;  // H <= 16384
 
@@ -83,14 +84,13 @@ __device__ __forceinline__ void load_cols(const T* p, float (&f)[kCols], bool ve
 }
 
 template <typename T, int PASSES>
-__global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const float* __restrict__ branch, int ldb,
-                                                                    const MoeSum m, const float* __restrict__ gain,
-                                                                    float* __restrict__ x, T* __restrict__ xb, int H,
-                                                                    int ldx, float eps) {
+__global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const exo_post_norm q, int ldb, const MoeSum m,
+                                                                    float* __restrict__ x, T* __restrict__ xb, int ldx) {
   __shared__ float tmp[kRowThreads / 64];
-  const int row = blockIdx.x;
+  const int row = blockIdx.x, H = q.H;
   float* xr = x + (size_t)row * H;
   const bool vec = H % kCols == 0 && (m.y ? m.ldy % kCols == 0 && m.lds % kCols == 0 : ldb % kCols == 0);
+  const bool gvec = H % kCols == 0;
   float v[PASSES][kCols], xv[PASSES][kCols];
   float pass = 0.f, sg = 0.f;  // weight of the input itself; gate of the shared expert
   const T *y = nullptr, *sh = nullptr;
@@ -127,24 +127,68 @@ __global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const float*
         for (int e = 0; e < kCols; ++e) v[i][e] = fmaf(sg, f[e], v[i][e]);
       }
     } else {
-      load_cols<float>(branch + (size_t)row * ldb + c, v[i], vec, left);
+      load_cols<float>(q.branch + (size_t)row * ldb + c, v[i], vec, left);
     }
 #pragma unroll
     for (int e = 0; e < kCols; ++e) ss += e < left ? v[i][e] * v[i][e] : 0.f;
   }
-  const float inv = 1.f / sqrtf(block_sum(ss, tmp) / H + eps);
+  if (q.branch2) {
+    float u[PASSES][kCols], su = 0.f;
+#pragma unroll
+    for (int i = 0; i < PASSES; ++i) {
+      const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
+      if (left <= 0) break;
+      load_cols<float>(q.branch2 + (size_t)row * ldb + c, u[i], vec, left);
+#pragma unroll
+      for (int e = 0; e < kCols; ++e) su += e < left ? u[i][e] * u[i][e] : 0.f;
+    }
+    const float ia = 0.5f / sqrtf(block_sum(ss, tmp) / H + q.eps), ib = 0.5f / sqrtf(block_sum(su, tmp) / H + q.eps);
+    ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < PASSES; ++i) {
+      const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
+      if (left <= 0) break;
+      float ga[kCols], gb[kCols];
+      load_cols<float>(q.gain_a + c, ga, gvec, left);
+      load_cols<float>(q.gain_b + c, gb, gvec, left);
+#pragma unroll
+      for (int e = 0; e < kCols; ++e) {
+        v[i][e] = v[i][e] * ia * ga[e] + u[i][e] * ib * gb[e];
+        ss += e < left ? v[i][e] * v[i][e] : 0.f;
+      }
+    }
+  }
+  const float inv = q.mult / sqrtf(block_sum(ss, tmp) / H + q.eps);
+  ss = 0.f;
 #pragma unroll
   for (int i = 0; i < PASSES; ++i) {
     const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
     if (left <= 0) break;
     float gn[kCols];
-    load_cols<float>(gain + c, gn, H % kCols == 0, left);
+    load_cols<float>(q.gain + c, gn, gvec, left);
+#pragma unroll
+    for (int e = 0; e < kCols; ++e) {
+      xv[i][e] += v[i][e] * inv * gn[e];
+      ss += e < left ? xv[i][e] * xv[i][e] : 0.f;
+    }
+  }
+  const float pinv = q.pre ? 1.f / sqrtf(block_sum(ss, tmp) / H + q.eps) : 1.f;
+#pragma unroll
+  for (int i = 0; i < PASSES; ++i) {
+    const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
+    if (left <= 0) break;
     float y[kCols];
 #pragma unroll
-    for (int e = 0; e < kCols; ++e) y[e] = xv[i][e] + v[i][e] * inv * gn[e];
+    for (int e = 0; e < kCols; ++e) y[e] = xv[i][e];
+    if (q.pre) {
+      float gp[kCols];
+      load_cols<float>(q.pre + c, gp, gvec, left);
+#pragma unroll
+      for (int e = 0; e < kCols; ++e) y[e] = y[e] * pinv * gp[e];
+    }
     T* bo = xb + (size_t)row * ldx + c;
     if (vec && ldx % kCols == 0) {
-      *reinterpret_cast<floatx4*>(xr + c) = floatx4{y[0], y[1], y[2], y[3]};
+      *reinterpret_cast<floatx4*>(xr + c) = floatx4{xv[i][0], xv[i][1], xv[i][2], xv[i][3]};
       if (sizeof(T) == 2)
         *reinterpret_cast<uint2*>(bo) = uint2{pack_bf2(y[0], y[1]), pack_bf2(y[2], y[3])};
       else
@@ -152,7 +196,7 @@ __global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const float*
     } else {
 #pragma unroll
       for (int e = 0; e < kCols; ++e)
-        if (e < left) xr[c + e] = y[e], bo[e] = Elem<T>::make(y[e]);
+        if (e < left) xr[c + e] = xv[i][e], bo[e] = Elem<T>::make(y[e]);
     }
   }
 }
@@ -452,18 +496,20 @@ extern "C" int exo_norm_rows(const float* x, const int32_t* rows, const float* g
   return EXO_OK;
 }
 
-static int post_norm(const float* branch, int ldb, const MoeSum& m, const float* gain, float* x, void* xb, int n, int H,
-                     int ldx, float eps, int dtype, exo_stream_t stream) {
-  EXO_REQUIRE(gain && x && xb && n >= 0 && H > 0 && H <= 16384 && ldx >= H, "exo_post_norm_add: bad argument (H=%d)", H);
+static int post_norm(const exo_post_norm* q, int ldb, const MoeSum& m, int n, int ldx, int dtype, exo_stream_t stream) {
+  EXO_TYPE_OK("exo_post_norm_add");
+  EXO_REQUIRE(q && q->gain && q->x && q->x == q->x_out && q->operand && n >= 0 && q->H > 0 && q->H <= 16384 && ldx >= q->H,
+              "exo_post_norm_add: bad argument (H=%d, x in place)", q ? q->H : 0);
+  EXO_REQUIRE(!q->branch2 || (q->gain_a && q->gain_b && !m.y), "exo_post_norm_add: two branches need a gain each");
   if (n == 0) return EXO_OK;
 #define EXO_POST(P)                                                                                              \
   do {                                                                                                           \
     if (dtype == 0)                                                                                              \
-      post_norm_add_kernel<bf16_t, P><<<n, kRowThreads, 0, (hipStream_t)stream>>>(branch, ldb, m, gain, x, (bf16_t*)xb, H, ldx, eps); \
+      post_norm_add_kernel<bf16_t, P><<<n, kRowThreads, 0, (hipStream_t)stream>>>(*q, ldb, m, q->x_out, (bf16_t*)q->operand, ldx); \
     else                                                                                                         \
-      post_norm_add_kernel<float, P><<<n, kRowThreads, 0, (hipStream_t)stream>>>(branch, ldb, m, gain, x, (float*)xb, H, ldx, eps);   \
+      post_norm_add_kernel<float, P><<<n, kRowThreads, 0, (hipStream_t)stream>>>(*q, ldb, m, q->x_out, (float*)q->operand, ldx);   \
   } while (0)
-  const int passes = exo_ceil_div(H, kRowThreads * kCols);
+  const int passes = exo_ceil_div(q->H, kRowThreads * kCols);
   if (passes <= 1) EXO_POST(1);
   else if (passes <= 2) EXO_POST(2);
   else if (passes <= 4) EXO_POST(4);
@@ -474,22 +520,17 @@ static int post_norm(const float* branch, int ldb, const MoeSum& m, const float*
   return EXO_OK;
 }
 
-extern "C" int exo_post_norm_add(const float* branch, int ldb, const float* gain, float* x, void* xb, int n, int H,
-                                 int ldx, float eps, int dtype, exo_stream_t stream) {
-  EXO_TYPE_OK("exo_post_norm_add");
-  EXO_REQUIRE(branch && ldb >= H, "exo_post_norm_add: bad branch");
-  return post_norm(branch, ldb, MoeSum{}, gain, x, xb, n, H, ldx, eps, dtype, stream);
+extern "C" int exo_post_norm_add(const exo_post_norm* q, int ldb, int n, int ldx, int dtype, exo_stream_t stream) {
+  EXO_REQUIRE(q && q->branch && ldb >= q->H, "exo_post_norm_add: bad branch");
+  return post_norm(q, ldb, MoeSum{}, n, ldx, dtype, stream);
 }
 
 extern "C" int exo_moe_sum_post_norm(const void* y, const int32_t* idx, const float* wt, const void* shared,
                                      const float* logits, int top, int experts, int ldy, int lds, int ldl, int gate_col,
-                                     const float* gain, float* x, void* xb, int n, int H, int ldx, float eps, int dtype,
-                                     exo_stream_t stream) {
-  EXO_TYPE_OK("exo_moe_sum_post_norm");
-  EXO_REQUIRE(y && idx && wt && top > 0 && experts > 0 && ldy >= H && (!shared || (logits && lds >= H && gate_col < ldl)),
+                                     const exo_post_norm* q, int n, int ldx, int dtype, exo_stream_t stream) {
+  EXO_REQUIRE(q && y && idx && wt && top > 0 && experts > 0 && ldy >= q->H && (!shared || (logits && lds >= q->H && gate_col < ldl)),
               "exo_moe_sum_post_norm: bad argument");
-  return post_norm(nullptr, 0, MoeSum{y, idx, wt, shared, logits, top, experts, ldy, lds, ldl, gate_col}, gain, x, xb, n,
-                   H, ldx, eps, dtype, stream);
+  return post_norm(q, 0, MoeSum{y, idx, wt, shared, logits, top, experts, ldy, lds, ldl, gate_col}, n, ldx, dtype, stream);
 }
 
 extern "C" int exo_moe_route(const float* logits, const float* correction, int32_t* idx, float* wt, int rows, int n,

@@ -1,6 +1,6 @@
 """Operators of the layer-list decoders on torch device tensors (C ABI of include/exo_mi355x.h):
-products with unquantised matrices, residual norms, routing, experts and attention over a paged
-pool.  Element type bf16 or float32 throughout (the tensors' dtype decides); like ``ops``, every
+products with unquantised matrices, residual norms, routing, experts, attention over a paged pool
+and recurrences over a state pool.  Element type bf16 or float32 throughout (the tensors' dtype decides); like ``ops``, every
 function launches on torch's current stream and never synchronises.
 
 Matrix operands have row strides of multiples of 64 elements with zeros past the logical size
@@ -50,18 +50,39 @@ def norm_rows(x, gain, eps: float, out, n: int, rows=None) -> None:
                                       _code(out), _stream()), "norm_rows")
 
 
-def post_norm_add(branch, gain, eps: float, x, xb, n: int) -> None:
-    """x += norm(branch); xb = x in the element type.  branch and x float32."""
-    check(native.load().exo_post_norm_add(_ptr(branch), branch.shape[1], _ptr(gain), _ptr(x), _ptr(xb), n,
-                                          gain.numel(), xb.shape[1], eps, _code(xb), _stream()), "post_norm_add")
+def _p(t):
+    return None if t is None else t.data_ptr()
 
 
-def moe_sum_post_norm(y, idx, wt, shared, logits, experts: int, gate_col: int, gain, eps: float, x, xb, n: int) -> None:
+class Branches:
+    """A sublayer's output on its way into the residual: ``branch``, or half the sum of two branches that
+    are normed each with a gain of its own first (``branch2``, ``gain_a``, ``gain_b``); then the norm with
+    ``gain``, times ``mult``.  All float32."""
+
+    def __init__(self, branch, gain, mult: float = 1.0, branch2=None, gain_a=None, gain_b=None):
+        self.branch, self.gain, self.mult = branch, gain, mult
+        self.branch2, self.gain_a, self.gain_b = branch2, gain_a, gain_b
+
+    def args(self, x, x_out, operand, eps: float, pre) -> native.PostNorm:
+        return native.PostNorm(x=x.data_ptr(), branch=_p(self.branch), branch2=_p(self.branch2), gain_a=_p(self.gain_a),
+                               gain_b=_p(self.gain_b), gain=self.gain.data_ptr(), pre=_p(pre), x_out=x_out.data_ptr(),
+                               operand=_p(operand), H=self.gain.numel(), eps=eps, mult=self.mult)
+
+
+def post_norm_add(br: Branches, eps: float, x, xb, n: int, pre=None) -> None:
+    """x += the normed branches; xb = x (or its norm with gain ``pre``) in the element type."""
+    check(native.load().exo_post_norm_add(C.byref(br.args(x, x, xb, eps, pre)), br.branch.shape[1], n, xb.shape[1],
+                                          _code(xb), _stream()), "post_norm_add")
+
+
+def moe_sum_post_norm(y, idx, wt, shared, logits, experts: int, gate_col: int, gain, eps: float, x, xb, n: int,
+                      mult: float = 1.0) -> None:
     """x += norm(weighted sum of the chosen experts' outputs y [n, top, ld] + gated shared)."""
+    q = Branches(None, gain, mult).args(x, x, xb, eps, None)
     check(native.load().exo_moe_sum_post_norm(
         _ptr(y), _ptr(idx), _ptr(wt), _ptr(shared), _ptr(logits), idx.shape[1], experts, y.shape[-1],
-        0 if shared is None else shared.shape[1], logits.shape[1], gate_col, _ptr(gain), _ptr(x), _ptr(xb), n,
-        gain.numel(), xb.shape[1], eps, _code(xb), _stream()), "moe_sum_post_norm")
+        0 if shared is None else shared.shape[1], logits.shape[1], gate_col, C.byref(q), n, xb.shape[1], _code(xb),
+        _stream()), "moe_sum_post_norm")
 
 
 def moe_route(logits, correction, scale: float, idx, wt, n: int) -> None:
@@ -81,40 +102,64 @@ def gemm_workspace(device) -> torch.Tensor:
     return _GEMM_WS[key]
 
 
-def linear(x, w, out, n: int, bias=None, force_gemm: bool = False) -> None:
-    """out[:n] = x[:n] @ w^T (+ bias float32); out in x's element type or float32."""
-    lib, N = native.load(), w.shape[0]
-    f32 = int(out.dtype == torch.float32)
+def _linear(x, w, out, n: int, bias=None, tail=None, up=None, spec=None) -> native.Linear:
+    """``tail``: float32 output of the columns past ``out``'s share (w's rows beyond N - tail's logical
+    columns; given as (tensor, columns)).  ``up``, ``spec``: the gated pair."""
+    N = w.shape[0]
+    t, nt = (None, 0) if tail is None else tail
+    return native.Linear(
+        x=_p(x), w=w.data_ptr(), w_up=_p(up), bias=_p(bias), y=out.data_ptr(), y2=_p(t), M=n, N=N, n1=N - nt,
+        ldx=w.shape[1] if x is None else x.stride(0), ldw=w.shape[1], ldy=out.stride(0), ldy2=0 if t is None else t.stride(0),
+        y_f32=int(out.dtype == torch.float32), dtype=_code(w), limit=spec.limit if spec else 0.0,
+        alpha=spec.alpha if spec else 0.0, shift=spec.shift if spec else 0.0)
+
+
+def linear(x, w, out, n: int, bias=None, force_gemm: bool = False, tail=None) -> None:
+    """out[:n] = x[:n] @ w^T (+ bias float32); out in x's element type or float32.  ``tail`` (tensor, columns):
+    the last columns go to that float32 tensor instead."""
+    _launch_linear(_linear(x, w, out, n, bias, tail), n, x.device, force_gemm)
+
+
+def _launch_linear(a, n: int, device, force_gemm: bool = False) -> None:
     if n <= GEMV_MAX_ROWS and not force_gemm:
-        check(lib.exo_dense_gemv(_ptr(x), _ptr(w), _ptr(bias), _ptr(out), f32, n, N, x.shape[1], w.shape[1],
-                                 out.shape[1], _code(x), _stream()), "linear")
-        return
-    ws = gemm_workspace(x.device)
-    check(lib.exo_dense_gemm(_ptr(x), _ptr(w), _ptr(bias), _ptr(out), f32, _ptr(ws), ws.numel(), n, N, x.shape[1],
-                             w.shape[1], out.shape[1], _code(x), _stream()), "linear(gemm)")
+        check(native.load().exo_linear_rows(C.byref(a), None, _stream()), "linear")
+    else:
+        ws = gemm_workspace(device)
+        check(native.load().exo_linear_gemm(C.byref(a), _ptr(ws), ws.numel(), _stream()), "linear(gemm)")
+
+
+def linear_pair(x0, w0, out0, x1, w1, out1, n: int) -> None:
+    """Two products over the same number of rows: one launch for few rows."""
+    a, b = _linear(x0, w0, out0, n), _linear(x1, w1, out1, n)
+    if n <= GEMV_MAX_ROWS:
+        check(native.load().exo_linear_rows(C.byref(a), C.byref(b), _stream()), "linear_pair")
+    else:
+        _launch_linear(a, n, x0.device)
+        _launch_linear(b, n, x1.device)
 
 
 POST_MAX_ROWS = 4  # beyond, every workgroup repeating the norm costs more than a launch
 
 
 def post_linear_fits(n: int, w, xb, H: int) -> bool:
-    return n <= POST_MAX_ROWS and bool(native.load().exo_post_gemv_fits(n, w.shape[0], H, xb.shape[1], _code(xb)))
+    return n <= POST_MAX_ROWS and bool(native.load().exo_post_linear_fits(n, w.shape[0], H, xb.shape[1], _code(xb)))
 
 
-def post_linear(x, branch, gain, eps: float, x_out, xb, w, out, n: int, bias=None) -> None:
-    """``post_norm_add`` and ``linear`` in one launch: x_out = x + norm(branch) (another buffer than
-    x), xb (may be None) its copy, out = x_out @ w^T (+ bias)."""
-    check(native.load().exo_post_gemv(
-        _ptr(x), _ptr(branch), _ptr(gain), eps, _ptr(x_out), _ptr(xb), _ptr(w), _ptr(bias), _ptr(out),
-        int(out.dtype == torch.float32), n, w.shape[0], gain.numel(), w.shape[1], w.shape[1], out.shape[1], _code(w),
-        _stream()), "post_linear")
+def post_linear(x, br: Branches, eps: float, x_out, xb, w, out, n: int, bias=None, tail=None, pre=None, up=None,
+                spec=None) -> None:
+    """``post_norm_add`` and ``linear`` (or the gated pair) in one launch: x_out = x + the normed branches
+    (another buffer than x), xb (may be None) the product's operand."""
+    q, a = br.args(x, x_out, xb, eps, pre), _linear(None, w, out, n, bias, tail, up, spec)
+    check(native.load().exo_post_linear(C.byref(q), C.byref(a), _stream()), "post_linear")
+
+
+def glu(x, gate, up, out, n: int, spec, force_gemm: bool = False) -> None:
+    """out[:n] = clamped gated unit of x[:n]."""
+    _launch_linear(_linear(x, gate, out, n, up=up, spec=spec), n, x.device, force_gemm)
 
 
 def glu_gemm(x, gate, up, out, n: int, spec) -> None:
-    """out[:n] = clamped gated unit of x[:n] (any n)."""
-    check(native.load().exo_dense_glu_gemm(
-        _ptr(x), _ptr(gate), _ptr(up), _ptr(out), spec.limit, spec.alpha, spec.shift, n, gate.shape[0], x.shape[1],
-        gate.shape[1], out.shape[1], _code(x), _stream()), "glu_gemm")
+    glu(x, gate, up, out, n, spec, force_gemm=True)
 
 
 def grouped_gemm(x, w, group_ws, out, T: int, topk: int, up=None, spec=None, x_per_pair: bool = False) -> None:
@@ -173,21 +218,22 @@ class PagedAttention:
     """Attention of one layer over a paged pool.  ``spec``: AttentionSpec; ``li``: index of the
     pool's layer that holds its keys and values."""
 
-    def __init__(self, spec, slopes, li: int, cache, eps: float):
-        self.spec, self.slopes, self.cache = spec, slopes, cache
+    def __init__(self, spec, slopes, li: int, cache, eps: float, q_gain=None, k_gain=None):
+        self.spec, self.slopes, self.cache, self.gains = spec, slopes, cache, (q_gain, k_gain)
         k, v = cache.k[li], cache.v[li]
         self.args = native.PagedAttn(
             k_pool=k.data_ptr(), v_pool=v.data_ptr(), table=cache.table.data_ptr(),
-            slopes=None if slopes is None else slopes.data_ptr(), scale=spec.scale, eps=eps,
+            slopes=_p(slopes), q_gain=_p(q_gain), k_gain=_p(k_gain), scale=spec.scale, eps=eps,
             heads=spec.heads, kv_heads=spec.kv_heads, dim=spec.dim, vdim=spec.vdim, ldk=k.shape[3], ldv=v.shape[2],
             max_pages=cache.table.shape[1], window=spec.window or 0, keep_first=spec.keep_first,
             unit_qk=int(spec.unit_qk), dtype=_code(k))
 
-    def _bind(self, qkv, out, slot, pos, lst, n: int):
+    def _bind(self, qkv, out, slot, pos, lst, n: int, gate=None):
         a = self.args
         assert qkv.dtype == self.cache.k[0].dtype
-        a.qkv, a.ldq, a.n = qkv.data_ptr(), qkv.shape[1], n
-        a.out, a.ldo = (None, 0) if out is None else (out.data_ptr(), out.shape[1])
+        a.qkv, a.ldq, a.n = qkv.data_ptr(), qkv.stride(0), n
+        a.out, a.ldo = (None, 0) if out is None else (out.data_ptr(), out.stride(0))
+        a.gate, a.ldg = (None, 0) if gate is None else (gate.data_ptr(), gate.stride(0))
         a.slot = None if slot is None else slot.data_ptr()
         a.pos = None if pos is None else pos.data_ptr()
         a.list = None if lst is None else lst.data_ptr()
@@ -201,9 +247,10 @@ class PagedAttention:
         s = self.spec
         return keys if s.window is None else min(keys, s.window + s.keep_first)
 
-    def rows(self, qkv, out, slot, pos, n: int, keys: int, append: bool, lst=None) -> None:
+    def rows(self, qkv, out, slot, pos, n: int, keys: int, append: bool, lst=None, gate=None) -> None:
         """One query position per row (``lst``: which rows, else the first n).  ``keys``: most keys
-        any of the sequences holds, as the host knows it (lays out the launch)."""
+        any of the sequences holds, as the host knows it (lays out the launch).  ``gate``: float32
+        [rows, heads], head h's output times its sigmoid."""
         s = self.spec
         tiles = -(-self.visible(keys) // 32) + 2
         wgs = n * s.kv_heads * (-(-(s.heads // s.kv_heads) // 16))
@@ -213,14 +260,81 @@ class PagedAttention:
         if n * s.heads > 16384:
             nsplit = 1
         ws = attn_workspace(n, s.heads, s.vdim, nsplit, qkv.device) if nsplit > 1 else None
-        check(native.load().exo_paged_attn_rows(self._bind(qkv, out, slot, pos, lst, n), nsplit, int(append), _ptr(ws),
+        check(native.load().exo_paged_attn_rows(self._bind(qkv, out, slot, pos, lst, n, gate), nsplit, int(append), _ptr(ws),
                                                 0 if ws is None else ws.numel(), _stream()), "paged_attn_rows")
 
     @staticmethod
     def prompt_block(spec) -> int:
         return native.load().exo_paged_prompt_block(spec.heads, spec.kv_heads)
 
-    def prompt(self, qkv, out, blocks, n: int) -> None:
+    def prompt(self, qkv, out, blocks, n: int, gate=None) -> None:
         """Portions of prompts: blocks int32 [n, 4] = first row, slot, first position, tokens."""
-        check(native.load().exo_paged_attn_prompt(self._bind(qkv, out, None, None, blocks, n), _stream()),
+        check(native.load().exo_paged_attn_prompt(self._bind(qkv, out, None, None, blocks, n, gate), _stream()),
               "paged_attn_prompt")
+
+
+_RECUR_WS: dict[int, torch.Tensor] = {}
+
+
+def recur_workspace(floats: int, device) -> torch.Tensor:
+    """Chunk states and scores of recurrences over prompts, one per device, grown on demand (work is in
+    stream order; single-token steps, which are captured, do not use it)."""
+    key = torch.device(device).index or 0
+    if key not in _RECUR_WS or _RECUR_WS[key].numel() < floats:
+        _RECUR_WS[key] = torch.empty(0, device=device)
+        _RECUR_WS[key] = torch.empty(floats, dtype=torch.float32, device=device)
+    return _RECUR_WS[key]
+
+
+def recur_chunk() -> int:
+    return native.load().exo_recur_chunk()
+
+
+class Recurrence:
+    """A recurrent mixer of one layer over a state pool.  ``core``: heads, key groups, key size, value size;
+    ``li``: index of the pool's layer; ``consts``: members of ``native.Recurrence`` that hold for every
+    launch (tensors stand for their addresses)."""
+
+    def __init__(self, core: tuple[int, int, int, int], li: int, cache, dtype, consts: dict):
+        self.heads, self.groups, self.dim, self.vdim = core
+        self.cache, self.consts = cache, consts
+        st, ring = cache.states.state[li], cache.states.ring[li]
+        self.args = native.Recurrence(
+            heads=self.heads, groups=self.groups, dim=self.dim, vdim=self.vdim, state=st.data_ptr(), lds=st.shape[3],
+            map=cache.states.map.data_ptr(), ring=_p(ring), taps=0 if ring is None else ring.shape[1],
+            channels=0 if ring is None else ring.shape[2], dtype=0 if dtype == torch.bfloat16 else 1,
+            **{k: v.data_ptr() if isinstance(v, torch.Tensor) else v for k, v in consts.items()})
+
+    def bind(self, y, **inputs) -> None:
+        """Where a step's inputs and outputs lie: ``y`` float32 [rows, heads * vdim]; ``inputs``: members
+        by name, tensors with their row strides (``ld`` member of the same name)."""
+        a = self.args
+        a.y, a.ldy = y.data_ptr(), y.stride(0)
+        for name, (t, ld) in inputs.items():
+            setattr(a, name, t.data_ptr())
+            setattr(a, ld, t.stride(0))
+
+    def step(self, slot, pos, n: int, lst=None) -> None:
+        """Single tokens: row i (``lst``: which rows, else the first n) is of cache row slot[i] at pos[i]."""
+        a = self.args
+        a.slot, a.pos, a.list, a.n = slot.data_ptr(), pos.data_ptr(), _p(lst), n
+        check(native.load().exo_recur_step(C.byref(a), _stream()), "recur_step")
+
+    def chunks(self, chunks, n_chunks: int, seqs, n_seqs: int, cum, dt) -> None:
+        """Portions of prompts (lists as the C ABI describes them).  ``cum``, ``dt``: scratch rows."""
+        a, lib = self.args, native.load()
+        ns = lib.exo_recur_state_floats(n_chunks, self.heads, self.dim, a.lds)
+        ws = recur_workspace(ns + lib.exo_recur_scores_floats(n_chunks, self.groups), chunks.device)
+        a.chunk_state, a.scores = ws.data_ptr(), ws.data_ptr() + 4 * ns
+        a.cum, a.ldcum, a.dt = cum.data_ptr(), cum.stride(0), _p(dt)
+        a.chunks, a.n_chunks, a.seqs, a.n_seqs = chunks.data_ptr(), n_chunks, seqs.data_ptr(), n_seqs
+        check(lib.exo_recur_chunks(C.byref(a), _stream()), "recur_chunks")
+
+
+def gated_norm(y, gate, gain, out, n: int, width: int, groups: int, eps: float, gate_first: bool) -> None:
+    """out[:n] = RMS norm of ``groups`` equal parts of y (gain repeating with its own length), with silu(gate)
+    ahead of the norm or behind it."""
+    a = native.GatedNorm(y=y.data_ptr(), gate=gate.data_ptr(), gain=gain.data_ptr(), out=out.data_ptr(), width=width,
+                         groups=groups, period=gain.numel(), ldy=y.stride(0), ldg=gate.stride(0), ldo=out.stride(0),
+                         gate_first=int(gate_first), dtype=_code(out), eps=eps)
+    check(native.load().exo_gated_norm_rows(C.byref(a), None, n, _stream()), "gated_norm")

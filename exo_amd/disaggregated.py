@@ -307,6 +307,8 @@ def send_kv_cache(stream: BinaryIO, cache: ShardKVCache, *, row: int = 0, dtype:
     cross PCIe."""
     if dtype != "bfloat16":
         raise ValueError("this engine's KV cache is bfloat16")
+    if not cache.trimmable:
+        raise ValueError("the wire carries keys and values, no recurrent states")
     offset = cache.offsets[row]
     if max_tokens is not None:
         offset = min(offset, max_tokens)
@@ -430,6 +432,8 @@ def ingest_into_cache(result: PrefillResult, cache: ShardKVCache, *, row: int = 
                       start_pos: int = 0) -> int:
     """Write the received chunks into pool row ``row`` behind its first ``start_pos``
     positions and set the fill level (client.py:112-154).  Returns the final offset."""
+    if not cache.trimmable:
+        raise ValueError("the wire carries keys and values, no recurrent states")
     received = max((sum(c.num_tokens for c in chunks) for chunks in result.kv_chunks.values()),
                    default=0)
     final_offset = start_pos + received

@@ -251,7 +251,8 @@ class ShardBatchGenerator:
                     logger.warning("failed to save prefix cache", exc_info=True)
 
         tps = 0.0
-        remote = len(remaining) > REMOTE_PREFILL_MIN_TOKENS and task_params.prefill_endpoint is not None
+        remote = (len(remaining) > REMOTE_PREFILL_MIN_TOKENS and task_params.prefill_endpoint is not None
+                  and self.cache.trimmable)  # (the wire carries no recurrent states)
         here = not self.mixed or remote  # the prompt is in the cache when submit returns
         if here:
             try:
@@ -759,6 +760,8 @@ class BatchGenerator(Engine):
             raise ValueError(f"prefill request of {n} tokens exceeds the cache ({self.max_seq})")
         if self._prefill_cache is None:
             self._prefill_cache = self.model.make_cache(1, self.max_seq)
+        if not self._prefill_cache.trimmable:
+            raise ValueError("a model with recurrent states cannot serve prefills: the wire carries keys and values only")
         cache = run_prefill_for_request(model=self.model, kv_prefix_cache=self.kv_prefix_cache,
                                         request=request, cache=self._prefill_cache, row=0)
         write_cache_to_wire(wfile, cache, row=0, request_id=request.request_id,

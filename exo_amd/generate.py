@@ -177,7 +177,8 @@ def prefill(model: DecoderShard, prompt_tokens, cache: ShardKVCache,
     n-1 tokens; token n-1 is then run as a single-token forward whose sample is
     discarded, the generator it came from had already computed one more single-token
     forward, and ``trim(2)`` removes both entries.  ``faithful_extra_steps=False``
-    skips those two forwards (same cache contents, less work).  ``graph_steps``: run them as
+    skips those two forwards (same cache contents, less work); so does a cache that cannot be
+    trimmed (recurrent states).  ``graph_steps``: run them as
     replays of the captured single-token step of this cache row instead of launch by launch
     (same kernels; worth it for a cache that serves many requests).
     Returns (tokens_per_sec, n)."""
@@ -194,7 +195,7 @@ def prefill(model: DecoderShard, prompt_tokens, cache: ShardKVCache,
         done += m
         if on_prefill_progress is not None:
             on_prefill_progress(done, n)
-    if faithful_extra_steps:
+    if faithful_extra_steps and cache.trimmable:
         if graph_steps and model.is_first and model.is_last:
             # the same two single-token forwards as graph replays (a cache that outlives the
             # call keeps its captured step per row): the second consumes the first's argmax

@@ -218,8 +218,9 @@ class DecoderShard:
                 # warm up outside capture (lazy module loads, attribute settings), then
                 # restore what the warm-up changed: the positions it advanced, the hidden
                 # state a later shard adds its residuals into in place, the input tokens
-                # the feedback overwrote, the sampler's counters and history ring
+                # the feedback overwrote, the sampler's counters and history ring, recurrent states
                 saved = cache.pos.clone()
+                saved_states = cache.save_states(range(row0, row0 + B))
                 saved_in = bf.tokens.clone() if self.is_first else bf.h.clone()
                 saved_sampler = sampler.snapshot() if sampler is not None else None
                 s = torch.cuda.Stream()
@@ -229,6 +230,7 @@ class DecoderShard:
                 torch.cuda.current_stream().wait_stream(s)
                 torch.cuda.synchronize()
                 cache.pos.copy_(saved)
+                cache.load_states(range(row0, row0 + B), saved_states)
                 (bf.tokens if self.is_first else bf.h).copy_(saved_in)
                 if sampler is not None:
                     sampler.restore(saved_sampler)

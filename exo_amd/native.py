@@ -27,14 +27,48 @@ class MoeRows(C.Structure):
                [(n, _f) for n in ("router_scale", "limit", "alpha", "shift", "shared_limit", "shared_alpha", "shared_shift")]
 
 
+class Linear(C.Structure):
+    """struct exo_linear: a product (or gated pair) with an unquantised matrix."""
+
+    _fields_ = [(n, _vp) for n in ("x", "w", "w_up", "bias", "y", "y2")] + \
+               [(n, _i) for n in ("M", "N", "n1", "ldx", "ldw", "ldy", "ldy2", "y_f32", "dtype")] + \
+               [(n, _f) for n in ("limit", "alpha", "shift")]
+
+
+class PostNorm(C.Structure):
+    """struct exo_post_norm: a sublayer's output on its way into the residual."""
+
+    _fields_ = [(n, _vp) for n in ("x", "branch", "branch2", "gain_a", "gain_b", "gain", "pre", "x_out", "operand")] + \
+               [("H", _i), ("eps", _f), ("mult", _f)]
+
+
 class PagedAttn(C.Structure):
     """struct exo_paged_attn: one attention layer over a paged pool."""
 
-    _fields_ = [(n, _vp) for n in ("qkv", "k_pool", "v_pool", "table", "slot", "pos", "list", "slopes", "out")] + \
+    _fields_ = [(n, _vp) for n in ("qkv", "k_pool", "v_pool", "table", "slot", "pos", "list", "slopes", "q_gain", "k_gain",
+                                   "gate", "out")] + \
                [("scale", _f), ("eps", _f)] + \
-               [(n, _i) for n in ("n", "heads", "kv_heads", "dim", "vdim", "ldq", "ldk", "ldv", "ldo", "max_pages",
+               [(n, _i) for n in ("n", "heads", "kv_heads", "dim", "vdim", "ldq", "ldk", "ldv", "ldo", "ldg", "max_pages",
                                   "window", "keep_first", "unit_qk", "dtype")]
 
+
+class Recurrence(C.Structure):
+    """struct exo_recurrence: one recurrent mixer."""
+
+    _fields_ = [(n, _vp) for n in (
+        "q", "k", "v", "low", "decay_w", "decay_b", "dt_raw", "dt_bias", "decay_rate", "skip", "raw", "conv_w", "conv_b",
+        "ring", "act", "cum", "dt", "scores", "chunk_state", "state", "y", "map", "slot", "pos", "list", "chunks", "seqs")] + \
+        [(n, _i) for n in (
+            "ldq", "ldk", "ldv", "ldlow", "rank", "lddt", "ldraw", "channels", "taps", "ldact", "ldcum", "lds", "ldy",
+            "q_channel", "k_channel", "v_channel", "heads", "groups", "dim", "vdim", "per_channel", "n", "n_chunks",
+            "n_seqs", "qk_vec", "v_vec", "dtype")] + [("q_scale", _f), ("inv_tau", _f)]
+
+
+class GatedNorm(C.Structure):
+    """struct exo_gated_norm: RMS norm of parts of a row with a silu gate."""
+
+    _fields_ = [(n, _vp) for n in ("y", "gate", "gain", "out")] + \
+               [(n, _i) for n in ("width", "groups", "period", "ldy", "ldg", "ldo", "gate_first", "dtype")] + [("eps", _f)]
 
 
 # name -> (restype, argtypes); mirrors include/exo_mi355x.h one to one
@@ -87,14 +121,13 @@ SIGNATURES: dict[str, tuple] = {
     "exo_argmax_logsumexp": (_i, [_vp] * 6 + [_i, _i, _vp]),
     "exo_embed_rows": (_i, [_vp] * 4 + [_i] * 6 + [_vp]),
     "exo_norm_rows": (_i, [_vp] * 4 + [_i] * 3 + [_f, _i, _vp]),
-    "exo_post_norm_add": (_i, [_vp, _i] + [_vp] * 3 + [_i] * 3 + [_f, _i, _vp]),
-    "exo_moe_sum_post_norm": (_i, [_vp] * 5 + [_i] * 6 + [_vp] * 3 + [_i] * 3 + [_f, _i, _vp]),
+    "exo_post_norm_add": (_i, [C.POINTER(PostNorm), _i, _i, _i, _i, _vp]),
+    "exo_moe_sum_post_norm": (_i, [_vp] * 5 + [_i] * 6 + [C.POINTER(PostNorm), _i, _i, _i, _vp]),
     "exo_moe_route": (_i, [_vp] * 4 + [_i] * 4 + [_f, _vp]),
-    "exo_dense_gemv": (_i, [_vp] * 4 + [_i] * 7 + [_vp]),
-    "exo_post_gemv_fits": (_i, [_i] * 5),
-    "exo_post_gemv": (_i, [_vp, _vp, _vp, _f] + [_vp] * 5 + [_i] * 8 + [_vp]),
-    "exo_dense_gemm": (_i, [_vp] * 4 + [_i, _vp, _i64] + [_i] * 6 + [_vp]),
-    "exo_dense_glu_gemm": (_i, [_vp] * 4 + [_f] * 3 + [_i] * 6 + [_vp]),
+    "exo_linear_rows": (_i, [C.POINTER(Linear), C.POINTER(Linear), _vp]),
+    "exo_linear_gemm": (_i, [C.POINTER(Linear), _vp, _i64, _vp]),
+    "exo_post_linear_fits": (_i, [_i] * 5),
+    "exo_post_linear": (_i, [C.POINTER(PostNorm), C.POINTER(Linear), _vp]),
     "exo_dense_grouped_gemm": (_i, [_vp] * 5 + [_f] * 3 + [_i] * 9 + [_vp]),
     "exo_moe_glu_rows": (_i, [C.POINTER(MoeRows), _vp]),
     "exo_moe_down_rows": (_i, [C.POINTER(MoeRows), _vp]),
@@ -103,6 +136,12 @@ SIGNATURES: dict[str, tuple] = {
     "exo_paged_attn_rows": (_i, [C.POINTER(PagedAttn), _i, _i, _vp, _i64, _vp]),
     "exo_paged_prompt_block": (_i, [_i, _i]),
     "exo_paged_attn_prompt": (_i, [C.POINTER(PagedAttn), _vp]),
+    "exo_recur_chunk": (_i, []),
+    "exo_recur_scores_floats": (_i64, [_i] * 2),
+    "exo_recur_state_floats": (_i64, [_i] * 4),
+    "exo_recur_chunks": (_i, [C.POINTER(Recurrence), _vp]),
+    "exo_recur_step": (_i, [C.POINTER(Recurrence), _vp]),
+    "exo_gated_norm_rows": (_i, [C.POINTER(GatedNorm), _vp, _i, _vp]),
     "exo_sample_workspace": (_i64, [_i]),
     "exo_sample": (_i, [_vp] * 13 + [_i64, _i, _i, _i, _i, _vp]),
 }

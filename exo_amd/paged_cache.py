@@ -3,7 +3,8 @@
 The cache protocol of ``ShardKVCache`` (rows, ``offsets``, ``pos``, trim / reset / copy_row) over a
 pool whose size is given in tokens, not rows x longest sequence: a row owns the pages its tokens
 need, through a page table on the device, and gives them back when it is trimmed, reset or
-released.  One table serves every layer.
+released.  One table serves every layer.  Recurrent layers keep their fixed-size states in slots beside
+the pages (``state_pool``); a row then cannot be cut back to an earlier position, only to none.
 
 Per layer with keys of its own (layers that use another layer's keys have no storage):
   k[i]  [pages, G, 64, ldk]   keys as attention uses them (normalised)
@@ -16,6 +17,7 @@ from __future__ import annotations
 import torch
 
 from .cache import LayerKV
+from .state_pool import StatePool, StateShape
 
 PAGE = 64
 
@@ -29,14 +31,14 @@ def pages_for(tokens: int) -> int:
 
 
 class PagedKVCache(list):
-    """list[LayerKV] (one per layer with keys of its own) plus the pool."""
+    """list[LayerKV] (one per layer with keys of its own and per recurrent state) plus the pools."""
 
     def __init__(self, layers: list[tuple[int, int, int]], rows: int, max_seq: int, device, dtype=torch.bfloat16,
-                 pool_tokens: int | None = None):
+                 pool_tokens: int | None = None, states: list[StateShape] = ()):
         """``layers``: (kv heads, key size, value size) per storing layer.  ``max_seq``: the longest
         sequence a row may hold; ``pool_tokens``: tokens all rows hold together, each row's count
-        rounded up to whole pages (default: every row at ``max_seq``)."""
-        super().__init__(LayerKV(self, i) for i in range(len(layers)))
+        rounded up to whole pages (default: every row at ``max_seq``); ``states``: the recurrent layers'."""
+        super().__init__(LayerKV(self, i) for i in range(len(layers) + len(states)))
         self.batch, self.max_seq, self.shapes = rows, max_seq, list(layers)
         self.n_pages = rows * pages_for(max_seq) if pool_tokens is None else pages_for(pool_tokens)
         self.max_pages = min(pages_for(max_seq), self.n_pages)
@@ -44,12 +46,25 @@ class PagedKVCache(list):
         z = dict(dtype=dtype, device=device)
         self.k = [torch.zeros(self.n_pages, g, PAGE, pad(d), **z) for g, d, _ in layers]
         self.v = [torch.zeros(self.n_pages, g, pad(e), PAGE, **z) for g, _, e in layers]
+        self.states = StatePool(states, rows, device, dtype)
         self.table = torch.zeros(rows, self.max_pages, dtype=torch.int32, device=device)
         self.pos = torch.zeros(rows, dtype=torch.int32, device=device)
         self.offsets = [0] * rows
         self.pages: list[list[int]] = [[] for _ in range(rows)]
         self._free = list(range(self.n_pages - 1, -1, -1))
         self._last_trim = 0
+
+    # -- recurrent states
+    @property
+    def trimmable(self) -> bool:
+        """Whether a row can go back to an earlier position (a recurrent state cannot)."""
+        return not len(self.states)
+
+    def save_states(self, rows) -> list[torch.Tensor]:
+        return self.states.read(rows)
+
+    def load_states(self, rows, saved: list[torch.Tensor]) -> None:
+        self.states.write(rows, saved)
 
     # -- pages
     @property
@@ -92,6 +107,8 @@ class PagedKVCache(list):
     def trim(self, n: int, rows=None) -> int:
         rows = range(self.batch) if rows is None else rows
         n = min([n] + [self.offsets[r] for r in rows])
+        if n and not self.trimmable and any(self.offsets[r] != n for r in rows):
+            raise ValueError("a recurrent state cannot be cut back to an earlier position")
         for r in rows:
             self.offsets[r] -= n
             self._give_back(r, self.offsets[r])
@@ -109,11 +126,13 @@ class PagedKVCache(list):
         self.reset(rows=[row])
 
     def copy_row(self, src: int, dst: int) -> None:
-        """Move one sequence to another row (slot compaction): the pages change hands, no key moves."""
+        """Move one sequence to another row (slot compaction): pages and state slot change hands,
+        no key or state moves."""
         self._give_back(dst, 0)
         self.pages[dst], self.pages[src] = self.pages[src], []
         self.table[dst].copy_(self.table[src])
         self.offsets[dst], self.offsets[src] = self.offsets[src], 0
+        self.states.swap(src, dst)
         self.sync_pos()
 
     def swap_rows(self, a: int, b: int) -> None:
@@ -122,10 +141,11 @@ class PagedKVCache(list):
         self.pages[a], self.pages[b] = self.pages[b], self.pages[a]
         self.offsets[a], self.offsets[b] = self.offsets[b], self.offsets[a]
         self.table[[a, b]] = self.table[[b, a]]
+        self.states.swap(a, b)
         self.sync_pos()
 
     def nbytes(self) -> int:
-        return sum(t.numel() * t.element_size() for t in self.k + self.v)
+        return sum(t.numel() * t.element_size() for t in self.k + self.v) + self.states.nbytes()
 
     # -- one row's contents as [n, G, size] tensors (prefix cache, wire)
     def _row_pages(self, row: int, lo: int, hi: int) -> torch.Tensor:
@@ -152,13 +172,17 @@ class PagedKVCache(list):
         self.v[layer][page, :, :e, at % PAGE] = v.to(self.v[layer].dtype)
 
     def snapshot(self, row: int) -> list[tuple[torch.Tensor, torch.Tensor]]:
-        """Detached copy of the row's positions, per layer (keys, values)."""
-        return [self.read_nhd(i, row, 0, self.offsets[row]) for i in range(len(self.k))]
+        """Detached copy of the row's positions, per layer (keys, values), then the recurrent
+        states (one entry of all of them, if there are any)."""
+        kv = [self.read_nhd(i, row, 0, self.offsets[row]) for i in range(len(self.k))]
+        return kv + ([tuple(self.states.read([row]))] if len(self.states) else [])
 
     def restore(self, row: int, layers: list[tuple[torch.Tensor, torch.Tensor]], length: int) -> None:
         self.reset(rows=[row])
         self.reserve([row], length)
-        for i, (k, v) in enumerate(layers):
+        if len(self.states):
+            self.states.write([row], list(layers[-1]))
+        for i, (k, v) in enumerate(layers[: len(self.k)]):
             self.write_nhd(i, row, 0, k[:length], v[:length])
         self.offsets[row] = length
         self.sync_pos()

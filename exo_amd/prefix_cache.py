@@ -99,8 +99,10 @@ def restore_row(stored: StoredKV, cache: ShardKVCache | PagedKVCache, row: int, 
         raise ValueError(f"restore of {length} positions from an entry of {stored.length}")
     if length > cache.max_seq:
         raise ValueError(f"restore of {length} positions into a cache of {cache.max_seq}")
-    if len(stored.layers) != len(cache.k):
+    if len(stored.layers) != len(cache.k) + (not cache.trimmable):
         raise ValueError("stored entry and cache differ in layer count")
+    if length != stored.length and not cache.trimmable:
+        raise ValueError(f"restore of {length} positions from a recurrent state after {stored.length}")
     cache.restore(row, stored.layers, length)
 
 
@@ -162,6 +164,8 @@ class KVPrefixCache:
         is_exact = False
         for i, cached_prompt in enumerate(self.prompts):
             length = get_prefix_length(toks, cached_prompt)
+            if not cache.trimmable and self.caches[i].length > min(length, max_length - 1):
+                continue  # a recurrent state serves only prompts that go on from where it stands
             if length >= max_length - 1 and length > 0:
                 best_index, best_length, is_exact = i, length, True
                 break

@@ -25,14 +25,83 @@ class AttentionSpec:
     window: int | None = None    # keys seen: fewer than this many positions back (None: all)
     keep_first: int = 0          # ... and the sequence's first positions, however far
     unit_qk: bool = False        # queries and keys divided by their RMS, per head
+    qk_gain: bool = False        # ... and multiplied by a gain per channel
+    head_gate: bool = False      # a head's output times sigmoid of a number of its own
     slopes: tuple[float, ...] | None = None  # per query head: score lowered by slope * distance
     bias: bool = False           # projections have biases
     kv_from: int | None = None   # keys and values of that layer instead of own ones
 
 
 @dataclass(frozen=True)
-class ExpertSpec:
-    """g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + shift)."""
+class LinearAttentionSpec:
+    """Recurrence S <- diag(a) S + k v^T per head with a decay per key channel, a = sigmoid(z)^(1/tau), z from
+    a low-rank product; the output RMS-normed per head, times silu of a gate."""
+
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+
+    @property
+    def core(self) -> tuple[int, int, int, int]:
+        """Heads, key groups, key size, value size of the recurrence."""
+        return self.heads, self.heads, self.dim, self.vdim
+
+
+@dataclass(frozen=True)
+class StateSpaceSpec:
+    """Recurrence S <- a S + dt k v^T per head with one decay per head and step, keys and queries shared by a
+    group of heads, a causal convolution in front and a skip; the output times silu of a gate, then
+    RMS-normed in ``norm_groups`` equal parts."""
+
+    heads: int
+    groups: int
+    state: int                   # key size
+    vdim: int
+    conv: int                    # taps
+    norm_groups: int
+
+    @property
+    def core(self) -> tuple[int, int, int, int]:
+        return self.heads, self.groups, self.state, self.vdim
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def channels(self) -> int:
+        """Convolved channels: values, keys, queries."""
+        return self.inner + 2 * self.groups * self.state
+
+
+@dataclass(frozen=True)
+class ParallelSpec:
+    """Two mixers over the same input, half the sum of their outputs, each RMS-normed first."""
+
+    left: AttentionSpec
+    right: StateSpaceSpec
+
+
+MixerSpec = AttentionSpec | LinearAttentionSpec | StateSpaceSpec | ParallelSpec
+
+
+def attention_of(m: MixerSpec) -> AttentionSpec | None:
+    """The part of a mixer that keeps keys and values."""
+    m = m.left if isinstance(m, ParallelSpec) else m
+    return m if isinstance(m, AttentionSpec) else None
+
+
+def recurrence_of(m: MixerSpec) -> LinearAttentionSpec | StateSpaceSpec | None:
+    """The part of a mixer that keeps a recurrent state."""
+    m = m.right if isinstance(m, ParallelSpec) else m
+    return m if isinstance(m, (LinearAttentionSpec, StateSpaceSpec)) else None
+
+
+@dataclass(frozen=True)
+class GluSpec:
+    """g = min(gate, limit), u = clamp(up, +-limit): g sigmoid(alpha g) (u + shift).  By itself a dense
+    feed-forward, and what an expert is."""
 
     ff: int
     limit: float
@@ -58,14 +127,28 @@ class RouterSpec:
 @dataclass(frozen=True)
 class MoeSpec:
     router: RouterSpec
-    expert: ExpertSpec
-    shared: ExpertSpec | None = None  # for every token, times sigmoid of one number per token
+    expert: GluSpec
+    shared: GluSpec | None = None  # for every token, times sigmoid of one number per token
 
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: AttentionSpec
-    mlp: MoeSpec | None
+    mixer: MixerSpec
+    mlp: MoeSpec | GluSpec | None
+
+
+@dataclass(frozen=True)
+class NormSpec:
+    """Where a layer's norms sit and what their stored weights mean."""
+
+    eps: float
+    pre: bool = False            # also on a sublayer's input (else only on its output)
+    offset: float = 0.0          # gain = stored weight + offset
+    mult: float = 1.0            # of a normed sublayer output in the residual sum
+
+    def names(self, sublayer: int) -> tuple[str | None, str]:
+        """Tensor names of the norms ahead of (None: none) and behind sublayer 1 or 2."""
+        return (f"norm{sublayer}", f"norm{sublayer}b") if self.pre else (None, f"norm{sublayer}")
 
 
 @dataclass
@@ -73,7 +156,7 @@ class StackConfig:
     architecture: str
     vocab_size: int
     hidden_size: int
-    eps: float
+    norm: NormSpec
     layers: tuple[LayerSpec, ...]
     raw: dict                    # config.json as read
 
@@ -81,19 +164,35 @@ class StackConfig:
         if min(self.vocab_size, self.hidden_size, len(self.layers)) <= 0:
             raise ValueError(f"{self.architecture}: vocab, width and the layer list must not be empty")
         for i, L in enumerate(self.layers):
-            m, f = L.mixer, L.mlp
+            m, f, r = attention_of(L.mixer), L.mlp, recurrence_of(L.mixer)
+            if r is not None:
+                h, g, d, e = r.core
+                if min(h, g, d, e) <= 0 or h % g:
+                    raise ValueError(f"layer {i}: {h} recurrent heads over {g} groups, sizes {d} and {e}")
+                if isinstance(r, StateSpaceSpec) and (r.conv <= 0 or r.norm_groups <= 0 or r.inner % r.norm_groups):
+                    raise ValueError(f"layer {i}: {r.conv} taps, {r.inner} channels in {r.norm_groups} norm groups")
+                if isinstance(r, LinearAttentionSpec) and not r.tau > 0:
+                    raise ValueError(f"layer {i}: tau {r.tau}")
+            if isinstance(f, MoeSpec) and self.norm.pre and f.router.identity:
+                raise ValueError(f"layer {i}: identity experts behind a norm of the input are not supported")
+            if isinstance(f, MoeSpec) and not 0 < f.router.top <= f.router.outputs:
+                raise ValueError(f"layer {i}: top {f.router.top} of {f.router.outputs} experts")
+            if m is None:
+                continue
             if min(m.heads, m.kv_heads, m.dim, m.vdim) <= 0 or m.heads % m.kv_heads:
                 raise ValueError(f"layer {i}: {m.heads} query heads over {m.kv_heads} key/value heads")
             if (m.window is not None and m.window <= 0) or m.keep_first < 0:
                 raise ValueError(f"layer {i}: window {m.window} with {m.keep_first} kept positions")
             if m.kv_from is not None:
-                src = self.layers[m.kv_from].mixer if 0 <= m.kv_from < i else None
+                src = attention_of(self.layers[m.kv_from].mixer) if 0 <= m.kv_from < i else None
                 if src is None or src.kv_from is not None:
                     raise ValueError(f"layer {i}: kv_from {m.kv_from} is no earlier layer with keys of its own")
                 if (src.kv_heads, src.dim, src.vdim) != (m.kv_heads, m.dim, m.vdim):
                     raise ValueError(f"layer {i}: head sizes differ from those of layer {m.kv_from}")
-            if f is not None and not 0 < f.router.top <= f.router.outputs:
-                raise ValueError(f"layer {i}: top {f.router.top} of {f.router.outputs} experts")
+
+    @property
+    def eps(self) -> float:
+        return self.norm.eps
 
     # -- what the engine asks of any configuration
     @property
@@ -149,8 +248,8 @@ def _gekazen(d: dict) -> StackConfig:
     clamped gated experts with a choice correction, identity experts and a gated shared expert;
     norms on the sublayers' outputs."""
 
-    def expert(e: dict) -> ExpertSpec:
-        return ExpertSpec(ff=int(e["ff"]), limit=float(e["limit"]))
+    def expert(e: dict) -> GluSpec:
+        return GluSpec(ff=int(e["ff"]), limit=float(e["limit"]))
 
     layers = []
     for i, L in enumerate(d["layers"]):
@@ -173,11 +272,42 @@ def _gekazen(d: dict) -> StackConfig:
                 RouterSpec(int(r["experts"]), int(r.get("identity") or 0), int(r["top"]), float(r["scale"])),
                 expert(f["expert"]), expert(f["shared"]) if f.get("shared") else None)
         layers.append(LayerSpec(mixer, mlp))
-    return StackConfig("Gekazen", int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]), tuple(layers),
-                       copy.deepcopy(d))
+    return StackConfig("Gekazen", int(d["vocab"]), int(d["width"]), NormSpec(float(d["norm"]["eps"]), offset=1.0),
+                       tuple(layers), copy.deepcopy(d))
 
 
-READERS = {"Gekazen": _gekazen}
+def _novosun(d: dict) -> StackConfig:
+    """Novosun: layers of gated linear attention, or of softmax attention (normed queries and keys, a gate
+    per head, no positions) side by side with a state-space recurrence; dense clamped gated
+    feed-forwards; norms on the sublayers' inputs and outputs, a constant on each sum."""
+
+    def linear(m: dict) -> LinearAttentionSpec:
+        return LinearAttentionSpec(int(m["heads"]), int(m["dim"]), int(m["vdim"]), float(m["tau"]))
+
+    def parallel(m: dict) -> ParallelSpec:
+        a, s = m["left"], m["right"]
+        return ParallelSpec(
+            AttentionSpec(heads=int(a["heads"]), kv_heads=int(a["kv_heads"]), dim=int(a["dim"]), vdim=int(a["vdim"]),
+                          scale=float(a["scale"]), unit_qk=True, qk_gain=True, head_gate=True),
+            StateSpaceSpec(heads=int(s["heads"]), groups=int(s["groups"]), state=int(s["state"]), vdim=int(s["vdim"]),
+                           conv=int(s["conv"]), norm_groups=int(s["norm_groups"])))
+
+    mixers = {"gla": linear, "parallel": parallel}
+    layers = []
+    for i, L in enumerate(d["layers"]):
+        if L["type"] not in mixers:
+            raise ValueError(f"layer {i}: mixer type {L['type']!r} not supported (have {tuple(mixers)})")
+        f, mlp = L.get("mlp"), None
+        if f is not None:
+            if f.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: feed-forward kind {f['kind']!r} not supported (have 'dense')")
+            mlp = GluSpec(ff=int(f["ff"]), limit=float(f["limit"]))
+        layers.append(LayerSpec(mixers[L["type"]](L["mixer"]), mlp))
+    norm = NormSpec(float(d["norm"]["eps"]), pre=True, mult=float(d["residual_mult"]))
+    return StackConfig("Novosun", int(d["vocab"]), int(d["width"]), norm, tuple(layers), copy.deepcopy(d))
+
+
+READERS = {"Gekazen": _gekazen, "Novosun": _novosun}
 
 
 def gekazen_dict(width: int, vocab: int, layers: int, *, heads: int, kv_heads: int, dim: int, vdim: int, experts: int,
@@ -198,3 +328,18 @@ def gekazen_dict(width: int, vocab: int, layers: int, *, heads: int, kv_heads: i
             mlp["shared"] = dict(ff=shared_ff, limit=limit)
         out.append(dict(type="attention", mixer=mixer, mlp=mlp))
     return dict(architecture="Gekazen", vocab=vocab, width=width, norm=dict(eps=eps), layers=out)
+
+
+def novosun_dict(width: int, vocab: int, kinds: str, *, heads: int, kv_heads: int, dim: int, vdim: int, ff: int | None,
+                 lin_heads: int, lin_dim: int, lin_vdim: int, ssm_heads: int, ssm_vdim: int, ssm_state: int,
+                 ssm_groups: int = 1, conv: int = 4, norm_groups: int = 1, tau: float = 16.0, limit: float = 7.0,
+                 mult: float = 1.0, eps: float = 1e-6) -> dict:
+    """A ``config.json`` of the design (benchmarks); ``kinds``: a letter per layer, g for linear attention, p
+    for the parallel mixer."""
+    linear = dict(type="gla", mixer=dict(heads=lin_heads, dim=lin_dim, vdim=lin_vdim, tau=tau))
+    parallel = dict(type="parallel", mixer=dict(
+        left=dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5),
+        right=dict(heads=ssm_heads, groups=ssm_groups, state=ssm_state, vdim=ssm_vdim, conv=conv, norm_groups=norm_groups)))
+    mlp = None if ff is None else dict(kind="dense", ff=ff, limit=limit)
+    layers = [dict(copy.deepcopy(linear if k == "g" else parallel), mlp=copy.deepcopy(mlp)) for k in kinds]
+    return dict(architecture="Novosun", vocab=vocab, width=width, norm=dict(eps=eps), residual_mult=mult, layers=layers)

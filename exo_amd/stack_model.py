@@ -6,19 +6,21 @@ one batch - runs them together and returns logits at the places asked for.  ``__
 ``decode_step`` (the graph-captured single-token step) are the protocol of ``ShardModel`` on top of
 the same launches, so the engines, ``prefill`` and ``generate`` drive either model class.
 
-Precision: the residual stream, norms, routing and attention weights are float32; matrix operands
-and the cache have the model's element type - bf16 as served, or float32 throughout
-(``dtype=torch.float32``).
+Precision: the residual stream, norms, routing, attention weights, decays, step sizes and recurrent
+states are float32; matrix operands and the cache have the model's element type - bf16 as served, or
+float32 throughout (``dtype=torch.float32``).
 
 Launches of a layer (rows R of the step):
-  R <= 16   q|k|v GEMV, attention (with norm and cache append inside when every row is a single
-            token), o GEMV, router GEMV, gated experts + shared expert in one launch that also
-            routes, weighted down-projections in one launch.  The norm of a sublayer's output and
-            its residual sum run inside the next product that reads the residual (up to 4 rows) or
-            as a launch of their own
+  R <= 16   the projection of all the mixer's parts as one GEMV; per part: attention (with norm and
+            cache append inside when every row is a single token) or the recurrence's step and gated
+            norm; the output projections of all parts as one GEMV; a dense feed-forward as a gated
+            pair and a down GEMV, or router GEMV, gated experts + shared expert in one launch that
+            also routes, weighted down-projections in one launch.  The norms of a sublayer's output,
+            its residual sum and the norm of the next input run inside the next product (up to 4 rows)
+            or as a launch of their own
   R > 16    the same with GEMMs, the experts grouped by expert, their weighted sum inside the
-            norm + residual launch; portions of prompts take the tiled attention, single tokens
-            beside them the split one
+            norm + residual launch; portions of prompts take the tiled attention and the chunked
+            recurrence, single tokens beside them the split attention and the step
 """
 
 from __future__ import annotations
@@ -31,64 +33,8 @@ from . import ops
 from .dense_ops import pad64, padded
 from .model import DecoderShard
 from .paged_cache import PagedKVCache
-from .stack_config import AttentionSpec, LayerSpec, StackConfig
-
-
-class _Layer:
-    """One layer's tensors on the device: projections concatenated, experts stacked, rows padded."""
-
-    def __init__(self, spec: LayerSpec, w: dict, i: int, H: int, dtype, device):
-        self.index, self.spec = i, spec
-        p, m, f = f"l{i}.", spec.mixer, spec.mlp
-
-        def get(name: str, *shape: int) -> torch.Tensor:
-            t = w[p + name]
-            if tuple(t.shape) != shape:
-                raise ValueError(f"{p}{name}: shape {tuple(t.shape)}, config says {shape}")
-            return t.to(device)
-
-        def mat(*parts) -> torch.Tensor:
-            return padded(torch.cat([get(*x) for x in parts]), dtype, device)
-
-        def gain(name: str) -> torch.Tensor:
-            return (1.0 + get(name, H).float()).contiguous()
-
-        outs = [("q", m.heads * m.dim)]
-        if m.kv_from is None:
-            outs += [("k", m.kv_heads * m.dim), ("v", m.kv_heads * m.vdim)]
-        self.qkv = mat(*((f"mix.{n}", rows, H) for n, rows in outs))
-        self.o = mat(("mix.o", H, m.heads * m.vdim))
-        self.qkv_b = self.o_b = None
-        if m.bias:
-            self.qkv_b = torch.cat([get(f"mix.{n}.b", rows) for n, rows in outs]).float().contiguous()
-            self.o_b = get("mix.o.b", H).float().contiguous()
-        self.slopes = None if m.slopes is None else torch.tensor(m.slopes, dtype=torch.float32, device=device)
-        self.norm1 = gain("norm1")
-        self.norm2 = self.router = None
-        if f is None:
-            return
-        self.norm2 = gain("norm2")
-        r, ff = f.router, f.expert.ff
-
-        def stack(name: str, n: int, k: int) -> torch.Tensor:
-            out = torch.zeros(r.experts, n, pad64(k), dtype=dtype, device=device)
-            for e in range(r.experts):
-                out[e, :, :k].copy_(get(f"mlp.e{e}.{name}", n, k))
-            return out
-
-        self.gate, self.up, self.down = stack("gate", ff, H), stack("up", ff, H), stack("down", H, ff)
-        self.correction = get("mlp.correction", r.outputs).float().contiguous()
-        # the shared expert's gate is one more output of the router product
-        rows = [("mlp.router", r.outputs, H)]
-        self.s_gate = self.s_up = self.s_down = None
-        if f.shared is not None:
-            rows.append(("mlp.shared.sg", 1, H))
-            self.s_gate, self.s_up = mat(("mlp.shared.gate", f.shared.ff, H)), mat(("mlp.shared.up", f.shared.ff, H))
-            self.s_down = mat(("mlp.shared.down", H, f.shared.ff))
-        self.router = mat(*rows)
-
-    def tensors(self) -> list[torch.Tensor]:
-        return [t for t in vars(self).values() if isinstance(t, torch.Tensor)]
+from .stack_config import GluSpec, MoeSpec, StackConfig, StateSpaceSpec, attention_of, recurrence_of
+from .stack_layers import AttentionPart, Layer, pad8
 
 
 class _Buffers:
@@ -108,6 +54,7 @@ class _Buffers:
         self.xb = self._z(rows, pad64(H))                    # its copy as matrix operand
         self.xn = self._z(rows, pad64(H))                    # rows entering the head
         self.branch = self._z(rows, H, dtype=torch.float32)  # a sublayer's output
+        self.branch2 = self._z(rows, H, dtype=torch.float32) if model.two_branches else None
         self.experts: dict[tuple[int, int], D.ExpertRows] = {}
         # outputs of a single-token step (last shard)
         self.logits = self.logits16 = None
@@ -126,11 +73,15 @@ class _Buffers:
             self._named[key] = self._z(*shape, dtype=self.model.dtype if dtype is None else dtype)
         return self._named[key]
 
-    def qkv(self, n: int) -> torch.Tensor:
-        return self._get("qkv", self.cap, -(-n // 8) * 8)
+    def f32(self, name: str, n: int) -> torch.Tensor:
+        return self._get(name, self.cap, n, dtype=torch.float32)
 
-    def attn(self, n: int) -> torch.Tensor:
-        return self._get("attn", self.cap, pad64(n))
+    def cols(self, name: str, n: int) -> torch.Tensor:
+        return self._get(name, self.cap, n)
+
+    def mixed(self, name: str, n: int) -> torch.Tensor:
+        """Rows of n columns that enter a product."""
+        return self._get(name, self.cap, pad64(n))
 
     def router_logits(self, n: int) -> torch.Tensor:
         return self._get("router", self.cap, n, dtype=torch.float32)
@@ -155,14 +106,18 @@ class _Buffers:
 
 
 class _Batch:
-    """What attention needs to know about the rows of a step, on the device."""
+    """What the mixers need to know about the rows of a step, on the device."""
 
     def __init__(self, rows: int, slot, pos, keys: int, single=None, n_single: int | None = None, blocks=None,
-                 want=None, n_want: int | None = None):
+                 want=None, n_want: int | None = None, chunks=None, n_chunks: int = 0, seqs=None, n_seqs: int = 0,
+                 alone=None, n_alone: int = 0):
         self.rows, self.slot, self.pos, self.keys = rows, slot, pos, keys
         self.single, self.n_single = single, rows if n_single is None else n_single  # rows alone (None: all)
         self.blocks = blocks or {}                                                   # tokens -> (list, count)
         self.want, self.n_want = want, rows if n_want is None else n_want            # rows with logits
+        # recurrences: portions of several tokens, cut into chunks; rows that are a portion by themselves
+        self.chunks, self.n_chunks, self.seqs, self.n_seqs = chunks, n_chunks, seqs, n_seqs
+        self.alone, self.n_alone = alone, n_alone
 
     @property
     def decode(self) -> bool:
@@ -181,13 +136,23 @@ class StackModel(DecoderShard):
         if not (0 <= self.start_layer < self.end_layer <= cfg.num_hidden_layers):
             raise ValueError(f"bad layer range [{start_layer},{end_layer}) of {cfg.num_hidden_layers}")
         H = cfg.hidden_size
-        self.layers = [_Layer(cfg.layers[i], weights, i, H, dtype, self.device)
+        self.layers = [Layer(cfg.layers[i], weights, i, H, cfg.norm, dtype, self.device)
                        for i in range(self.start_layer, self.end_layer)]
-        # layer -> index of the pool's layer that holds its keys and values
+        self.two_branches = any(len(L.parts) > 1 for L in self.layers)
+        # layer -> index of the pool's layer that holds its keys and values, its recurrent state
         self.kv_index: dict[int, int] = {}
         self.kv_shapes: list[tuple[int, int, int]] = []
+        self.state_index: dict[int, int] = {}
+        self.state_shapes: list[tuple[int, int, int, int, int]] = []
         for L in self.layers:
-            m = L.spec.mixer
+            r = recurrence_of(L.spec.mixer)
+            if r is not None:
+                h, _, d, e = r.core
+                self.state_index[L.index] = len(self.state_shapes)
+                self.state_shapes.append((h, d, e, *((r.conv, r.channels) if isinstance(r, StateSpaceSpec) else (0, 0))))
+            m = attention_of(L.spec.mixer)
+            if m is None:
+                continue
             if m.kv_from is None:
                 self.kv_index[L.index] = len(self.kv_shapes)
                 self.kv_shapes.append((m.kv_heads, m.dim, m.vdim))
@@ -200,11 +165,11 @@ class StackModel(DecoderShard):
         if self.is_first:
             self.embed = padded(weights["embed"].to(self.device), dtype, self.device)
         if self.is_last:
-            self.norm = (1.0 + weights["final.norm"].to(self.device).float()).contiguous()
+            self.norm = (cfg.norm.offset + weights["final.norm"].to(self.device).float()).contiguous()
             self.head = padded(weights["head"].to(self.device), dtype, self.device)
         self._bufs: dict[tuple, _Buffers] = {}
         self._graphs: dict[tuple, tuple] = {}
-        self._attn: tuple | None = None  # (cache, per-layer argument blocks)
+        self._bound: tuple | None = None  # (cache, per layer and part the argument blocks)
         self._row_ids: dict[tuple[int, int], torch.Tensor] = {}
         self.layer_hook = None  # called with (layer index, residual rows) after every layer (eager steps)
 
@@ -216,7 +181,7 @@ class StackModel(DecoderShard):
         return sum(t.numel() * t.element_size() for t in ts)
 
     def make_cache(self, batch: int = 1, max_seq: int = 4096, pool_tokens: int | None = None) -> PagedKVCache:
-        return PagedKVCache(self.kv_shapes, batch, max_seq, self.device, self.dtype, pool_tokens)
+        return PagedKVCache(self.kv_shapes, batch, max_seq, self.device, self.dtype, pool_tokens, self.state_shapes)
 
     def _buffers(self, B: int, T: int) -> _Buffers:
         """Activations of B x T rows: single-token steps (T = 1) have a set per batch size - a
@@ -246,71 +211,82 @@ class StackModel(DecoderShard):
         bf.logits16.copy_(logits)
         return bf.logits16
 
-    def _attention(self, cache: PagedKVCache) -> list[D.PagedAttention]:
-        if self._attn is None or self._attn[0] is not cache:
-            self._attn = (cache, [D.PagedAttention(L.spec.mixer, L.slopes, self.kv_index[L.index], cache, self.cfg.eps)
-                                  for L in self.layers])
-        return self._attn[1]
+    def _mixers(self, cache: PagedKVCache) -> list[list]:
+        """Per layer, the bound operator of each part of its mixer."""
+        if self._bound is None or self._bound[0] is not cache:
+            self._bound = (cache, [[p.bind(cache, (self.kv_index if isinstance(p, AttentionPart) else self.state_index)[L.index],
+                                           self.dtype, self.cfg.eps) for p in L.parts] for L in self.layers])
+        return self._bound[1]
 
     # ------------------------------------------------------------------ the launches
-    def _settle(self, bf: _Buffers, n: int, gain: torch.Tensor | None) -> None:
-        """residual += norm(branch), if a sublayer's output is still outstanding (``gain``)"""
-        if gain is not None:
-            D.post_norm_add(bf.branch, gain, self.cfg.eps, bf.h, bf.xb, n)
+    def _settle(self, bf: _Buffers, n: int, due: D.Branches | None, pre: torch.Tensor | None) -> None:
+        """residual += normed sublayer output, if one is still outstanding (``due``); bf.xb <- the
+        residual, or its norm (``pre``)"""
+        if due is not None:
+            D.post_norm_add(due, self.cfg.eps, bf.h, bf.xb, n, pre)
+        elif pre is not None:
+            D.norm_rows(bf.h, pre, self.cfg.eps, bf.xb, n)
 
-    def _product(self, bf: _Buffers, n: int, gain: torch.Tensor | None, w, out, bias=None, keep_copy: bool = False) -> None:
-        """out <- residual @ w^T, after the outstanding norm and sum; ``keep_copy``: bf.xb is read
-        by later launches too"""
-        if gain is not None and len(bf.hs) > 1 and D.post_linear_fits(n, w, bf.xb, self.cfg.hidden_size):
+    def _product(self, bf: _Buffers, n: int, due: D.Branches | None, pre, w, out, bias=None, tail=None, up=None, spec=None,
+                 keep_operand: bool = False) -> None:
+        """out <- operand @ w^T (or the gated pair), after the outstanding norms and sum;
+        ``keep_operand``: bf.xb is read by later launches too"""
+        if due is not None and len(bf.hs) > 1 and D.post_linear_fits(n, w, bf.xb, self.cfg.hidden_size):
             x = bf.h
             bf.cur ^= 1
-            D.post_linear(x, bf.branch, gain, self.cfg.eps, bf.h, bf.xb if keep_copy else None, w, out, n, bias)
+            D.post_linear(x, due, self.cfg.eps, bf.h, bf.xb if keep_operand else None, w, out, n, bias, tail, pre, up, spec)
             return
-        self._settle(bf, n, gain)
-        D.linear(bf.xb, w, out, n, bias=bias)
-
-    def _mixer(self, L: _Layer, att: D.PagedAttention, bf: _Buffers, b: _Batch, gain: torch.Tensor | None) -> None:
-        """bf.branch <- attention of the residual"""
-        m: AttentionSpec = L.spec.mixer
-        n, own = b.rows, m.kv_from is None
-        qkv, out = bf.qkv(L.qkv.shape[0]), bf.attn(m.heads * m.vdim)
-        self._product(bf, n, gain, L.qkv, qkv, bias=L.qkv_b)
-        if b.decode:
-            att.rows(qkv, out, b.slot, b.pos, n, b.keys, append=own)
+        self._settle(bf, n, due, pre)
+        if up is not None:
+            D.glu(bf.xb, w, up, out, n, spec)
         else:
-            if own:
-                att.append(qkv, b.slot, b.pos, n)
-            if b.blocks:
-                att.prompt(qkv, out, *b.blocks[att.prompt_block(m)])
-            if b.n_single:
-                att.rows(qkv, out, b.slot, b.pos, b.n_single, b.keys, append=False, lst=b.single)
-        D.linear(out, L.o, bf.branch, n, bias=L.o_b)
+            D.linear(bf.xb, w, out, n, bias=bias, tail=tail)
 
-    def _mlp(self, L: _Layer, bf: _Buffers, n: int, gain: torch.Tensor | None) -> torch.Tensor | None:
-        """The experts of the residual: bf.branch (returns the gain of the norm still outstanding),
-        or already normed and added (returns None)"""
-        f, H = L.spec.mlp, self.cfg.hidden_size
-        r, eps = f.router, self.cfg.eps
-        logits, idx, wt = bf.router_logits(L.router.shape[0]), bf.idx(r.top), bf.wt(r.top)
-        self._product(bf, n, gain, L.router, logits, keep_copy=True)
+    def _mixer(self, L: Layer, bound: list, bf: _Buffers, b: _Batch, due: D.Branches | None) -> D.Branches:
+        """The mixer of the residual; returns its output on the way into the residual"""
+        n, eps = b.rows, self.cfg.eps
+        y = bf.cols("proj", pad8(L.n_main))
+        y2 = bf.f32("proj_tail", L.n_tail) if L.n_tail else None
+        self._product(bf, n, due, L.pre1, L.proj, y, bias=L.proj_b, tail=(y2, L.n_tail) if L.n_tail else None)
+        outs = [p.run(op, bf, b, y, y2, eps) for p, op in zip(L.parts, bound)]
+        p = L.parts[0]
+        if len(L.parts) == 1:
+            D.linear(outs[0], p.o, bf.branch, n, bias=p.o_b)
+            return D.Branches(bf.branch, L.norm1, self.cfg.norm.mult)
+        D.linear_pair(outs[0], p.o, bf.branch, outs[1], L.parts[1].o, bf.branch2, n)
+        return D.Branches(bf.branch, L.norm1, self.cfg.norm.mult, bf.branch2, L.gain_a, L.gain_b)
+
+    def _dense(self, L: Layer, bf: _Buffers, n: int, due: D.Branches) -> D.Branches:
+        f: GluSpec = L.spec.mlp
+        act = bf.mixed("ff", f.ff)
+        self._product(bf, n, due, L.pre2, L.ff.gate, act, up=L.ff.up, spec=f)
+        D.linear(act, L.ff.down, bf.branch, n)
+        return D.Branches(bf.branch, L.norm2, self.cfg.norm.mult)
+
+    def _moe(self, L: Layer, bf: _Buffers, n: int, due: D.Branches) -> D.Branches | None:
+        """The experts of the residual: bf.branch, or already normed and added (returns None)"""
+        f, H, w = L.spec.mlp, self.cfg.hidden_size, L.ff
+        r, mult = f.router, self.cfg.norm.mult
+        logits, idx, wt = bf.router_logits(w.router.shape[0]), bf.idx(r.top), bf.wt(r.top)
+        self._product(bf, n, due, L.pre2, w.router, logits, keep_operand=True)
         if n <= D.GEMV_MAX_ROWS:
             key = (L.index, bf.cur)
             if key not in bf.experts:
-                bf.experts[key] = D.ExpertRows(f, L, bf, H, bf.h)
+                bf.experts[key] = D.ExpertRows(f, w, bf, H, bf.h)
             bf.experts[key].glu(n)
             bf.experts[key].down(n)
-            return L.norm2
-        D.moe_route(logits, L.correction, r.scale, idx, wt, n)
+            return D.Branches(bf.branch, L.norm2, mult)
+        D.moe_route(logits, w.correction, r.scale, idx, wt, n)
         act, out = bf.act(r.top, f.expert.ff), bf.expert_out(r.top)
         ws = ops.moe_group(idx[:n], r.experts, check_indices=False)  # identity ids are past the end: left out
-        D.grouped_gemm(bf.xb, L.gate, ws, act, n, r.top, up=L.up, spec=f.expert)
-        D.grouped_gemm(act, L.down, ws, out, n, r.top, x_per_pair=True)
+        D.grouped_gemm(bf.xb, w.gate, ws, act, n, r.top, up=w.up, spec=f.expert)
+        D.grouped_gemm(act, w.down, ws, out, n, r.top, x_per_pair=True)
         shared = None
         if f.shared is not None:
             sact, shared = bf.shared_act(f.shared.ff), bf.shared_out()
-            D.glu_gemm(bf.xb, L.s_gate, L.s_up, sact, n, f.shared)
-            D.linear(sact, L.s_down, shared, n)
-        D.moe_sum_post_norm(out, idx, wt, shared, logits, r.experts, r.outputs, L.norm2, eps, bf.h, bf.xb, n)
+            D.glu_gemm(bf.xb, w.s_gate, w.s_up, sact, n, f.shared)
+            D.linear(sact, w.s_down, shared, n)
+        D.moe_sum_post_norm(out, idx, wt, shared, logits, r.experts, r.outputs, L.norm2, self.cfg.eps, bf.h, bf.xb, n, mult)
         return None
 
     def _forward(self, cache: PagedKVCache, bf: _Buffers, b: _Batch, logits: bool) -> torch.Tensor:
@@ -322,17 +298,16 @@ class StackModel(DecoderShard):
             D.embed_rows(bf.tokens[:n], self.embed, bf.h, bf.xb, H)
         else:
             bf.xb[:n, :H].copy_(bf.h[:n])
-        gain = None  # of the norm that the latest sublayer's output still has to pass
-        for L, att in zip(self.layers, self._attention(cache)):
-            self._mixer(L, att, bf, b, gain)
-            gain = L.norm1
-            if L.spec.mlp is not None:
-                gain = self._mlp(L, bf, n, gain)
+        due = None  # the latest sublayer's output, which still has to pass its norm
+        for L, bound in zip(self.layers, self._mixers(cache)):
+            due = self._mixer(L, bound, bf, b, due)
+            if L.ff is not None:
+                due = (self._moe if isinstance(L.spec.mlp, MoeSpec) else self._dense)(L, bf, n, due)
             if self.layer_hook is not None:
-                self._settle(bf, n, gain)
-                gain = None
+                self._settle(bf, n, due, None)
+                due = None
                 self.layer_hook(L.index, bf.h[:n])
-        self._settle(bf, n, gain)
+        self._settle(bf, n, due, None)
         if not self.is_last or not logits:
             if bf.cur:  # callers find the residual where they put it
                 bf.hs[0][:n].copy_(bf.h[:n])
@@ -362,8 +337,10 @@ class StackModel(DecoderShard):
         """``counts``: (cache row, tokens) per entry, in batch order; ``want``: batch rows with logits."""
         n = sum(c for _, c in counts)
         slot, pos, single = np.empty(n, np.int32), np.empty(n, np.int32), []
-        sizes = {D.PagedAttention.prompt_block(L.spec.mixer) for L in self.layers}
+        sizes = {D.PagedAttention.prompt_block(m) for m in (attention_of(L.spec.mixer) for L in self.layers) if m is not None}
         blocks: dict[int, list] = {s: [] for s in sizes}
+        chunks, seqs, alone = [], [], []
+        C = D.recur_chunk() if self.state_shapes else 0
         at, keys = 0, 1
         tiled = self.dtype == torch.bfloat16  # the 32-bit mode runs every position by itself
         for row, c in counts:
@@ -376,8 +353,13 @@ class StackModel(DecoderShard):
             else:
                 for s in sizes:
                     blocks[s] += [(at + o, row, p0 + o, min(s, c - o)) for o in range(0, c, s)]
+            if C and c == 1:
+                alone.append(at)
+            elif C:
+                seqs.append((len(chunks), -(-c // C), 0, 0))
+                chunks += [(at + o, row, p0 + o, min(C, c - o), p0, 0, 0, 0) for o in range(0, c, C)]
             at += c
-        parts = [slot, pos, np.asarray(single, np.int32), np.asarray(want, np.int32)]
+        parts = [slot, pos] + [np.asarray(x, np.int32).reshape(-1) for x in (single, want, chunks, seqs, alone)]
         have = [s for s in sizes if blocks[s]]
         parts += [np.asarray(blocks[s], np.int32).reshape(-1) for s in have]
         starts, total = [], 0
@@ -391,8 +373,9 @@ class StackModel(DecoderShard):
         t = [dev[s0 : s0 + p.size] for s0, p in zip(starts, parts)]
         one_each = all(c == 1 for _, c in counts)
         return _Batch(n, t[0], t[1], keys, single=None if one_each else t[2], n_single=len(single),
-                      blocks={s: (t[4 + i], len(blocks[s])) for i, s in enumerate(have)},
-                      want=t[3], n_want=len(want))
+                      blocks={s: (t[7 + i], len(blocks[s])) for i, s in enumerate(have)},
+                      want=t[3], n_want=len(want), chunks=t[4], n_chunks=len(chunks), seqs=t[5], n_seqs=len(seqs),
+                      alone=t[6], n_alone=len(alone))
 
     def step(self, cache: PagedKVCache, entries: list[tuple[int, list[int], list[int]]]) -> torch.Tensor | None:
         """One batch: ``entries`` are (cache row, its next tokens, places among them whose logits are

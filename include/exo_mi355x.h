@@ -443,36 +443,48 @@ int exo_embed_rows(const int32_t* ids, const void* table, float* x, void* xb, in
 /* y[i] = x[rows[i]] / rms * gain (rows null: row i); x float32 [.., H]. */
 int exo_norm_rows(const float* x, const int32_t* rows, const float* gain, void* y, int n, int H,
                   int ldy, float eps, int dtype, exo_stream_t stream);
-/* Norm of a sublayer's output, then the residual sum: x += gain * branch / rms(branch), xb = x. */
-int exo_post_norm_add(const float* branch, int ldb, const float* gain, float* x, void* xb, int n,
-                      int H, int ldx, float eps, int dtype, exo_stream_t stream);
+/* Norm of a sublayer's output, then the residual sum: x_out = x + mult * gain * v / rms(v), where v
+ * is the branch, or (branch2) half the sum of two branches normed each with a gain of its own; the
+ * next product's operand is x_out, or (pre) x_out / rms(x_out) * pre.  Branches and x float32 [.., H]. */
+typedef struct {
+  const float *x, *branch, *branch2, *gain_a, *gain_b, *gain, *pre;
+  float* x_out;
+  void* operand; /* element type */
+  int H;
+  float eps, mult;
+} exo_post_norm;
+/* ... as a launch of its own, in place (x_out == x); operand [n][ldx]. */
+int exo_post_norm_add(const exo_post_norm* q, int ldb, int n, int ldx, int dtype,
+                      exo_stream_t stream);
 /* The same with the branch formed from a token's experts: sum of wt * y over the chosen experts
  * (idx >= experts: the input x itself), plus sigmoid(logits[gate_col]) * shared. */
 int exo_moe_sum_post_norm(const void* y, const int32_t* idx, const float* wt, const void* shared,
                           const float* logits, int top, int experts, int ldy, int lds, int ldl,
-                          int gate_col, const float* gain, float* x, void* xb, int n, int H,
-                          int ldx, float eps, int dtype, exo_stream_t stream);
+                          int gate_col, const exo_post_norm* q, int n, int ldx, int dtype,
+                          exo_stream_t stream);
 /* softmax over n logits; the `top` largest of score + correction; weight = score * scale. */
 int exo_moe_route(const float* logits, const float* correction, int32_t* idx, float* wt, int rows,
                   int n, int ldl, int top, float scale, exo_stream_t stream);
 
-/* y[M,N] = x[M,K] @ w[N,K]^T (+ bias), y in the element type or (y_f32) float32. */
-int exo_dense_gemv(const void* x, const void* w, const float* bias, void* y, int y_f32, int M,
-                   int N, int ldx, int ldw, int ldy, int dtype, exo_stream_t stream); /* M <= 16 */
-/* exo_post_norm_add and the product in one launch (few rows: exo_post_gemv_fits): the residual
- * x + gain * branch / rms(branch) goes to x_out (not x) and, in the element type, to xb_out (may be
- * null), and is the product's input. */
-int exo_post_gemv_fits(int M, int N, int H, int ldx, int dtype);
-int exo_post_gemv(const float* x, const float* branch, const float* gain, float eps, float* x_out,
-                  void* xb_out, const void* w, const float* bias, void* y, int y_f32, int M, int N,
-                  int H, int ldx, int ldw, int ldy, int dtype, exo_stream_t stream);
-int exo_dense_gemm(const void* x, const void* w, const float* bias, void* y, int y_f32,
-                   float* workspace, int64_t workspace_floats, int M, int N, int ldx, int ldw,
-                   int ldy, int dtype, exo_stream_t stream);
-/* g = min(x @ w^T, limit), u = clamp(x @ w_up^T, +-limit): y = g sigmoid(alpha g) (u + shift). */
-int exo_dense_glu_gemm(const void* x, const void* w, const void* w_up, void* y, float limit,
-                       float alpha, float shift, int M, int N, int ldx, int ldw, int ldy,
-                       int dtype, exo_stream_t stream);
+/* y[M,N] = x[M,K] @ w[N,K]^T (+ bias): columns below n1 to y (element type, or float32 if y_f32),
+ * the rest to y2 (float32; n1 = N: none).  w_up non-null: the gated pair instead, with g = min(x @ w^T,
+ * limit), u = clamp(x @ w_up^T, +-limit): y = g sigmoid(alpha g) (u + shift). */
+typedef struct {
+  const void *x, *w, *w_up;
+  const float* bias;
+  void* y;
+  float* y2;
+  int M, N, n1, ldx, ldw, ldy, ldy2, y_f32, dtype;
+  float limit, alpha, shift;
+} exo_linear;
+/* up to 16 rows; b non-null: a second product over the same number of rows in the same launch */
+int exo_linear_rows(const exo_linear* a, const exo_linear* b, exo_stream_t stream);
+int exo_linear_gemm(const exo_linear* a, float* workspace, int64_t workspace_floats,
+                    exo_stream_t stream);
+/* exo_post_norm_add and the product in one launch (few rows: exo_post_linear_fits): a->x is not
+ * read, the residual goes to q->x_out (not q->x), the operand also to q->operand (may be null). */
+int exo_post_linear_fits(int M, int N, int H, int ldx, int dtype);
+int exo_post_linear(const exo_post_norm* q, const exo_linear* a, exo_stream_t stream);
 /* Experts of a prompt by (token, slot) pair through exo_moe_group's workspace; w_up null: the
  * plain product.  x_per_pair: x has a row per pair, else per token. */
 int exo_dense_grouped_gemm(const void* x, const void* w, const void* w_up, const void* group_ws,
@@ -500,15 +512,17 @@ int exo_moe_down_rows(const exo_moe_rows* args, exo_stream_t stream);
 /* Attention over a paged KV pool: keys [page][kv_heads][64][ldk], values transposed
  * [page][kv_heads][ldv][64]; table [slots][max_pages]; row i of qkv belongs to slot[i] at
  * position pos[i].  window 0: causal; else a key is seen if fewer than `window` positions back or
- * among the first keep_first positions.  slopes: per-head distance penalty, or null. */
+ * among the first keep_first positions.  slopes: per-head distance penalty, or null.  q_gain, k_gain
+ * [dim]: gains of the query / key norm (unit_qk), or null.  gate [rows][ldg]: head h's output times
+ * sigmoid(gate[h]), or null. */
 typedef struct {
   const void* qkv;
   void *k_pool, *v_pool;
   const int32_t *table, *slot, *pos, *list;
-  const float* slopes;
+  const float *slopes, *q_gain, *k_gain, *gate;
   void* out;
   float scale, eps;
-  int n, heads, kv_heads, dim, vdim, ldq, ldk, ldv, ldo, max_pages, window, keep_first, unit_qk, dtype;
+  int n, heads, kv_heads, dim, vdim, ldq, ldk, ldv, ldo, ldg, max_pages, window, keep_first, unit_qk, dtype;
 } exo_paged_attn;
 /* keys (normalised if unit_qk) and values of all n rows into the pool */
 int exo_paged_append(const exo_paged_attn* args, exo_stream_t stream);
@@ -522,6 +536,55 @@ int exo_paged_attn_rows(const exo_paged_attn* args, int nsplit, int append, void
  * at most exo_paged_prompt_block(heads, kv_heads) tokens of one sequence */
 int exo_paged_prompt_block(int heads, int kv_heads);
 int exo_paged_attn_prompt(const exo_paged_attn* args, exo_stream_t stream);
+
+/* Recurrent mixers.  Per head, from S = 0: S <- diag(a_t) S + k_t v_t^T, o_t = S^T (q_scale q_t), S
+ * [dim][vdim] float32.  per_channel: a_t per key channel = sigmoid(z)^(inv_tau) with z = low @ decay_w +
+ * decay_b (low float32 [rows][rank], decay_w [rank][heads * dim]), queries and keys per head (groups =
+ * heads).  Else: dt = softplus(dt_raw + dt_bias), a_t = exp(-decay_rate dt) per head, values scaled by
+ * dt, queries and keys shared by heads / groups heads, o_t += skip v_t, and all three come from `raw`
+ * [rows][channels] (at q_channel, k_channel, v_channel) through a causal convolution per channel (conv_w
+ * [taps][channels], the current input's weight last) and silu.
+ * Cache row r's state is state[map[r]], [heads][dim][lds] (lds a multiple of 4, columns from vdim on zero), the
+ * convolution's latest inputs ring[map[r]], [taps][channels], position p at p % taps; position 0
+ * starts from zero. */
+typedef struct {
+  const void *q, *k, *v; /* element type; convolved inputs: parts of act */
+  const float *low, *decay_w, *decay_b;
+  const float *dt_raw, *dt_bias, *decay_rate, *skip;
+  const void* raw;
+  const float *conv_w, *conv_b;
+  void *ring, *act;
+  float *cum, *dt;            /* [rows][ldcum] scratch of prompts */
+  float *scores, *chunk_state; /* exo_recur_scores_floats, exo_recur_state_floats */
+  float *state, *y;            /* y [rows][ldy] */
+  const int32_t *map, *slot, *pos, *list; /* single tokens: row i of cache row slot[i] at pos[i]; list: which rows, or null */
+  const int32_t *chunks, *seqs;
+  int ldq, ldk, ldv, ldlow, rank, lddt, ldraw, channels, taps, ldact, ldcum, lds, ldy;
+  int q_channel, k_channel, v_channel;
+  int heads, groups, dim, vdim, per_channel, n, n_chunks, n_seqs, qk_vec, v_vec, dtype;
+  float q_scale, inv_tau;
+} exo_recurrence;
+/* portions of prompts: chunks [n_chunks][8] = first row, cache row, first position, tokens (at most
+ * exo_recur_chunk()), first position of its portion, 0, 0, 0, a portion's chunks one after the other;
+ * seqs [n_seqs][4] = first chunk, chunks, 0, 0 */
+int exo_recur_chunk(void);
+int64_t exo_recur_scores_floats(int n_chunks, int groups);
+int64_t exo_recur_state_floats(int n_chunks, int heads, int dim, int lds);
+int exo_recur_chunks(const exo_recurrence* args, exo_stream_t stream);
+/* single tokens of n sequences */
+int exo_recur_step(const exo_recurrence* args, exo_stream_t stream);
+/* RMS norm of `groups` equal parts of y, gain repeating with `period`, and silu(gate) ahead of the
+ * norm (gate_first) or behind it; rows null: the first n */
+typedef struct {
+  const float* y;
+  const void* gate;
+  const float* gain;
+  void* out;
+  int width, groups, period, ldy, ldg, ldo, gate_first, dtype;
+  float eps;
+} exo_gated_norm;
+int exo_gated_norm_rows(const exo_gated_norm* args, const int32_t* rows, int n,
+                        exo_stream_t stream);
 
 #ifdef __cplusplus
 }

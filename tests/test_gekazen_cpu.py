@@ -243,9 +243,11 @@ def test_can_admit_counts_requests_to_their_end(monkeypatch):
 
 def test_new_entry_points_check_their_arguments():
     lib = native.load()
-    assert lib.exo_dense_gemv(None, None, None, None, 0, 1, 8, 64, 64, 8, 0, None) == -1
-    assert lib.exo_dense_gemv(16, 16, None, 16, 0, 17, 8, 64, 64, 8, 0, None) == -1
-    assert lib.exo_dense_gemv(16, 16, None, 16, 0, 1, 8, 72, 72, 8, 0, None) == -1
+    lin = dict(x=16, w=16, y=16, M=1, N=8, n1=8, ldx=64, ldw=64, ldy=8)
+    assert lib.exo_linear_rows(native.Linear(**dict(lin, w=None)), None, None) == -1
+    assert lib.exo_linear_rows(native.Linear(**dict(lin, M=17)), None, None) == -1
+    assert lib.exo_linear_rows(native.Linear(**dict(lin, n1=4)), None, None) == -1  # no second output
+    assert lib.exo_linear_rows(native.Linear(**dict(lin, ldx=72, ldw=72)), None, None) == -1
     assert b"multiples of 64" in lib.exo_last_error()
     assert lib.exo_moe_route(16, 16, 16, 16, 1, 600, 600, 2, 1.0, None) == -1
     a = native.PagedAttn(qkv=16, k_pool=16, v_pool=16, table=16, slot=16, pos=16, out=16, n=1, heads=3, kv_heads=2,

@@ -19,7 +19,7 @@ from exo_amd.generate import generate
 from exo_amd.paged_cache import PAGE, PagedKVCache
 from exo_amd.prefix_cache import KVPrefixCache
 from exo_amd.registry import build_model, config_from_dict
-from exo_amd.stack_config import AttentionSpec, ExpertSpec, MoeSpec, RouterSpec, distance_slopes
+from exo_amd.stack_config import AttentionSpec, GluSpec, MoeSpec, RouterSpec, distance_slopes
 from exo_amd.types import GenerationTask, TextGenerationTaskParams
 from oracle import gekazen as O
 from oracle.affine import bf16_round
@@ -86,7 +86,7 @@ def test_linear(device, dtype, M, N, K):
 def test_gated_pair(device, dtype, M, N, K):
     say("glu", dtype, M, N, K)
     x, g, u = rand((M, K), 1), rand((N, K), 2, 2 * K**-0.5), rand((N, K), 3, 2 * K**-0.5)
-    spec = ExpertSpec(N, 1.3)
+    spec = GluSpec(N, 1.3)
     out = torch.zeros(M, D.pad64(N), dtype=dtype, device="cuda")
     D.glu_gemm(mat(x, dtype), mat(g, dtype), mat(u, dtype), out, M, spec)
     want = O.clamped_glu(x.astype(np.float64) @ g.T, x.astype(np.float64) @ u.T, 1.3)
@@ -103,7 +103,7 @@ def test_residual_norm(device, dtype, n, H):
     say("post norm", dtype, n, H)
     x, y, w, eps = rand((n, H), 1), rand((n, H), 2, 3e-3), rand((H,), 3), 1e-5  # eps of the order of mean(y^2)
     xt, xb = dev(x), torch.zeros(n, D.pad64(H), dtype=dtype, device="cuda")
-    D.post_norm_add(dev(y), dev(1 + w), eps, xt, xb, n)
+    D.post_norm_add(D.Branches(dev(y), dev(1 + w)), eps, xt, xb, n)
     want = x + O.rms_norm_offset(y.astype(np.float64), w, eps)
     close(host(xt), want, 1e-5, "residual")
     close(host(xb[:, :H]), want, TOL[dtype], "its copy")
@@ -123,7 +123,7 @@ def test_residual_norm_inside_a_product(device, dtype, n, H, N):
         assert dtype == F32 or N == 20000  # too many columns for the launch's registers or LDS
         return
     xt, xo, out = dev(x), torch.zeros(n, H, device="cuda"), torch.zeros(n, N, device="cuda")
-    D.post_linear(xt, dev(y), dev(1 + g), 1e-5, xo, xb, W, out, n, bias=dev(b))
+    D.post_linear(xt, D.Branches(dev(y), dev(1 + g)), 1e-5, xo, xb, W, out, n, bias=dev(b))
     want = x + O.rms_norm_offset(y.astype(np.float64), g, 1e-5)
     close(host(xo), want, 1e-5, "residual")
     close(host(xb[:, :H]), want, TOL[dtype], "its copy")
@@ -169,7 +169,7 @@ def test_feed_forward(device, dtype, H, E, I, top, ff, sff, n):
     bf = model._buffers(1, max(n, 2))
     bf.h[:n].copy_(dev(x))
     bf.xb[:n, :H].copy_(dev(x))
-    model._settle(bf, n, model._mlp(model.layers[0], bf, n, None))
+    model._settle(bf, n, model._moe(model.layers[0], bf, n, None), None)
     ww = O.to_float64(w)
     want = O.moe(x.astype(np.float64), ww, "l0.mlp.", m)
     want = x + O.rms_norm_offset(want, ww["l0.norm2"], cfg.eps)
