@@ -303,7 +303,7 @@ def _novosun(d: dict) -> StackConfig:
                 raise ValueError(f"layer {i}: feed-forward kind {f['kind']!r} not supported (have 'dense')")
             mlp = GluSpec(ff=int(f["ff"]), limit=float(f["limit"]))
         layers.append(LayerSpec(mixers[L["type"]](L["mixer"]), mlp))
-    norm = NormSpec(float(d["norm"]["eps"]), pre=True, mult=float(d["residual_mult"]))
+    norm = NormSpec(float(d["norm"]["eps"]), pre=True, mult=float(d.get("residual_mult", 1.0)))
     return StackConfig("Novosun", int(d["vocab"]), int(d["width"]), norm, tuple(layers), copy.deepcopy(d))
 
 

@@ -1,0 +1,109 @@
+"""What the tests of the layer-list designs share: tensors in and out, schedules of steps through the
+trace replay, tasks through an engine."""
+
+from __future__ import annotations
+
+import numpy as np
+import torch
+
+from exo_amd import dense_ops as D
+from exo_amd.engine import BatchGenerator
+from exo_amd.types import GenerationTask, TextGenerationTaskParams
+from oracle.affine import bf16_round
+from tests.util import rng
+
+BF, F32 = torch.bfloat16, torch.float32
+DTYPES = [BF, F32]
+TOL = {BF: 1.2e-2, F32: 2e-5}  # one operator: rounding of a bf16 output / float32 sums
+
+
+def rand(shape, seed, scale=1.0):
+    return bf16_round((rng(seed).standard_normal(shape) * scale).astype(np.float32))
+
+
+def dev(a, dtype=F32):
+    return torch.from_numpy(np.ascontiguousarray(a)).to("cuda").to(dtype)
+
+
+def mat(a, dtype):
+    return D.padded(torch.from_numpy(np.ascontiguousarray(a)), dtype, "cuda")
+
+
+def host(t):
+    return t.float().cpu().numpy()
+
+
+def close(got, want, tol, what):
+    want = np.asarray(want, np.float64)
+    err = (np.abs(np.asarray(got, np.float64) - want) / np.maximum(np.abs(want), np.sqrt(np.mean(want**2)))).max()
+    assert err < tol, f"{what}: {err:.2e} of the larger of value and RMS"
+
+
+def play(model, toks, steps, max_tokens=1024, rows=4):
+    """Run a schedule [[(name, tokens), ...], ...] with all places wanted; sequences end when their
+    tokens are used up.  Returns {name: logits}."""
+    from exo_amd.trace import Replay
+
+    rp, at, got = Replay(model, max_tokens, rows), {}, {}
+    for step in steps:
+        entries, end = [], []
+        for name, n in step:
+            base, a = name.split("#")[0], at.get(name, 0)
+            n = min(n, len(toks[base]) - a)
+            if n <= 0:
+                continue
+            entries.append(dict(id=name, tokens=toks[base][a : a + n], want=list(range(n))))
+            at[name] = a + n
+            if at[name] == len(toks[base]):
+                end.append(name)
+        lg = rp.step(entries, end)
+        o = 0
+        for e in entries:
+            k = len(e["tokens"])
+            got.setdefault(e["id"], []).append(lg[o : o + k])
+            o += k
+    assert len(rp.cache._free) == rp.cache.n_pages  # everything was given back
+    return {k: np.concatenate(v) for k, v in got.items()}
+
+
+# portions beside single tokens, requests that pause, end and are admitted again; over sequences of
+# a 300, b 141, c 64, d 23 and e 1 tokens
+SCHEDULE = [[("d", 5)], [("d", 1), ("a", 40)], [("d", 1), ("a", 2), ("b", 64)], [("a", 100), ("b", 1), ("d", 1)],
+            [("b", 1), ("d", 1)], [("d", 14), ("a", 1), ("b", 3), ("c", 33)], [("c", 31), ("a", 29), ("b", 2), ("e", 1)],
+            [("e#2", 1), ("a", 1)], [("a", 1), ("c#2", 2), ("b", 70)], [("a", 126), ("c#2", 50)], [("d#2", 23), ("c#2", 1)],
+            [("c#2", 11), ("b#2", 141)]] + [[("a#2", 7), ("d#3", 1)]] * 50
+
+
+def greedy_agrees(forward, prompt, got, dtype):
+    """Tokens are the arg max of ``forward`` (the oracle's logits of a whole sequence) given the tokens
+    before, or within rounding of it."""
+    lg = forward(list(prompt) + list(got))[len(prompt) - 1 : -1]
+    rms = np.sqrt(np.mean(lg**2, -1))
+    short = (lg.max(-1) - lg[np.arange(len(got)), got]) / rms
+    assert short.max() < (2e-2 if dtype == F32 else 0.3), f"{short.max():.3f} at {int(short.argmax())}"
+    assert np.mean(short == 0) > (0.9 if dtype == F32 else 0.6)
+
+
+def engine(model, **kw):
+    return BatchGenerator(model=model, tokenizer=None, model_id="m", max_seq=512, **kw)
+
+
+def task(i, prompt, n, **kw):
+    return GenerationTask(f"t{i}", f"c{i}", TextGenerationTaskParams(
+        model="m", input=prompt, max_output_tokens=n, temperature=0.0, bench=True, **kw))
+
+
+def drain(eng, tasks, join_at=None):
+    out = {t.task_id: [] for t in tasks}
+    todo, done, k = list(tasks), 0, 0
+    while done < len(tasks):
+        while todo and (join_at is None or k >= join_at[len(tasks) - len(todo)]):
+            eng.submit(todo.pop(0))
+        for tid, ev in eng.step():
+            if hasattr(ev, "token_id"):
+                out[tid].append(ev.token_id)
+            else:
+                done += 1
+        k += 1
+        assert k < 2000
+    return out

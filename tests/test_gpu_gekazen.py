@@ -14,48 +14,25 @@ import torch
 
 from exo_amd import dense_ops as D
 from exo_amd import native, ops
-from exo_amd.engine import BatchGenerator, SequentialGenerator, ShardBatchGenerator
+from exo_amd.engine import SequentialGenerator, ShardBatchGenerator
 from exo_amd.generate import generate
 from exo_amd.paged_cache import PAGE, PagedKVCache
 from exo_amd.prefix_cache import KVPrefixCache
 from exo_amd.registry import build_model, config_from_dict
 from exo_amd.stack_config import AttentionSpec, GluSpec, MoeSpec, RouterSpec, distance_slopes
-from exo_amd.types import GenerationTask, TextGenerationTaskParams
+from exo_amd.types import TextGenerationTaskParams
 from oracle import gekazen as O
 from oracle.affine import bf16_round
 from tests import gekazen_util as U
+from tests import stack_util as S
+from tests.stack_util import BF, DTYPES, F32, SCHEDULE, TOL, close, dev, drain, engine, host, mat, play, rand, task
 from tests.util import rng
 
 pytestmark = pytest.mark.gpu
-BF, F32 = torch.bfloat16, torch.float32
-DTYPES = [BF, F32]
-TOL = {BF: 1.2e-2, F32: 2e-5}  # one operator: rounding of a bf16 output / float32 sums
 
 
 def say(*a):
     print("[gekazen]", *a, flush=True)
-
-
-def rand(shape, seed, scale=1.0):
-    return bf16_round((rng(seed).standard_normal(shape) * scale).astype(np.float32))
-
-
-def dev(a, dtype=F32):
-    return torch.from_numpy(np.ascontiguousarray(a)).to("cuda").to(dtype)
-
-
-def mat(a, dtype):
-    return D.padded(torch.from_numpy(a), dtype, "cuda")
-
-
-def host(t):
-    return t.float().cpu().numpy()
-
-
-def close(got, want, tol, what):
-    want = np.asarray(want, np.float64)
-    err = (np.abs(np.asarray(got, np.float64) - want) / np.maximum(np.abs(want), np.sqrt(np.mean(want**2)))).max()
-    assert err < tol, f"{what}: {err:.2e} of the larger of value and RMS"
 
 
 # ------------------------------------------------------------------ products
@@ -357,33 +334,6 @@ def check_rows(built, dtype, name, places, logits, what):
     assert (err[~tied] < 6e-2).all() and err.max() < 1.0, f"{what}: {err.max():.2e}"
 
 
-def play(model, toks, steps, max_tokens=1024, rows=4):
-    """Run a schedule [[(name, tokens), ...], ...] with all places wanted; sequences end when their
-    tokens are used up.  Returns {name: logits}."""
-    from exo_amd.trace import Replay
-
-    rp, at, got = Replay(model, max_tokens, rows), {}, {}
-    for step in steps:
-        entries, end = [], []
-        for name, n in step:
-            base, a = name.split("#")[0], at.get(name, 0)
-            n = min(n, len(toks[base]) - a)
-            if n <= 0:
-                continue
-            entries.append(dict(id=name, tokens=toks[base][a : a + n], want=list(range(n))))
-            at[name] = a + n
-            if at[name] == len(toks[base]):
-                end.append(name)
-        lg = rp.step(entries, end)
-        o = 0
-        for e in entries:
-            k = len(e["tokens"])
-            got.setdefault(e["id"], []).append(lg[o : o + k])
-            o += k
-    assert len(rp.cache._free) == rp.cache.n_pages  # everything was given back
-    return {k: np.concatenate(v) for k, v in got.items()}
-
-
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("portion", [300, 1, 2, 3, 17, 64, 65, 128])
 def test_model_in_portions(built, dtype, portion):
@@ -406,12 +356,6 @@ def test_model_layers(built, dtype):
     for i, (g, w) in enumerate(zip(outs, want)):
         err = U.rel_rms(g, w)
         assert np.median(err) < 3e-2 and (dtype == BF or err.max() < 2e-5), f"layer {i}: {err.max():.2e}"
-
-
-SCHEDULE = [[("d", 5)], [("d", 1), ("a", 40)], [("d", 1), ("a", 2), ("b", 64)], [("a", 100), ("b", 1), ("d", 1)],
-            [("b", 1), ("d", 1)], [("d", 14), ("a", 1), ("b", 3), ("c", 33)], [("c", 31), ("a", 29), ("b", 2), ("e", 1)],
-            [("e#2", 1), ("a", 1)], [("a", 1), ("c#2", 2), ("b", 70)], [("a", 126), ("c#2", 50)], [("d#2", 23), ("c#2", 1)],
-            [("c#2", 11), ("b#2", 141)]] + [[("a#2", 7), ("d#3", 1)]] * 50
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -508,37 +452,7 @@ def test_step_errors(built):
 
 
 def greedy_agrees(built, prompt, got, dtype):
-    """Tokens are the oracle's arg max given the tokens before, or within rounding of it."""
-    lg = O.forward(built.cfg, built.w, list(prompt) + list(got))[len(prompt) - 1 : -1]
-    rms = np.sqrt(np.mean(lg**2, -1))
-    short = (lg.max(-1) - lg[np.arange(len(got)), got]) / rms
-    assert short.max() < (2e-2 if dtype == F32 else 0.3), f"{short.max():.3f} at {int(short.argmax())}"
-    assert np.mean(short == 0) > (0.9 if dtype == F32 else 0.6)
-
-
-def engine(model, **kw):
-    return BatchGenerator(model=model, tokenizer=None, model_id="gekazen", max_seq=512, **kw)
-
-
-def task(i, prompt, n, **kw):
-    return GenerationTask(f"t{i}", f"c{i}", TextGenerationTaskParams(
-        model="gekazen", input=prompt, max_output_tokens=n, temperature=0.0, bench=True, **kw))
-
-
-def drain(eng, tasks, join_at=None):
-    out = {t.task_id: [] for t in tasks}
-    todo, done, k = list(tasks), 0, 0
-    while done < len(tasks):
-        while todo and (join_at is None or k >= join_at[len(tasks) - len(todo)]):
-            eng.submit(todo.pop(0))
-        for tid, ev in eng.step():
-            if hasattr(ev, "token_id"):
-                out[tid].append(ev.token_id)
-            else:
-                done += 1
-        k += 1
-        assert k < 2000
-    return out
+    S.greedy_agrees(lambda toks: O.forward(built.cfg, built.w, toks), prompt, got, dtype)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
