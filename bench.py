@@ -33,6 +33,14 @@ GEKAZEN_SIZES = {
     "4k": (4096, 6, 64, 4, 128, 128, 8, 8, 1536, 151936, 8),
 }
 
+# Novosun layers beside a Gekazen of that size: kinds of the layers (g linear attention, p attention beside a
+# state-space recurrence), linear attention heads / key size / value size, recurrence heads / value size / state / groups, ff
+NOVOSUN_SIZES = {
+    "1k": ("gp" * 12, 4, 128, 256, 32, 64, 128, 1, 2560),
+    "2k": ("gp" * 8, 4, 256, 512, 64, 64, 128, 1, 6912),
+    "4k": ("gp" * 3, 8, 256, 512, 128, 64, 128, 8, 13824),
+}
+
 
 def parse_args():
     ap = argparse.ArgumentParser()
@@ -52,11 +60,12 @@ def parse_args():
     ap.add_argument("--pmc-copy", action="store_true",
                     help="also launch one plain 256 MiB copy kernel: the known-size dispatch that "
                          "calibrates FETCH_SIZE / WRITE_SIZE in a rocprofv3 --pmc pass")
-    ap.add_argument("--workload", default="decode", choices=["decode", "qmatmul_sweep", "gekazen"],
-                    help="decode (default, the headline), the quantised-matmul shape sweep, or the Gekazen "
-                         "design beside a Qwen3-MoE of equal size, whole steps and launch by launch")
-    ap.add_argument("--gekazen-size", default="all", choices=["all"] + list(GEKAZEN_SIZES),
-                    help="sizes of the gekazen workload")
+    ap.add_argument("--workload", default="decode", choices=["decode", "qmatmul_sweep", "gekazen", "novosun"],
+                    help="decode (default, the headline), the quantised-matmul shape sweep, or a layer-list design "
+                         "beside the closest other model of equal size, whole steps and launch by launch: Gekazen "
+                         "beside a Qwen3-MoE, Novosun beside a Gekazen")
+    ap.add_argument("--gekazen-size", "--size", dest="size", default="all", choices=["all"] + list(GEKAZEN_SIZES),
+                    help="sizes of the gekazen and novosun workloads")
     return ap.parse_args()
 
 
@@ -633,62 +642,223 @@ def qwen_launches(torch, m, B, ctx):
     return rows
 
 
-def gekazen_workload(args):
+class RandomTensors(dict):
+    """Tensors of a layer-list checkpoint, drawn when the model asks for them; ``shape_of``: name -> shape."""
+
+    def __init__(self, torch, shape_of):
+        super().__init__()
+        self.torch, self.shape_of = torch, shape_of
+        self.g = torch.Generator(device="cuda").manual_seed(0)
+
+    def __missing__(self, key):
+        shape, mean, std = self.shape_of(key)
+        t = self.torch.empty(shape, dtype=self.torch.bfloat16, device="cuda").normal_(0.0, std, generator=self.g)
+        return t.add_(mean)
+
+
+def novosun_model(torch, size, novo):
+    from exo_amd.stack_config import StackConfig, novosun_dict
+    from exo_amd.stack_model import StackModel
+
+    H, _, hq, hkv, hd, _, _, _, _, V, _ = size
+    kinds, lh, ld, lv, sh, sv, sn, sg, ff = novo
+    cfg = StackConfig.from_dict(novosun_dict(H, V, kinds, heads=hq, kv_heads=hkv, dim=hd, vdim=hd, ff=ff, lin_heads=lh,
+                                             lin_dim=ld, lin_vdim=lv, ssm_heads=sh, ssm_vdim=sv, ssm_state=sn,
+                                             ssm_groups=sg, mult=0.5))
+    inner, rank = sh * sv, 16
+    ch = inner + 2 * sg * sn
+    vectors = {"norm1": H, "norm2": H, "norm1b": H, "norm2b": H, "left.out": H, "right.out": H, "final.norm": H, "q.norm": hd,
+               "k.norm": hd, "right.norm": inner, "mix.norm": lv, "A_log": sh, "D": sh}
+    mats = {"embed": (V, H), "head": (V, H), "mlp.gate": (ff, H), "mlp.up": (ff, H), "mlp.down": (H, ff),
+            "left.q": (hq * hd, H), "left.k": (hkv * hd, H), "left.v": (hkv * hd, H), "left.g": (hq, H), "left.o": (H, hq * hd),
+            "right.in": (inner + ch + sh, H), "right.conv": (ch, 4), "right.o": (H, inner), "mix.q": (lh * ld, H),
+            "mix.k": (lh * ld, H), "mix.v": (lh * lv, H), "mix.g": (lh * lv, H), "mix.o": (H, lh * lv), "mix.a1": (rank, H),
+            "mix.a2": (lh * ld, rank)}
+
+    def shape_of(key):
+        for name, n in vectors.items():
+            if key == name or key.endswith("." + name):
+                return (n,), 1.0, 0.1
+        for name, n in (("a2.b", lh * ld), ("conv.b", ch), ("dt_bias", sh)):
+            if key.endswith(name):
+                return (n,), {"a2.b": 2.0, "conv.b": 0.0, "dt_bias": -3.0}[name], 0.5
+        for name, shape in mats.items():
+            if key == name or key.endswith("." + name):
+                return shape, 0.0, 0.3 if name in ("right.conv", "mix.a2") else 0.02
+        raise KeyError(key)
+
+    w = RandomTensors(torch, shape_of)
+    for i, k in enumerate(kinds):  # (its size says the rank)
+        if k == "g":
+            w[f"l{i}.mix.a1"] = w[f"l{i}.mix.a1"]
+    return StackModel(cfg, w)
+
+
+def novosun_launches(torch, m, B, ctx):
+    """Per-launch times of a step of B rows (B <= 16: single tokens at context ctx; else one prompt)."""
+    from exo_amd import dense_ops as D
+    from exo_amd.stack_layers import LinearAttentionPart
+    from exo_amd.stack_model import _Batch
+
+    c, prompt = m.cfg, B > 16
+    H, eps = c.hidden_size, c.eps
+    cache = m.make_cache(1 if prompt else B, ctx + B + 64)
+    g = torch.Generator().manual_seed(7)
+    toks = lambda n: torch.randint(0, c.vocab_size, (n,), generator=g).tolist()  # noqa: E731
+    if prompt:
+        cache.reserve([0], B)
+        batch, bf = m._batch(cache, [(0, B)], []), m._buffers(1, B)
+        bf.tokens[:B].copy_(torch.tensor(toks(B), dtype=torch.int32))
+    else:
+        for r in range(B):
+            m.step(cache, [(r, toks(ctx), [])])
+        bf = m._buffers(B, 1)
+        bf.tokens.copy_(torch.tensor(toks(B), dtype=torch.int32))
+        m.decode_step(cache, B, use_graph=False)
+        batch = _Batch(B, torch.arange(B, dtype=torch.int32, device="cuda"), cache.pos[:B] - 1, m._keys_hint(cache, slice(0, B)))
+    m._forward(cache, bf, batch, False)
+    lin = [(L, o) for L, o in zip(m.layers, m._mixers(cache)) if isinstance(L.parts[0], LinearAttentionPart)]
+    par = [(L, o) for L, o in zip(m.layers, m._mixers(cache)) if len(L.parts) > 1]
+    every = [(L, None) for L in m.layers]
+    rows, fused = [], not prompt and D.post_linear_fits(B, m.layers[0].proj, bf.xb, H, True)
+    other = torch.empty_like(bf.h)
+
+    def add(name, which, fn, nbytes, flops):
+        rows.append(row_of(name, time_launches(torch, [(lambda L=L, o=o: fn(L, o)) for L, o in which]), nbytes, flops))
+
+    def mm(n, k):
+        return 2 * n * k + 2 * B * (n + k), 2 * B * n * k
+
+    def due(L, two):
+        return D.Branches(bf.branch, L.norm1, c.norm.mult, *((bf.branch2, L.gain_a, L.gain_b) if two else ()))
+
+    def product(L, w, out, two=False, **kw):
+        pre = L.pre2 if "up" in kw else L.pre1
+        if fused:
+            D.post_linear(bf.h, due(L, two), eps, other, None, w, out, B, pre=pre, **kw)
+        elif "up" in kw:
+            D.glu(bf.xb, w, kw["up"], out, B, kw["spec"])
+        else:
+            D.linear(bf.xb, w, out, B, **kw)
+    head = "norms, residual, " if fused else ""
+    for name, which in (("linear attention", lin), ("attention | state space", par)):
+        L0 = which[0][0]
+        y = bf.cols("proj", -(-L0.n_main // 8) * 8)
+        y2 = bf.f32("proj_tail", L0.n_tail)
+        add(f"{head}{name}: projection", which, lambda L, o: product(L, L.proj, y, tail=(y2, L.n_tail)), *mm(L0.proj.shape[0], H))
+        for i, p in enumerate(L0.parts):
+            s = p.spec
+            if hasattr(s, "kv_heads"):
+                vis = [j + 1 for j in range(B)] if prompt else [ctx] * B
+                kvb = 2 * s.kv_heads * (s.dim + s.vdim) * (B if prompt else sum(vis))
+                fl = 2 * sum(vis) * s.heads * (s.dim + s.vdim)
+                out = bf.mixed("attn", p.width)
+                gate = y2[:, p.tcol :]
+                if prompt:
+                    add("append keys, values", which, lambda L, o: o[i].append(y[:, p.col :], batch.slot, batch.pos, B), 2 * kvb, 0)
+                    add("attention", which, lambda L, o: o[i].prompt(y[:, p.col :], out, *batch.blocks[o[i].prompt_block(s)], gate=gate),
+                        kvb + 4 * B * s.heads * s.dim, fl)
+                else:
+                    add("norm, append, attention", which, lambda L, o: o[i].rows(y[:, p.col :], out, batch.slot, batch.pos, B, batch.keys,
+                                                                                append=True, gate=gate), kvb, fl)
+                continue
+            h, grp, d, e = s.core
+            ins = 2 * (s.channels if hasattr(s, "channels") else h * (2 * d + e))
+            part = "state space" if hasattr(s, "channels") else "linear attention"
+            state = 8 * h * d * e * (1 if prompt else B)
+            # at least: inputs and outputs once, the state in and out; two products with it per token
+            add(f"{part}: recurrence", which, lambda L, o: L.parts[i]._recur(o[i], bf, batch, h * d if part[0] == "l" else h, part[0] == "s"),
+                B * (ins + 4 * h * e) + state, 4 * B * h * d * e)
+            z = y[:, p.col :] if part[0] == "s" else y[:, p.col + 2 * h * d + h * e :]
+            ro, oo = bf.f32("recur", h * e), bf.mixed("recur_out", h * e)
+            add(f"{part}: gated norm", which, lambda L, o: D.gated_norm(ro, z, L.parts[i].norm, oo, B, h * e, s.norm_groups if part[0] == "s" else h,
+                                                                       eps, part[0] == "s"), B * h * e * 8, 0)
+        if len(L0.parts) == 1:
+            add(f"{name}: o", which, lambda L, o: D.linear(bf.mixed("recur_out", L.parts[0].width), L.parts[0].o, bf.branch, B),
+                *mm(H, L0.parts[0].width))
+        else:
+            a, b = L0.parts[0].width, L0.parts[1].width
+            nb, fl = mm(H, a + b)
+            add(f"{name}: both o", which, lambda L, o: D.linear_pair(bf.mixed("attn", a), L.parts[0].o, bf.branch, bf.mixed("recur_out", b),
+                                                                    L.parts[1].o, bf.branch2, B), nb, fl)
+    if not fused:
+        add("norms + residual", lin, lambda L, o: D.post_norm_add(due(L, False), eps, bf.h, bf.xb, B, L.pre2), B * H * 14, 0)
+        add("norms of two branches + residual", par, lambda L, o: D.post_norm_add(due(L, True), eps, bf.h, bf.xb, B, L.pre2), B * H * 18, 0)
+    f = c.layers[0].mlp
+    act = bf.mixed("ff", f.ff)
+    add(f"{head}gate, up", every, lambda L, o: product(L, L.ff.gate, act, len(L.parts) > 1, up=L.ff.up, spec=f), *mm(2 * f.ff, H))
+    add("down", every, lambda L, o: D.linear(act, L.ff.down, bf.branch, B), *mm(H, f.ff))
+    return rows
+
+
+def step_rates(torch, m, args, tag) -> dict:
+    """Whole steps: prompt and decode throughput at batch 1, 4, 8 and 16."""
+    from exo_amd.generate import prefill
+
+    g = torch.Generator().manual_seed(1234)
+    out = dict(weights_GB=round(m.weight_bytes() / 1e9, 2))
+    prompt = torch.randint(0, m.cfg.vocab_size, (args.prompt,), generator=g).tolist()
+    for B in (1, 4, 8, 16):
+        cache = m.make_cache(B, args.prompt + args.steps + args.warmup + 64)
+        for row in range(B):
+            if row < 2:  # (the second time is the timed one: buffers and code objects are there)
+                for _ in range(2):
+                    cache.reset(rows=range(row, row + 1))
+                    tps, n = prefill(m, prompt, cache, row=row, faithful_extra_steps=False)
+                out["prefill_tok_s"], out["prefill_tokens"] = round(tps), n
+            else:
+                prefill(m, prompt, cache, row=row, faithful_extra_steps=False)
+        bufs = m._buffers(B, 1)
+        bufs.tokens.fill_(1)
+        for _ in range(max(args.warmup, 1)):
+            m.decode_step(cache, B, feedback=True)
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        for _ in range(args.steps):
+            m.decode_step(cache, B, feedback=True)
+        torch.cuda.synchronize()
+        dt = (time.perf_counter() - t0) / args.steps
+        out[f"decode_tok_s_b{B}"], out[f"us_per_step_b{B}"] = round(B / dt, 1), round(dt * 1e6, 1)
+        print(f"[bench] {tag} batch {B}: {dt * 1e6:.0f} us/step, prompt {out['prefill_tok_s']} tok/s", file=sys.stderr, flush=True)
+        m._graphs.clear()
+        del cache
+    return out
+
+
+def stack_workload(args):
+    """A layer-list design beside the closest other model of equal size."""
     import torch
 
     from exo_amd import native
-    from exo_amd.generate import prefill
 
     native.load()
     torch.cuda.set_device(0)
+    kinds = {"gekazen": (lambda size, name: gekazen_model(torch, size, 4096), gekazen_launches),
+             "novosun": (lambda size, name: novosun_model(torch, size, NOVOSUN_SIZES[name]), novosun_launches),
+             "qwen3_moe": (lambda size, name: qwen_model(torch, size), qwen_launches)}
+    pair = ("gekazen", "qwen3_moe") if args.workload == "gekazen" else ("novosun", "gekazen")
     report = {}
-    for name in (GEKAZEN_SIZES if args.gekazen_size == "all" else [args.gekazen_size]):
+    for name in (GEKAZEN_SIZES if args.size == "all" else [args.size]):
         size, res = GEKAZEN_SIZES[name], {}
-        for kind in ("gekazen", "qwen3_moe"):
-            m = gekazen_model(torch, size, 4096) if kind == "gekazen" else qwen_model(torch, size)
-            g = torch.Generator().manual_seed(1234)
-            out = res[kind] = dict(weights_GB=round(m.weight_bytes() / 1e9, 2))
-            prompt = torch.randint(0, m.cfg.vocab_size, (args.prompt,), generator=g).tolist()
-            for B in (1, 4, 8, 16):
-                cache = m.make_cache(B, args.prompt + args.steps + args.warmup + 64)
-                for row in range(B):
-                    if row < 2:  # (the second time is the timed one: buffers and code objects are there)
-                        for _ in range(2):
-                            cache.reset(rows=range(row, row + 1))
-                            tps, n = prefill(m, prompt, cache, row=row, faithful_extra_steps=False)
-                        out["prefill_tok_s"], out["prefill_tokens"] = round(tps), n
-                    else:
-                        prefill(m, prompt, cache, row=row, faithful_extra_steps=False)
-                bufs = m._buffers(B, 1)
-                bufs.tokens.fill_(1)
-                for _ in range(max(args.warmup, 1)):
-                    m.decode_step(cache, B, feedback=True)
-                torch.cuda.synchronize()
-                t0 = time.perf_counter()
-                for _ in range(args.steps):
-                    m.decode_step(cache, B, feedback=True)
-                torch.cuda.synchronize()
-                dt = (time.perf_counter() - t0) / args.steps
-                out[f"decode_tok_s_b{B}"], out[f"us_per_step_b{B}"] = round(B / dt, 1), round(dt * 1e6, 1)
-                print(f"[gekazen] {name} {kind} batch {B}: {dt * 1e6:.0f} us/step, prompt {out['prefill_tok_s']} tok/s",
-                      file=sys.stderr, flush=True)
-                m._graphs.clear()
-                del cache
-            launches = gekazen_launches if kind == "gekazen" else qwen_launches
+        for kind in pair:
+            build, launches = kinds[kind]
+            m = build(size, name)
+            out = res[kind] = step_rates(torch, m, args, f"{name} {kind}")
             for B in (1, 8, args.prompt):
                 out[f"launches_{B}_rows"] = launches(torch, m, B, args.prompt)
                 for r in out[f"launches_{B}_rows"]:
-                    print(f"[gekazen] {name} {kind} rows {B}: {r}", file=sys.stderr, flush=True)
-            del m, bufs
+                    print(f"[bench] {name} {kind} rows {B}: {r}", file=sys.stderr, flush=True)
+            del m
             torch.cuda.empty_cache()
         report[name] = res
-    first = next(iter(report.values()))["gekazen"]
+    first = next(iter(report.values()))[pair[0]]
+    sizes = {k: GEKAZEN_SIZES[k] if args.workload == "gekazen" else GEKAZEN_SIZES[k] + NOVOSUN_SIZES[k] for k in report}
     print(json.dumps({
-        "metric": "decode tok/s, Gekazen design, batch 1", "value": first["decode_tok_s_b1"], "unit": "tok/s", "n_gpus": 1,
-        "steps": args.steps, "warmup": args.warmup, "ms_per_step": first["us_per_step_b1"] * 1e-3, "higher_is_better": True,
-        "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
-        "config": {"workload": f"Gekazen layers of real size, random weights, context {args.prompt}, beside a Qwen3-MoE of equal "
-                               "size (quantised); x = launch time over its roofline", "sizes": {k: GEKAZEN_SIZES[k] for k in report}},
+        "metric": f"decode tok/s, {pair[0].capitalize()} design, batch 1", "value": first["decode_tok_s_b1"], "unit": "tok/s",
+        "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "ms_per_step": first["us_per_step_b1"] * 1e-3,
+        "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": f"{pair[0].capitalize()} layers of real size, random weights, context {args.prompt}, beside a "
+                               f"{pair[1]} of equal size; x = launch time over its roofline", "sizes": sizes},
         "results": report}))
 
 
@@ -701,8 +871,8 @@ def main():
         sys.exit(2)
     if args.workload == "qmatmul_sweep":
         return qmatmul_sweep(args)
-    if args.workload == "gekazen":
-        return gekazen_workload(args)
+    if args.workload in ("gekazen", "novosun"):
+        return stack_workload(args)
     import torch
 
     from exo_amd import native

@@ -11,27 +11,39 @@
 // sequence at position 0 starts from zero whatever its slot holds.
 //
 // Single tokens: recur_step_kernel does it all, a workgroup per (row, head, range of value columns).
-// Portions of prompts, cut into chunks of 64 tokens, c_t = sum of the logarithms of the decays of the
-// chunk's tokens up to t (every exponent below is <= 0):
-//   recur_prep_*    c, dt, and the convolved inputs
-//   recur_state     per chunk  U = sum_t exp(c_end - c_t) k_t v_t^T
-//   recur_scores    per chunk  A[i][j] = sum_d q_i k_j exp(c_i - c_j), j <= i; decay per head: q_i . k_j
-//   recur_scan      per portion, elementwise over the state: U <- state ahead of the chunk; the end state
-//   recur_out       per chunk  o_i = exp(c_i) q_i S + sum_j A[i][j] v_j (+ D v_i)
+// Portions of prompts, cut into chunks of 64 tokens, c_t = sum of the binary logarithms of the decays of
+// the chunk's tokens up to t (every exponent below is <= 0):
+//   recur_prep / recur_conv   c, dt, and the convolved inputs
+//   recur_scores  per chunk   A[i][j] = sum_d q_i k_j 2^(c_i - c_j), j <= i; decay per head: q_i . k_j
+//   recur_carry   per portion, tiles of the state in registers: leaves the state ahead of every chunk,
+//                             S <- 2^c_end S + sum_t 2^(c_end - c_t) k_t v_t^T
+//   recur_out     per chunk   o_i = 2^c_i q_i S + sum_j A[i][j] v_j (+ D v_i)
 // A decay per channel does not factor out of a score without overflow, so its scores are formed for
 // 16-token blocks: between blocks both factors are taken to the query block's start, inside a block
-// each pair has its own exponentials.
+// each pair has its own exponentials.  That launch also leaves 2^c q and, transposed, 2^(c_end - c) k as
+// matrix operands; recur_carry leaves the states as operands too (value columns x keys).
 #include "../../include/exo_mi355x.h"
 #include "dense.h"
 
 namespace {
 
+typedef __attribute__((__vector_size__(4 * sizeof(int)))) int int4v;
+
 constexpr int kChunk = 64;
 constexpr int kRec = 8;  // ints of a chunk's record: row, cache row, position, tokens, portion's first position
 
-typedef exo_recurrence Rec;
+// the arguments and where the parts of the workspace lie
+struct Rec : exo_recurrence {
+  float* scores;         // [chunk][group][64][64]
+  void* states;          // T [terms][chunk][head][lds][dp]: the state ahead of a chunk, value columns x keys
+  void *qhat, *khat;     // decay per channel: T [terms][chunk][head][64][dp], [terms][chunk][head][dp][64]
+  size_t nstates, nhat;  // elements of a term
+  int dp;                // dim rounded up to 64, zeros behind dim
+};
 
 __device__ __forceinline__ float softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+constexpr float kLog2e = 1.4426950408889634f;
+__device__ __forceinline__ float pow2(float x) { return __builtin_amdgcn_exp2f(x); }
 __device__ __forceinline__ float sigmoidf(float z) { return 1.f / (1.f + expf(-z)); }
 
 template <typename T>
@@ -61,6 +73,26 @@ struct Split<float> {
   uint4 hi;
   __device__ __forceinline__ void set(const float (&f)[4]) { hi = __builtin_bit_cast(uint4, floatx4{f[0], f[1], f[2], f[3]}); }
 };
+// its value term from p, the remainder term (bf16) n elements behind
+template <typename T>
+__device__ __forceinline__ Split<T> split_at(const void* p, size_t at, size_t n) {
+  Split<T> s;
+  s.hi = *reinterpret_cast<const uint4*>(reinterpret_cast<const T*>(p) + at);
+  if constexpr (sizeof(T) == 2) s.lo = *reinterpret_cast<const uint4*>(reinterpret_cast<const T*>(p) + n + at);
+  return s;
+}
+// four consecutive elements of such an operand
+template <typename T>
+__device__ __forceinline__ void split_store(void* p, size_t at, size_t n, const float (&f)[4]) {
+  if constexpr (sizeof(T) == 2) {
+    const uint32_t h0 = pack_bf2(f[0], f[1]), h1 = pack_bf2(f[2], f[3]);
+    *reinterpret_cast<uint2*>(reinterpret_cast<T*>(p) + at) = uint2{h0, h1};
+    *reinterpret_cast<uint2*>(reinterpret_cast<T*>(p) + n + at) =
+        uint2{pack_bf2(f[0] - bf_lo(h0), f[1] - bf_hi(h0)), pack_bf2(f[2] - bf_lo(h1), f[3] - bf_hi(h1))};
+  } else {
+    *reinterpret_cast<floatx4*>(reinterpret_cast<T*>(p) + at) = floatx4{f[0], f[1], f[2], f[3]};
+  }
+}
 template <typename T>
 __device__ __forceinline__ floatx4 mma(const Split<T>& a, const uint4& b, floatx4 c) {
   if constexpr (sizeof(T) == 2) c = Elem<T>::mma16(a.lo, b, c);
@@ -139,10 +171,11 @@ __global__ __launch_bounds__(256) void recur_prep_channel_kernel(const Rec p) {
         for (int e = 0; e < 4; ++e) acc[t] = fmaf(w[j + e], l[e], acc[t]);
       }
   }
+  const float scale = p.inv_tau * kLog2e;
   float sum = 0.f;
 #pragma unroll
   for (int t = 0; t < kSeg; ++t) {
-    sum -= softplus(-acc[t]) * p.inv_tau;
+    sum -= softplus(-acc[t]) * scale;
     acc[t] = sum;
   }
   total[wave][lane] = sum;
@@ -156,32 +189,36 @@ __global__ __launch_bounds__(256) void recur_prep_channel_kernel(const Rec p) {
 }
 
 // c and dt per head: a wave per head, a lane per token
-__global__ __launch_bounds__(256) void recur_prep_head_kernel(const Rec p) {
-  const Chunk ck(p.chunks, blockIdx.x);
-  const int lane = threadIdx.x & 63, h = blockIdx.y * 4 + (threadIdx.x >> 6);
+__device__ __forceinline__ void prep_heads(const Rec& p, const Chunk& ck, int h) {
+  const int lane = threadIdx.x & 63;
   if (h >= p.heads) return;
   const bool on = lane < ck.n;
   const size_t row = (size_t)ck.row + min(lane, ck.n - 1);
   const float dt = softplus(p.dt_raw[row * p.lddt + h] + p.dt_bias[h]);
-  float s = on ? -p.decay_rate[h] * dt : 0.f;
+  float s = on ? -p.decay_rate[h] * dt * kLog2e : 0.f;
 #pragma unroll
   for (int o = 1; o < 64; o *= 2) {
     const float u = __shfl_up(s, o, 64);
     if (lane >= o) s += u;
   }
   if (on) {
-    p.cum[row * p.ldcum + h] = s;
-    p.dt[row * p.ldcum + h] = dt;
+    p.cum[(size_t)h * p.ldcum + row] = s;
+    p.dt[(size_t)h * p.ldcum + row] = dt;
   }
 }
 
-// causal convolution per channel and silu, 16 tokens per thread
+// causal convolution per channel and silu, 16 tokens per thread; the last rows of workgroups: prep_heads
 constexpr int kConvTokens = 16;
 
 template <typename T, int TM>
 __global__ __launch_bounds__(256) void recur_conv_kernel(const Rec p) {
   const Chunk ck(p.chunks, blockIdx.x / (kChunk / kConvTokens));
-  const int t0 = (blockIdx.x % (kChunk / kConvTokens)) * kConvTokens, c = blockIdx.y * 256 + threadIdx.x;
+  const int part = blockIdx.x % (kChunk / kConvTokens), t0 = part * kConvTokens, c = blockIdx.y * 256 + threadIdx.x;
+  const int conv_rows = (p.channels + 255) / 256;
+  if ((int)blockIdx.y >= conv_rows) {
+    prep_heads(p, ck, (((int)blockIdx.y - conv_rows) * (kChunk / kConvTokens) + part) * 4 + (threadIdx.x >> 6));
+    return;
+  }
   if (t0 >= ck.n || c >= p.channels) return;
   float w[TM], x[TM];  // the latest TM inputs, oldest first (taps < TM: zero weights in front)
 #pragma unroll
@@ -221,83 +258,43 @@ __global__ __launch_bounds__(256) void recur_conv_kernel(const Rec p) {
 template <typename T>
 constexpr int kVStride = kChunk + 16 / (int)sizeof(T);
 
+// one element, as the bits of the low half or of a whole register
 template <typename T>
-__device__ __forceinline__ void stage_values(const Rec& p, const Chunk& ck, int h, int e0, T* vt, int tid) {
-  const int q = (tid & 15) * 4, t0 = (tid >> 4) * 4;
-  struct alignas(4 * sizeof(T)) Quad {
-    T e[4];
-  };
-  Quad in[4];
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int t = t0 + i;
-    load_n<T, 4>(as<T>(p.v) + (size_t)(ck.row + min(t, ck.n - 1)) * p.ldv + h * p.vdim + e0 + q, in[i].e, p.v_vec != 0,
-                 t < ck.n ? p.vdim - e0 - q : 0);
-  }
-#pragma unroll
-  for (int e = 0; e < 4; ++e) {
-    Quad out;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) out.e[i] = in[i].e[e];
-    *reinterpret_cast<Quad*>(vt + (q + e) * kVStride<T> + t0) = out;
-  }
+__device__ __forceinline__ uint32_t raw_one(__amdgpu_buffer_rsrc_t rs, uint32_t voff, uint32_t soff) {
+  if constexpr (sizeof(T) == 2)
+    return __builtin_amdgcn_raw_buffer_load_b16(rs, voff, soff, 0);
+  else
+    return __builtin_amdgcn_raw_buffer_load_b32(rs, voff, soff, 0);
 }
-
-// 64 channels x 64 value columns of a chunk's own contribution to the state
-template <typename T, bool CHANNEL>
-__global__ __launch_bounds__(256) void recur_state_kernel(const Rec p) {
-  constexpr int KV = Elem<T>::kVec;
-  __shared__ __attribute__((aligned(16))) T vt[64 * kVStride<T>];
-  __shared__ float wt[kChunk];
-  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int r = lane & 15, g = lane >> 4;
-  const Chunk ck(p.chunks, blockIdx.x);
-  const int h = blockIdx.y, gk = h / (p.heads / p.groups);
-  const int ne = (p.lds + 63) / 64, e0 = ((int)blockIdx.z % ne) * 64, d0 = ((int)blockIdx.z / ne) * 64;
-  stage_values<T>(p, ck, h, e0, vt, tid);
-  const size_t last = (size_t)(ck.row + ck.n - 1) * p.ldcum;
-  if (!CHANNEL && tid < kChunk) {
-    const size_t at = (size_t)(ck.row + min(tid, ck.n - 1)) * p.ldcum + h;
-    wt[tid] = tid < ck.n ? expf(p.cum[last + h] - p.cum[at]) * p.dt[at] : 0.f;
-  }
-  __syncthreads();
-  const int d = d0 + wave * 16 + r;
-  const bool on = d < p.dim;
-  const int dc = min(d, p.dim - 1);
-  const float cend = CHANNEL ? p.cum[last + h * p.dim + dc] : 0.f;
-  const T* kp = as<T>(p.k) + (size_t)ck.row * p.ldk + gk * p.dim + dc;
-  const float* cp = p.cum + (size_t)ck.row * p.ldcum + h * p.dim + dc;
-  floatx4 acc[4];
+// four value (or key) columns of a token on their way to LDS.  VEC: whole 8- or 16-byte loads through a range-
+// checked buffer, so that nothing branches and nothing is waited for before the columns are used.
+template <typename T, bool VEC>
+struct Quad4 {
+  uint32_t w[VEC ? (int)sizeof(T) : 4];
+  // voff: the thread's place (kPastEnd: none), soff: the same for all
+  __device__ __forceinline__ void request(__amdgpu_buffer_rsrc_t rv, uint32_t voff, uint32_t soff, int left) {
+    if constexpr (VEC) {
+      if constexpr (sizeof(T) == 2) {
+        const uint2 v = __builtin_bit_cast(uint2, __builtin_amdgcn_raw_buffer_load_b64(rv, voff, soff, 0));
+        w[0] = v.x, w[1] = v.y;
+      } else {
+        const uint4 v = buf_load16(rv, voff, soff);
+        w[0] = v.x, w[1] = v.y, w[2] = v.z, w[3] = v.w;
+      }
+    } else {
 #pragma unroll
-  for (int j = 0; j < 4; ++j) acc[j] = floatx4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-  for (int s = 0; s < kChunk; s += 4 * KV) {
-    if (s >= ck.n) break;
-    float f[KV];
-#pragma unroll
-    for (int e = 0; e < KV; ++e) {
-      const int t = s + g * KV + e, tc = min(t, ck.n - 1);
-      const float k = Elem<T>::load(kp[(size_t)tc * p.ldk]);
-      const float w = CHANNEL ? expf(cend - cp[(size_t)tc * p.ldcum]) : wt[t];
-      f[e] = on && t < ck.n ? k * w : 0.f;
-    }
-    Split<T> a;
-    a.set(f);
-#pragma unroll
-    for (int j = 0; j < 4; ++j)
-      acc[j] = mma<T>(a, *reinterpret_cast<const uint4*>(vt + (j * 16 + r) * kVStride<T> + s + g * KV), acc[j]);
-  }
-  float* u = p.chunk_state + ((size_t)blockIdx.x * p.heads + h) * p.dim * p.lds;
-#pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int col = e0 + j * 16 + r;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int dd = d0 + wave * 16 + 4 * g + e;
-      if (dd < p.dim && col < p.lds) u[(size_t)dd * p.lds + col] = acc[j][e];
+      for (int e = 0; e < 4; ++e) w[e] = raw_one<T>(rv, e < left ? voff + e * (uint32_t)sizeof(T) : kPastEnd, soff);
     }
   }
-}
+  __device__ __forceinline__ T at(int e) const {
+    if constexpr (VEC && sizeof(T) == 2)
+      return T(w[e / 2] >> (16 * (e & 1)));
+    else if constexpr (sizeof(T) == 2)
+      return T(w[e]);
+    else
+      return __builtin_bit_cast(T, w[e]);
+  }
+};
 
 // scores of a chunk, decay per head: the plain products of a group's queries and keys
 template <typename T>
@@ -337,224 +334,414 @@ __global__ __launch_bounds__(256) void recur_scores_head_kernel(const Rec p) {
     }
 }
 
-// scores of a chunk, decay per key channel (queries and keys per head); 64 channels at a time in LDS
+// scores of 16 queries of a chunk, decay per key channel (queries and keys per head); 64 channels at a
+// time in LDS.  Wave j takes the keys of block j ahead of the queries' own; that one is dealt out over
+// the waves by channels.
 template <typename T>
 __global__ __launch_bounds__(256) void recur_scores_channel_kernel(const Rec p) {
   constexpr int KV = Elem<T>::kVec, ST = 68;
-  __shared__ __attribute__((aligned(16))) float qs[kChunk][ST], ks[kChunk][ST], cs[kChunk][ST];
+  __shared__ __attribute__((aligned(16))) float qs[16][ST], ks[kChunk][ST], cs[kChunk][ST];
+  __shared__ float part[4][256];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r = lane & 15, g = lane >> 4;
   const Chunk ck(p.chunks, blockIdx.x);
-  const int h = blockIdx.y, i0 = wave * 16;
-  floatx4 acc[4];
+  const int h = blockIdx.y, block = 3 - (int)blockIdx.z, i0 = block * 16;  // (the longest first)
+  if (i0 >= ck.n) return;
+  floatx4 acc = {0.f, 0.f, 0.f, 0.f};
+  float own[4] = {0.f, 0.f, 0.f, 0.f};
+  T kr[16], qr[4];
+  float cr[16];
+  auto request = [&](int d) {
+    const int dc = h * p.dim + min(d, p.dim - 1);
 #pragma unroll
-  for (int j = 0; j < 4; ++j) acc[j] = floatx4{0.f, 0.f, 0.f, 0.f};
-  for (int d0 = 0; d0 < p.dim; d0 += 64) {
-    __syncthreads();
-    {
-      const int c = lane, d = d0 + c;
-      const bool on = d < p.dim;
-#pragma unroll 4
-      for (int t = wave; t < kChunk; t += 4) {
-        const bool live = on && t < ck.n;
-        const size_t row = (size_t)ck.row + t;
-        qs[t][c] = live ? Elem<T>::load(as<T>(p.q)[row * p.ldq + h * p.dim + d]) * p.q_scale : 0.f;
-        ks[t][c] = live ? Elem<T>::load(as<T>(p.k)[row * p.ldk + h * p.dim + d]) : 0.f;
-        cs[t][c] = live ? p.cum[row * p.ldcum + h * p.dim + d] : 0.f;
-      }
+    for (int j = 0; j < 16; ++j) {
+      const size_t row = (size_t)ck.row + min(min(wave + 4 * j, i0 + 15), ck.n - 1);
+      kr[j] = as<T>(p.k)[row * p.ldk + dc];
+      cr[j] = p.cum[row * p.ldcum + dc];
     }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) qr[j] = as<T>(p.q)[((size_t)ck.row + min(i0 + wave + 4 * j, ck.n - 1)) * p.ldq + dc];
+  };
+  request(lane);
+  for (int d0 = 0; d0 < p.dim; d0 += 64) {
+    const bool on = d0 + lane < p.dim;
+    __syncthreads();  // (the channels before have been read)
+#pragma unroll
+    for (int j = 0; j < 16; ++j)
+    {
+      ks[wave + 4 * j][lane] = on ? Elem<T>::load(kr[j]) : 0.f;
+      cs[wave + 4 * j][lane] = on ? cr[j] : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) qs[wave + 4 * j][lane] = on ? Elem<T>::load(qr[j]) * p.q_scale : 0.f;
     __syncthreads();
-    if (i0 >= ck.n) continue;
-    const int db = min(64, p.dim - d0);
-    // earlier blocks: both factors relative to the last token ahead of this wave's queries
-    if (wave > 0) {
-      for (int s = 0; s < db; s += 4 * KV) {
-        const int d = s + g * KV;
-        float base[KV], f[KV];
-        Split<T> a, b;
+    request(min(d0 + 64, p.dim - 1) + lane);
+    {
+      const int i = tid >> 4, c = (tid & 15) * 4;
+      float f[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) f[e] = qs[i][c + e] * pow2(cs[i0 + i][c + e]);
+      split_store<T>(p.qhat, (((size_t)blockIdx.x * p.heads + h) * kChunk + i0 + i) * p.dp + d0 + c, p.nhat, f);
+    }
+    if (i0 + 16 >= ck.n) {  // (the last block has all the keys)
+      const int c = tid >> 2, t0 = (tid & 3) * 16;
+      const float cend = cs[ck.n - 1][c];
+#pragma unroll
+      for (int tk = 0; tk < 16; tk += KV) {
+        float f[KV];
 #pragma unroll
         for (int e = 0; e < KV; ++e) {
-          base[e] = cs[i0 - 1][d + e];
-          f[e] = qs[i0 + r][d + e] * expf(fminf(cs[i0 + r][d + e] - base[e], 0.f));
+          const int t = t0 + tk + e;
+          f[e] = t < ck.n ? ks[t][c] * pow2(cend - cs[t][c]) : 0.f;
         }
-        a.set(f);
+        Split<T> out;
+        out.set(f);
+        T* dst = reinterpret_cast<T*>(p.khat) + (((size_t)blockIdx.x * p.heads + h) * p.dp + d0 + c) * kChunk + t0 + tk;
+        *reinterpret_cast<uint4*>(dst) = out.hi;
+        if constexpr (sizeof(T) == 2) *reinterpret_cast<uint4*>(dst + p.nhat) = out.lo;
+      }
+    }
+    const int db = min(64, p.dim - d0);
+    // an earlier block: both factors relative to the last token ahead of the queries
+    if (wave < block) {
+      for (int s = 0; s < db; s += 4 * KV) {
+        const int dd = s + g * KV;
+        float fa[KV], fb[KV];
 #pragma unroll
-        for (int j = 0; j < 3; ++j)
-          if (j < wave) {
-#pragma unroll
-            for (int e = 0; e < KV; ++e) f[e] = ks[j * 16 + r][d + e] * expf(base[e] - cs[j * 16 + r][d + e]);
-            b.set(f);
-            acc[j] = mma<T>(a, b, acc[j]);
-          }
+        for (int e = 0; e < KV; ++e) {
+          const float base = cs[i0 - 1][dd + e];
+          fa[e] = qs[r][dd + e] * pow2(cs[i0 + r][dd + e] - base);
+          fb[e] = ks[wave * 16 + r][dd + e] * pow2(base - cs[wave * 16 + r][dd + e]);
+        }
+        Split<T> a, b;
+        a.set(fa);
+        b.set(fb);
+        acc = mma<T>(a, b, acc);
       }
     }
     // the own block, pair by pair: lane (g, r) has queries 4g .. 4g + 3 and key r
-    float own[4] = {0.f, 0.f, 0.f, 0.f};
-    for (int d = 0; d < db; d += 4) {
-      const floatx4 k = *reinterpret_cast<const floatx4*>(&ks[i0 + r][d]), c = *reinterpret_cast<const floatx4*>(&cs[i0 + r][d]);
+    for (int dd = wave * 16; dd < min(db, wave * 16 + 16); dd += 4) {
+      const floatx4 k = *reinterpret_cast<const floatx4*>(&ks[i0 + r][dd]), c = *reinterpret_cast<const floatx4*>(&cs[i0 + r][dd]);
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        const floatx4 q = *reinterpret_cast<const floatx4*>(&qs[i0 + 4 * g + e][d]), b = *reinterpret_cast<const floatx4*>(&cs[i0 + 4 * g + e][d]);
+        const floatx4 q = *reinterpret_cast<const floatx4*>(&qs[4 * g + e][dd]), b = *reinterpret_cast<const floatx4*>(&cs[i0 + 4 * g + e][dd]);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) own[e] = fmaf(q[i] * k[i], expf(fminf(b[i] - c[i], 0.f)), own[e]);
+        for (int i = 0; i < 4; ++i) own[e] = fmaf(q[i] * k[i], pow2(fminf(b[i] - c[i], 0.f)), own[e]);
       }
     }
-#pragma unroll
-    for (int j = 0; j < 4; ++j)
-      if (j == wave) {
-#pragma unroll
-        for (int e = 0; e < 4; ++e) acc[j][e] += own[e];
-      }
   }
-  if (i0 >= ck.n) return;
-  float* out = p.scores + ((size_t)blockIdx.x * p.heads + h) * kChunk * kChunk;
 #pragma unroll
-  for (int j = 0; j < 4; ++j)
-    if (j <= wave) {
+  for (int e = 0; e < 4; ++e) part[wave][(4 * g + e) * 16 + r] = own[e];
+  float* out = p.scores + (((size_t)blockIdx.x * p.heads + h) * kChunk + i0) * kChunk;
+  if (wave < block) {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) out[(i0 + 4 * g + e) * kChunk + j * 16 + r] = acc[j][e];
-    }
+    for (int e = 0; e < 4; ++e) out[(4 * g + e) * kChunk + wave * 16 + r] = acc[e];
+  }
+  __syncthreads();
+  out[(tid >> 4) * kChunk + i0 + (tid & 15)] = part[0][tid] + part[1][tid] + part[2][tid] + part[3][tid];
 }
 
-// along a portion's chunks: chunk_state becomes the state ahead of its chunk, the slot gets the last
-// one.  blockIdx.y == heads: the convolution's ring takes the portion's last inputs.
-template <typename T, bool CHANNEL>
-__global__ __launch_bounds__(256) void recur_scan_kernel(const Rec p) {
+// Along a portion's chunks with a tile of the state, 64 keys x (16 NE) value columns, in registers.  One
+// workgroup per CU at most, so the loop is kept short: every address is a thread's fixed offset plus a
+// scalar that steps with the chunk, and the ends of rows and of the portion are the buffers' ends.
+// blockIdx.y == heads: the convolution's ring takes the portion's last inputs.
+template <typename T, bool CHANNEL, int NE, bool VEC>
+__global__ __launch_bounds__(256) void recur_carry_kernel(const Rec p) {
+  constexpr int KV = Elem<T>::kVec, KS = kChunk / (4 * KV), VS = kVStride<T>, EB = sizeof(T), NT = sizeof(T) == 2 ? 2 : 1;
+  __shared__ __attribute__((aligned(16))) T vt[2][16 * NE * VS];
+  __shared__ __attribute__((aligned(16))) T kt[CHANNEL ? 1 : 2][CHANNEL ? 16 : 64 * VS];
+  __shared__ __attribute__((aligned(16))) T sv[2][NT][16 * NE * VS];  // the state on its way out [column][key]
+  __shared__ __attribute__((aligned(16))) float wt[2][kChunk];
   const int32_t* seq = p.seqs + 4 * (size_t)blockIdx.z;
   const int first = seq[0], count = seq[1];
-  const Chunk c0(p.chunks, first);
+  const Chunk c0(p.chunks, first), cl(p.chunks, first + count - 1);
   const int slot = p.map[c0.crow];
   if ((int)blockIdx.y == p.heads) {
-    const int c = blockIdx.x * 256 + threadIdx.x;
-    if (c >= p.channels) return;
-    const Chunk cl(p.chunks, first + count - 1);
     const int end = cl.pos + cl.n;  // one past the last position
-    T* ring = reinterpret_cast<T*>(p.ring) + (size_t)slot * p.taps * p.channels + c;
-    for (int at = max(end - p.taps, c0.pos0); at < end; ++at)
-      ring[(size_t)(at % p.taps) * p.channels] = as<T>(p.raw)[(size_t)(c0.row + at - c0.pos0) * p.ldraw + c];
+    for (int c = blockIdx.x * 256 + threadIdx.x; c < p.channels; c += gridDim.x * 256) {
+      T* ring = reinterpret_cast<T*>(p.ring) + (size_t)slot * p.taps * p.channels + c;
+      for (int at = max(end - p.taps, c0.pos0); at < end; ++at)
+        ring[(size_t)(at % p.taps) * p.channels] = as<T>(p.raw)[(size_t)(c0.row + at - c0.pos0) * p.ldraw + c];
+    }
     return;
   }
-  const int h = blockIdx.y, i = (blockIdx.x * 256 + threadIdx.x) * 4, size = p.dim * p.lds;
-  if (i >= size) return;
-  const int d = i / p.lds;
-  float* st = p.state + ((size_t)slot * p.heads + h) * size + i;
-  floatx4 s = {0.f, 0.f, 0.f, 0.f};
-  if (c0.pos0 > 0) s = *reinterpret_cast<const floatx4*>(st);
-  constexpr int kAhead = 4;
-  for (int b = 0; b < count; b += kAhead) {
-    floatx4 u[kAhead];
-    float e[kAhead];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int h = blockIdx.y, gk = h / (p.heads / p.groups), ne = (p.lds + 16 * NE - 1) / (16 * NE);
+  const int e0 = ((int)blockIdx.x % ne) * 16 * NE, d0 = ((int)blockIdx.x / ne) * 64 + wave * 16;
+  const int total = cl.row + cl.n - c0.row;  // tokens: a portion's chunks lie one behind the other
+  // the state tile: lane (g, r) has keys d0 + 4g .. + 3 of column r
+  floatx4 s[NE];
+  float* st = p.state + ((size_t)slot * p.heads + h) * p.dim * p.lds;
 #pragma unroll
-    for (int j = 0; j < kAhead; ++j) {
-      const int ci = first + min(b + j, count - 1);
-      const Chunk ck(p.chunks, ci);
-      u[j] = *reinterpret_cast<const floatx4*>(p.chunk_state + ((size_t)ci * p.heads + h) * size + i);
-      e[j] = p.cum[(size_t)(ck.row + ck.n - 1) * p.ldcum + (CHANNEL ? h * p.dim + d : h)];
+  for (int j = 0; j < NE; ++j)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int d = d0 + 4 * g + e, col = e0 + j * 16 + r;
+      s[j][e] = c0.pos0 > 0 && d < p.dim && col < p.lds ? st[(size_t)d * p.lds + col] : 0.f;
+    }
+  // ---- where a chunk's parts lie
+  constexpr int CQ = 4 * NE, TP = kChunk * CQ / 256;  // quads of columns, tokens per thread
+  const int q = (tid % CQ) * 4, t0 = (tid / CQ) * TP;
+  auto rows = [&](const void* base, int ld, int bytes) {  // the portion's rows of a matrix, from its first
+    return buf_of(reinterpret_cast<const char*>(base) + (size_t)c0.row * ld * bytes, (uint32_t)total * ld * bytes);
+  };
+  const __amdgpu_buffer_rsrc_t rv = rows(p.v, p.ldv, EB), rk = rows(p.k, p.ldk, EB);
+  const size_t mine = (size_t)h * p.ldcum + c0.row;  // decay per head: a head's tokens in a run
+  const __amdgpu_buffer_rsrc_t rc = CHANNEL ? rows(p.cum, p.ldcum, 4) : buf_of(p.cum + mine, total * 4u),
+                               rd = CHANNEL ? rc : buf_of(p.dt + mine, total * 4u);
+  uint32_t voff[TP], koff[4];
+#pragma unroll
+  for (int k = 0; k < TP; ++k)
+    voff[k] = e0 + q < p.vdim ? ((uint32_t)(t0 + k) * p.ldv + h * p.vdim + e0 + q) * EB : kPastEnd;
+  const int kq = (tid & 15) * 4, kt0 = (tid >> 4) * 4, dq = ((int)blockIdx.x / ne) * 64 + kq;  // decay per head: the keys
+#pragma unroll
+  for (int k = 0; k < 4; ++k) koff[k] = dq < p.dim ? ((uint32_t)(kt0 + k) * p.ldk + gk * p.dim + dq) * EB : kPastEnd;
+  const uint32_t cstep = (uint32_t)p.heads * p.dp * kChunk * EB;  // khat, per chunk
+  const __amdgpu_buffer_rsrc_t rh = buf_of(as<T>(p.khat) + ((size_t)first * p.heads + h) * p.dp * kChunk, CHANNEL ? count * cstep : 0u);
+  const __amdgpu_buffer_rsrc_t rl =
+      buf_of(as<T>(p.khat) + p.nhat + ((size_t)first * p.heads + h) * p.dp * kChunk, CHANNEL ? count * cstep : 0u);
+  const uint32_t hoff = ((uint32_t)(d0 + r) * kChunk + g * KV) * EB;
+  const uint32_t eoff = (h * p.dim + d0 + 4 * g) * 4u, woff = lane * 4u;
+  const uint32_t sstep = (uint32_t)p.heads * p.lds * p.dp * EB;  // states, per chunk
+  const __amdgpu_buffer_rsrc_t sh = buf_of(as<T>(p.states) + ((size_t)first * p.heads + h) * p.lds * p.dp, count * sstep);
+  const __amdgpu_buffer_rsrc_t sl = buf_of(as<T>(p.states) + p.nstates + ((size_t)first * p.heads + h) * p.lds * p.dp, count * sstep);
+  // 16-byte pieces of the tile's columns, 64 keys each: whole lines
+  constexpr int PIECES = kChunk / KV, SP = 16 * NE * PIECES / 256;  // per column, per thread
+  uint32_t soff[SP];
+#pragma unroll
+  for (int k = 0; k < SP; ++k) {
+    const int col = (tid + 256 * k) / PIECES, piece = (tid + 256 * k) % PIECES;
+    soff[k] = e0 + col < p.lds ? ((uint32_t)(e0 + col) * p.dp + ((int)blockIdx.x / ne) * 64 + piece * KV) * EB : kPastEnd;
+  }
+
+  struct Request {
+    Quad4<T, VEC> vin[TP];
+    Split<T> kh[CHANNEL ? KS : 1];
+    Quad4<T, VEC> kin[CHANNEL ? 1 : 4];
+    floatx4 end;
+    float w_c, w_end, w_dt;
+  };
+  constexpr int AHEAD = VEC ? 4 : 2;  // (at most 63 loads and stores can be told apart)
+  Request rq[AHEAD];
+  // Requests past the last chunk re-read it: every load is unconditional, so the waits count exactly
+  // the loads in front of the ones they are for.
+  auto request = [&](Request& q_, int i_) {
+    const int i = min(i_, count - 1);
+    const uint32_t row = i * kChunk, last = min(row + kChunk, (uint32_t)total) - 1;
+#pragma unroll
+    for (int k = 0; k < TP; ++k) q_.vin[k].request(rv, voff[k], row * p.ldv * EB, p.vdim - e0 - q);
+    if constexpr (CHANNEL) {
+#pragma unroll
+      for (int k = 0; k < KS; ++k) {
+        q_.kh[k].hi = buf_load16(rh, hoff + k * 4 * KV * EB, i * cstep);
+        if constexpr (sizeof(T) == 2) q_.kh[k].lo = buf_load16(rl, hoff + k * 4 * KV * EB, i * cstep);
+      }
+      q_.end = __builtin_bit_cast(floatx4, buf_load16(rc, eoff, last * p.ldcum * 4));
+    } else {
+#pragma unroll
+      for (int k = 0; k < 4; ++k) q_.kin[k].request(rk, koff[k], row * p.ldk * EB, p.dim - dq);
+      q_.w_end = __builtin_bit_cast(float, __builtin_amdgcn_raw_buffer_load_b32(rc, 0u, last * 4, 0));
+      q_.w_c = __builtin_bit_cast(float, __builtin_amdgcn_raw_buffer_load_b32(rc, woff, row * 4, 0));
+      q_.w_dt = __builtin_bit_cast(float, __builtin_amdgcn_raw_buffer_load_b32(rd, woff, row * 4, 0));  // zero past the end
+    }
+  };
+  auto chunk = [&](Request& q_, int i) {
+    const int b = i & 1;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      struct alignas(TP * sizeof(T)) Run {
+        T t[TP];
+      } out;
+#pragma unroll
+      for (int k = 0; k < TP; ++k) out.t[k] = q_.vin[k].at(e);
+      *reinterpret_cast<Run*>(&vt[b][(q + e) * VS + t0]) = out;
+    }
+    if constexpr (!CHANNEL) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        struct alignas(4 * sizeof(T)) Run {
+          T t[4];
+        } out;
+#pragma unroll
+        for (int k = 0; k < 4; ++k) out.t[k] = q_.kin[k].at(e);
+        *reinterpret_cast<Run*>(&kt[b][(kq + e) * VS + kt0]) = out;
+      }
+      wt[b][lane] = pow2(q_.w_end - q_.w_c) * q_.w_dt;  // (every wave the same)
+    }
+    float f[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) f[e] = pow2(CHANNEL ? q_.end[e] : q_.w_end);
+#pragma unroll
+    for (int j = 0; j < NE; ++j) {
+      const float x[4] = {s[j][0], s[j][1], s[j][2], s[j][3]};
+      split_store<T>(&sv[b][0][0], (j * 16 + r) * VS + wave * 16 + 4 * g, 16 * NE * VS, x);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s[j][e] *= f[e];
+    }
+    __syncthreads();  // this chunk is complete in its buffer; the other one has been read
+#pragma unroll
+    for (int k = 0; k < SP; ++k) {
+      const int at = (tid + 256 * k) / PIECES * VS + (tid + 256 * k) % PIECES * KV;
+      __builtin_amdgcn_raw_buffer_store_b128(__builtin_bit_cast(int4v, *reinterpret_cast<const uint4*>(&sv[b][0][at])), sh, soff[k], i * sstep, 0);
+      if constexpr (sizeof(T) == 2)
+        __builtin_amdgcn_raw_buffer_store_b128(__builtin_bit_cast(int4v, *reinterpret_cast<const uint4*>(&sv[b][NT - 1][at])), sl, soff[k],
+                                               i * sstep, 0);
     }
 #pragma unroll
-    for (int j = 0; j < kAhead; ++j) {
-      if (b + j >= count) break;
-      *reinterpret_cast<floatx4*>(p.chunk_state + ((size_t)(first + b + j) * p.heads + h) * size + i) = s;
-      const float a = expf(e[j]);
+    for (int k = 0; k < KS; ++k) {
+      const int t = k * 4 * KV + g * KV;
+      Split<T> a;
+      if constexpr (CHANNEL) {
+        a = q_.kh[k];
+      } else {
+        float x[KV];
+        unpack_vec<T>(*reinterpret_cast<const uint4*>(&kt[b][(wave * 16 + r) * VS + t]), x);
 #pragma unroll
-      for (int k = 0; k < 4; ++k) s[k] = fmaf(a, s[k], u[j][k]);
+        for (int e = 0; e < KV; ++e) x[e] *= wt[b][t + e];
+        a.set(x);
+      }
+#pragma unroll
+      for (int j = 0; j < NE; ++j) s[j] = mma<T>(a, *reinterpret_cast<const uint4*>(&vt[b][(j * 16 + r) * VS + t]), s[j]);
+    }
+  };
+#pragma unroll
+  for (int u = 0; u < AHEAD; ++u) {
+    request(rq[u], u);
+    __builtin_amdgcn_sched_barrier(0);  // (in this order: the first wait is for the first of them only)
+  }
+  int i = 0;
+  for (; i + AHEAD <= count; i += AHEAD) {  // (no way out in between: a set's registers stay where they are)
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) {
+      chunk(rq[u], i + u);
+      request(rq[u], i + u + AHEAD);
+      __builtin_amdgcn_sched_barrier(0);
     }
   }
-  *reinterpret_cast<floatx4*>(st) = s;
+#pragma unroll
+  for (int u = 0; u < AHEAD - 1; ++u)
+    if (i + u < count) chunk(rq[u], i + u);
+#pragma unroll
+  for (int j = 0; j < NE; ++j)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int d = d0 + 4 * g + e, col = e0 + j * 16 + r;
+      if (d < p.dim && col < p.lds) st[(size_t)d * p.lds + col] = s[j][e];
+    }
 }
 
 // 64 value columns of a chunk's outputs
-template <typename T, bool CHANNEL>
+template <typename T, bool CHANNEL, bool VEC>
 __global__ __launch_bounds__(256) void recur_out_kernel(const Rec p) {
-  constexpr int KV = Elem<T>::kVec, DB = 32, SS = DB + 16 / (int)sizeof(T), NT = sizeof(T) == 2 ? 2 : 1;
+  constexpr int KV = Elem<T>::kVec, NT = sizeof(T) == 2 ? 2 : 1;
   __shared__ __attribute__((aligned(16))) T vt[64 * kVStride<T>];
-  __shared__ __attribute__((aligned(16))) T st[NT][64 * SS];  // state columns [column][key], as (value, remainder)
+  __shared__ __attribute__((aligned(16))) T st[NT][64 * 9 * KV];  // [column][keys], value and remainder
   __shared__ float cl[kChunk], dl[kChunk];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r = lane & 15, g = lane >> 4;
   const Chunk ck(p.chunks, blockIdx.x);
   const int h = blockIdx.y, grp = h / (p.heads / p.groups), e0 = (int)blockIdx.z * 64, i0 = wave * 16;
-  const bool active = i0 < ck.n;
-  stage_values<T>(p, ck, h, e0, vt, tid);
-  if (!CHANNEL && tid < kChunk) {
-    const size_t at = (size_t)(ck.row + min(tid, ck.n - 1)) * p.ldcum + h;
-    cl[tid] = p.cum[at];
-    dl[tid] = p.dt[at];
+  // the values, scores and step sizes are requested ahead of the product with the state
+  const int q4 = (tid & 15) * 4, t0 = (tid >> 4) * 4;
+  const __amdgpu_buffer_rsrc_t rv = buf_of(as<T>(p.v) + (size_t)ck.row * p.ldv, (uint32_t)ck.n * p.ldv * (uint32_t)sizeof(T));
+  Quad4<T, VEC> values[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    values[i].request(rv, e0 + q4 < p.vdim ? ((uint32_t)(t0 + i) * p.ldv + h * p.vdim + e0 + q4) * (uint32_t)sizeof(T) : kPastEnd, 0,
+                      p.vdim - e0 - q4);
+  constexpr int SQ = kChunk / 16;  // quads of scores per lane
+  const float* A = p.scores + ((size_t)blockIdx.x * p.groups + grp) * kChunk * kChunk + (i0 + r) * kChunk;
+  floatx4 sc[SQ];
+#pragma unroll
+  for (int i = 0; i < SQ; ++i) {
+    const int j = (i * 4 / KV) * 4 * KV + g * KV + (i * 4) % KV;
+    sc[i] = *reinterpret_cast<const floatx4*>(A + j);  // (those of later keys are not written: any values)
   }
-  // ---- from the state ahead of the chunk
+  float c_own = 0.f, dt_own = 0.f;
+  if (!CHANNEL) {
+    const size_t at = (size_t)h * p.ldcum + ck.row + min(lane, ck.n - 1);
+    c_own = p.cum[at];
+    dt_own = p.dt[at];
+  }
   floatx4 acc[4];
 #pragma unroll
   for (int j = 0; j < 4; ++j) acc[j] = floatx4{0.f, 0.f, 0.f, 0.f};
-  const float* S = p.chunk_state + ((size_t)blockIdx.x * p.heads + h) * p.dim * p.lds;
-  const bool start = ck.pos == 0;  // (nothing ahead of the sequence's first token)
-  const int lr = ck.row + min(i0 + r, ck.n - 1);
-  const T* qp = as<T>(p.q) + (size_t)lr * p.ldq + grp * p.dim;
-  const float* cp = p.cum + (size_t)lr * p.ldcum + h * p.dim;
-  const int q4 = (tid & 15) * 4, dp = (tid >> 4) * 2;
-  floatx4 in[2];
-  auto load_state = [&](int s) {
+  const size_t head = (size_t)blockIdx.x * p.heads + h;
+  // ---- from the state ahead of the chunk (nothing is ahead of the sequence's first token); 128 bytes of
+  // keys per column at a time through LDS
+  if (ck.pos > 0) {
+    constexpr int DB = 8 * KV, SS = DB + KV;
+    const T* qp = as<T>(p.q) + (size_t)(ck.row + min(i0 + r, ck.n - 1)) * p.ldq + grp * p.dim;
+    const size_t qh = (head * kChunk + i0 + r) * p.dp + g * KV;
+    const int piece = tid & 7, col = tid >> 3;  // 16-byte pieces of columns col and col + 32
+    const T* src[2];
 #pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      in[k] = floatx4{0.f, 0.f, 0.f, 0.f};
-      if (s + dp + k < p.dim && e0 + q4 < p.lds) in[k] = *reinterpret_cast<const floatx4*>(S + (size_t)(s + dp + k) * p.lds + e0 + q4);
-    }
-  };
-  if (!start) load_state(0);
-  for (int s0 = 0; s0 < p.dim && !start; s0 += DB) {
-    __syncthreads();  // (the previous block has been read)
+    for (int k = 0; k < 2; ++k) src[k] = as<T>(p.states) + (head * p.lds + min(e0 + col + 32 * k, p.lds - 1)) * p.dp + piece * KV;
+    Split<T> in[2];
+    auto load_state = [&](int s) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int at = (q4 + e) * SS + dp;
-      if constexpr (sizeof(T) == 2) {
-        const uint32_t hi = pack_bf2(in[0][e], in[1][e]);
-        *reinterpret_cast<uint32_t*>(&st[0][at]) = hi;
-        *reinterpret_cast<uint32_t*>(&st[NT - 1][at]) = pack_bf2(in[0][e] - bf_lo(hi), in[1][e] - bf_hi(hi));
-      } else {
-        st[0][at] = in[0][e];
-        st[0][at + 1] = in[1][e];
+      for (int k = 0; k < 2; ++k) in[k] = split_at<T>(src[k], s, p.nstates);
+    };
+    load_state(0);
+    for (int s0 = 0; s0 < p.dim; s0 += DB) {
+      __syncthreads();  // (the keys before have been read)
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        *reinterpret_cast<uint4*>(&st[0][(col + 32 * k) * SS + piece * KV]) = in[k].hi;
+        if constexpr (sizeof(T) == 2) *reinterpret_cast<uint4*>(&st[NT - 1][(col + 32 * k) * SS + piece * KV]) = in[k].lo;
       }
-    }
-    __syncthreads();
-    if (s0 + DB < p.dim) load_state(s0 + DB);
-    if (!active) continue;
-#pragma unroll
-    for (int s = 0; s < DB; s += 4 * KV) {
-      const int d = s0 + s + g * KV, left = p.dim - d;
+      Split<T> a[2];
       struct alignas(16) Vec {
         T e[KV];
-      } a;
-      load_n<T, KV>(qp + d, a.e, p.qk_vec != 0, left);
-      Split<T> sa;
-      if (CHANNEL) {
-        float f[KV];
+      } raw[2];
 #pragma unroll
-        for (int e = 0; e < KV; ++e) f[e] = e < left ? Elem<T>::load(a.e[e]) * p.q_scale * expf(cp[d + e]) : 0.f;
-        sa.set(f);
-      }
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        Split<T> b;
-        b.hi = *reinterpret_cast<const uint4*>(&st[0][(j * 16 + r) * SS + s + g * KV]);
-        if constexpr (sizeof(T) == 2) b.lo = *reinterpret_cast<const uint4*>(&st[NT - 1][(j * 16 + r) * SS + s + g * KV]);
-        if (CHANNEL)
-          acc[j] = mma<T>(sa, b, acc[j]);
+      for (int u = 0; u < 2; ++u) {
+        const int su = s0 + u * 4 * KV;
+        if constexpr (CHANNEL)
+          a[u] = split_at<T>(p.qhat, qh + su, p.nhat);
         else
-          acc[j] = mma<T>(__builtin_bit_cast(uint4, a), b, acc[j]);
+          load_n<T, KV>(qp + su + g * KV, raw[u].e, VEC, p.dim - su - g * KV);
       }
+      load_state(min(s0 + DB, p.dp - DB));
+      __syncthreads();
+      if (i0 >= ck.n) continue;
+#pragma unroll
+      for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int at = (j * 16 + r) * SS + u * 4 * KV + g * KV;
+          Split<T> b;
+          b.hi = *reinterpret_cast<const uint4*>(&st[0][at]);
+          if constexpr (sizeof(T) == 2) b.lo = *reinterpret_cast<const uint4*>(&st[NT - 1][at]);
+          if constexpr (CHANNEL)
+            acc[j] = mma<T>(a[u], b, acc[j]);
+          else
+            acc[j] = mma<T>(__builtin_bit_cast(uint4, raw[u]), b, acc[j]);
+        }
     }
-  }
-  __syncthreads();
-  if (!active) return;
-  if (!CHANNEL) {
+    if (!CHANNEL) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const float f = expf(cl[i0 + 4 * g + e]) * p.q_scale;
+      for (int e = 0; e < 4; ++e) {
+        const float f = pow2(__shfl(c_own, i0 + 4 * g + e, 64)) * p.q_scale;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) acc[j][e] *= f;
+        for (int j = 0; j < 4; ++j) acc[j][e] *= f;
+      }
     }
   }
   // ---- from the chunk's own tokens
-  const float* A = p.scores + ((size_t)blockIdx.x * p.groups + grp) * kChunk * kChunk + (i0 + r) * kChunk;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    struct alignas(4 * sizeof(T)) Run {
+      T t[4];
+    } out;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) out.t[i] = values[i].at(e);
+    *reinterpret_cast<Run*>(vt + (q4 + e) * kVStride<T> + t0) = out;
+  }
+  if (!CHANNEL && wave == 0) cl[lane] = c_own, dl[lane] = dt_own;
+  __syncthreads();
+  if (i0 >= ck.n) return;
 #pragma unroll
   for (int s = 0; s < kChunk; s += 4 * KV) {
     if (s > i0 + 15) break;
@@ -562,12 +749,11 @@ __global__ __launch_bounds__(256) void recur_out_kernel(const Rec p) {
 #pragma unroll
     for (int e4 = 0; e4 < KV; e4 += 4) {
       const int j = s + g * KV + e4;
-      // (blocks of 16 keys behind the query's own are not written)
-      const floatx4 v = j <= i0 + 15 ? *reinterpret_cast<const floatx4*>(A + j) : floatx4{0.f, 0.f, 0.f, 0.f};
+      const floatx4 v = sc[(s / (4 * KV)) * (KV / 4) + e4 / 4];
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int jj = j + e;
-        const float w = CHANNEL ? 1.f : expf(fminf(cl[i0 + r] - cl[jj], 0.f)) * dl[jj];
+        const float w = CHANNEL ? 1.f : pow2(fminf(cl[i0 + r] - cl[jj], 0.f)) * dl[jj];
         f[e4 + e] = jj <= i0 + r && jj < ck.n ? v[e] * w : 0.f;
       }
     }
@@ -595,24 +781,31 @@ __global__ __launch_bounds__(256) void recur_out_kernel(const Rec p) {
 
 // ------------------------------------------------------------------------------ single tokens
 // One convolved input: the current one from its row, the others from the ring; `keep`: the current one
-// takes its place in the ring.
+// takes its place in the ring (`here` = pos % taps).
 template <typename T>
-__device__ __forceinline__ float conv_one(const Rec& p, int row, int slot, int pos, int c, bool keep) {
+__device__ __forceinline__ float conv_one(const Rec& p, int row, int slot, int pos, int here, int c, bool keep) {
   T* ring = reinterpret_cast<T*>(p.ring) + (size_t)slot * p.taps * p.channels + c;
   const T cur = as<T>(p.raw)[(size_t)row * p.ldraw + c];
   float y = p.conv_b[c];
-  for (int i = 0; i < p.taps - 1; ++i) {
-    const int at = pos - (p.taps - 1) + i;
-    if (at >= 0) y = fmaf(p.conv_w[(size_t)i * p.channels + c], Elem<T>::load(ring[(size_t)(at % p.taps) * p.channels]), y);
+  for (int b0 = 1; b0 < p.taps; b0 += 4) {  // four requests together
+    float w[4], x[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int back = b0 + i, bc = min(back, p.taps - 1), at = here - bc;
+      x[i] = Elem<T>::load(ring[(size_t)(at < 0 ? at + p.taps : at) * p.channels]);
+      w[i] = back < p.taps && pos >= back ? p.conv_w[(size_t)(p.taps - 1 - bc) * p.channels + c] : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) y = fmaf(w[i], x[i], y);
   }
   y = fmaf(p.conv_w[(size_t)(p.taps - 1) * p.channels + c], Elem<T>::load(cur), y);
-  if (keep) ring[(size_t)(pos % p.taps) * p.channels] = cur;
+  if (keep) ring[(size_t)here * p.channels] = cur;
   return Elem<T>::load(Elem<T>::make(y * sigmoidf(y)));
 }
 
 template <typename T, bool CHANNEL>
 __global__ __launch_bounds__(256) void recur_step_kernel(const Rec p, int cols) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];  // q, k, decay [dim]; values [64]; partials [1024]
+  extern __shared__ __attribute__((aligned(16))) float lds[];  // q, k, decay [dim]; values [64]; partials [4][cols]
   const int tid = threadIdx.x, D = p.dim, h = blockIdx.y, e0 = blockIdx.x * cols;
   const int Dp = (D + 3) / 4 * 4;
   float *qs = lds, *ks = qs + Dp, *as_ = ks + Dp, *vs = as_ + Dp, *red = vs + 64;
@@ -641,7 +834,13 @@ __global__ __launch_bounds__(256) void recur_step_kernel(const Rec p, int cols) 
     for (int d = tid; d < D; d += 256) {
       const int c = h * D + d;
       float z = p.decay_b[c];
-      for (int j = 0; j < p.rank; ++j) z = fmaf(p.decay_w[(size_t)j * C + c], low[j], z);
+      for (int j0 = 0; j0 < p.rank; j0 += 16) {  // (16 requests together)
+        float w[16];
+#pragma unroll
+        for (int j = 0; j < 16; ++j) w[j] = p.decay_w[(size_t)min(j0 + j, p.rank - 1) * C + c];
+#pragma unroll
+        for (int j = 0; j < 16; ++j) z = fmaf(w[j], j0 + j < p.rank ? low[j0 + j] : 0.f, z);
+      }
       as_[d] = expf(-softplus(-z) * p.inv_tau);
       qs[d] = Elem<T>::load(as<T>(p.q)[(size_t)row * p.ldq + grp * D + d]) * p.q_scale;
       ks[d] = Elem<T>::load(as<T>(p.k)[(size_t)row * p.ldk + grp * D + d]);
@@ -649,13 +848,20 @@ __global__ __launch_bounds__(256) void recur_step_kernel(const Rec p, int cols) 
     if (tid < cols) vs[tid] = e0 + tid < p.vdim ? Elem<T>::load(as<T>(p.v)[(size_t)row * p.ldv + h * p.vdim + e0 + tid]) : 0.f;
   } else {
     const bool keep = blockIdx.x == 0 && h == grp * hpg;  // a group's keys and queries: one workgroup's to keep
-    for (int d = tid; d < D; d += 256) {
-      ks[d] = conv_one<T>(p, row, slot, pos, p.k_channel + grp * D + d, keep);
-      qs[d] = conv_one<T>(p, row, slot, pos, p.q_channel + grp * D + d, keep) * p.q_scale;
-    }
-    if (tid >= 192 && tid - 192 < cols) {
-      const int e = e0 + tid - 192;
-      vs[tid - 192] = e < p.vdim ? conv_one<T>(p, row, slot, pos, p.v_channel + h * p.vdim + e, true) : 0.f;
+    const int here = pos % p.taps;
+    for (int i = tid; i < 2 * D + cols; i += 256) {  // keys, queries, values
+      if (i < 2 * D) {
+        const bool key = i < D;
+        const int d = key ? i : i - D;
+        const float f = conv_one<T>(p, row, slot, pos, here, (key ? p.k_channel : p.q_channel) + grp * D + d, keep);
+        if (key)
+          ks[d] = f;
+        else
+          qs[d] = f * p.q_scale;
+      } else {
+        const int e = i - 2 * D;
+        vs[e] = e0 + e < p.vdim ? conv_one<T>(p, row, slot, pos, here, p.v_channel + h * p.vdim + e0 + e, true) : 0.f;
+      }
     }
     vscale = softplus(p.dt_raw[(size_t)row * p.lddt + h] + p.dt_bias[h]);
     const float a = expf(-p.decay_rate[h] * vscale);
@@ -681,56 +887,116 @@ __global__ __launch_bounds__(256) void recur_step_kernel(const Rec p, int cols) 
     }
     if (d0 + kAhead * rpp < D) load_state(d0 + kAhead * rpp);
   }
-  *reinterpret_cast<floatx4*>(red + dr * cols + cq) = o;
+  // over the wave's rows (lanes with the same columns), then over the waves
+  for (int step = lpr; step < 64; step *= 2) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] += __shfl_xor(o[e], step, 64);
+  }
+  if ((tid & 63) < lpr) *reinterpret_cast<floatx4*>(red + (tid >> 6) * cols + cq) = o;
   __syncthreads();
   if (tid < cols && e0 + tid < p.vdim) {
     float y = 0.f;
-    for (int i = 0; i < rpp; ++i) y += red[i * cols + tid];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) y += red[i * cols + tid];
     p.y[(size_t)row * p.ldy + h * p.vdim + e0 + tid] = fmaf(skip, vs[tid], y);
   }
 }
 
 // ------------------------------------------------------------------------------ gated norm
 // out = norm of equal parts of y, with the gate silu(z) ahead of the norm or behind it; the gain
-// repeats with `period`.  A team of TEAM threads per part.
-template <typename T, int TEAM>
-__global__ __launch_bounds__(256) void gated_norm_kernel(const exo_gated_norm p, const int32_t* __restrict__ rows) {
-  __shared__ float part[4];
+// repeats with `period`.  TEAM threads per part, each with PASSES runs of VEC columns.
+template <typename T, int TEAM, int BLOCK, int VEC, int PASSES>
+__global__ __launch_bounds__(BLOCK) void gated_norm_kernel(const exo_gated_norm p, const int32_t* __restrict__ rows) {
+  __shared__ float part[BLOCK / 64];
   const int tid = threadIdx.x, team = tid / TEAM, l = tid % TEAM;
-  const int gi = blockIdx.x * (256 / TEAM) + team;
+  const int gi = blockIdx.x * (BLOCK / TEAM) + team;
   const int row = rows ? rows[blockIdx.y] : (int)blockIdx.y;
   const int size = p.width / p.groups;
-  const bool on = gi < p.groups;
-  const float* y = p.y + (size_t)row * p.ldy + (size_t)gi * size;
-  const T* z = as<T>(p.gate) + (size_t)row * p.ldg + (size_t)gi * size;
-  float ss = 0.f;
-  if (on)
-    for (int c = l; c < size; c += TEAM) {
-      float v = y[c];
-      if (p.gate_first) {
-        const float zz = Elem<T>::load(z[c]);
-        v *= zz * sigmoidf(zz);
+  const size_t at = (size_t)min(gi, p.groups - 1) * size;
+  const float* y = p.y + (size_t)row * p.ldy + at;
+  const T* z = as<T>(p.gate) + (size_t)row * p.ldg + at;
+  float v[PASSES][VEC], gate[PASSES][VEC], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < PASSES; ++i) {
+    const int c = (l + i * TEAM) * VEC;
+    T zz[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[i][e] = 0.f, zz[e] = T(0);
+    if (c < size) {
+      if constexpr (VEC == 4) {
+        const floatx4 f = *reinterpret_cast<const floatx4*>(y + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[i][e] = f[e];
+        load_n<T, 4>(z + c, zz, true, 4);
+      } else {
+        v[i][0] = y[c];
+        zz[0] = z[c];
       }
-      ss += v * v;
     }
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      const float f = Elem<T>::load(zz[e]);
+      gate[i][e] = f * sigmoidf(f);
+      if (p.gate_first) v[i][e] *= gate[i][e];
+      ss += v[i][e] * v[i][e];
+    }
+  }
   ss = wave_sum(ss);
-  if (TEAM == 256) {
+  if (TEAM > 64) {
     if ((tid & 63) == 0) part[tid >> 6] = ss;
     __syncthreads();
-    ss = part[0] + part[1] + part[2] + part[3];
+    ss = 0.f;
+#pragma unroll
+    for (int w = 0; w < TEAM / 64; ++w) ss += part[w];
   }
-  if (!on) return;
+  if (gi >= p.groups) return;
   const float inv = 1.f / sqrtf(ss / size + p.eps);
-  T* out = reinterpret_cast<T*>(p.out) + (size_t)row * p.ldo + (size_t)gi * size;
-  for (int c = l; c < size; c += TEAM) {
-    const float zz = Elem<T>::load(z[c]), gate = zz * sigmoidf(zz);
-    const float v = p.gate_first ? y[c] * gate : y[c];
-    const float w = p.gain[(gi * size + c) % p.period];
-    out[c] = Elem<T>::make(p.gate_first ? v * inv * w : v * inv * w * gate);
+  T* out = reinterpret_cast<T*>(p.out) + (size_t)row * p.ldo + at;
+  const int g0 = (int)(at % p.period);
+#pragma unroll
+  for (int i = 0; i < PASSES; ++i) {
+    const int c = (l + i * TEAM) * VEC;
+    if (c >= size) break;
+    int gc = g0 + c;
+    if (gc >= p.period) gc %= p.period;  // (VEC divides the period)
+    T o[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      const float w = v[i][e] * inv * p.gain[gc + e];
+      o[e] = Elem<T>::make(p.gate_first ? w : w * gate[i][e]);
+    }
+    if constexpr (VEC == 4 && sizeof(T) == 2)
+      *reinterpret_cast<uint2*>(out + c) = uint2{(uint32_t)o[0] | (uint32_t)o[1] << 16, (uint32_t)o[2] | (uint32_t)o[3] << 16};
+    else
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) out[c + e] = o[e];
   }
 }
 
-int check(const Rec* a, const char* what) {
+template <typename T, int VEC>
+int launch_gated_norm(const exo_gated_norm& a, const int32_t* rows, int n, hipStream_t st) {
+  const int size = a.width / a.groups, per = exo_ceil_div(size, VEC);  // runs of VEC columns per part
+  const dim3 small(exo_ceil_div(a.groups, 4), n), wide(a.groups, n);
+  if (per <= 64)
+    gated_norm_kernel<T, 64, 256, VEC, 1><<<small, 256, 0, st>>>(a, rows);
+  else if (per <= 128)
+    gated_norm_kernel<T, 64, 256, VEC, 2><<<small, 256, 0, st>>>(a, rows);
+  else if (per <= 512)
+    gated_norm_kernel<T, 256, 256, VEC, 2><<<wide, 256, 0, st>>>(a, rows);
+  else if (per <= 1024)
+    gated_norm_kernel<T, 1024, 1024, VEC, 1><<<wide, 1024, 0, st>>>(a, rows);
+  else if (per <= 2048)
+    gated_norm_kernel<T, 1024, 1024, VEC, 2><<<wide, 1024, 0, st>>>(a, rows);
+  else if (per <= 8192)
+    gated_norm_kernel<T, 1024, 1024, VEC, 8><<<wide, 1024, 0, st>>>(a, rows);
+  else {
+    exo_set_error("exo_gated_norm_rows: parts of %d columns are too long", size);
+    return EXO_ERR_ARG;
+  }
+  return EXO_OK;
+}
+
+int check(const exo_recurrence* a, const char* what) {
   EXO_REQUIRE(a && (a->dtype == 0 || a->dtype == 1), "%s: bad dtype", what);
   EXO_REQUIRE(a->heads > 0 && a->groups > 0 && a->heads % a->groups == 0 && a->dim > 0 && a->dim <= 1024 && a->vdim > 0 &&
                   a->lds >= a->vdim && a->lds % 4 == 0,
@@ -757,65 +1023,88 @@ bool vec_ok(const void* p, int ld, int part, int n) {
   return part % n == 0 && ld % n == 0 && (uintptr_t)p % (n * sizeof(T)) == 0;
 }
 
+int64_t chunk_bytes(const exo_recurrence* a, int n_chunks, Rec* out, char* ws) {
+  const int dp = exo_ceil_div(a->dim, 64) * 64, terms = a->dtype == 0 ? 2 : 1, esz = a->dtype == 0 ? 2 : 4;
+  const int64_t scores = (int64_t)n_chunks * a->groups * kChunk * kChunk * 4;
+  const int64_t nstates = (int64_t)n_chunks * a->heads * a->lds * dp, nhat = a->per_channel ? (int64_t)n_chunks * a->heads * kChunk * dp : 0;
+  const int64_t states = nstates * terms * esz, hat = nhat * terms * esz;
+  if (out) {
+    out->scores = reinterpret_cast<float*>(ws);
+    out->states = ws + scores;
+    out->qhat = ws + scores + states;
+    out->khat = ws + scores + states + hat;
+    out->nstates = nstates;
+    out->nhat = nhat;
+    out->dp = dp;
+  }
+  return scores + states + 2 * hat;
+}
+
 template <typename T, bool CHANNEL>
 void launch_chunks(Rec p, hipStream_t st) {
-  constexpr int KV = Elem<T>::kVec;
+  constexpr int KV = Elem<T>::kVec, NE = 2;
   p.qk_vec = vec_ok<T>(p.q, p.ldq, p.dim, KV) && vec_ok<T>(p.k, p.ldk, p.dim, KV);
   p.v_vec = vec_ok<T>(p.v, p.ldv, p.vdim, 4);
   if constexpr (CHANNEL) {
     recur_prep_channel_kernel<<<dim3(p.n_chunks, exo_ceil_div(p.heads * p.dim, 64)), 256, 0, st>>>(p);
+    recur_scores_channel_kernel<T><<<dim3(p.n_chunks, p.heads, 4), 256, 0, st>>>(p);
   } else {
-    recur_prep_head_kernel<<<dim3(p.n_chunks, exo_ceil_div(p.heads, 4)), 256, 0, st>>>(p);
-    const dim3 grid(p.n_chunks * (kChunk / kConvTokens), exo_ceil_div(p.channels, 256));
+    const int parts = kChunk / kConvTokens;
+    const dim3 grid(p.n_chunks * parts, exo_ceil_div(p.channels, 256) + exo_ceil_div(p.heads, 4 * parts));
     if (p.taps <= 4)
       recur_conv_kernel<T, 4><<<grid, 256, 0, st>>>(p);
     else if (p.taps <= 8)
       recur_conv_kernel<T, 8><<<grid, 256, 0, st>>>(p);
     else
       recur_conv_kernel<T, 16><<<grid, 256, 0, st>>>(p);
-  }
-  const int ne = exo_ceil_div(p.lds, 64);
-  recur_state_kernel<T, CHANNEL><<<dim3(p.n_chunks, p.heads, ne * exo_ceil_div(p.dim, 64)), 256, 0, st>>>(p);
-  if constexpr (CHANNEL)
-    recur_scores_channel_kernel<T><<<dim3(p.n_chunks, p.heads), 256, 0, st>>>(p);
-  else
     recur_scores_head_kernel<T><<<dim3(p.n_chunks, p.groups), 256, 0, st>>>(p);
-  int gx = exo_ceil_div((int64_t)p.dim * p.lds, 1024);
-  if (p.taps > 0 && gx < exo_ceil_div(p.channels, 256)) gx = exo_ceil_div(p.channels, 256);
-  recur_scan_kernel<T, CHANNEL><<<dim3(gx, p.heads + (p.taps > 0 ? 1 : 0), p.n_seqs), 256, 0, st>>>(p);
-  recur_out_kernel<T, CHANNEL><<<dim3(p.n_chunks, p.heads, exo_ceil_div(p.vdim, 64)), 256, 0, st>>>(p);
+  }
+  const dim3 grid(exo_ceil_div(p.lds, 16 * NE) * (p.dp / 64), p.heads + (p.taps > 0 ? 1 : 0), p.n_seqs);
+  const dim3 out_grid(p.n_chunks, p.heads, exo_ceil_div(p.vdim, 64));
+  if (p.v_vec && p.qk_vec) {
+    recur_carry_kernel<T, CHANNEL, NE, true><<<grid, 256, 0, st>>>(p);
+    recur_out_kernel<T, CHANNEL, true><<<out_grid, 256, 0, st>>>(p);
+  } else {
+    recur_carry_kernel<T, CHANNEL, NE, false><<<grid, 256, 0, st>>>(p);
+    recur_out_kernel<T, CHANNEL, false><<<out_grid, 256, 0, st>>>(p);
+  }
 }
 
 template <typename T, bool CHANNEL>
 void launch_step(const Rec& p, hipStream_t st) {
   int cols = 64;
   while (cols > 16 && (int64_t)p.n * p.heads * exo_ceil_div(p.lds, cols) < 256) cols /= 2;
-  const int lds = (3 * ((p.dim + 3) / 4 * 4) + 64 + 1024) * 4;
+  const int lds = (3 * ((p.dim + 3) / 4 * 4) + 64 + 4 * cols) * 4;
   recur_step_kernel<T, CHANNEL><<<dim3(exo_ceil_div(p.lds, cols), p.heads, p.n), 256, lds, st>>>(p, cols);
 }
 
 }  // namespace
 
-extern "C" int64_t exo_recur_scores_floats(int n_chunks, int groups) { return (int64_t)n_chunks * groups * kChunk * kChunk; }
-extern "C" int64_t exo_recur_state_floats(int n_chunks, int heads, int dim, int lds) {
-  return (int64_t)n_chunks * heads * dim * lds;
-}
 extern "C" int exo_recur_chunk(void) { return kChunk; }
+extern "C" int64_t exo_recur_workspace(const exo_recurrence* a) {
+  return a && a->n_chunks > 0 && a->dim > 0 ? chunk_bytes(a, a->n_chunks, nullptr, nullptr) : 0;
+}
 
-extern "C" int exo_recur_chunks(const exo_recurrence* a, exo_stream_t stream) {
+extern "C" int exo_recur_chunks(const exo_recurrence* a, void* workspace, int64_t workspace_bytes, exo_stream_t stream) {
   const int rc = check(a, "exo_recur_chunks");
   if (rc) return rc;
   EXO_REQUIRE(a->n_chunks > 0 && a->n_chunks <= 65535 && a->n_seqs > 0 && a->n_seqs <= 65535 && a->chunks && a->seqs,
               "exo_recur_chunks: bad lists (%d chunks, %d portions)", a->n_chunks, a->n_seqs);
-  EXO_REQUIRE(a->q && a->k && a->v && a->cum && a->scores && a->chunk_state &&
-                  a->ldcum >= (a->per_channel ? a->heads * a->dim : a->heads) && a->ldq >= a->groups * a->dim &&
-                  a->ldk >= a->groups * a->dim && a->ldv >= a->heads * a->vdim && (((uintptr_t)a->scores | (uintptr_t)a->chunk_state) & 15) == 0,
-              "exo_recur_chunks: bad inputs or workspace");
+  EXO_REQUIRE(a->q && a->k && a->v && a->cum && a->ldcum >= (a->per_channel ? a->heads * a->dim : 1) &&
+                  a->ldq >= a->groups * a->dim && a->ldk >= a->groups * a->dim && a->ldv >= a->heads * a->vdim,
+              "exo_recur_chunks: bad inputs");
   EXO_REQUIRE(a->per_channel || (a->act && a->dt && a->ldact >= a->channels), "exo_recur_chunks: no place for the convolved inputs");
+  EXO_REQUIRE((int64_t)a->n_chunks * a->heads * (a->lds > kChunk ? a->lds : kChunk) * exo_ceil_div(a->dim, 64) * 256 < (1ll << 31) &&
+                  (int64_t)a->n_chunks * kChunk * (a->per_channel && a->ldcum > a->ldv ? a->ldcum : a->ldv) * 4 < (1ll << 31) &&
+                  (int64_t)a->n_chunks * kChunk * a->ldk * 4 < (1ll << 31),
+              "exo_recur_chunks: %d chunks exceed 31-bit byte offsets", a->n_chunks);
+  EXO_REQUIRE(workspace && (uintptr_t)workspace % 16 == 0 && workspace_bytes >= exo_recur_workspace(a), "exo_recur_chunks: workspace too small");
+  Rec p{*a};
+  chunk_bytes(a, a->n_chunks, &p, reinterpret_cast<char*>(workspace));
   if (a->dtype == 0)
-    a->per_channel ? launch_chunks<bf16_t, true>(*a, (hipStream_t)stream) : launch_chunks<bf16_t, false>(*a, (hipStream_t)stream);
+    a->per_channel ? launch_chunks<bf16_t, true>(p, (hipStream_t)stream) : launch_chunks<bf16_t, false>(p, (hipStream_t)stream);
   else
-    a->per_channel ? launch_chunks<float, true>(*a, (hipStream_t)stream) : launch_chunks<float, false>(*a, (hipStream_t)stream);
+    a->per_channel ? launch_chunks<float, true>(p, (hipStream_t)stream) : launch_chunks<float, false>(p, (hipStream_t)stream);
   EXO_CHECK_LAUNCH("exo_recur_chunks");
   return EXO_OK;
 }
@@ -826,10 +1115,11 @@ extern "C" int exo_recur_step(const exo_recurrence* a, exo_stream_t stream) {
   EXO_REQUIRE(a->n > 0 && a->n <= 65535 && a->slot && a->pos, "exo_recur_step: bad rows (n=%d)", a->n);
   EXO_REQUIRE(!a->per_channel || (a->q && a->k && a->v && a->ldq >= a->heads * a->dim && a->ldk >= a->heads * a->dim && a->ldv >= a->heads * a->vdim),
               "exo_recur_step: bad inputs");
+  const Rec p{*a};
   if (a->dtype == 0)
-    a->per_channel ? launch_step<bf16_t, true>(*a, (hipStream_t)stream) : launch_step<bf16_t, false>(*a, (hipStream_t)stream);
+    a->per_channel ? launch_step<bf16_t, true>(p, (hipStream_t)stream) : launch_step<bf16_t, false>(p, (hipStream_t)stream);
   else
-    a->per_channel ? launch_step<float, true>(*a, (hipStream_t)stream) : launch_step<float, false>(*a, (hipStream_t)stream);
+    a->per_channel ? launch_step<float, true>(p, (hipStream_t)stream) : launch_step<float, false>(p, (hipStream_t)stream);
   EXO_CHECK_LAUNCH("exo_recur_step");
   return EXO_OK;
 }
@@ -841,13 +1131,16 @@ extern "C" int exo_gated_norm_rows(const exo_gated_norm* a, const int32_t* rows,
                   a->ldy >= a->width && a->ldg >= a->width && a->ldo >= a->width,
               "exo_gated_norm_rows: bad sizes (width=%d groups=%d period=%d)", a->width, a->groups, a->period);
   if (n == 0) return EXO_OK;
-  const bool wide = a->width / a->groups > 512;
-  const dim3 grid(wide ? a->groups : exo_ceil_div(a->groups, 4), n);
+  const int esz = a->dtype == 0 ? 2 : 4;
+  const bool vec = (a->width / a->groups) % 4 == 0 && a->period % 4 == 0 && a->ldy % 4 == 0 && a->ldg % 4 == 0 && a->ldo % 4 == 0 &&
+                   (uintptr_t)a->y % 16 == 0 && (uintptr_t)a->gate % (4 * esz) == 0 && (uintptr_t)a->out % (4 * esz) == 0;
   const hipStream_t st = (hipStream_t)stream;
+  int rc;
   if (a->dtype == 0)
-    wide ? gated_norm_kernel<bf16_t, 256><<<grid, 256, 0, st>>>(*a, rows) : gated_norm_kernel<bf16_t, 64><<<grid, 256, 0, st>>>(*a, rows);
+    rc = vec ? launch_gated_norm<bf16_t, 4>(*a, rows, n, st) : launch_gated_norm<bf16_t, 1>(*a, rows, n, st);
   else
-    wide ? gated_norm_kernel<float, 256><<<grid, 256, 0, st>>>(*a, rows) : gated_norm_kernel<float, 64><<<grid, 256, 0, st>>>(*a, rows);
+    rc = vec ? launch_gated_norm<float, 4>(*a, rows, n, st) : launch_gated_norm<float, 1>(*a, rows, n, st);
+  if (rc) return rc;
   EXO_CHECK_LAUNCH("exo_gated_norm_rows");
   return EXO_OK;
 }

@@ -10,7 +10,8 @@ namespace {
 
 constexpr int kRowThreads = 256;
 
-// sum over a workgroup of kRowThreads threads, in every thread
+// sum over a workgroup of TH threads, in every thread
+template <int TH = kRowThreads>
 __device__ __forceinline__ float block_sum(float v, float* tmp) {
   v = wave_sum(v);
   const int wave = threadIdx.x >> 6;
@@ -19,7 +20,7 @@ __device__ __forceinline__ float block_sum(float v, float* tmp) {
   __syncthreads();
   float s = 0.f;
 #pragma unroll
-  for (int w = 0; w < kRowThreads / 64; ++w) s += tmp[w];
+  for (int w = 0; w < TH / 64; ++w) s += tmp[w];
   return s;
 }
 
@@ -38,18 +39,16 @@ __global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const T* __re
 
 // ------------------------------------------------------------------------------ norms
 // y = x / rms(x) * gain, rows given by an index list (null: row i)
-template <typename T>
-__global__ __launch_bounds__(kRowThreads) void norm_rows_kernel(const float* __restrict__ x,
-                                                                const int32_t* __restrict__ rows,
-                                                                const float* __restrict__ gain, T* __restrict__ y,
-                                                                int H, int ldy, float eps) {
-  __shared__ float tmp[kRowThreads / 64];
+template <typename T, int TH>
+__global__ __launch_bounds__(TH) void norm_rows_kernel(const float* __restrict__ x, const int32_t* __restrict__ rows,
+                                                       const float* __restrict__ gain, T* __restrict__ y, int H, int ldy,
+                                                       float eps) {
+  __shared__ float tmp[TH / 64];
   const float* xr = x + (size_t)(rows ? rows[blockIdx.x] : (int)blockIdx.x) * H;
   float ss = 0.f;
-  for (int c = threadIdx.x; c < H; c += kRowThreads) ss += xr[c] * xr[c];
-  const float inv = 1.f / sqrtf(block_sum(ss, tmp) / H + eps);
-  for (int c = threadIdx.x; c < H; c += kRowThreads)
-    y[(size_t)blockIdx.x * ldy + c] = Elem<T>::make(xr[c] * inv * gain[c]);
+  for (int c = threadIdx.x; c < H; c += TH) ss += xr[c] * xr[c];
+  const float inv = 1.f / sqrtf(block_sum<TH>(ss, tmp) / H + eps);
+  for (int c = threadIdx.x; c < H; c += TH) y[(size_t)blockIdx.x * ldy + c] = Elem<T>::make(xr[c] * inv * gain[c]);
 }
 
 struct MoeSum {        // the feed-forward's output as a sum over a token's experts
@@ -83,10 +82,10 @@ __device__ __forceinline__ void load_cols(const T* p, float (&f)[kCols], bool ve
   }
 }
 
-template <typename T, int PASSES>
-__global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const exo_post_norm q, int ldb, const MoeSum m,
+template <typename T, int TH, int PASSES>
+__global__ __launch_bounds__(TH) void post_norm_add_kernel(const exo_post_norm q, int ldb, const MoeSum m,
                                                                     float* __restrict__ x, T* __restrict__ xb, int ldx) {
-  __shared__ float tmp[kRowThreads / 64];
+  __shared__ float tmp[TH / 64];
   const int row = blockIdx.x, H = q.H;
   float* xr = x + (size_t)row * H;
   const bool vec = H % kCols == 0 && (m.y ? m.ldy % kCols == 0 && m.lds % kCols == 0 : ldb % kCols == 0);
@@ -106,7 +105,7 @@ __global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const exo_po
   float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < PASSES; ++i) {
-    const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
+    const int c = (threadIdx.x + i * TH) * kCols, left = H - c;
     if (left <= 0) break;
     load_cols<float>(xr + c, xv[i], vec, left);
     if (m.y) {
@@ -136,17 +135,17 @@ __global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const exo_po
     float u[PASSES][kCols], su = 0.f;
 #pragma unroll
     for (int i = 0; i < PASSES; ++i) {
-      const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
+      const int c = (threadIdx.x + i * TH) * kCols, left = H - c;
       if (left <= 0) break;
       load_cols<float>(q.branch2 + (size_t)row * ldb + c, u[i], vec, left);
 #pragma unroll
       for (int e = 0; e < kCols; ++e) su += e < left ? u[i][e] * u[i][e] : 0.f;
     }
-    const float ia = 0.5f / sqrtf(block_sum(ss, tmp) / H + q.eps), ib = 0.5f / sqrtf(block_sum(su, tmp) / H + q.eps);
+    const float ia = 0.5f / sqrtf(block_sum<TH>(ss, tmp) / H + q.eps), ib = 0.5f / sqrtf(block_sum<TH>(su, tmp) / H + q.eps);
     ss = 0.f;
 #pragma unroll
     for (int i = 0; i < PASSES; ++i) {
-      const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
+      const int c = (threadIdx.x + i * TH) * kCols, left = H - c;
       if (left <= 0) break;
       float ga[kCols], gb[kCols];
       load_cols<float>(q.gain_a + c, ga, gvec, left);
@@ -158,11 +157,11 @@ __global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const exo_po
       }
     }
   }
-  const float inv = q.mult / sqrtf(block_sum(ss, tmp) / H + q.eps);
+  const float inv = q.mult / sqrtf(block_sum<TH>(ss, tmp) / H + q.eps);
   ss = 0.f;
 #pragma unroll
   for (int i = 0; i < PASSES; ++i) {
-    const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
+    const int c = (threadIdx.x + i * TH) * kCols, left = H - c;
     if (left <= 0) break;
     float gn[kCols];
     load_cols<float>(q.gain + c, gn, gvec, left);
@@ -172,10 +171,10 @@ __global__ __launch_bounds__(kRowThreads) void post_norm_add_kernel(const exo_po
       ss += e < left ? xv[i][e] * xv[i][e] : 0.f;
     }
   }
-  const float pinv = q.pre ? 1.f / sqrtf(block_sum(ss, tmp) / H + q.eps) : 1.f;
+  const float pinv = q.pre ? 1.f / sqrtf(block_sum<TH>(ss, tmp) / H + q.eps) : 1.f;
 #pragma unroll
   for (int i = 0; i < PASSES; ++i) {
-    const int c = (threadIdx.x + i * kRowThreads) * kCols, left = H - c;
+    const int c = (threadIdx.x + i * TH) * kCols, left = H - c;
     if (left <= 0) break;
     float y[kCols];
 #pragma unroll
@@ -488,10 +487,16 @@ extern "C" int exo_norm_rows(const float* x, const int32_t* rows, const float* g
   EXO_TYPE_OK("exo_norm_rows");
   EXO_REQUIRE(x && gain && y && n >= 0 && H > 0 && ldy >= H, "exo_norm_rows: bad argument");
   if (n == 0) return EXO_OK;
-  if (dtype == 0)
-    norm_rows_kernel<bf16_t><<<n, kRowThreads, 0, (hipStream_t)stream>>>(x, rows, gain, (bf16_t*)y, H, ldy, eps);
+  const hipStream_t st = (hipStream_t)stream;
+  if (n <= 256 && H > 1024) {
+    if (dtype == 0)
+      norm_rows_kernel<bf16_t, 1024><<<n, 1024, 0, st>>>(x, rows, gain, (bf16_t*)y, H, ldy, eps);
+    else
+      norm_rows_kernel<float, 1024><<<n, 1024, 0, st>>>(x, rows, gain, (float*)y, H, ldy, eps);
+  } else if (dtype == 0)
+    norm_rows_kernel<bf16_t, 256><<<n, 256, 0, st>>>(x, rows, gain, (bf16_t*)y, H, ldy, eps);
   else
-    norm_rows_kernel<float><<<n, kRowThreads, 0, (hipStream_t)stream>>>(x, rows, gain, (float*)y, H, ldy, eps);
+    norm_rows_kernel<float, 256><<<n, 256, 0, st>>>(x, rows, gain, (float*)y, H, ldy, eps);
   EXO_CHECK_LAUNCH("exo_norm_rows");
   return EXO_OK;
 }
@@ -502,19 +507,23 @@ static int post_norm(const exo_post_norm* q, int ldb, const MoeSum& m, int n, in
               "exo_post_norm_add: bad argument (H=%d, x in place)", q ? q->H : 0);
   EXO_REQUIRE(!q->branch2 || (q->gain_a && q->gain_b && !m.y), "exo_post_norm_add: two branches need a gain each");
   if (n == 0) return EXO_OK;
-#define EXO_POST(P)                                                                                              \
+#define EXO_POST(TH, P)                                                                                          \
   do {                                                                                                           \
     if (dtype == 0)                                                                                              \
-      post_norm_add_kernel<bf16_t, P><<<n, kRowThreads, 0, (hipStream_t)stream>>>(*q, ldb, m, q->x_out, (bf16_t*)q->operand, ldx); \
+      post_norm_add_kernel<bf16_t, TH, P><<<n, TH, 0, (hipStream_t)stream>>>(*q, ldb, m, q->x_out, (bf16_t*)q->operand, ldx); \
     else                                                                                                         \
-      post_norm_add_kernel<float, P><<<n, kRowThreads, 0, (hipStream_t)stream>>>(*q, ldb, m, q->x_out, (float*)q->operand, ldx);   \
+      post_norm_add_kernel<float, TH, P><<<n, TH, 0, (hipStream_t)stream>>>(*q, ldb, m, q->x_out, (float*)q->operand, ldx);   \
   } while (0)
   const int passes = exo_ceil_div(q->H, kRowThreads * kCols);
-  if (passes <= 1) EXO_POST(1);
-  else if (passes <= 2) EXO_POST(2);
-  else if (passes <= 4) EXO_POST(4);
-  else if (passes <= 8) EXO_POST(8);
-  else EXO_POST(16);
+  if (n <= 256 && passes > 1) {  // few rows: the length of a row's chain counts, not the workgroups per CU
+    if (passes <= 4) EXO_POST(1024, 1);
+    else if (passes <= 8) EXO_POST(1024, 2);
+    else EXO_POST(1024, 4);
+  } else if (passes <= 1) EXO_POST(256, 1);
+  else if (passes <= 2) EXO_POST(256, 2);
+  else if (passes <= 4) EXO_POST(256, 4);
+  else if (passes <= 8) EXO_POST(256, 8);
+  else EXO_POST(256, 16);
 #undef EXO_POST
   EXO_CHECK_LAUNCH("exo_post_norm_add");
   return EXO_OK;

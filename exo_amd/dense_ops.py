@@ -138,10 +138,13 @@ def linear_pair(x0, w0, out0, x1, w1, out1, n: int) -> None:
         _launch_linear(b, n, x1.device)
 
 
-POST_MAX_ROWS = 4  # beyond, every workgroup repeating the norm costs more than a launch
+POST_MAX_ROWS = 4  # (rows of a buffer set that keeps two residuals)
 
 
-def post_linear_fits(n: int, w, xb, H: int) -> bool:
+def post_linear_fits(n: int, w, xb, H: int, pre: bool = False) -> bool:
+    """Whether (and by measurement) the norms belong inside the product: every workgroup repeats them."""
+    if n * H > 4096 or (pre and H > 2048):
+        return False
     return n <= POST_MAX_ROWS and bool(native.load().exo_post_linear_fits(n, w.shape[0], H, xb.shape[1], _code(xb)))
 
 
@@ -276,13 +279,13 @@ class PagedAttention:
 _RECUR_WS: dict[int, torch.Tensor] = {}
 
 
-def recur_workspace(floats: int, device) -> torch.Tensor:
-    """Chunk states and scores of recurrences over prompts, one per device, grown on demand (work is in
+def recur_workspace(nbytes: int, device) -> torch.Tensor:
+    """Scores and states of recurrences over prompts, one per device, grown on demand (work is in
     stream order; single-token steps, which are captured, do not use it)."""
     key = torch.device(device).index or 0
-    if key not in _RECUR_WS or _RECUR_WS[key].numel() < floats:
-        _RECUR_WS[key] = torch.empty(0, device=device)
-        _RECUR_WS[key] = torch.empty(floats, dtype=torch.float32, device=device)
+    if key not in _RECUR_WS or _RECUR_WS[key].numel() < nbytes:
+        _RECUR_WS.pop(key, None)
+        _RECUR_WS[key] = torch.empty(nbytes, dtype=torch.uint8, device=device)
     return _RECUR_WS[key]
 
 
@@ -321,14 +324,13 @@ class Recurrence:
         check(native.load().exo_recur_step(C.byref(a), _stream()), "recur_step")
 
     def chunks(self, chunks, n_chunks: int, seqs, n_seqs: int, cum, dt) -> None:
-        """Portions of prompts (lists as the C ABI describes them).  ``cum``, ``dt``: scratch rows."""
+        """Portions of prompts (lists as the C ABI describes them).  ``cum``: scratch, a row per token; with
+        ``dt`` both are [heads, rows]."""
         a, lib = self.args, native.load()
-        ns = lib.exo_recur_state_floats(n_chunks, self.heads, self.dim, a.lds)
-        ws = recur_workspace(ns + lib.exo_recur_scores_floats(n_chunks, self.groups), chunks.device)
-        a.chunk_state, a.scores = ws.data_ptr(), ws.data_ptr() + 4 * ns
         a.cum, a.ldcum, a.dt = cum.data_ptr(), cum.stride(0), _p(dt)
         a.chunks, a.n_chunks, a.seqs, a.n_seqs = chunks.data_ptr(), n_chunks, seqs.data_ptr(), n_seqs
-        check(lib.exo_recur_chunks(C.byref(a), _stream()), "recur_chunks")
+        ws = recur_workspace(lib.exo_recur_workspace(C.byref(a)), chunks.device)
+        check(lib.exo_recur_chunks(C.byref(a), ws.data_ptr(), ws.numel(), _stream()), "recur_chunks")
 
 
 def gated_norm(y, gate, gain, out, n: int, width: int, groups: int, eps: float, gate_first: bool) -> None:

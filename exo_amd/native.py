@@ -57,7 +57,7 @@ class Recurrence(C.Structure):
 
     _fields_ = [(n, _vp) for n in (
         "q", "k", "v", "low", "decay_w", "decay_b", "dt_raw", "dt_bias", "decay_rate", "skip", "raw", "conv_w", "conv_b",
-        "ring", "act", "cum", "dt", "scores", "chunk_state", "state", "y", "map", "slot", "pos", "list", "chunks", "seqs")] + \
+        "ring", "act", "cum", "dt", "state", "y", "map", "slot", "pos", "list", "chunks", "seqs")] + \
         [(n, _i) for n in (
             "ldq", "ldk", "ldv", "ldlow", "rank", "lddt", "ldraw", "channels", "taps", "ldact", "ldcum", "lds", "ldy",
             "q_channel", "k_channel", "v_channel", "heads", "groups", "dim", "vdim", "per_channel", "n", "n_chunks",
@@ -137,9 +137,8 @@ SIGNATURES: dict[str, tuple] = {
     "exo_paged_prompt_block": (_i, [_i, _i]),
     "exo_paged_attn_prompt": (_i, [C.POINTER(PagedAttn), _vp]),
     "exo_recur_chunk": (_i, []),
-    "exo_recur_scores_floats": (_i64, [_i] * 2),
-    "exo_recur_state_floats": (_i64, [_i] * 4),
-    "exo_recur_chunks": (_i, [C.POINTER(Recurrence), _vp]),
+    "exo_recur_workspace": (_i64, [C.POINTER(Recurrence)]),
+    "exo_recur_chunks": (_i, [C.POINTER(Recurrence), _vp, _i64, _vp]),
     "exo_recur_step": (_i, [C.POINTER(Recurrence), _vp]),
     "exo_gated_norm_rows": (_i, [C.POINTER(GatedNorm), _vp, _i, _vp]),
     "exo_sample_workspace": (_i64, [_i]),

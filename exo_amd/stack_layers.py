@@ -110,7 +110,10 @@ class _RecurrentPart(_Part):
             rec.step(b.slot, b.pos, b.rows)
             return
         if b.n_chunks:
-            rec.chunks(b.chunks, b.n_chunks, b.seqs, b.n_seqs, bf.f32("cum", cum), bf.f32("dt", cum) if dt else None)
+            c, d = bf.f32("cum", cum), bf.f32("dt", cum) if dt else None
+            if dt:  # a head's tokens in a run
+                c, d = c.view(cum, -1), d.view(cum, -1)
+            rec.chunks(b.chunks, b.n_chunks, b.seqs, b.n_seqs, c, d)
         if b.n_alone:
             rec.step(b.slot, b.pos, b.n_alone, lst=b.alone)
 

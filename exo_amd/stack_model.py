@@ -231,7 +231,7 @@ class StackModel(DecoderShard):
                  keep_operand: bool = False) -> None:
         """out <- operand @ w^T (or the gated pair), after the outstanding norms and sum;
         ``keep_operand``: bf.xb is read by later launches too"""
-        if due is not None and len(bf.hs) > 1 and D.post_linear_fits(n, w, bf.xb, self.cfg.hidden_size):
+        if due is not None and len(bf.hs) > 1 and D.post_linear_fits(n, w, bf.xb, self.cfg.hidden_size, pre is not None):
             x = bf.h
             bf.cur ^= 1
             D.post_linear(x, due, self.cfg.eps, bf.h, bf.xb if keep_operand else None, w, out, n, bias, tail, pre, up, spec)

@@ -554,8 +554,7 @@ typedef struct {
   const void* raw;
   const float *conv_w, *conv_b;
   void *ring, *act;
-  float *cum, *dt;            /* [rows][ldcum] scratch of prompts */
-  float *scores, *chunk_state; /* exo_recur_scores_floats, exo_recur_state_floats */
+  float *cum, *dt;            /* scratch of prompts: per_channel cum [rows][ldcum], else both [heads][ldcum >= rows] */
   float *state, *y;            /* y [rows][ldy] */
   const int32_t *map, *slot, *pos, *list; /* single tokens: row i of cache row slot[i] at pos[i]; list: which rows, or null */
   const int32_t *chunks, *seqs;
@@ -568,9 +567,9 @@ typedef struct {
  * exo_recur_chunk()), first position of its portion, 0, 0, 0, a portion's chunks one after the other;
  * seqs [n_seqs][4] = first chunk, chunks, 0, 0 */
 int exo_recur_chunk(void);
-int64_t exo_recur_scores_floats(int n_chunks, int groups);
-int64_t exo_recur_state_floats(int n_chunks, int heads, int dim, int lds);
-int exo_recur_chunks(const exo_recurrence* args, exo_stream_t stream);
+int64_t exo_recur_workspace(const exo_recurrence* args); /* bytes, for its n_chunks */
+int exo_recur_chunks(const exo_recurrence* args, void* workspace, int64_t workspace_bytes,
+                     exo_stream_t stream);
 /* single tokens of n sequences */
 int exo_recur_step(const exo_recurrence* args, exo_stream_t stream);
 /* RMS norm of `groups` equal parts of y, gain repeating with `period`, and silu(gate) ahead of the

@@ -242,7 +242,7 @@ def test_new_entry_points_check_their_arguments():
     head = dict(heads=4, groups=2, dim=8, vdim=8, lds=16, state=16, map=16, y=16, ldy=32, dt_raw=16, dt_bias=16, decay_rate=16,
                 lddt=4, taps=4, channels=64, ldraw=64, raw=16, ring=16, conv_w=16, conv_b=16, k_channel=32, q_channel=48)
     for change in (dict(taps=17), dict(channels=60), dict(q_channel=50), dict(lddt=3)):
-        assert lib.exo_recur_chunks(native.Recurrence(**{**head, **change}), None) == -1
+        assert lib.exo_recur_chunks(native.Recurrence(**{**head, **change}), None, 0, None) == -1
         assert b"exo_recur_chunks" in lib.exo_last_error()
     assert lib.exo_gated_norm_rows(native.GatedNorm(y=16, gate=16, gain=16, out=16, width=10, groups=3, period=10, ldy=10, ldg=10,
                                                     ldo=10), None, 1, None) == -1
