@@ -41,9 +41,15 @@ struct Rec : exo_recurrence {
   int dp;                // dim rounded up to 64, zeros behind dim
 };
 
-__device__ __forceinline__ float softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
-constexpr float kLog2e = 1.4426950408889634f;
+constexpr float kLog2e = 1.4426950408889634f, kLn2 = 0.6931471805599453f;
 __device__ __forceinline__ float pow2(float x) { return __builtin_amdgcn_exp2f(x); }
+// max(z, 0) + log(1 + e), e = exp(-|z|).  u = 1 + e rounds, so log(u) belongs to u - 1 instead of e: taken
+// times e / (u - 1) it keeps its relative precision for small e.
+__device__ __forceinline__ float softplus(float z) {
+  const float e = pow2(-fabsf(z) * kLog2e), u = 1.f + e, d = u - 1.f;
+  const float l = d == 0.f ? e : __builtin_amdgcn_logf(u) * kLn2 * (e * __builtin_amdgcn_rcpf(d));
+  return fmaxf(z, 0.f) + l;
+}
 __device__ __forceinline__ float sigmoidf(float z) { return 1.f / (1.f + expf(-z)); }
 
 template <typename T>
@@ -441,6 +447,12 @@ __global__ __launch_bounds__(256) void recur_scores_channel_kernel(const Rec p) 
   out[(tid >> 4) * kChunk + i0 + (tid & 15)] = part[0][tid] + part[1][tid] + part[2][tid] + part[3][tid];
 }
 
+template <typename T, bool CHANNEL, int NE>
+constexpr int carry_lds() {
+  constexpr int tile = 16 * NE * kVStride<T> * (int)sizeof(T);
+  return 2 * tile + 2 * tile * (sizeof(T) == 2 ? 2 : 1) + (CHANNEL ? 0 : 2 * 64 * kVStride<T> * (int)sizeof(T)) + 2 * kChunk * 4;
+}
+
 // Along a portion's chunks with a tile of the state, 64 keys x (16 NE) value columns, in registers.  One
 // workgroup per CU at most, so the loop is kept short: every address is a thread's fixed offset plus a
 // scalar that steps with the chunk, and the ends of rows and of the portion are the buffers' ends.
@@ -448,10 +460,14 @@ __global__ __launch_bounds__(256) void recur_scores_channel_kernel(const Rec p) 
 template <typename T, bool CHANNEL, int NE, bool VEC>
 __global__ __launch_bounds__(256) void recur_carry_kernel(const Rec p) {
   constexpr int KV = Elem<T>::kVec, KS = kChunk / (4 * KV), VS = kVStride<T>, EB = sizeof(T), NT = sizeof(T) == 2 ? 2 : 1;
-  __shared__ __attribute__((aligned(16))) T vt[2][16 * NE * VS];
-  __shared__ __attribute__((aligned(16))) T kt[CHANNEL ? 1 : 2][CHANNEL ? 16 : 64 * VS];
-  __shared__ __attribute__((aligned(16))) T sv[2][NT][16 * NE * VS];  // the state on its way out [column][key]
-  __shared__ __attribute__((aligned(16))) float wt[2][kChunk];
+  // two buffers each: values [column][token], keys [key][token] (decay per head), the state on its way
+  // out [term][column][key], weights of the tokens (decay per head)
+  extern __shared__ __attribute__((aligned(16))) char lds_raw[];
+  constexpr int TILE = 16 * NE * VS;
+  T(*vt)[TILE] = reinterpret_cast<T(*)[TILE]>(lds_raw);
+  T(*sv)[NT][TILE] = reinterpret_cast<T(*)[NT][TILE]>(vt + 2);
+  T(*kt)[64 * VS] = reinterpret_cast<T(*)[64 * VS]>(sv + 2);
+  float(*wt)[kChunk] = reinterpret_cast<float(*)[kChunk]>(kt + (CHANNEL ? 0 : 2));
   const int32_t* seq = p.seqs + 4 * (size_t)blockIdx.z;
   const int first = seq[0], count = seq[1];
   const Chunk c0(p.chunks, first), cl(p.chunks, first + count - 1);
@@ -522,7 +538,7 @@ __global__ __launch_bounds__(256) void recur_carry_kernel(const Rec p) {
     floatx4 end;
     float w_c, w_end, w_dt;
   };
-  constexpr int AHEAD = VEC ? 4 : 2;  // (at most 63 loads and stores can be told apart)
+  constexpr int AHEAD = !VEC || NE > 2 ? 2 : 4;  // (at most 63 loads and stores can be told apart)
   Request rq[AHEAD];
   // Requests past the last chunk re-read it: every load is unconditional, so the waits count exactly
   // the loads in front of the ones they are for.
@@ -1040,9 +1056,26 @@ int64_t chunk_bytes(const exo_recurrence* a, int n_chunks, Rec* out, char* ws) {
   return scores + states + 2 * hat;
 }
 
+template <typename T, bool CHANNEL, int NE, bool VEC>
+int launch_carry(const Rec& p, hipStream_t st) {
+  constexpr int lds = carry_lds<T, CHANNEL, NE>();
+  const auto fn = recur_carry_kernel<T, CHANNEL, NE, VEC>;
+  static bool done = false;
+  if (!done && lds > 64 * 1024) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    if (e != hipSuccess) {
+      exo_set_error("exo_recur_chunks: cannot raise the dynamic LDS limit: %s", hipGetErrorString(e));
+      return EXO_ERR_HIP;
+    }
+  }
+  done = true;
+  fn<<<dim3(exo_ceil_div(p.lds, 16 * NE) * (p.dp / 64), p.heads + (p.taps > 0 ? 1 : 0), p.n_seqs), 256, lds, st>>>(p);
+  return EXO_OK;
+}
+
 template <typename T, bool CHANNEL>
-void launch_chunks(Rec p, hipStream_t st) {
-  constexpr int KV = Elem<T>::kVec, NE = 2;
+int launch_chunks(Rec p, hipStream_t st) {
+  constexpr int KV = Elem<T>::kVec;
   p.qk_vec = vec_ok<T>(p.q, p.ldq, p.dim, KV) && vec_ok<T>(p.k, p.ldk, p.dim, KV);
   p.v_vec = vec_ok<T>(p.v, p.ldv, p.vdim, 4);
   if constexpr (CHANNEL) {
@@ -1059,15 +1092,20 @@ void launch_chunks(Rec p, hipStream_t st) {
       recur_conv_kernel<T, 16><<<grid, 256, 0, st>>>(p);
     recur_scores_head_kernel<T><<<dim3(p.n_chunks, p.groups), 256, 0, st>>>(p);
   }
-  const dim3 grid(exo_ceil_div(p.lds, 16 * NE) * (p.dp / 64), p.heads + (p.taps > 0 ? 1 : 0), p.n_seqs);
   const dim3 out_grid(p.n_chunks, p.heads, exo_ceil_div(p.vdim, 64));
+  // wide tiles of the state (a key tile is read by fewer workgroups) once they leave a workgroup per CU
+  const bool wide = (int64_t)exo_ceil_div(p.lds, 64) * (p.dp / 64) * p.heads * p.n_seqs >= 256;
+  int rc;
   if (p.v_vec && p.qk_vec) {
-    recur_carry_kernel<T, CHANNEL, NE, true><<<grid, 256, 0, st>>>(p);
+    rc = wide ? launch_carry<T, CHANNEL, 4, true>(p, st) : launch_carry<T, CHANNEL, 2, true>(p, st);
+    if (rc) return rc;
     recur_out_kernel<T, CHANNEL, true><<<out_grid, 256, 0, st>>>(p);
   } else {
-    recur_carry_kernel<T, CHANNEL, NE, false><<<grid, 256, 0, st>>>(p);
+    rc = launch_carry<T, CHANNEL, 2, false>(p, st);
+    if (rc) return rc;
     recur_out_kernel<T, CHANNEL, false><<<out_grid, 256, 0, st>>>(p);
   }
+  return EXO_OK;
 }
 
 template <typename T, bool CHANNEL>
@@ -1101,10 +1139,13 @@ extern "C" int exo_recur_chunks(const exo_recurrence* a, void* workspace, int64_
   EXO_REQUIRE(workspace && (uintptr_t)workspace % 16 == 0 && workspace_bytes >= exo_recur_workspace(a), "exo_recur_chunks: workspace too small");
   Rec p{*a};
   chunk_bytes(a, a->n_chunks, &p, reinterpret_cast<char*>(workspace));
+  const hipStream_t st = (hipStream_t)stream;
+  int rc2;
   if (a->dtype == 0)
-    a->per_channel ? launch_chunks<bf16_t, true>(p, (hipStream_t)stream) : launch_chunks<bf16_t, false>(p, (hipStream_t)stream);
+    rc2 = a->per_channel ? launch_chunks<bf16_t, true>(p, st) : launch_chunks<bf16_t, false>(p, st);
   else
-    a->per_channel ? launch_chunks<float, true>(p, (hipStream_t)stream) : launch_chunks<float, false>(p, (hipStream_t)stream);
+    rc2 = a->per_channel ? launch_chunks<float, true>(p, st) : launch_chunks<float, false>(p, st);
+  if (rc2) return rc2;
   EXO_CHECK_LAUNCH("exo_recur_chunks");
   return EXO_OK;
 }

@@ -446,6 +446,19 @@ def test_other_orders_and_sizes(device, dtype, layers):
             assert rel_rms(lg, want[k]).max() < LIMIT[dtype]
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_recurrences_with_many_heads(device, dtype):
+    """Enough heads that a portion's states are carried in wide tiles."""
+    for layer in (U.linear(heads=64, dim=64, vdim=256), U.parallel(ssm_heads=128, ssm_vdim=64, state=128, groups=2, norm_groups=4)):
+        cfg = U.config([dict(layer, mlp=None)], width=64)
+        w = U.weights(cfg, 7)
+        m = build_model(config_from_dict(cfg), torch_weights(w, "cuda"), dtype=dtype)
+        toks = {"a": rng(1).integers(0, cfg["vocab"], 200).tolist()}
+        want = O.forward(cfg, w, toks["a"])
+        for sched in ([[("a", 200)]], [[("a", 70)], [("a", 129)], [("a", 1)]]):
+            assert rel_rms(play(m, toks, sched)["a"], want).max() < (3e-2 if dtype == BF else 1e-4)
+
+
 def test_model_pipeline_shards(built):
     w = torch_weights({k: np.asarray(v, np.float32) for k, v in built.w.items()}, "cuda")
     c = config_from_dict(built.cfg)
