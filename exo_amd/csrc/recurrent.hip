@@ -341,20 +341,22 @@ __global__ __launch_bounds__(256) void recur_scores_head_kernel(const Rec p) {
 }
 
 // scores of 16 queries of a chunk, decay per key channel (queries and keys per head); 64 channels at a
-// time in LDS.  Wave j takes the keys of block j ahead of the queries' own; that one is dealt out over
-// the waves by channels.
+// time in LDS.  Wave j takes the keys of block j ahead of the queries' own.  Of that one, wave 3 takes the
+// later eight queries with the earlier eight keys like an earlier block; the two squares of eight are
+// dealt out over the waves by channels.
 template <typename T>
 __global__ __launch_bounds__(256) void recur_scores_channel_kernel(const Rec p) {
   constexpr int KV = Elem<T>::kVec, ST = 68;
   __shared__ __attribute__((aligned(16))) float qs[16][ST], ks[kChunk][ST], cs[kChunk][ST];
-  __shared__ float part[4][256];
+  __shared__ float part[4][128], cross[256];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r = lane & 15, g = lane >> 4;
+  const int sk = (lane >> 5) * 8 + (lane & 7), sq = (lane >> 5) * 8 + ((lane >> 3) & 3) * 2;  // a square's key, two queries
   const Chunk ck(p.chunks, blockIdx.x);
   const int h = blockIdx.y, block = 3 - (int)blockIdx.z, i0 = block * 16;  // (the longest first)
   if (i0 >= ck.n) return;
   floatx4 acc = {0.f, 0.f, 0.f, 0.f};
-  float own[4] = {0.f, 0.f, 0.f, 0.f};
+  float own[2] = {0.f, 0.f};
   T kr[16], qr[4];
   float cr[16];
   auto request = [&](int d) {
@@ -408,16 +410,18 @@ __global__ __launch_bounds__(256) void recur_scores_channel_kernel(const Rec p) 
       }
     }
     const int db = min(64, p.dim - d0);
-    // an earlier block: both factors relative to the last token ahead of the queries
-    if (wave < block) {
+    // earlier keys: both factors relative to the last token ahead of the queries
+    if (wave < block || wave == 3) {
+      const int ref = wave < block ? i0 - 1 : i0 + 7, key = wave < block ? wave * 16 + r : i0 + r;
+      const float qon = wave < block || r >= 8 ? 1.f : 0.f, kon = wave < block || r < 8 ? 1.f : 0.f;
       for (int s = 0; s < db; s += 4 * KV) {
         const int dd = s + g * KV;
         float fa[KV], fb[KV];
 #pragma unroll
         for (int e = 0; e < KV; ++e) {
-          const float base = cs[i0 - 1][dd + e];
-          fa[e] = qs[r][dd + e] * pow2(cs[i0 + r][dd + e] - base);
-          fb[e] = ks[wave * 16 + r][dd + e] * pow2(base - cs[wave * 16 + r][dd + e]);
+          const float base = cs[ref][dd + e];
+          fa[e] = qon * qs[r][dd + e] * pow2(fminf(cs[i0 + r][dd + e] - base, 0.f));
+          fb[e] = kon * ks[key][dd + e] * pow2(fminf(base - cs[key][dd + e], 0.f));
         }
         Split<T> a, b;
         a.set(fa);
@@ -425,26 +429,30 @@ __global__ __launch_bounds__(256) void recur_scores_channel_kernel(const Rec p) 
         acc = mma<T>(a, b, acc);
       }
     }
-    // the own block, pair by pair: lane (g, r) has queries 4g .. 4g + 3 and key r
+    // the squares, pair by pair
     for (int dd = wave * 16; dd < min(db, wave * 16 + 16); dd += 4) {
-      const floatx4 k = *reinterpret_cast<const floatx4*>(&ks[i0 + r][dd]), c = *reinterpret_cast<const floatx4*>(&cs[i0 + r][dd]);
+      const floatx4 k = *reinterpret_cast<const floatx4*>(&ks[i0 + sk][dd]), c = *reinterpret_cast<const floatx4*>(&cs[i0 + sk][dd]);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const floatx4 q = *reinterpret_cast<const floatx4*>(&qs[4 * g + e][dd]), b = *reinterpret_cast<const floatx4*>(&cs[i0 + 4 * g + e][dd]);
+      for (int e = 0; e < 2; ++e) {
+        const floatx4 q = *reinterpret_cast<const floatx4*>(&qs[sq + e][dd]), b = *reinterpret_cast<const floatx4*>(&cs[i0 + sq + e][dd]);
 #pragma unroll
         for (int i = 0; i < 4; ++i) own[e] = fmaf(q[i] * k[i], pow2(fminf(b[i] - c[i], 0.f)), own[e]);
       }
     }
   }
 #pragma unroll
-  for (int e = 0; e < 4; ++e) part[wave][(4 * g + e) * 16 + r] = own[e];
+  for (int e = 0; e < 2; ++e) part[wave][(sq + e) * 8 + (sk & 7)] = own[e];
   float* out = p.scores + (((size_t)blockIdx.x * p.heads + h) * kChunk + i0) * kChunk;
-  if (wave < block) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) out[(4 * g + e) * kChunk + wave * 16 + r] = acc[e];
+  for (int e = 0; e < 4; ++e) {
+    if (wave < block)
+      out[(4 * g + e) * kChunk + wave * 16 + r] = acc[e];
+    else if (wave == 3)
+      cross[(4 * g + e) * 16 + r] = acc[e];
   }
   __syncthreads();
-  out[(tid >> 4) * kChunk + i0 + (tid & 15)] = part[0][tid] + part[1][tid] + part[2][tid] + part[3][tid];
+  const int qi = tid >> 4, kj = tid & 15, at = qi * 8 + (kj & 7);
+  out[qi * kChunk + i0 + kj] = (qi ^ kj) & 8 ? cross[tid] : part[0][at] + part[1][at] + part[2][at] + part[3][at];
 }
 
 template <typename T, bool CHANNEL, int NE>
