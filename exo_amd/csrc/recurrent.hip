@@ -19,8 +19,8 @@
 //                             S <- 2^c_end S + sum_t 2^(c_end - c_t) k_t v_t^T
 //   recur_out     per chunk   o_i = 2^c_i q_i S + sum_j A[i][j] v_j (+ D v_i)
 // A decay per channel does not factor out of a score without overflow, so its scores are formed for
-// 16-token blocks: between blocks both factors are taken to the query block's start, inside a block
-// each pair has its own exponentials.  That launch also leaves 2^c q and, transposed, 2^(c_end - c) k as
+// 16-token blocks: between blocks both factors are taken to the query block's start, between a block's
+// halves to its middle, and inside a half each pair has its own exponentials.  That launch also leaves 2^c q and, transposed, 2^(c_end - c) k as
 // matrix operands; recur_carry leaves the states as operands too (value columns x keys).
 #include "../../include/exo_mi355x.h"
 #include "dense.h"

@@ -63,7 +63,7 @@ struct MoeSum {        // the feed-forward's output as a sum over a token's expe
 // x += mult * gain * v / rms(v), v = the branch row, half the sum of two branches normed each with a
 // gain of its own, or the weighted sum over the experts; xb = x, or x / rms(x) * pre.
 // Four columns per thread and pass (VEC: rows of four columns are aligned), v in registers.
-constexpr int kCols = 4, kPasses = 16;  // H <= 16384
+constexpr int kCols = 4;  // at most 16 passes: H <= 16384
 
 template <typename T>
 __device__ __forceinline__ void load_cols(const T* p, float (&f)[kCols], bool vec, int left) {
