@@ -16,7 +16,7 @@ PKG = Path(__file__).resolve().parent
 CSRC = PKG / "csrc"
 LIB = PKG / "libexo_mi355x.so"
 SOURCES = ["quant.hip", "qmv.hip", "qmv_mfma.hip", "qmv_quad.hip", "qmv_w16.hip", "qmm.hip", "sdpa.hip", "sdpa_prefill.hip", "elementwise.hip", "kvwire.hip", "sampling.hip",
-           "dense.hip", "stack.hip", "paged_attn.hip", "recurrent.hip"]
+           "dense.hip", "stack.hip", "paged_attn.hip", "latent_attn.hip", "recurrent.hip"]
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 FLAGS = [

@@ -75,6 +75,32 @@ __device__ __forceinline__ float clamped_glu(float g, float u, const GluConst& c
   return g / (1.f + expf(-c.alpha * g)) * (u + c.shift);
 }
 
+// What happens to a product's result ahead of its store: an activation, then a factor out of a table
+// (element type) whose row is given by an index list (null: the result's own row).
+struct Epilogue {
+  int act;  // 0 none, 1 square of relu, 2 gelu (tanh form)
+  const void* mul;
+  const int32_t* mul_rows;
+  int ldmul;
+};
+template <typename T>
+__device__ __forceinline__ float finish(float v, size_t m, int n, const Epilogue& e) {
+  if (e.act == 1) {
+    v = fmaxf(v, 0.f);
+    v *= v;
+  } else if (e.act == 2) {
+    v = 0.5f * v * (1.f + tanhf(0.79788456080286536f * (v + 0.044715f * v * v * v)));
+  }
+  if (e.mul) v *= Elem<T>::load(reinterpret_cast<const T*>(e.mul)[(e.mul_rows ? (size_t)e.mul_rows[m] : m) * e.ldmul + n]);
+  return v;
+}
+
+// 16 bytes as one vector value (a struct copy of a uint4 may end up in scratch memory)
+typedef __attribute__((__vector_size__(4 * sizeof(uint32_t)))) uint32_t u32x4_t;
+__device__ __forceinline__ uint4 load16(const void* p) {
+  return __builtin_bit_cast(uint4, *reinterpret_cast<const u32x4_t*>(p));
+}
+
 // range-checked buffer over `bytes` bytes: reads past the end return zero and move nothing
 __device__ __forceinline__ __amdgpu_buffer_rsrc_t buf_of(const void* base, uint32_t bytes) {
   return __builtin_amdgcn_make_buffer_rsrc(const_cast<void*>(base), 0, bytes, 0x00020000);

@@ -35,6 +35,7 @@ struct GemvParams {
   float* y2;       // columns from n1 on
   int M, N, n1, ldx, ldw, ldy, ldy2, y_f32;
   GluConst glu;
+  Epilogue ep;
 };
 
 template <typename T>
@@ -46,22 +47,23 @@ __device__ __forceinline__ void store_out(void* y, size_t i, float v, int y_f32)
 }
 
 // Norm of the previous sublayer's output and residual sum, in front of the product that reads the
-// residual: every workgroup forms y = x + mult * gain * v / rms(v) for itself and from it the product's
-// operand (in LDS, element type): y, or y / rms(y) * pre.  v is the branch, or half the sum of two
-// branches that are normed each with a gain of its own.  Workgroup 0 also writes y out - to another
+// residual: every workgroup forms y = x + mult * gain * v / rms(v), or (sum) y = gain * norm(keep * x + v),
+// for itself and from it the product's operand (in LDS, element type): y, or y / rms(y) * pre.  v is the
+// branch, or half the sum of two branches that are normed each with a gain of its own.  `norm` divides by
+// the RMS, after the mean was taken off if `center`.  x null: only the branch is normed.  Workgroup 0 also writes y out - to another
 // buffer than x is read from, since the others may still be reading.
 struct PostNorm {
-  const float* x;        // [M][H]
-  const float* branch;   // [M][H]
-  const float* branch2;  // [M][H], or null
+  const float* x;        // [M][H], or null
+  const float* branch;   // [M][ldb]
+  const float* branch2;  // [M][ldb], or null
   const float* gain_a;   // [H] gains of two branches
   const float* gain_b;
   const float* gain;     // [H]
   const float* pre;      // [H], or null
-  float* x_out;          // [M][H]
+  float* x_out;          // [M][H] (null with x)
   void* xb_out;          // T [M][ldx] the operand, or null
-  int H;
-  float eps, mult;
+  int H, ldb, sum, center;
+  float eps, mult, keep;
 };
 constexpr int kPostPasses = 4;  // at most so many float4 per lane of a row's waves
 
@@ -136,17 +138,17 @@ __global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p0
     // a row's columns over wpr waves; its inputs are requested ahead of the first weights
     const int wpr = post_waves_per_row(p.M, NW), rpi = NW / wpr;  // rows per iteration
     const uint32_t lrow = xrow + 16;
-    const bool vec = q.H % 4 == 0;
+    const bool vec = q.H % 4 == 0 && q.ldb % 4 == 0;
     for (int m0 = 0; m0 < p.M; m0 += rpi) {
       const int m = m0 + wave / wpr, c0 = ((wave % wpr) * 64 + lane) * 4, cs = wpr * 256;
       const bool on = m < p.M;
-      const size_t o = (size_t)m * q.H;
+      const size_t o = (size_t)m * q.H, ob = (size_t)m * q.ldb;
       floatx4 v[NP], x[NP], u[NU];
 #pragma unroll
       for (int i = 0; i < NP; ++i) {
-        v[i] = row4(q.branch + o, c0 + i * cs, q.H, on, vec);
-        if (TWO) u[TWO ? i : 0] = row4(q.branch2 + o, c0 + i * cs, q.H, on, vec);
-        x[i] = row4(q.x + o, c0 + i * cs, q.H, on, vec);
+        v[i] = row4(q.branch + ob, c0 + i * cs, q.H, on, vec);
+        if (TWO) u[TWO ? i : 0] = row4(q.branch2 + ob, c0 + i * cs, q.H, on, vec);
+        x[i] = row4(q.x + o, c0 + i * cs, q.H, on && q.x, vec);
       }
       if (m0 == 0) load_w(s0);
       float ss = 0.f, su = 0.f;
@@ -165,12 +167,32 @@ __global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p0
         }
         ss = su = 0.f;
       }
+      if (q.sum) {  // the sum itself is normed
+#pragma unroll
+        for (int i = 0; i < NP; ++i)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            v[i][e] = fmaf(q.keep, x[i][e], v[i][e]);
+            x[i][e] = 0.f;
+            su += v[i][e];
+          }
+        if (q.center) {
+          row_sums<NW>(ss, su, part, wave, wpr, lane);
+          const float mean = su / q.H;
+#pragma unroll
+          for (int i = 0; i < NP; ++i)
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (c0 + i * cs + e < q.H) v[i][e] -= mean;
+        }
+        ss = su = 0.f;
+      }
 #pragma unroll
       for (int i = 0; i < NP; ++i)
 #pragma unroll
         for (int e = 0; e < 4; ++e) ss += v[i][e] * v[i][e];
       row_sums<NW>(ss, su, part, wave, wpr, lane);
-      const float inv = q.mult / sqrtf(ss / q.H + q.eps);
+      const float inv = (q.sum ? 1.f : q.mult) / sqrtf(ss / q.H + q.eps);
       ss = 0.f;
 #pragma unroll
       for (int i = 0; i < NP; ++i) {
@@ -201,7 +223,7 @@ __global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p0
         for (int e = 0; e < 4; ++e) {
           out[e] = Elem<T>::make(y[e]);
           if (blockIdx.x == 0 && c + e < q.H) {
-            q.x_out[o + c + e] = x[i][e];
+            if (q.x_out) q.x_out[o + c + e] = x[i][e];
             if (q.xb_out) reinterpret_cast<T*>(q.xb_out)[(size_t)m * p.ldx + c + e] = out[e];
           }
         }
@@ -252,7 +274,7 @@ __global__ __launch_bounds__(64 * NW) void dense_gemv_kernel(const GemvParams p0
     }
     if (p.bias) v += p.bias[n0 + n];
     if (n0 + n < p.n1)
-      store_out<T>(p.y, (size_t)m * p.ldy + n0 + n, v, p.y_f32);
+      store_out<T>(p.y, (size_t)m * p.ldy + n0 + n, finish<T>(v, m, n0 + n, p.ep), p.y_f32);
     else
       p.y2[(size_t)m * p.ldy2 + n0 + n - p.n1] = v;
   }
@@ -268,6 +290,7 @@ struct GemmParams {
   float* y2;       // columns from n1 on
   int M, N, n1, ldx, ldw, ldy, ldy2, y_f32;
   GluConst glu;
+  Epilogue ep;
   // grouped
   const int32_t* sorted;
   const int32_t* tiles;
@@ -434,7 +457,7 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const GemmParams p) 
           } else {
             const float v = acc[i][j][e] + (p.bias ? p.bias[n] : 0.f);
             if (GROUPED || n < p.n1)
-              store_out<T>(p.y, row * p.ldy + n, v, p.y_f32);
+              store_out<T>(p.y, row * p.ldy + n, finish<T>(v, row, n, p.ep), p.y_f32);
             else
               p.y2[row * p.ldy2 + n - p.n1] = v;
           }
@@ -451,7 +474,7 @@ __global__ __launch_bounds__(256) void dense_reduce_kernel(const GemmParams p) {
   float v = p.bias ? p.bias[n] : 0.f;
   for (int z = 0; z < p.ksplit; ++z) v += p.part[((size_t)z * p.M + m) * p.N + n];
   if (n < p.n1)
-    store_out<T>(p.y, (size_t)m * p.ldy + n, v, p.y_f32);
+    store_out<T>(p.y, (size_t)m * p.ldy + n, finish<T>(v, m, n, p.ep), p.y_f32);
   else
     p.y2[(size_t)m * p.ldy2 + n - p.n1] = v;
 }
@@ -590,6 +613,8 @@ static int linear_check(const exo_linear* a, const char* what) {
   EXO_REQUIRE(a->n1 > 0 && a->n1 <= a->N && a->ldy >= a->n1 && (a->n1 == a->N || (a->y2 && a->ldy2 >= a->N - a->n1)),
               "%s: outputs do not hold %d columns (%d in the first: %d, %d)", what, a->N, a->n1, a->ldy, a->ldy2);
   EXO_REQUIRE(!a->w_up || (a->n1 == a->N && !a->bias), "%s: a gated pair has one output and no bias", what);
+  EXO_REQUIRE(a->act >= 0 && a->act <= 2 && (!a->mul || a->ldmul >= a->N) && (!(a->act || a->mul) || (!a->w_up && a->n1 == a->N)),
+              "%s: an activation (%d) or factor belongs to one plain output", what, a->act);
   return EXO_OK;
 }
 static GemvParams gemv_of(const exo_linear* a) {
@@ -597,6 +622,7 @@ static GemvParams gemv_of(const exo_linear* a) {
   p.x = a->x, p.w = a->w, p.w2 = a->w_up, p.bias = a->bias, p.y = a->y, p.y2 = a->y2;
   p.M = a->M, p.N = a->N, p.n1 = a->n1, p.ldx = a->ldx, p.ldw = a->ldw, p.ldy = a->ldy, p.ldy2 = a->ldy2, p.y_f32 = a->y_f32;
   p.glu = GluConst{a->limit, a->alpha, a->shift};
+  p.ep = Epilogue{a->act, a->mul, a->mul_rows, a->ldmul};
   return p;
 }
 
@@ -627,12 +653,16 @@ extern "C" int exo_post_linear_fits(int M, int N, int H, int ldx, int dtype) {
 extern "C" int exo_post_linear(const exo_post_norm* q, const exo_linear* a, exo_stream_t stream) {
   int rc = linear_check(a, "exo_post_linear");
   if (rc) return rc;
-  EXO_REQUIRE(q && q->x && q->branch && q->gain && q->x_out && q->x_out != q->x, "exo_post_linear: null pointer or x_out == x");
+  EXO_REQUIRE(q && q->branch && q->gain && (q->x ? q->x_out && q->x_out != q->x : !q->x_out && !q->sum),
+              "exo_post_linear: null pointer or x_out == x");
+  EXO_REQUIRE(q->ldb >= q->H && !(q->sum && q->branch2) && (q->sum || !q->center),
+              "exo_post_linear: branch stride %d of %d columns, or a norm of the sum of two branches", q->ldb, q->H);
   EXO_REQUIRE(!q->branch2 || (q->gain_a && q->gain_b), "exo_post_linear: two branches need a gain each");
   EXO_REQUIRE(post_fits(a->M, a->N, q->H, a->ldx, a->dtype == 0 ? 2 : 4), "exo_post_linear: %d rows of %d columns do not fit one launch",
               a->M, q->H);
   const GemvParams p = gemv_of(a);
-  const PostNorm n{q->x, q->branch, q->branch2, q->gain_a, q->gain_b, q->gain, q->pre, q->x_out, q->operand, q->H, q->eps, q->mult};
+  const PostNorm n{q->x, q->branch, q->branch2, q->gain_a, q->gain_b, q->gain, q->pre, q->x_out, q->operand, q->H, q->ldb,
+                   q->sum, q->center, q->eps, q->mult, q->keep};
   rc = EXO_BY_TYPE(a->dtype, launch_gemv<bf16_t>(p, nullptr, &n, (hipStream_t)stream),
                    launch_gemv<float>(p, nullptr, &n, (hipStream_t)stream));
   if (rc) return rc;
@@ -648,6 +678,7 @@ extern "C" int exo_linear_gemm(const exo_linear* a, float* workspace, int64_t wo
   p.x = a->x, p.w = a->w, p.w2 = a->w_up, p.bias = a->bias, p.y = a->y, p.y2 = a->y2;
   p.M = a->M, p.N = a->N, p.n1 = a->n1, p.ldx = a->ldx, p.ldw = a->ldw, p.ldy = a->ldy, p.ldy2 = a->ldy2, p.y_f32 = a->y_f32;
   p.glu = GluConst{a->limit, a->alpha, a->shift};
+  p.ep = Epilogue{a->act, a->mul, a->mul_rows, a->ldmul};
   p.part = a->w_up ? nullptr : workspace;
   EXO_REQUIRE(!a->w_up || a->y_f32 == (a->dtype == 1), "exo_linear_gemm: a gated pair leaves in the element type");
   if (a->w_up)

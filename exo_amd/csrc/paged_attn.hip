@@ -1,8 +1,9 @@
 // Attention over a paged KV pool, for batches that mix portions of prompts with single decoded
 // tokens.  Options, each a parameter of the layer: unit-RMS queries and keys (with a gain per
-// channel), a gate per head on the output (sigmoid of a given number), a per-head linear
-// distance penalty, a sliding window with kept first tokens, value size other than key size, keys
-// and values of another layer.  Scores, penalty, softmax and sums are float32; where the weights
+// channel), per head or over the whole projection, rotary positions (interleaved pairs), scores bent
+// to cap * tanh(score / cap), values mixed with another layer's values of the token, a gate per head on
+// the output (sigmoid of a given number), a per-head linear distance penalty, a sliding window with kept
+// first tokens, value size other than key size, keys and values of another layer.  Scores, penalty, softmax and sums are float32; where the weights
 // enter a bf16 matrix product they go in as two bf16 terms (high and remainder), so that they keep
 // 16 bits.
 //
@@ -20,12 +21,16 @@
 //   tiles that hold a visible key are dealt (kept first tokens, then the window).  Splits meet
 //   through device-scope partials and an arrival counter.  FUSE: the launch also normalises and
 //   stores the row's own key and value (the workgroup that owns the last tile does).
+// paged_prepare_kernel: norm over whole projections, rotation and value mixing of all rows of a step
+//   ahead of the other two (queries in place, keys and values into the pool); a step of single tokens
+//   does the same inside paged_rows_kernel.
 // paged_prompt_kernel: 32 query positions of one head per wave, four such units of one kv head and
 //   one sequence per workgroup sharing page-sized key tiles through LDS (two buffers, the next tile
 //   in registers meanwhile); 32x32 products, transposed like above so that running maximum, sum and
 //   rescale factor are per-lane scalars.
 #include "../../include/exo_mi355x.h"
 #include "dense.h"
+#include "rotary.h"
 
 namespace {
 
@@ -42,15 +47,26 @@ struct Params {
   const int32_t* pos;   // [R]
   const int32_t* list;  // rows: row indices (null: all); prompt: blocks of {row, slot, pos, n}
   const float* slopes;  // [H], or null
-  const float* qgain;   // [D], or null
-  const float* kgain;   // [D], or null
+  const float* qgain;   // [D] (whole: [H * D]), or null
+  const float* kgain;   // [D] (whole: [G * D]), or null
+  const double* freq;   // [rot / 2] turns per position
+  const void* vmix;     // T [R][ldmix] values mixed in, or null
   const float* gate;    // [R][ldg] a number per head, or null
   void* out;            // T [R][ldo]
   float* ws;
   int* counters;
-  float scale, eps;
-  int n, H, G, D, E, ldq, ldk, ldv, ldo, ldg, max_pages, size, keep, unit, nsplit, gsz, hgroups;
+  float scale, eps, cap, mix;  // cap 0: none
+  int n, H, G, D, E, ldq, ldk, ldv, ldo, ldg, ldmix, max_pages, size, keep, unit, whole, rot, nsplit, gsz, hgroups;
 };
+// expanded latent keys and values (latent_attn.hip) in place of the pool: rows of a sequence from its
+// block's second entry on
+struct Expanded {
+  const bf16_t* k;      // [keys][ldk]: head h's d8 entries at h * d8
+  const bf16_t* kr;     // [keys][r8]: shared by the heads
+  const bf16_t* v;      // [heads * E][ldv]: positions in a run
+  int ldk, ldv, d8, r8, qs, rot_col;  // queries: head h's at h * qs, its rotated part at rot_col + h * r8
+};
+constexpr int kMaxRot = 256;
 
 __device__ __forceinline__ void st_dev(float* p, float v) {
   __hip_atomic_store(p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
@@ -92,18 +108,42 @@ __device__ __forceinline__ void unit_row(const T* __restrict__ src, T* dst, int 
   for (int d = lane; d < D; d += 64) dst[d] = Elem<T>::make(Elem<T>::load(src[d]) * inv * (gain ? gain[d] : 1.f));
 }
 
+// one wave: the pairs of src[0..D) times inv and gain, the first `rot` entries turned -> dst (may be src)
+template <typename T>
+__device__ __forceinline__ void turn_row(const T* src, T* dst, int D, float inv, const float* __restrict__ gain,
+                                         const float2* cs, int rot, int lane) {
+  for (int i = lane; 2 * i < D; i += 64) {
+    const bool two = 2 * i + 1 < D;
+    float2 x{Elem<T>::load(src[2 * i]) * inv, two ? Elem<T>::load(src[2 * i + 1]) * inv : 0.f};
+    if (gain) x.x *= gain[2 * i], x.y *= two ? gain[2 * i + 1] : 0.f;
+    if (2 * i < rot) x = turn_pair(x.x, x.y, cs[i]);
+    dst[2 * i] = Elem<T>::make(x.x);
+    if (two) dst[2 * i + 1] = Elem<T>::make(x.y);
+  }
+}
+// the token's value column, mixed with the other layer's
+template <typename T>
+__device__ __forceinline__ T mixed_value(const Params& p, T v, int row, int c) {
+  if (!p.vmix) return v;
+  const float o = Elem<T>::load(reinterpret_cast<const T*>(p.vmix)[(size_t)row * p.ldmix + c]);
+  return Elem<T>::make((1.f - p.mix) * Elem<T>::load(v) + p.mix * o);
+}
+
 // key and value of one (row, kv head) into the pool, by one wave each
 template <typename T>
-__device__ __forceinline__ void put_key(const Params& p, int row, int g, int page, int at, int lane) {
+__device__ __forceinline__ void put_key(const Params& p, int row, int g, int page, int at, int lane, float inv, const float2* cs) {
   const T* src = reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + p.H * p.D + g * p.D;
   T* dst = reinterpret_cast<T*>(p.kpool) + (((size_t)page * p.G + g) * kPage + at) * p.ldk;
-  unit_row<T>(src, dst, p.D, p.unit, p.eps, p.kgain, lane);
+  if (p.whole || p.rot)
+    turn_row<T>(src, dst, p.D, inv, p.kgain ? p.kgain + g * p.D : nullptr, cs, p.rot, lane);
+  else
+    unit_row<T>(src, dst, p.D, p.unit, p.eps, p.kgain, lane);
 }
 template <typename T>
 __device__ __forceinline__ void put_value(const Params& p, int row, int g, int page, int at, int lane) {
   const T* src = reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + (p.H + p.G) * p.D + g * p.E;
   T* dst = reinterpret_cast<T*>(p.vpool) + ((size_t)page * p.G + g) * p.ldv * kPage + at;
-  for (int d = lane; d < p.E; d += 64) dst[(size_t)d * kPage] = src[d];
+  for (int d = lane; d < p.E; d += 64) dst[(size_t)d * kPage] = mixed_value<T>(p, src[d], row, g * p.E + d);
 }
 
 // A wave takes eight rows of one head: the keys' loads go out together, and the values of eight
@@ -203,6 +243,105 @@ __global__ __launch_bounds__(256) void paged_append_kernel(const Params p) {
   }
 }
 
+// Norm over whole projections, rotation and value mixing of eight rows, a wave each; then the values of
+// all kv heads, eight positions of a column per store where they lie in one run.  Queries stay in qkv.
+template <typename T>
+__device__ __forceinline__ void prepare_run(T* src, T* dst, int ldd, int heads, int D, float inv, const float* gain, const float2* cs,
+                                            int rot, bool vec, int lane) {
+  constexpr int VEC = Elem<T>::kVec;
+  if (vec) {
+    for (int c = lane * VEC; c < heads * D; c += 64 * VEC) {
+      const int h = c / D, d = c - h * D;
+      float f[VEC];
+      unpack_vec<T>(*reinterpret_cast<const uint4*>(src + c), f);
+      struct alignas(16) Vec {
+        T e[VEC];
+      } w;
+#pragma unroll
+      for (int e = 0; e < VEC; e += 2) {
+        float2 x{f[e] * inv, f[e + 1] * inv};
+        if (gain) x.x *= gain[c + e], x.y *= gain[c + e + 1];
+        if (d + e < rot) x = turn_pair(x.x, x.y, cs[(d + e) / 2]);
+        w.e[e] = Elem<T>::make(x.x), w.e[e + 1] = Elem<T>::make(x.y);
+      }
+      *reinterpret_cast<uint4*>(dst + (size_t)h * ldd + d) = __builtin_bit_cast(uint4, w);
+    }
+  } else {
+    for (int h = 0; h < heads; ++h)
+      turn_row<T>(src + h * D, dst + (size_t)h * ldd, D, inv, gain ? gain + h * D : nullptr, cs, rot, lane);
+  }
+}
+template <typename T>
+__device__ __forceinline__ float row_square_sum(const T* src, int n, bool vec, int lane) {
+  constexpr int VEC = Elem<T>::kVec;
+  float ss = 0.f;
+  if (vec) {
+    for (int c = lane * VEC; c < n; c += 64 * VEC) {
+      float f[VEC];
+      unpack_vec<T>(*reinterpret_cast<const uint4*>(src + c), f);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss += f[e] * f[e];
+    }
+  } else {
+    for (int c = lane; c < n; c += 64) ss += Elem<T>::load(src[c]) * Elem<T>::load(src[c]);
+  }
+  return wave_sum(ss);
+}
+
+template <typename T>
+__global__ __launch_bounds__(64 * kAppendRows) void paged_prepare_kernel(const Params p) {
+  __shared__ float2 cs[kAppendRows][kMaxRot / 2];
+  __shared__ int s_page[kAppendRows], s_pos[kAppendRows];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x >> 6);
+  const int row0 = blockIdx.x * kAppendRows, n = min(kAppendRows, p.n - row0);
+  constexpr int VEC = Elem<T>::kVec;
+  if (wave < n) {
+    const int row = row0 + wave, pos = p.pos[row];
+    const int page = p.table[(size_t)p.slot[row] * p.max_pages + pos / kPage];
+    if (lane == 0) s_page[wave] = page, s_pos[wave] = pos;
+    for (int i = lane; 2 * i < p.rot; i += 64) cs[wave][i] = turn_of(pos, p.freq[i]);  // (read by this wave only)
+    T* q = const_cast<T*>(reinterpret_cast<const T*>(p.qkv)) + (size_t)row * p.ldq;
+    T* k = q + p.H * p.D;
+    const bool vec = p.D % VEC == 0 && p.ldq % VEC == 0;
+    const float iq = p.whole ? 1.f / sqrtf(row_square_sum<T>(q, p.H * p.D, vec, lane) / (p.H * p.D) + p.eps) : 1.f;
+    const float ik = p.whole ? 1.f / sqrtf(row_square_sum<T>(k, p.G * p.D, vec, lane) / (p.G * p.D) + p.eps) : 1.f;
+    prepare_run<T>(q, q, p.D, p.H, p.D, iq, p.qgain, cs[wave], p.rot, vec, lane);
+    T* dst = reinterpret_cast<T*>(p.kpool) + ((size_t)page * p.G * kPage + pos % kPage) * p.ldk;
+    prepare_run<T>(k, dst, kPage * p.ldk, p.G, p.D, ik, p.kgain, cs[wave], p.rot, vec, lane);
+  }
+  __syncthreads();
+  bool run = n == kAppendRows && s_pos[0] % kAppendRows == 0;
+#pragma unroll
+  for (int i = 1; i < kAppendRows; ++i)
+    if (i < n) run = run && s_page[i] == s_page[0] && s_pos[i] == s_pos[0] + i;
+  for (int c = threadIdx.x; c < p.G * p.E; c += 64 * kAppendRows) {
+    const int g = c / p.E, d = c - g * p.E;
+    T v[kAppendRows];
+#pragma unroll
+    for (int i = 0; i < kAppendRows; ++i) {
+      const int row = row0 + min(i, n - 1);
+      v[i] = mixed_value<T>(p, reinterpret_cast<const T*>(p.qkv)[(size_t)row * p.ldq + (p.H + p.G) * p.D + c], row, c);
+    }
+    if (run) {
+      T* dst = reinterpret_cast<T*>(p.vpool) + (((size_t)s_page[0] * p.G + g) * p.ldv + d) * kPage + s_pos[0] % kPage;
+      constexpr int per = 16 / (int)sizeof(T);
+#pragma unroll
+      for (int k = 0; k < kAppendRows; k += per) {
+        struct alignas(16) Vec {
+          T e[per];
+        } w;
+#pragma unroll
+        for (int i = 0; i < per; ++i) w.e[i] = v[k + i];
+        *reinterpret_cast<uint4*>(dst + k) = __builtin_bit_cast(uint4, w);
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < kAppendRows; ++i)
+        if (i < n) reinterpret_cast<T*>(p.vpool)[(((size_t)s_page[i] * p.G + g) * p.ldv + d) * kPage + s_pos[i] % kPage] = v[i];
+    }
+  }
+}
+
 template <typename T>
 struct PTerms;  // softmax weights of 32 keys as B operands
 template <>
@@ -262,6 +401,7 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
   T* qs = reinterpret_cast<T*>(lds_raw);                          // [16][QS]
   float* os = reinterpret_cast<float*>(lds_raw);                  // later: [waves][gsz][ldv]
   __shared__ float ms[kRowWaves][16], ls[kRowWaves][16];
+  __shared__ float2 cs[kMaxRot / 2];
   __shared__ int s_last;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane((int)threadIdx.x >> 6);
   const int r = lane & 15, g = lane >> 4;
@@ -302,14 +442,39 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
   if (early) load_tile(tile, tl.at(j) * 32);
 
   // ---- queries (and the row's own key and value) through float32 norms
+  float iq = 1.f, ik = 1.f;
+  const bool turned = p.whole || p.rot;
+  if (turned) {  // angles, and the RMS of the whole projections, once per workgroup
+    const T* src = reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq;
+    for (int i = threadIdx.x; 2 * i < p.rot; i += 64 * kRowWaves) cs[i] = turn_of(pos, p.freq[i]);
+    if (p.whole) {
+      float sq = 0.f, sk = 0.f;
+      for (int c = threadIdx.x; c < p.H * p.D; c += 64 * kRowWaves) sq += Elem<T>::load(src[c]) * Elem<T>::load(src[c]);
+      if (FUSE)
+        for (int c = p.H * p.D + threadIdx.x; c < (p.H + p.G) * p.D; c += 64 * kRowWaves)
+          sk += Elem<T>::load(src[c]) * Elem<T>::load(src[c]);
+      sq = wave_sum(sq), sk = wave_sum(sk);
+      if (lane == 0) ms[wave][0] = sq, ms[wave][1] = sk;
+    }
+    __syncthreads();
+    if (p.whole) {
+      float sq = 0.f, sk = 0.f;
+#pragma unroll
+      for (int w = 0; w < kRowWaves; ++w) sq += ms[w][0], sk += ms[w][1];
+      iq = 1.f / sqrtf(sq / (p.H * p.D) + p.eps), ik = 1.f / sqrtf(sk / (p.G * p.D) + p.eps);
+    }
+  }
   for (int h = wave; h < 16; h += kRowWaves) {
     T* dst = qs + h * QS;
-    if (h < gs) unit_row<T>(reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + (h0 + h) * p.D, dst, p.D, p.unit, p.eps, p.qgain, lane);
+    if (h < gs && turned)
+      turn_row<T>(reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + (h0 + h) * p.D, dst, p.D, iq,
+                  p.qgain ? p.qgain + (h0 + h) * p.D : nullptr, cs, p.rot, lane);
+    else if (h < gs) unit_row<T>(reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq + (h0 + h) * p.D, dst, p.D, p.unit, p.eps, p.qgain, lane);
     for (int d = (h < gs ? p.D : 0) + lane; d < QS; d += 64) dst[d] = Elem<T>::make(0.f);
   }
   if (FUSE && split == ((tl.n - 1) % stride) / kRowWaves) {
     const int page = table[pos / kPage];
-    if (wave == kRowWaves - 1) put_key<T>(p, row, kvh, page, pos % kPage, lane);
+    if (wave == kRowWaves - 1) put_key<T>(p, row, kvh, page, pos % kPage, lane, ik, cs);
     if (wave == kRowWaves - 2) put_value<T>(p, row, kvh, page, pos % kPage, lane);
     wait_own_stores_done();
   }
@@ -320,7 +485,7 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
   for (int s = 0; s < KST; ++s)
     q[s] = *reinterpret_cast<const uint4*>(reinterpret_cast<const char*>(qs + r * QS) + s * 64 + g * 16);
 
-  const float sc = p.scale * kLog2e;
+  const float sc = p.cap > 0.f ? p.scale / p.cap : p.scale * kLog2e, cap2 = p.cap * kLog2e;
   const float slope = p.slopes && r < gs ? p.slopes[h0 + r] * kLog2e : 0.f;
   floatx4 o[VT];
 #pragma unroll
@@ -338,12 +503,18 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
       }
     float x0[4], x1[4], mx = -INFINITY;
 #pragma unroll
+    for (int e = 0; e < 4; ++e) s0[e] *= sc, s1[e] *= sc;
+    if (p.cap > 0.f) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s0[e] = cap2 * tanhf(s0[e]), s1[e] = cap2 * tanhf(s1[e]);
+    }
+#pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int ja = key0 + 4 * g + e, jb = ja + 16;
       const bool va = ja <= pos && (pos - ja < p.size || ja < p.keep);
       const bool vb = jb <= pos && (pos - jb < p.size || jb < p.keep);
-      x0[e] = va ? s0[e] * sc - slope * (float)(pos - ja) : -INFINITY;
-      x1[e] = vb ? s1[e] * sc - slope * (float)(pos - jb) : -INFINITY;
+      x0[e] = va ? s0[e] - slope * (float)(pos - ja) : -INFINITY;
+      x1[e] = vb ? s1[e] - slope * (float)(pos - jb) : -INFINITY;
       mx = fmaxf(mx, fmaxf(x0[e], x1[e]));
     }
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -459,17 +630,18 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
 // ------------------------------------------------------------------------------ prompts
 constexpr int kPadK = 8;
 
-template <int D>
+template <int DK, int DV>
 constexpr int prompt_lds() {
-  return 2 * (kPage * (D + kPadK) + D * (kPage + kPadK)) * 2;
+  return 2 * (kPage * (DK + kPadK) + DV * (kPage + kPadK)) * 2;
 }
 
-// HW: query heads per workgroup (4, 2, 1); its other factor is token tiles of 32
-template <int D, int HW>
-__global__ __launch_bounds__(256, D > 128 ? 1 : 2) void paged_prompt_kernel(const Params p) {
-  constexpr int STEPS = D / 16, DT = D / 32, KS = D + kPadK, VS = kPage + kPadK;
-  constexpr int VEC = D / 8, LOADS = kPage * VEC / 256;
-  constexpr int BUF = kPage * KS + D * VS;
+// DK, DV: key and value size at most; HW: query heads per workgroup (4, 2, 1), its other factor is token
+// tiles of 32; ROWS: expanded keys and values instead of the pool's (HW 1)
+template <int DK, int DV, int HW, bool ROWS>
+__global__ __launch_bounds__(256, DK > 128 ? 1 : 2) void paged_prompt_kernel(const Params p, const Expanded x) {
+  constexpr int STEPS = DK / 16, DT = DV / 32, KS = DK + kPadK, VS = kPage + kPadK;
+  constexpr int VEC = DK / 8, LOADS = kPage * VEC / 256, VLOADS = DV / 32;
+  constexpr int BUF = kPage * KS + DV * VS;
   constexpr int TT = 4 / HW;  // token tiles per workgroup
   extern __shared__ __attribute__((aligned(16))) bf16_t lds[];  // [2][BUF]
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -483,20 +655,25 @@ __global__ __launch_bounds__(256, D > 128 ? 1 : 2) void paged_prompt_kernel(cons
   const int t_lane = min(tt * 32 + n, blk.w - 1);  // this lane's token of the block
   const int row = blk.x + t_lane, qpos = blk.z + t_lane;
   const int wfirst = blk.z + min(tt * 32, blk.w - 1), wlast = blk.z + min(tt * 32 + 31, blk.w - 1);
-  const int32_t* table = p.table + (size_t)blk.y * p.max_pages;
+  const int32_t* table = ROWS ? nullptr : p.table + (size_t)blk.y * p.max_pages;
   const Tiles tl = tiles_of(blk.z, blk.z + blk.w - 1, p.size, p.keep, kPage);
 
   // Q^T operand: lane (query n, half kq) holds d = 16 step + 8 kq .. + 8, normalised in float32
   uint4 q[STEPS];
   {
-    const bf16_t* qp = reinterpret_cast<const bf16_t*>(p.qkv) + (size_t)row * p.ldq + (size_t)hq * p.D;
+    const bf16_t* qp = reinterpret_cast<const bf16_t*>(p.qkv) + (size_t)row * p.ldq + (size_t)hq * (ROWS ? x.qs : p.D);
     float ss = 0.f;
     const bool vec = p.D % 8 == 0 && p.ldq % 8 == 0;
 #pragma unroll
     for (int s = 0; s < STEPS; ++s) {
       const int d0 = 16 * s + 8 * kq;
       uint32_t w[4];
-      if (vec) {
+      if (ROWS) {
+        const bf16_t* at = d0 < x.d8 ? qp + d0
+                                     : reinterpret_cast<const bf16_t*>(p.qkv) + (size_t)row * p.ldq + x.rot_col + hq * x.r8 + (d0 - x.d8);
+        const uint4 v = d0 < x.d8 + x.r8 ? *reinterpret_cast<const uint4*>(at) : uint4{0, 0, 0, 0};
+        w[0] = v.x, w[1] = v.y, w[2] = v.z, w[3] = v.w;
+      } else if (vec) {
         const uint4 v = d0 < p.D ? *reinterpret_cast<const uint4*>(qp + d0) : uint4{0, 0, 0, 0};
         w[0] = v.x, w[1] = v.y, w[2] = v.z, w[3] = v.w;
       } else {
@@ -528,9 +705,24 @@ __global__ __launch_bounds__(256, D > 128 ? 1 : 2) void paged_prompt_kernel(cons
     }
   }
 
-  uint4 kreg[LOADS], vreg[LOADS];
+  uint4 kreg[LOADS], vreg[VLOADS];
   const uint32_t kbytes = kPage * (uint32_t)p.ldk * 2, vbytes = (uint32_t)p.ldv * kPage * 2;
-  auto load_tile = [&](int j) {
+  auto load_tile = [&](int j) __attribute__((always_inline)) {
+    if (ROWS) {  // (columns past a key's and rows past the values': any finite ones)
+      const int key = blk.y + tl.at(j) * kPage;
+#pragma unroll
+      for (int i = 0; i < LOADS; ++i) {
+        const int vi = tid + i * 256, kr = key + vi / VEC, kc = vi % VEC * 8;
+        const bf16_t* at = kc < x.d8 ? x.k + (size_t)kr * x.ldk + hq * x.d8 + kc : x.kr + (size_t)kr * x.r8 + min(kc - x.d8, x.r8 - 8);
+        kreg[i] = load16(at);
+      }
+#pragma unroll
+      for (int i = 0; i < VLOADS; ++i) {
+        const int vi = tid + i * 256;
+        vreg[i] = load16(x.v + (size_t)(hq * p.E + min(vi >> 3, p.E - 1)) * x.ldv + key + (vi & 7) * 8);
+      }
+      return;
+    }
     const size_t head = (size_t)table[tl.at(j)] * p.G + kvh;
     const __amdgpu_buffer_rsrc_t rk = buf_of(reinterpret_cast<const bf16_t*>(p.kpool) + head * kPage * p.ldk, kbytes);
     const __amdgpu_buffer_rsrc_t rv = buf_of(reinterpret_cast<const bf16_t*>(p.vpool) + head * p.ldv * kPage, vbytes);
@@ -538,8 +730,9 @@ __global__ __launch_bounds__(256, D > 128 ? 1 : 2) void paged_prompt_kernel(cons
     for (int i = 0; i < LOADS; ++i) {
       const int vi = tid + i * 256, kr = vi / VEC, kc = vi % VEC;
       kreg[i] = buf_load16(rk, kc * 8 < p.ldk ? (kr * p.ldk + kc * 8) * 2 : kPastEnd, 0);
-      vreg[i] = buf_load16(rv, vi * 16, 0);  // rows of 64 positions; rows past ldv read as zero
     }
+#pragma unroll
+    for (int i = 0; i < VLOADS; ++i) vreg[i] = buf_load16(rv, (tid + i * 256) * 16, 0);  // rows of 64 positions; rows past ldv read as zero
   };
   auto store_tile = [&](int b) {
     bf16_t* kl = lds + b * BUF;
@@ -548,6 +741,10 @@ __global__ __launch_bounds__(256, D > 128 ? 1 : 2) void paged_prompt_kernel(cons
     for (int i = 0; i < LOADS; ++i) {
       const int vi = tid + i * 256;
       *reinterpret_cast<uint4*>(&kl[(vi / VEC) * KS + (vi % VEC) * 8]) = kreg[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VLOADS; ++i) {
+      const int vi = tid + i * 256;
       *reinterpret_cast<uint4*>(&vl[(vi >> 3) * VS + (vi & 7) * 8]) = vreg[i];
     }
   };
@@ -555,7 +752,7 @@ __global__ __launch_bounds__(256, D > 128 ? 1 : 2) void paged_prompt_kernel(cons
   // lane half kq are keys 16s + 8kq .. + 8 (the B operand order of the second product)
   const int jr = n >> 3;
   const int key_of_row = 16 * (jr >> 1) + 8 * ((n >> 2) & 1) + 4 * (jr & 1) + (n & 3);
-  const float sc = p.scale * kLog2e;
+  const float sc = p.scale * kLog2e, cap2 = p.cap * kLog2e, icap = p.cap > 0.f ? 2.f * kLog2e * p.scale / p.cap : 0.f;
   const float slope = p.slopes ? p.slopes[hq] * kLog2e : 0.f;
 
   floatx16 o[DT];
@@ -594,15 +791,23 @@ __global__ __launch_bounds__(256, D > 128 ? 1 : 2) void paged_prompt_kernel(cons
     const int rel = qpos - key0 - 8 * kq;  // distance to the lane's first key
     const float base = -slope * (float)rel;
     float mx = -INFINITY;
+    if (p.cap > 0.f) {  // tanh(y) = 1 - 2 / (e^2y + 1)
+#pragma unroll
+      for (int ks = 0; ks < 2; ++ks)
+#pragma unroll
+        for (int e = 0; e < 16; ++e)
+          s[ks][e] = cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s[ks][e] * icap) + 1.f);
+    }
+    const float scl = p.cap > 0.f ? 1.f : sc;
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks)
 #pragma unroll
       for (int e = 0; e < 16; ++e) {
         const int k = ks * 32 + 16 * (e >> 3) + (e & 7);
-        float x = fmaf(s[ks][e], sc, fmaf(slope, (float)k, base));
-        if (partial && (k > rel || (rel - k >= p.size && key0 + 8 * kq + k >= p.keep))) x = -INFINITY;
-        s[ks][e] = x;
-        mx = fmaxf(mx, x);
+        float sv = fmaf(s[ks][e], scl, fmaf(slope, (float)k, base));
+        if (partial && (k > rel || (rel - k >= p.size && key0 + 8 * kq + k >= p.keep))) sv = -INFINITY;
+        s[ks][e] = sv;
+        mx = fmaxf(mx, sv);
       }
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
     const float mn = fmaxf(m, mx), mr = mn == -INFINITY ? 0.f : mn;  // (a query may see none of the tile)
@@ -673,6 +878,8 @@ Params params_of(const exo_paged_attn* a) {
   p.ldq = a->ldq, p.ldk = a->ldk, p.ldv = a->ldv, p.ldo = a->ldo, p.max_pages = a->max_pages;
   p.size = a->window > 0 ? a->window : 0x3FFFFFFF;
   p.keep = a->keep_first, p.unit = a->unit_qk;
+  p.freq = a->freq, p.vmix = a->v_mix, p.ldmix = a->ldmix, p.mix = a->mix, p.cap = a->softcap, p.whole = a->whole_norm, p.rot = a->rot;
+  if (a->prepared) p.unit = p.whole = p.rot = 0, p.qgain = p.kgain = nullptr;
   p.nsplit = 1;
   return p;
 }
@@ -687,7 +894,11 @@ int check(const exo_paged_attn* a, const char* what) {
               "%s: pool strides %d / %d do not fit head sizes %d / %d", what, a->ldk, a->ldv, a->dim, a->vdim);
   EXO_REQUIRE(a->qkv && a->k_pool && a->v_pool && a->table && a->max_pages > 0, "%s: null pointer", what);
   EXO_REQUIRE(!a->gate || a->ldg >= a->heads, "%s: %d gates per row for %d heads", what, a->ldg, a->heads);
-  EXO_REQUIRE(a->unit_qk || (!a->q_gain && !a->k_gain), "%s: a query / key gain belongs to the norm", what);
+  EXO_REQUIRE(a->rot >= 0 && a->rot % 2 == 0 && a->rot <= a->dim && a->rot <= kMaxRot && (!a->rot || a->freq) && !(a->rot && a->unit_qk),
+              "%s: %d rotated dimensions of %d (an even number, angles given, no norm per head)", what, a->rot, a->dim);
+  EXO_REQUIRE(!a->whole_norm || (!a->unit_qk && a->q_gain && a->k_gain), "%s: one norm, with gains over the whole projections", what);
+  EXO_REQUIRE(a->softcap >= 0.f && (!a->v_mix || a->ldmix >= a->kv_heads * a->vdim), "%s: bad cap or mixed values", what);
+  EXO_REQUIRE(a->unit_qk || a->whole_norm || (!a->q_gain && !a->k_gain), "%s: a query / key gain belongs to the norm", what);
   EXO_REQUIRE(a->keep_first >= 0 && a->window >= 0, "%s: negative window", what);
   return EXO_OK;
 }
@@ -722,11 +933,11 @@ int launch_rows_d(const Params& p, int d, bool fuse, hipStream_t st) {
   return d <= 64 ? launch_rows_f<T, 64>(p, fuse, st) : d <= 128 ? launch_rows_f<T, 128>(p, fuse, st) : launch_rows_f<T, 256>(p, fuse, st);
 }
 
-template <int D, int HW>
-int launch_prompt(const Params& p, hipStream_t st) {
-  constexpr int lds = prompt_lds<D>();
+template <int DK, int DV, int HW, bool ROWS = false>
+int launch_prompt(const Params& p, hipStream_t st, const Expanded& x = Expanded{}) {
+  constexpr int lds = prompt_lds<DK, DV>();
   static bool done = false;
-  const auto fn = paged_prompt_kernel<D, HW>;
+  const auto fn = paged_prompt_kernel<DK, DV, HW, ROWS>;
   if (!done && lds > 64 * 1024) {
     const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     if (e != hipSuccess) {
@@ -737,14 +948,14 @@ int launch_prompt(const Params& p, hipStream_t st) {
   done = true;
   const int group = p.H / p.G;
   const dim3 grid(p.n, p.G * ((group + HW - 1) / HW));
-  exo_note_variant("paged_prompt<%d,%d> grid=%dx%d", D, HW, (int)grid.x, (int)grid.y);
-  fn<<<grid, 256, lds, st>>>(p);
+  exo_note_variant("paged_prompt<%d,%d,%d,%s> grid=%dx%d", DK, DV, HW, ROWS ? "rows" : "pool", (int)grid.x, (int)grid.y);
+  fn<<<grid, 256, lds, st>>>(p, x);
   return EXO_OK;
 }
 template <int D>
 int launch_prompt_h(const Params& p, hipStream_t st) {
   const int group = p.H / p.G;
-  return group >= 3 ? launch_prompt<D, 4>(p, st) : group == 2 ? launch_prompt<D, 2>(p, st) : launch_prompt<D, 1>(p, st);
+  return group >= 3 ? launch_prompt<D, D, 4>(p, st) : group == 2 ? launch_prompt<D, D, 2>(p, st) : launch_prompt<D, D, 1>(p, st);
 }
 
 }  // namespace
@@ -754,6 +965,7 @@ extern "C" int exo_paged_append(const exo_paged_attn* a, exo_stream_t stream) {
   if (rc) return rc;
   EXO_REQUIRE(a->slot && a->pos && a->ldq >= (a->heads + a->kv_heads) * a->dim + a->kv_heads * a->vdim,
               "exo_paged_append: rows of %d elements do not hold q, k and v", a->ldq);
+  EXO_REQUIRE(!a->whole_norm && !a->rot && !a->v_mix, "exo_paged_append: a norm over whole projections, rotations and mixed values need exo_paged_prepare");
   const Params p = params_of(a);
   const dim3 grid((p.n + kAppendRows - 1) / kAppendRows, (2 * p.G + 3) / 4);
   if (a->dtype == 0)
@@ -761,6 +973,21 @@ extern "C" int exo_paged_append(const exo_paged_attn* a, exo_stream_t stream) {
   else
     paged_append_kernel<float><<<grid, 256, 0, (hipStream_t)stream>>>(p);
   EXO_CHECK_LAUNCH("exo_paged_append");
+  return EXO_OK;
+}
+
+extern "C" int exo_paged_prepare(const exo_paged_attn* a, exo_stream_t stream) {
+  const int rc = check(a, "exo_paged_prepare");
+  if (rc) return rc;
+  EXO_REQUIRE(a->slot && a->pos && !a->prepared && !a->unit_qk && a->ldq >= (a->heads + a->kv_heads) * a->dim + a->kv_heads * a->vdim,
+              "exo_paged_prepare: rows of %d elements do not hold q, k and v, or a norm per head", a->ldq);
+  const Params p = params_of(a);
+  const int grid = (p.n + kAppendRows - 1) / kAppendRows;
+  if (a->dtype == 0)
+    paged_prepare_kernel<bf16_t><<<grid, 64 * kAppendRows, 0, (hipStream_t)stream>>>(p);
+  else
+    paged_prepare_kernel<float><<<grid, 64 * kAppendRows, 0, (hipStream_t)stream>>>(p);
+  EXO_CHECK_LAUNCH("exo_paged_prepare");
   return EXO_OK;
 }
 
@@ -808,6 +1035,7 @@ extern "C" int exo_paged_attn_prompt(const exo_paged_attn* a, exo_stream_t strea
   const int rc = check(a, "exo_paged_attn_prompt");
   if (rc) return rc;
   EXO_REQUIRE(a->dtype == 0, "exo_paged_attn_prompt: bf16 only");
+  EXO_REQUIRE(a->prepared || !(a->whole_norm || a->rot), "exo_paged_attn_prompt: queries must be prepared (exo_paged_prepare)");
   EXO_REQUIRE(a->list && a->out && a->ldo >= a->heads * a->vdim && a->ldq >= a->heads * a->dim && a->ldo % 4 == 0 &&
                   a->ldk % 8 == 0,
               "exo_paged_attn_prompt: bad rows or output");
@@ -817,5 +1045,28 @@ extern "C" int exo_paged_attn_prompt(const exo_paged_attn* a, exo_stream_t strea
   const int rc2 = d <= 64 ? launch_prompt_h<64>(p, st) : d <= 128 ? launch_prompt_h<128>(p, st) : launch_prompt_h<256>(p, st);
   if (rc2) return rc2;
   EXO_CHECK_LAUNCH("exo_paged_attn_prompt");
+  return EXO_OK;
+}
+
+extern "C" int exo_latent_prompt(const exo_latent_prompt_args* a, exo_stream_t stream) {
+  EXO_REQUIRE(a && a->q && a->k && a->k_rot && a->v && a->list && a->out && a->n > 0 && a->heads > 0 && a->heads <= 65535 && a->vdim > 0,
+              "exo_latent_prompt: null pointer or bad counts");
+  EXO_REQUIRE(a->d8 > 0 && a->d8 % 8 == 0 && a->r8 >= 8 && a->r8 % 8 == 0 && a->d8 + a->r8 <= 256 && a->vdim <= 256,
+              "exo_latent_prompt: key parts %d and %d (multiples of 8, at most 256 together), values %d", a->d8, a->r8, a->vdim);
+  EXO_REQUIRE(a->ldk >= a->heads * a->d8 && a->ldk % 8 == 0 && a->ldv % 64 == 0 && a->ldq % 8 == 0 && a->q_head % 8 == 0 &&
+                  a->q_head >= a->d8 && a->rot_col % 8 == 0 && a->rot_col >= a->heads * a->q_head &&
+                  a->ldq >= a->rot_col + a->heads * a->r8 && a->ldo >= a->heads * a->vdim && a->ldo % 4 == 0,
+              "exo_latent_prompt: bad row strides");
+  Params p{};
+  p.qkv = a->q, p.list = a->list, p.out = a->out, p.scale = a->scale, p.n = a->n, p.H = p.G = a->heads, p.D = a->d8, p.E = a->vdim;
+  p.ldq = a->ldq, p.ldo = a->ldo, p.size = 0x3FFFFFFF, p.nsplit = 1;
+  const Expanded x{(const bf16_t*)a->k, (const bf16_t*)a->k_rot, (const bf16_t*)a->v, a->ldk, a->ldv, a->d8, a->r8, a->q_head, a->rot_col};
+  const int dk = a->d8 + a->r8;
+  const hipStream_t st = (hipStream_t)stream;
+  const int rc = dk <= 128 && a->vdim <= 128   ? launch_prompt<128, 128, 1, true>(p, st, x)
+                 : dk <= 192 && a->vdim <= 128 ? launch_prompt<192, 128, 1, true>(p, st, x)
+                                               : launch_prompt<256, 256, 1, true>(p, st, x);
+  if (rc) return rc;
+  EXO_CHECK_LAUNCH("exo_latent_prompt");
   return EXO_OK;
 }

@@ -1,0 +1,16 @@
+// Rotary positions in the interleaved layout: the pair (x[2i], x[2i+1]) turned by position * f_i.  f_i is
+// given in turns per position as a double, so that the angle keeps float32 accuracy at any position:
+// the product is exact to 2^-53 of a turn count, whole turns fall away, and the rest is a float.
+#pragma once
+#include "common.h"
+
+__device__ __forceinline__ float2 turn_of(int pos, double turns_per_position) {
+  double t = (double)pos * turns_per_position;
+  t -= floor(t);
+  float2 cs;
+  sincospif(2.f * (float)t, &cs.y, &cs.x);
+  return cs;  // cos, sin
+}
+__device__ __forceinline__ float2 turn_pair(float u, float v, float2 cs) {
+  return float2{u * cs.x - v * cs.y, v * cs.x + u * cs.y};
+}

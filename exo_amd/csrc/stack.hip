@@ -27,28 +27,32 @@ __device__ __forceinline__ float block_sum(float v, float* tmp) {
 // ------------------------------------------------------------------------------ embedding
 template <typename T>
 __global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const T* __restrict__ table, float* __restrict__ x,
-                                  T* __restrict__ xb, int V, int H, int ldt, int ldx) {
+                                  T* __restrict__ xb, int V, int H, int ldt, int ldx, float scale) {
   const int row = blockIdx.x;
   const int id = min(max(ids[row], 0), V - 1);
   for (int c = threadIdx.x; c < H; c += blockDim.x) {
-    const T v = table[(size_t)id * ldt + c];
-    x[(size_t)row * H + c] = Elem<T>::load(v);
-    xb[(size_t)row * ldx + c] = v;
+    const float v = Elem<T>::load(table[(size_t)id * ldt + c]) * scale;
+    x[(size_t)row * H + c] = v;
+    xb[(size_t)row * ldx + c] = Elem<T>::make(v);
   }
 }
 
 // ------------------------------------------------------------------------------ norms
-// y = x / rms(x) * gain, rows given by an index list (null: row i)
+// y = x / rms(x) * gain (center: the mean is taken off x first), rows given by an index list (null: row i)
 template <typename T, int TH>
 __global__ __launch_bounds__(TH) void norm_rows_kernel(const float* __restrict__ x, const int32_t* __restrict__ rows,
-                                                       const float* __restrict__ gain, T* __restrict__ y, int H, int ldy,
-                                                       float eps) {
+                                                       const float* __restrict__ gain, T* __restrict__ y, int H, int ldx,
+                                                       int ldy, float eps, int center) {
   __shared__ float tmp[TH / 64];
-  const float* xr = x + (size_t)(rows ? rows[blockIdx.x] : (int)blockIdx.x) * H;
-  float ss = 0.f;
-  for (int c = threadIdx.x; c < H; c += TH) ss += xr[c] * xr[c];
+  const float* xr = x + (size_t)(rows ? rows[blockIdx.x] : (int)blockIdx.x) * ldx;
+  float mean = 0.f, ss = 0.f;
+  if (center) {
+    for (int c = threadIdx.x; c < H; c += TH) mean += xr[c];
+    mean = block_sum<TH>(mean, tmp) / H;
+  }
+  for (int c = threadIdx.x; c < H; c += TH) ss += (xr[c] - mean) * (xr[c] - mean);
   const float inv = 1.f / sqrtf(block_sum<TH>(ss, tmp) / H + eps);
-  for (int c = threadIdx.x; c < H; c += TH) y[(size_t)blockIdx.x * ldy + c] = Elem<T>::make(xr[c] * inv * gain[c]);
+  for (int c = threadIdx.x; c < H; c += TH) y[(size_t)blockIdx.x * ldy + c] = Elem<T>::make((xr[c] - mean) * inv * gain[c]);
 }
 
 struct MoeSum {        // the feed-forward's output as a sum over a token's experts
@@ -57,11 +61,12 @@ struct MoeSum {        // the feed-forward's output as a sum over a token's expe
   const float* wt;     // [R][top]
   const void* shared;  // T [R][lds] output of the shared expert, or null
   const float* logits; // router logits; column E + identity is the shared expert's gate
-  int top, experts, ldy, lds, ldl, gate_col;
+  int top, experts, ldy, lds, ldl, gate_col;  // gate_col < 0: the shared expert as it is
 };
 
 // x += mult * gain * v / rms(v), v = the branch row, half the sum of two branches normed each with a
-// gain of its own, or the weighted sum over the experts; xb = x, or x / rms(x) * pre.
+// gain of its own, or the weighted sum over the experts; or (sum) x = gain * norm(keep * x + v); xb = x,
+// or x / rms(x) * pre.
 // Four columns per thread and pass (VEC: rows of four columns are aligned), v in registers.
 constexpr int kCols = 4;  // at most 16 passes: H <= 16384
 
@@ -83,12 +88,12 @@ __device__ __forceinline__ void load_cols(const T* p, float (&f)[kCols], bool ve
 }
 
 template <typename T, int TH, int PASSES>
-__global__ __launch_bounds__(TH) void post_norm_add_kernel(const exo_post_norm q, int ldb, const MoeSum m,
+__global__ __launch_bounds__(TH) void post_norm_add_kernel(const exo_post_norm q, const MoeSum m,
                                                                     float* __restrict__ x, T* __restrict__ xb, int ldx) {
   __shared__ float tmp[TH / 64];
   const int row = blockIdx.x, H = q.H;
   float* xr = x + (size_t)row * H;
-  const bool vec = H % kCols == 0 && (m.y ? m.ldy % kCols == 0 && m.lds % kCols == 0 : ldb % kCols == 0);
+  const bool vec = H % kCols == 0 && (m.y ? m.ldy % kCols == 0 && m.lds % kCols == 0 : q.ldb % kCols == 0);
   const bool gvec = H % kCols == 0;
   float v[PASSES][kCols], xv[PASSES][kCols];
   float pass = 0.f, sg = 0.f;  // weight of the input itself; gate of the shared expert
@@ -97,7 +102,7 @@ __global__ __launch_bounds__(TH) void post_norm_add_kernel(const exo_post_norm q
     y = reinterpret_cast<const T*>(m.y) + (size_t)row * m.top * m.ldy;
     if (m.shared) {
       sh = reinterpret_cast<const T*>(m.shared) + (size_t)row * m.lds;
-      sg = 1.f / (1.f + expf(-m.logits[(size_t)row * m.ldl + m.gate_col]));
+      sg = m.gate_col < 0 ? 1.f : 1.f / (1.f + expf(-m.logits[(size_t)row * m.ldl + m.gate_col]));
     }
     for (int j = 0; j < m.top; ++j)
       if (m.idx[row * m.top + j] >= m.experts) pass += m.wt[row * m.top + j];
@@ -126,7 +131,7 @@ __global__ __launch_bounds__(TH) void post_norm_add_kernel(const exo_post_norm q
         for (int e = 0; e < kCols; ++e) v[i][e] = fmaf(sg, f[e], v[i][e]);
       }
     } else {
-      load_cols<float>(q.branch + (size_t)row * ldb + c, v[i], vec, left);
+      load_cols<float>(q.branch + (size_t)row * q.ldb + c, v[i], vec, left);
     }
 #pragma unroll
     for (int e = 0; e < kCols; ++e) ss += e < left ? v[i][e] * v[i][e] : 0.f;
@@ -137,7 +142,7 @@ __global__ __launch_bounds__(TH) void post_norm_add_kernel(const exo_post_norm q
     for (int i = 0; i < PASSES; ++i) {
       const int c = (threadIdx.x + i * TH) * kCols, left = H - c;
       if (left <= 0) break;
-      load_cols<float>(q.branch2 + (size_t)row * ldb + c, u[i], vec, left);
+      load_cols<float>(q.branch2 + (size_t)row * q.ldb + c, u[i], vec, left);
 #pragma unroll
       for (int e = 0; e < kCols; ++e) su += e < left ? u[i][e] * u[i][e] : 0.f;
     }
@@ -157,7 +162,33 @@ __global__ __launch_bounds__(TH) void post_norm_add_kernel(const exo_post_norm q
       }
     }
   }
-  const float inv = q.mult / sqrtf(block_sum<TH>(ss, tmp) / H + q.eps);
+  if (q.sum) {  // the sum itself is normed
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < PASSES; ++i) {
+      const int c = (threadIdx.x + i * TH) * kCols, left = H - c;
+      if (left <= 0) break;
+#pragma unroll
+      for (int e = 0; e < kCols; ++e) {
+        v[i][e] = fmaf(q.keep, xv[i][e], v[i][e]);
+        xv[i][e] = 0.f;
+        s += e < left ? v[i][e] : 0.f;
+      }
+    }
+    const float mean = q.center ? block_sum<TH>(s, tmp) / H : 0.f;
+    ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < PASSES; ++i) {
+      const int c = (threadIdx.x + i * TH) * kCols, left = H - c;
+      if (left <= 0) break;
+#pragma unroll
+      for (int e = 0; e < kCols; ++e) {
+        v[i][e] -= mean;
+        ss += e < left ? v[i][e] * v[i][e] : 0.f;
+      }
+    }
+  }
+  const float inv = (q.sum ? 1.f : q.mult) / sqrtf(block_sum<TH>(ss, tmp) / H + q.eps);
   ss = 0.f;
 #pragma unroll
   for (int i = 0; i < PASSES; ++i) {
@@ -202,12 +233,13 @@ __global__ __launch_bounds__(TH) void post_norm_add_kernel(const exo_post_norm q
 
 // ------------------------------------------------------------------------------ routing
 // One wave per token: softmax over all N <= 64 NR outputs, the `top` largest of score + correction
-// (equals: the lower index), weight = score * scale.  On return lane j < top holds the j-th choice.
+// (equals: the lower index), weight = score * scale.  renorm: the largest of logit + correction instead,
+// weights = softmax over the chosen logits alone, times scale.  On return lane j < top holds the j-th choice.
 // Reductions on the DPP path; the winner's lane comes from a ballot, so a choice costs about a
 // hundred cycles.
 template <int NR>
 __device__ __forceinline__ void route_choose(const float* __restrict__ logits, const float* __restrict__ corr, int N,
-                                             int top, float scale, int lane, int& my_id, float& my_wt) {
+                                             int top, float scale, int renorm, int lane, int& my_id, float& my_wt) {
   float s[NR], c[NR];
   float mx = -INFINITY;
 #pragma unroll
@@ -218,7 +250,8 @@ __device__ __forceinline__ void route_choose(const float* __restrict__ logits, c
   }
 #pragma unroll
   for (int i = 0; i < NR; ++i) {
-    if (lane + 64 * i >= N) s[i] = -INFINITY;
+    if (lane + 64 * i >= N) s[i] = c[i] = -INFINITY;
+    if (renorm) c[i] += s[i];
     mx = fmaxf(mx, s[i]);
   }
   mx = wave_max_f32_uniform(mx);
@@ -231,8 +264,9 @@ __device__ __forceinline__ void route_choose(const float* __restrict__ logits, c
   sum = wave_sum_uniform(sum);
 #pragma unroll
   for (int i = 0; i < NR; ++i) {
+    if (renorm) continue;
     s[i] = s[i] / sum;
-    c[i] = lane + 64 * i < N ? s[i] + c[i] : -INFINITY;
+    c[i] += s[i];
   }
   my_id = 0;
   my_wt = 0.f;
@@ -254,16 +288,17 @@ __device__ __forceinline__ void route_choose(const float* __restrict__ logits, c
       }
     }
   }
+  if (renorm) my_wt = my_wt * scale / wave_sum_uniform(my_wt);
 }
 
 template <int NR>
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ logits, const float* __restrict__ corr,
                                                        int32_t* __restrict__ idx, float* __restrict__ wt, int N, int ldl,
-                                                       int top, float scale) {
+                                                       int top, float scale, int renorm) {
   const int row = blockIdx.x, lane = threadIdx.x;
   int id;
   float w;
-  route_choose<NR>(logits + (size_t)row * ldl, corr, N, top, scale, lane, id, w);
+  route_choose<NR>(logits + (size_t)row * ldl, corr, N, top, scale, renorm, lane, id, w);
   if (lane < top) {
     idx[(size_t)row * top + lane] = id;
     wt[(size_t)row * top + lane] = w;
@@ -286,7 +321,7 @@ struct MoeRows {
   const float* logits; // [R][ldl]
   const float* corr;   // routing inside the gated launch (null: idx and wt are given)
   float rscale;
-  int outputs;
+  int outputs, renorm;
   int R, top, experts, ff, sff, H, ldx, lda, ldsa, ldl, gate_col;
   GluConst glu, sglu;
 };
@@ -315,7 +350,7 @@ __global__ __launch_bounds__(64 * kGuWaves) void moe_glu_rows_kernel(const MoeRo
     if constexpr (NR > 0) {
       int id;
       float w;
-      route_choose<NR>(p.logits + (size_t)t * p.ldl, p.corr, p.outputs, p.top, p.rscale, lane, id, w);
+      route_choose<NR>(p.logits + (size_t)t * p.ldl, p.corr, p.outputs, p.top, p.rscale, p.renorm, lane, id, w);
       if (b == 0 && slot == 0 && wave == 0 && lane < p.top) {
         p.idx[pair + lane] = id;
         p.wt[pair + lane] = w;
@@ -413,7 +448,7 @@ __global__ __launch_bounds__(64 * kDnWaves) void moe_down_rows_kernel(const MoeR
     const char *w, *a;
     uint32_t rowb;
     if (sh) {
-      wt = 1.f / (1.f + expf(-p.logits[(size_t)t * p.ldl + p.gate_col]));
+      wt = p.gate_col < 0 ? 1.f : 1.f / (1.f + expf(-p.logits[(size_t)t * p.ldl + p.gate_col]));
       w = reinterpret_cast<const char*>(p.sdown);
       a = reinterpret_cast<const char*>(p.sact) + (size_t)t * srow;
       rowb = srow;
@@ -470,49 +505,50 @@ __global__ __launch_bounds__(64 * kDnWaves) void moe_down_rows_kernel(const MoeR
   } while (0)
 
 extern "C" int exo_embed_rows(const int32_t* ids, const void* table, float* x, void* xb, int n, int V, int H, int ldt,
-                              int ldx, int dtype, exo_stream_t stream) {
+                              int ldx, float scale, int dtype, exo_stream_t stream) {
   EXO_TYPE_OK("exo_embed_rows");
   EXO_REQUIRE(ids && table && x && xb && n >= 0 && V > 0 && H > 0 && ldt >= H && ldx >= H, "exo_embed_rows: bad argument");
   if (n == 0) return EXO_OK;
   if (dtype == 0)
-    embed_rows_kernel<bf16_t><<<n, 256, 0, (hipStream_t)stream>>>(ids, (const bf16_t*)table, x, (bf16_t*)xb, V, H, ldt, ldx);
+    embed_rows_kernel<bf16_t><<<n, 256, 0, (hipStream_t)stream>>>(ids, (const bf16_t*)table, x, (bf16_t*)xb, V, H, ldt, ldx, scale);
   else
-    embed_rows_kernel<float><<<n, 256, 0, (hipStream_t)stream>>>(ids, (const float*)table, x, (float*)xb, V, H, ldt, ldx);
+    embed_rows_kernel<float><<<n, 256, 0, (hipStream_t)stream>>>(ids, (const float*)table, x, (float*)xb, V, H, ldt, ldx, scale);
   EXO_CHECK_LAUNCH("exo_embed_rows");
   return EXO_OK;
 }
 
-extern "C" int exo_norm_rows(const float* x, const int32_t* rows, const float* gain, void* y, int n, int H, int ldy,
-                             float eps, int dtype, exo_stream_t stream) {
+extern "C" int exo_norm_rows(const float* x, const int32_t* rows, const float* gain, void* y, int n, int H, int ldx,
+                             int ldy, float eps, int center, int dtype, exo_stream_t stream) {
   EXO_TYPE_OK("exo_norm_rows");
-  EXO_REQUIRE(x && gain && y && n >= 0 && H > 0 && ldy >= H, "exo_norm_rows: bad argument");
+  EXO_REQUIRE(x && gain && y && n >= 0 && H > 0 && ldx >= H && ldy >= H, "exo_norm_rows: bad argument");
   if (n == 0) return EXO_OK;
   const hipStream_t st = (hipStream_t)stream;
   if (n <= 256 && H > 1024) {
     if (dtype == 0)
-      norm_rows_kernel<bf16_t, 1024><<<n, 1024, 0, st>>>(x, rows, gain, (bf16_t*)y, H, ldy, eps);
+      norm_rows_kernel<bf16_t, 1024><<<n, 1024, 0, st>>>(x, rows, gain, (bf16_t*)y, H, ldx, ldy, eps, center);
     else
-      norm_rows_kernel<float, 1024><<<n, 1024, 0, st>>>(x, rows, gain, (float*)y, H, ldy, eps);
+      norm_rows_kernel<float, 1024><<<n, 1024, 0, st>>>(x, rows, gain, (float*)y, H, ldx, ldy, eps, center);
   } else if (dtype == 0)
-    norm_rows_kernel<bf16_t, 256><<<n, 256, 0, st>>>(x, rows, gain, (bf16_t*)y, H, ldy, eps);
+    norm_rows_kernel<bf16_t, 256><<<n, 256, 0, st>>>(x, rows, gain, (bf16_t*)y, H, ldx, ldy, eps, center);
   else
-    norm_rows_kernel<float, 256><<<n, 256, 0, st>>>(x, rows, gain, (float*)y, H, ldy, eps);
+    norm_rows_kernel<float, 256><<<n, 256, 0, st>>>(x, rows, gain, (float*)y, H, ldx, ldy, eps, center);
   EXO_CHECK_LAUNCH("exo_norm_rows");
   return EXO_OK;
 }
 
-static int post_norm(const exo_post_norm* q, int ldb, const MoeSum& m, int n, int ldx, int dtype, exo_stream_t stream) {
+static int post_norm(const exo_post_norm* q, const MoeSum& m, int n, int ldx, int dtype, exo_stream_t stream) {
   EXO_TYPE_OK("exo_post_norm_add");
   EXO_REQUIRE(q && q->gain && q->x && q->x == q->x_out && q->operand && n >= 0 && q->H > 0 && q->H <= 16384 && ldx >= q->H,
               "exo_post_norm_add: bad argument (H=%d, x in place)", q ? q->H : 0);
+  EXO_REQUIRE(!(q->sum && q->branch2) && (q->sum || !q->center), "exo_post_norm_add: a norm of the sum takes one branch");
   EXO_REQUIRE(!q->branch2 || (q->gain_a && q->gain_b && !m.y), "exo_post_norm_add: two branches need a gain each");
   if (n == 0) return EXO_OK;
 #define EXO_POST(TH, P)                                                                                          \
   do {                                                                                                           \
     if (dtype == 0)                                                                                              \
-      post_norm_add_kernel<bf16_t, TH, P><<<n, TH, 0, (hipStream_t)stream>>>(*q, ldb, m, q->x_out, (bf16_t*)q->operand, ldx); \
+      post_norm_add_kernel<bf16_t, TH, P><<<n, TH, 0, (hipStream_t)stream>>>(*q, m, q->x_out, (bf16_t*)q->operand, ldx); \
     else                                                                                                         \
-      post_norm_add_kernel<float, TH, P><<<n, TH, 0, (hipStream_t)stream>>>(*q, ldb, m, q->x_out, (float*)q->operand, ldx);   \
+      post_norm_add_kernel<float, TH, P><<<n, TH, 0, (hipStream_t)stream>>>(*q, m, q->x_out, (float*)q->operand, ldx);   \
   } while (0)
   const int passes = exo_ceil_div(q->H, kRowThreads * kCols);
   if (n <= 256 && passes > 1) {  // few rows: the length of a row's chain counts, not the workgroups per CU
@@ -529,27 +565,27 @@ static int post_norm(const exo_post_norm* q, int ldb, const MoeSum& m, int n, in
   return EXO_OK;
 }
 
-extern "C" int exo_post_norm_add(const exo_post_norm* q, int ldb, int n, int ldx, int dtype, exo_stream_t stream) {
-  EXO_REQUIRE(q && q->branch && ldb >= q->H, "exo_post_norm_add: bad branch");
-  return post_norm(q, ldb, MoeSum{}, n, ldx, dtype, stream);
+extern "C" int exo_post_norm_add(const exo_post_norm* q, int n, int ldx, int dtype, exo_stream_t stream) {
+  EXO_REQUIRE(q && q->branch && q->ldb >= q->H, "exo_post_norm_add: bad branch");
+  return post_norm(q, MoeSum{}, n, ldx, dtype, stream);
 }
 
 extern "C" int exo_moe_sum_post_norm(const void* y, const int32_t* idx, const float* wt, const void* shared,
                                      const float* logits, int top, int experts, int ldy, int lds, int ldl, int gate_col,
                                      const exo_post_norm* q, int n, int ldx, int dtype, exo_stream_t stream) {
-  EXO_REQUIRE(q && y && idx && wt && top > 0 && experts > 0 && ldy >= q->H && (!shared || (logits && lds >= q->H && gate_col < ldl)),
+  EXO_REQUIRE(q && y && idx && wt && top > 0 && experts > 0 && ldy >= q->H && (!shared || (lds >= q->H && (gate_col < 0 || (logits && gate_col < ldl)))),
               "exo_moe_sum_post_norm: bad argument");
-  return post_norm(q, 0, MoeSum{y, idx, wt, shared, logits, top, experts, ldy, lds, ldl, gate_col}, n, ldx, dtype, stream);
+  return post_norm(q, MoeSum{y, idx, wt, shared, logits, top, experts, ldy, lds, ldl, gate_col}, n, ldx, dtype, stream);
 }
 
 extern "C" int exo_moe_route(const float* logits, const float* correction, int32_t* idx, float* wt, int rows, int n,
-                             int ldl, int top, float scale, exo_stream_t stream) {
+                             int ldl, int top, float scale, int renorm, exo_stream_t stream) {
   EXO_REQUIRE(logits && correction && idx && wt, "exo_moe_route: null pointer");
   EXO_REQUIRE(rows >= 0 && n > 0 && n <= 512 && ldl >= n && top > 0 && top <= 64 && top <= n,
               "exo_moe_route: need 0 < n <= %d and 0 < top <= min(64, n); got n=%d top=%d", 512, n, top);
   if (rows == 0) return EXO_OK;
   const auto fn = n <= 64 ? moe_route_kernel<1> : n <= 128 ? moe_route_kernel<2> : n <= 256 ? moe_route_kernel<4> : moe_route_kernel<8>;
-  fn<<<rows, 64, 0, (hipStream_t)stream>>>(logits, correction, idx, wt, n, ldl, top, scale);
+  fn<<<rows, 64, 0, (hipStream_t)stream>>>(logits, correction, idx, wt, n, ldl, top, scale, renorm);
   EXO_CHECK_LAUNCH("exo_moe_route");
   return EXO_OK;
 }
@@ -560,7 +596,7 @@ static MoeRows moe_rows_of(const exo_moe_rows* a) {
   p.sgate = a->shared_gate, p.sup = a->shared_up, p.sdown = a->shared_down;
   p.act = a->act, p.sact = a->shared_act, p.out = a->out, p.xres = a->x_res;
   p.idx = a->idx, p.wt = a->wt, p.logits = a->logits, p.corr = a->correction, p.rscale = a->router_scale;
-  p.outputs = a->outputs;
+  p.outputs = a->outputs, p.renorm = a->renorm;
   p.R = a->rows, p.top = a->top, p.experts = a->experts, p.ff = a->ff, p.sff = a->shared_ff, p.H = a->H;
   p.ldx = a->ldx, p.lda = a->lda, p.ldsa = a->ldsa, p.ldl = a->ldl, p.gate_col = a->gate_col;
   p.glu = GluConst{a->limit, a->alpha, a->shift};
@@ -577,7 +613,7 @@ static int moe_rows_check(const exo_moe_rows* a) {
               "exo_moe_rows: row strides must be multiples of 64 (ldx=%d lda=%d)", a->ldx, a->lda);
   EXO_REQUIRE(a->x && a->gate && a->up && a->down && a->act && a->out && a->x_res && a->idx && a->wt,
               "exo_moe_rows: null pointer");
-  EXO_REQUIRE(!a->shared_gate || (a->shared_up && a->shared_down && a->shared_act && a->logits && a->shared_ff > 0 &&
+  EXO_REQUIRE(!a->shared_gate || (a->shared_up && a->shared_down && a->shared_act && (a->gate_col < 0 || a->logits) && a->shared_ff > 0 &&
                                   a->ldsa % 64 == 0 && a->ldsa >= a->shared_ff && a->gate_col < a->ldl),
               "exo_moe_rows: incomplete shared expert");
   return EXO_OK;

@@ -39,15 +39,16 @@ def _code(t: torch.Tensor) -> int:
     raise ValueError(f"element type {t.dtype} not supported (bfloat16, float32)")
 
 
-def embed_rows(ids, table, x, xb, H: int) -> None:
+def embed_rows(ids, table, x, xb, H: int, scale: float = 1.0) -> None:
     n = ids.numel()
     check(native.load().exo_embed_rows(_ptr(ids), _ptr(table), _ptr(x), _ptr(xb), n, table.shape[0], H,
-                                       table.shape[1], xb.shape[1], _code(xb), _stream()), "embed_rows")
+                                       table.shape[1], xb.shape[1], scale, _code(xb), _stream()), "embed_rows")
 
 
-def norm_rows(x, gain, eps: float, out, n: int, rows=None) -> None:
-    check(native.load().exo_norm_rows(_ptr(x), _ptr(rows), _ptr(gain), _ptr(out), n, gain.numel(), out.shape[1], eps,
-                                      _code(out), _stream()), "norm_rows")
+def norm_rows(x, gain, eps: float, out, n: int, rows=None, center: bool = False) -> None:
+    """out[i] = x[i] (rows: x[rows[i]]) / rms * gain; ``center``: its mean is taken off first."""
+    check(native.load().exo_norm_rows(x.data_ptr(), _ptr(rows), _ptr(gain), _ptr(out), n, gain.numel(), x.stride(0),
+                                      out.shape[1], eps, int(center), _code(out), _stream()), "norm_rows")
 
 
 def _p(t):
@@ -57,37 +58,42 @@ def _p(t):
 class Branches:
     """A sublayer's output on its way into the residual: ``branch``, or half the sum of two branches that
     are normed each with a gain of its own first (``branch2``, ``gain_a``, ``gain_b``); then the norm with
-    ``gain``, times ``mult``.  All float32."""
+    ``gain``, times ``mult``.  ``norm``: a NormSpec that asks for the norm of the sum instead (the residual times
+    ``norm.keep``).  All float32."""
 
-    def __init__(self, branch, gain, mult: float = 1.0, branch2=None, gain_a=None, gain_b=None):
+    def __init__(self, branch, gain, mult: float = 1.0, branch2=None, gain_a=None, gain_b=None, norm=None):
         self.branch, self.gain, self.mult = branch, gain, mult
         self.branch2, self.gain_a, self.gain_b = branch2, gain_a, gain_b
+        self.of_sum = norm is not None and norm.of_sum
+        self.center, self.keep = self.of_sum and norm.center, norm.keep if self.of_sum else 1.0
 
     def args(self, x, x_out, operand, eps: float, pre) -> native.PostNorm:
-        return native.PostNorm(x=x.data_ptr(), branch=_p(self.branch), branch2=_p(self.branch2), gain_a=_p(self.gain_a),
-                               gain_b=_p(self.gain_b), gain=self.gain.data_ptr(), pre=_p(pre), x_out=x_out.data_ptr(),
-                               operand=_p(operand), H=self.gain.numel(), eps=eps, mult=self.mult)
+        return native.PostNorm(x=_p(x), branch=_p(self.branch), branch2=_p(self.branch2), gain_a=_p(self.gain_a),
+                               gain_b=_p(self.gain_b), gain=self.gain.data_ptr(), pre=_p(pre), x_out=_p(x_out),
+                               operand=_p(operand), H=self.gain.numel(), ldb=0 if self.branch is None else self.branch.stride(0),
+                               sum=int(self.of_sum), center=int(self.center), eps=eps, mult=self.mult, keep=self.keep)
 
 
 def post_norm_add(br: Branches, eps: float, x, xb, n: int, pre=None) -> None:
     """x += the normed branches; xb = x (or its norm with gain ``pre``) in the element type."""
-    check(native.load().exo_post_norm_add(C.byref(br.args(x, x, xb, eps, pre)), br.branch.shape[1], n, xb.shape[1],
+    check(native.load().exo_post_norm_add(C.byref(br.args(x, x, xb, eps, pre)), n, xb.shape[1],
                                           _code(xb), _stream()), "post_norm_add")
 
 
 def moe_sum_post_norm(y, idx, wt, shared, logits, experts: int, gate_col: int, gain, eps: float, x, xb, n: int,
-                      mult: float = 1.0) -> None:
-    """x += norm(weighted sum of the chosen experts' outputs y [n, top, ld] + gated shared)."""
-    q = Branches(None, gain, mult).args(x, x, xb, eps, None)
+                      mult: float = 1.0, norm=None) -> None:
+    """x += norm(weighted sum of the chosen experts' outputs y [n, top, ld] + shared, gated by the logits'
+    ``gate_col`` unless that is negative); ``norm`` as for ``Branches``."""
+    q = Branches(None, gain, mult, norm=norm).args(x, x, xb, eps, None)
     check(native.load().exo_moe_sum_post_norm(
         _ptr(y), _ptr(idx), _ptr(wt), _ptr(shared), _ptr(logits), idx.shape[1], experts, y.shape[-1],
         0 if shared is None else shared.shape[1], logits.shape[1], gate_col, C.byref(q), n, xb.shape[1], _code(xb),
         _stream()), "moe_sum_post_norm")
 
 
-def moe_route(logits, correction, scale: float, idx, wt, n: int) -> None:
+def moe_route(logits, correction, scale: float, idx, wt, n: int, renorm: bool = False) -> None:
     check(native.load().exo_moe_route(_ptr(logits), _ptr(correction), _ptr(idx), _ptr(wt), n, correction.numel(),
-                                      logits.shape[1], idx.shape[1], scale, _stream()), "moe_route")
+                                      logits.shape[1], idx.shape[1], scale, int(renorm), _stream()), "moe_route")
 
 
 _GEMM_WS: dict[int, torch.Tensor] = {}
@@ -102,22 +108,35 @@ def gemm_workspace(device) -> torch.Tensor:
     return _GEMM_WS[key]
 
 
-def _linear(x, w, out, n: int, bias=None, tail=None, up=None, spec=None) -> native.Linear:
+ACTS = {None: 0, "relu2": 1, "gelu_tanh": 2}
+
+
+class After:
+    """What happens to a product's result ahead of its store: ``act``, then times row ``rows[m]`` (or m) of
+    ``mul`` (element type)."""
+
+    def __init__(self, act: str | None = None, mul=None, rows=None):
+        self.act, self.mul, self.rows = act, mul, rows
+
+
+def _linear(x, w, out, n: int, bias=None, tail=None, up=None, spec=None, after: After | None = None) -> native.Linear:
     """``tail``: float32 output of the columns past ``out``'s share (w's rows beyond N - tail's logical
     columns; given as (tensor, columns)).  ``up``, ``spec``: the gated pair."""
     N = w.shape[0]
     t, nt = (None, 0) if tail is None else tail
+    f = after or After()
     return native.Linear(
         x=_p(x), w=w.data_ptr(), w_up=_p(up), bias=_p(bias), y=out.data_ptr(), y2=_p(t), M=n, N=N, n1=N - nt,
         ldx=w.shape[1] if x is None else x.stride(0), ldw=w.shape[1], ldy=out.stride(0), ldy2=0 if t is None else t.stride(0),
         y_f32=int(out.dtype == torch.float32), dtype=_code(w), limit=spec.limit if spec else 0.0,
-        alpha=spec.alpha if spec else 0.0, shift=spec.shift if spec else 0.0)
+        alpha=spec.alpha if spec else 0.0, shift=spec.shift if spec else 0.0, act=ACTS[f.act], mul=_p(f.mul),
+        mul_rows=_p(f.rows), ldmul=0 if f.mul is None else f.mul.stride(0))
 
 
-def linear(x, w, out, n: int, bias=None, force_gemm: bool = False, tail=None) -> None:
+def linear(x, w, out, n: int, bias=None, force_gemm: bool = False, tail=None, after: After | None = None) -> None:
     """out[:n] = x[:n] @ w^T (+ bias float32); out in x's element type or float32.  ``tail`` (tensor, columns):
     the last columns go to that float32 tensor instead."""
-    _launch_linear(_linear(x, w, out, n, bias, tail), n, x.device, force_gemm)
+    _launch_linear(_linear(x, w, out, n, bias, tail, after=after), n, x.device, force_gemm)
 
 
 def _launch_linear(a, n: int, device, force_gemm: bool = False) -> None:
@@ -149,11 +168,22 @@ def post_linear_fits(n: int, w, xb, H: int, pre: bool = False) -> bool:
 
 
 def post_linear(x, br: Branches, eps: float, x_out, xb, w, out, n: int, bias=None, tail=None, pre=None, up=None,
-                spec=None) -> None:
+                spec=None, after: After | None = None) -> None:
     """``post_norm_add`` and ``linear`` (or the gated pair) in one launch: x_out = x + the normed branches
-    (another buffer than x), xb (may be None) the product's operand."""
-    q, a = br.args(x, x_out, xb, eps, pre), _linear(None, w, out, n, bias, tail, up, spec)
+    (another buffer than x), xb (may be None) the product's operand.  x and x_out None: the normed branch
+    alone is the operand."""
+    q, a = br.args(x, x_out, xb, eps, pre), _linear(None, w, out, n, bias, tail, up, spec, after)
     check(native.load().exo_post_linear(C.byref(q), C.byref(a), _stream()), "post_linear")
+
+
+def norm_linear(x, gain, eps: float, operand, w, out, n: int) -> None:
+    """out[:n] = (x / rms * gain) @ w^T, x float32 rows; ``operand``: scratch for the normed rows."""
+    br = Branches(x, gain)
+    if post_linear_fits(n, w, operand, gain.numel()):
+        post_linear(None, br, eps, None, None, w, out, n)
+    else:
+        norm_rows(x, gain, eps, operand, n)
+        linear(operand, w, out, n)
 
 
 def glu(x, gate, up, out, n: int, spec, force_gemm: bool = False) -> None:
@@ -190,7 +220,8 @@ class ExpertRows:
             x_res=p(h), idx=p(bf.idx(r.top)), wt=p(bf.wt(r.top)), logits=p(bf.router_logits(w.router.shape[0])),
             correction=p(w.correction),
             top=r.top, experts=r.experts, ff=e.ff, shared_ff=s.ff if s else 0, H=H, ldx=bf.xb.shape[1],
-            lda=pad64(e.ff), ldsa=pad64(s.ff) if s else 0, ldl=w.router.shape[0], gate_col=r.outputs, outputs=r.outputs, router_scale=r.scale,
+            lda=pad64(e.ff), ldsa=pad64(s.ff) if s else 0, ldl=w.router.shape[0], gate_col=w.gate_col, outputs=r.outputs,
+            renorm=int(r.renorm), router_scale=r.scale,
             dtype=_code(bf.xb), limit=e.limit, alpha=e.alpha, shift=e.shift,
             shared_limit=s.limit if s else 0.0, shared_alpha=s.alpha if s else 0.0, shared_shift=s.shift if s else 0.0)
 
@@ -219,20 +250,24 @@ def attn_workspace(n: int, heads: int, vdim: int, nsplit: int, device) -> torch.
 
 class PagedAttention:
     """Attention of one layer over a paged pool.  ``spec``: AttentionSpec; ``li``: index of the
-    pool's layer that holds its keys and values."""
+    pool's layer that holds its keys and values; ``freq``: float64 turns per position of each rotated pair."""
 
-    def __init__(self, spec, slopes, li: int, cache, eps: float, q_gain=None, k_gain=None):
-        self.spec, self.slopes, self.cache, self.gains = spec, slopes, cache, (q_gain, k_gain)
+    def __init__(self, spec, slopes, li: int, cache, eps: float, q_gain=None, k_gain=None, freq=None):
+        self.spec, self.slopes, self.cache, self.keep = spec, slopes, cache, (q_gain, k_gain, freq)
         k, v = cache.k[li], cache.v[li]
+        # whether queries and keys of a step need a launch of their own ahead of prompt attention
+        self.prepares = spec.whole_norm or spec.rot is not None or spec.v_mix
         self.args = native.PagedAttn(
             k_pool=k.data_ptr(), v_pool=v.data_ptr(), table=cache.table.data_ptr(),
             slopes=_p(slopes), q_gain=_p(q_gain), k_gain=_p(k_gain), scale=spec.scale, eps=eps,
             heads=spec.heads, kv_heads=spec.kv_heads, dim=spec.dim, vdim=spec.vdim, ldk=k.shape[3], ldv=v.shape[2],
             max_pages=cache.table.shape[1], window=spec.window or 0, keep_first=spec.keep_first,
-            unit_qk=int(spec.unit_qk), dtype=_code(k))
+            unit_qk=int(spec.unit_qk), whole_norm=int(spec.whole_norm), rot=spec.rot.dims if spec.rot else 0, freq=_p(freq),
+            softcap=spec.softcap or 0.0, dtype=_code(k))
 
-    def _bind(self, qkv, out, slot, pos, lst, n: int, gate=None):
+    def _bind(self, qkv, out, slot, pos, lst, n: int, gate=None, prepared: bool = False):
         a = self.args
+        a.prepared = int(prepared and self.prepares)
         assert qkv.dtype == self.cache.k[0].dtype
         a.qkv, a.ldq, a.n = qkv.data_ptr(), qkv.stride(0), n
         a.out, a.ldo = (None, 0) if out is None else (out.data_ptr(), out.stride(0))
@@ -242,8 +277,18 @@ class PagedAttention:
         a.list = None if lst is None else lst.data_ptr()
         return C.byref(a)
 
+    def mix_values(self, v, weight: float) -> None:
+        """Own values become (1 - weight) own + weight ``v`` (element type, a row per row of the step)."""
+        self.args.v_mix, self.args.ldmix, self.args.mix = v.data_ptr(), v.stride(0), weight
+
     def append(self, qkv, slot, pos, n: int) -> None:
-        check(native.load().exo_paged_append(self._bind(qkv, None, slot, pos, None, n), _stream()), "paged_append")
+        """Keys and values of n rows into the pool; a design that prepares also turns the queries in place,
+        and says ``prepared`` to what follows."""
+        a = self._bind(qkv, None, slot, pos, None, n)
+        if self.prepares:
+            check(native.load().exo_paged_prepare(a, _stream()), "paged_prepare")
+        else:
+            check(native.load().exo_paged_append(a, _stream()), "paged_append")
 
     def visible(self, keys: int) -> int:
         """Most keys one query sees when its sequence holds ``keys``."""
@@ -263,7 +308,7 @@ class PagedAttention:
         if n * s.heads > 16384:
             nsplit = 1
         ws = attn_workspace(n, s.heads, s.vdim, nsplit, qkv.device) if nsplit > 1 else None
-        check(native.load().exo_paged_attn_rows(self._bind(qkv, out, slot, pos, lst, n, gate), nsplit, int(append), _ptr(ws),
+        check(native.load().exo_paged_attn_rows(self._bind(qkv, out, slot, pos, lst, n, gate, not append), nsplit, int(append), _ptr(ws),
                                                 0 if ws is None else ws.numel(), _stream()), "paged_attn_rows")
 
     @staticmethod
@@ -272,8 +317,96 @@ class PagedAttention:
 
     def prompt(self, qkv, out, blocks, n: int, gate=None) -> None:
         """Portions of prompts: blocks int32 [n, 4] = first row, slot, first position, tokens."""
-        check(native.load().exo_paged_attn_prompt(self._bind(qkv, out, None, None, blocks, n, gate), _stream()),
+        check(native.load().exo_paged_attn_prompt(self._bind(qkv, out, None, None, blocks, n, gate, True), _stream()),
               "paged_attn_prompt")
+
+
+_LATENT_WS: dict[tuple, list[torch.Tensor]] = {}
+
+
+def latent_workspace(kind: str, n: int, dtype, device) -> torch.Tensor:
+    """Partials of split rows ("parts", float32) and expanded latents, one per kind and device, grown on
+    demand (replaced partials stay alive: a captured graph may point at them)."""
+    key = (kind, dtype, torch.device(device).index or 0)
+    have = _LATENT_WS.setdefault(key, [])
+    if not have or have[-1].numel() < n:
+        if kind != "parts":
+            have.clear()
+        have.append(torch.empty(n, dtype=dtype, device=device))
+    return have[-1][:n]
+
+
+LATENT_BLOCK = 128  # tokens of a block of expanded prompt attention
+LATENT_SHORT = 32   # portions below this many tokens go through the absorbed rows
+
+
+class LatentAttention:
+    """Latent attention of one layer over a paged pool.  ``spec``: LatentSpec; ``w``: the layer's tensors
+    (``stack_layers.LatentPart``); ``li``: index of the pool's layer."""
+
+    def __init__(self, spec, w, li: int, cache, eps: float):
+        self.spec, self.w, self.cache = spec, w, cache
+        pool = cache.k[li]
+        self.args = native.LatentAttn(
+            gain=w.kv_gain.data_ptr(), freq=_p(w.freq), pool=pool.data_ptr(), table=cache.table.data_ptr(), scale=spec.scale,
+            eps=eps, heads=spec.heads, rank=spec.kv_rank, rot=spec.rot_dim, rot_col=w.rot_col, ldk=pool.shape[3],
+            max_pages=cache.table.shape[1], dtype=_code(pool))
+
+    def _bind(self, q, kv, slot, pos, n: int, lst=None, prepared: bool = False):
+        a = self.args
+        a.q, a.ldq, a.kv, a.ldkv, a.n = q.data_ptr(), q.stride(0), kv.data_ptr(), kv.stride(0), n
+        a.slot, a.pos, a.list, a.prepared = slot.data_ptr(), pos.data_ptr(), _p(lst), int(prepared)
+        return a
+
+    def prepare(self, q, kv, slot, pos, n: int) -> None:
+        """Latents and shared key parts of n rows into the pool; the queries' rotated parts in place."""
+        check(native.load().exo_latent_prepare(C.byref(self._bind(q, kv, slot, pos, n)), _stream()), "latent_prepare")
+
+    def rows(self, q, kv, ql, ol, out, slot, pos, n: int, keys: int, append: bool, lst=None) -> None:
+        """One query position per row (``lst``: which rows, else the first n): ``out`` [rows, heads * vdim].
+        ``ql``, ``ol``: scratch, [rows, heads * pad64(kv_rank)]; ``keys``: most keys any sequence holds."""
+        s, w, lib = self.spec, self.w, native.load()
+        head_linear(q, w.nope_pad, w.uk, ql, pad64(s.kv_rank), n, s.dim, lst)
+        tiles, wgs = -(-keys // 64), n * (-(-s.heads // 16))
+        nsplit = max(1, min(-(-tiles // 2), 256 // wgs, 32))
+        a = self._bind(q, kv, slot, pos, n, lst, not append)
+        a.q_latent, a.ldql, a.nsplit = ql.data_ptr(), ql.stride(0), nsplit
+        parts = None
+        if nsplit == 1:
+            a.out, a.ldo = ol.data_ptr(), ol.stride(0)
+        else:
+            parts = latent_workspace("parts", lib.exo_latent_parts(n, s.heads, s.kv_rank, nsplit), torch.float32, q.device)
+            a.parts, a.parts_floats = parts.data_ptr(), parts.numel()
+        check(lib.exo_latent_rows(C.byref(a), int(append), _stream()), "latent_rows")
+        head_linear(ol, pad64(s.kv_rank), w.uv, out, s.vdim, n, s.kv_rank, lst, parts, nsplit)
+
+    def prompt(self, q, kv, out, slot, pos, blocks, n_blocks: int, pages, n_pages: int) -> None:
+        """Portions of prompts over expanded keys and values: ``pages`` int32 [n, 2] (cache row, page of its
+        sequence), ``blocks`` int32 [n, 4] (first row, first gathered key row, first position, tokens)."""
+        s, w, lib, dev = self.spec, self.w, native.load(), q.device
+        n, H, r8 = 64 * n_pages, s.heads, -(-s.rot_dim // 8) * 8
+        new = lambda kind, *shape: latent_workspace(kind, shape[0] * shape[1], torch.bfloat16, dev).view(*shape)  # noqa: E731
+        c, kr = new("latents", n, pad64(s.kv_rank)), new("rotated", n, r8)
+        k, v = new("keys", n, H * w.d8), new("values", H * s.vdim, n)
+        a = self._bind(q, kv, slot, pos, 1)
+        check(lib.exo_latent_gather(C.byref(a), pages.data_ptr(), n_pages, c.data_ptr(), kr.data_ptr(), _stream()), "latent_gather")
+        linear(c, w.uk_rows, k, n, force_gemm=True)
+        linear(w.uv_rows, c, v, H * s.vdim, force_gemm=True)
+        p = native.LatentPrompt(
+            q=q.data_ptr(), k=k.data_ptr(), k_rot=kr.data_ptr(), v=v.data_ptr(), list=blocks.data_ptr(), out=out.data_ptr(),
+            scale=s.scale, n=n_blocks, heads=H, vdim=s.vdim, d8=w.d8, r8=r8, ldq=q.stride(0), q_head=w.nope_pad,
+            rot_col=w.rot_col, ldk=k.stride(0), ldv=v.stride(0), ldo=out.stride(0))
+        check(lib.exo_latent_prompt(C.byref(p), _stream()), "latent_prompt")
+
+
+def head_linear(x, x_head: int, w, y, y_head: int, n: int, K: int, lst=None, parts=None, nsplit: int = 1) -> None:
+    """y[row][h] = w[h] x[row][h] for n rows (``lst``: which): w [heads, N, pad64(K)], head h at h * x_head and
+    h * y_head; ``parts``: x is merged from the partials of split latent rows."""
+    a = native.HeadLinear(
+        x=x.data_ptr(), w=w.data_ptr(), parts=_p(parts), parts_floats=0 if parts is None else parts.numel(), y=y.data_ptr(),
+        list=_p(lst), n=n, heads=w.shape[0], N=w.shape[1], K=K, ldx=x.stride(0), x_head=x_head, ldw=w.shape[2], ldy=y.stride(0),
+        y_head=y_head, nsplit=nsplit, dtype=_code(w))
+    check(native.load().exo_head_linear(C.byref(a), _stream()), "head_linear")
 
 
 _RECUR_WS: dict[int, torch.Tensor] = {}

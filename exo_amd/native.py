@@ -23,15 +23,15 @@ class MoeRows(C.Structure):
     _fields_ = [(n, _vp) for n in ("x", "gate", "up", "down", "shared_gate", "shared_up", "shared_down", "act",
                                    "shared_act", "out", "x_res", "idx", "wt", "logits", "correction")] + \
                [(n, _i) for n in ("rows", "top", "experts", "ff", "shared_ff", "H", "ldx", "lda", "ldsa", "ldl",
-                                  "gate_col", "outputs", "dtype")] + \
+                                  "gate_col", "outputs", "renorm", "dtype")] + \
                [(n, _f) for n in ("router_scale", "limit", "alpha", "shift", "shared_limit", "shared_alpha", "shared_shift")]
 
 
 class Linear(C.Structure):
     """struct exo_linear: a product (or gated pair) with an unquantised matrix."""
 
-    _fields_ = [(n, _vp) for n in ("x", "w", "w_up", "bias", "y", "y2")] + \
-               [(n, _i) for n in ("M", "N", "n1", "ldx", "ldw", "ldy", "ldy2", "y_f32", "dtype")] + \
+    _fields_ = [(n, _vp) for n in ("x", "w", "w_up", "bias", "y", "y2", "mul", "mul_rows")] + \
+               [(n, _i) for n in ("M", "N", "n1", "ldx", "ldw", "ldy", "ldy2", "y_f32", "dtype", "act", "ldmul")] + \
                [(n, _f) for n in ("limit", "alpha", "shift")]
 
 
@@ -39,17 +39,41 @@ class PostNorm(C.Structure):
     """struct exo_post_norm: a sublayer's output on its way into the residual."""
 
     _fields_ = [(n, _vp) for n in ("x", "branch", "branch2", "gain_a", "gain_b", "gain", "pre", "x_out", "operand")] + \
-               [("H", _i), ("eps", _f), ("mult", _f)]
+               [(n, _i) for n in ("H", "ldb", "sum", "center")] + [(n, _f) for n in ("eps", "mult", "keep")]
 
 
 class PagedAttn(C.Structure):
     """struct exo_paged_attn: one attention layer over a paged pool."""
 
     _fields_ = [(n, _vp) for n in ("qkv", "k_pool", "v_pool", "table", "slot", "pos", "list", "slopes", "q_gain", "k_gain",
-                                   "gate", "out")] + \
-               [("scale", _f), ("eps", _f)] + \
+                                   "gate", "freq", "v_mix", "out")] + \
+               [(n, _f) for n in ("scale", "eps", "softcap", "mix")] + \
                [(n, _i) for n in ("n", "heads", "kv_heads", "dim", "vdim", "ldq", "ldk", "ldv", "ldo", "ldg", "max_pages",
-                                  "window", "keep_first", "unit_qk", "dtype")]
+                                  "window", "keep_first", "unit_qk", "whole_norm", "rot", "ldmix", "prepared", "dtype")]
+
+
+class LatentAttn(C.Structure):
+    """struct exo_latent_attn: one latent-attention layer over a paged pool."""
+
+    _fields_ = [(n, _vp) for n in ("q", "q_latent", "kv", "gain", "freq", "pool", "table", "slot", "pos", "list", "out",
+                                   "parts")] + \
+               [("parts_floats", _i64), ("scale", _f), ("eps", _f)] + \
+               [(n, _i) for n in ("n", "heads", "rank", "rot", "rot_col", "ldq", "ldql", "ldkv", "ldk", "ldo", "max_pages",
+                                  "prepared", "nsplit", "dtype")]
+
+
+class HeadLinear(C.Structure):
+    """struct exo_head_linear_args: a product with a matrix per head."""
+
+    _fields_ = [("x", _vp), ("w", _vp), ("parts", _vp), ("parts_floats", _i64), ("y", _vp), ("list", _vp)] + \
+               [(n, _i) for n in ("n", "heads", "N", "K", "ldx", "x_head", "ldw", "ldy", "y_head", "nsplit", "dtype")]
+
+
+class LatentPrompt(C.Structure):
+    """struct exo_latent_prompt_args: portions of prompts over expanded keys and values."""
+
+    _fields_ = [(n, _vp) for n in ("q", "k", "k_rot", "v", "list", "out")] + [("scale", _f)] + \
+               [(n, _i) for n in ("n", "heads", "vdim", "d8", "r8", "ldq", "q_head", "rot_col", "ldk", "ldv", "ldo")]
 
 
 class Recurrence(C.Structure):
@@ -119,11 +143,11 @@ SIGNATURES: dict[str, tuple] = {
     "exo_moe_combine": (_i, [_vp, _vp, _vp, _vp, _i, _i, _i, _vp]),
     "exo_argmax_workspace": (_i64, [_i]),
     "exo_argmax_logsumexp": (_i, [_vp] * 6 + [_i, _i, _vp]),
-    "exo_embed_rows": (_i, [_vp] * 4 + [_i] * 6 + [_vp]),
-    "exo_norm_rows": (_i, [_vp] * 4 + [_i] * 3 + [_f, _i, _vp]),
-    "exo_post_norm_add": (_i, [C.POINTER(PostNorm), _i, _i, _i, _i, _vp]),
+    "exo_embed_rows": (_i, [_vp] * 4 + [_i] * 5 + [_f, _i, _vp]),
+    "exo_norm_rows": (_i, [_vp] * 4 + [_i] * 4 + [_f, _i, _i, _vp]),
+    "exo_post_norm_add": (_i, [C.POINTER(PostNorm), _i, _i, _i, _vp]),
     "exo_moe_sum_post_norm": (_i, [_vp] * 5 + [_i] * 6 + [C.POINTER(PostNorm), _i, _i, _i, _vp]),
-    "exo_moe_route": (_i, [_vp] * 4 + [_i] * 4 + [_f, _vp]),
+    "exo_moe_route": (_i, [_vp] * 4 + [_i] * 4 + [_f, _i, _vp]),
     "exo_linear_rows": (_i, [C.POINTER(Linear), C.POINTER(Linear), _vp]),
     "exo_linear_gemm": (_i, [C.POINTER(Linear), _vp, _i64, _vp]),
     "exo_post_linear_fits": (_i, [_i] * 5),
@@ -131,11 +155,18 @@ SIGNATURES: dict[str, tuple] = {
     "exo_dense_grouped_gemm": (_i, [_vp] * 5 + [_f] * 3 + [_i] * 9 + [_vp]),
     "exo_moe_glu_rows": (_i, [C.POINTER(MoeRows), _vp]),
     "exo_moe_down_rows": (_i, [C.POINTER(MoeRows), _vp]),
+    "exo_paged_prepare": (_i, [C.POINTER(PagedAttn), _vp]),
     "exo_paged_append": (_i, [C.POINTER(PagedAttn), _vp]),
     "exo_paged_attn_workspace": (_i64, [_i] * 4),
     "exo_paged_attn_rows": (_i, [C.POINTER(PagedAttn), _i, _i, _vp, _i64, _vp]),
     "exo_paged_prompt_block": (_i, [_i, _i]),
     "exo_paged_attn_prompt": (_i, [C.POINTER(PagedAttn), _vp]),
+    "exo_latent_prepare": (_i, [C.POINTER(LatentAttn), _vp]),
+    "exo_latent_parts": (_i64, [_i] * 4),
+    "exo_latent_rows": (_i, [C.POINTER(LatentAttn), _i, _vp]),
+    "exo_head_linear": (_i, [C.POINTER(HeadLinear), _vp]),
+    "exo_latent_gather": (_i, [C.POINTER(LatentAttn), _vp, _i, _vp, _vp, _vp]),
+    "exo_latent_prompt": (_i, [C.POINTER(LatentPrompt), _vp]),
     "exo_recur_chunk": (_i, []),
     "exo_recur_workspace": (_i64, [C.POINTER(Recurrence)]),
     "exo_recur_chunks": (_i, [C.POINTER(Recurrence), _vp, _i64, _vp]),

@@ -9,7 +9,8 @@ the pages (``state_pool``); a row then cannot be cut back to an earlier position
 Per layer with keys of its own (layers that use another layer's keys have no storage):
   k[i]  [pages, G, 64, ldk]   keys as attention uses them (normalised)
   v[i]  [pages, G, ldv, 64]   values, transposed inside the page (matrix-core operand order)
-with ldk, ldv the head sizes rounded up to 32; the padding stays zero.
+with ldk, ldv the head sizes rounded up to 32; the padding stays zero.  Latent attention keeps one "key" per
+position - the normed latent, and behind it the shared rotated key part - and no values.
 """
 
 from __future__ import annotations
@@ -155,8 +156,9 @@ class PagedKVCache(list):
         """Keys [n, G, D] and values [n, G, E] of positions [start, start + n)."""
         g, d, e = self.shapes[layer]
         idx, off = self._row_pages(row, start, start + n), start % PAGE
-        k = self.k[layer][idx].permute(0, 2, 1, 3).reshape(-1, g, self.k[layer].shape[-1])
-        v = self.v[layer][idx].permute(0, 3, 1, 2).reshape(-1, g, self.v[layer].shape[2])
+        rows = len(idx) * PAGE
+        k = self.k[layer][idx].permute(0, 2, 1, 3).reshape(rows, g, self.k[layer].shape[-1])
+        v = self.v[layer][idx].permute(0, 3, 1, 2).reshape(rows, g, self.v[layer].shape[2])
         return k[off : off + n, :, :d].contiguous(), v[off : off + n, :, :e].contiguous()
 
     def write_nhd(self, layer: int, row: int, start: int, k: torch.Tensor, v: torch.Tensor) -> None:

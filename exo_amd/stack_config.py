@@ -11,8 +11,21 @@ from __future__ import annotations
 
 import copy
 import json
+import math
 from dataclasses import dataclass
 from pathlib import Path
+
+
+@dataclass(frozen=True)
+class RotarySpec:
+    """Pairs (2i, 2i + 1) of a head's first ``dims`` entries turned by position * base^(-2i / dims)."""
+
+    base: float
+    dims: int
+
+    def turns(self) -> list[float]:
+        """Turns per position of each pair."""
+        return [self.base ** (-2.0 * i / self.dims) / (2.0 * math.pi) for i in range(self.dims // 2)]
 
 
 @dataclass(frozen=True)
@@ -30,6 +43,35 @@ class AttentionSpec:
     slopes: tuple[float, ...] | None = None  # per query head: score lowered by slope * distance
     bias: bool = False           # projections have biases
     kv_from: int | None = None   # keys and values of that layer instead of own ones
+    whole_norm: bool = False     # RMS norm of the whole query and key projections, with gains
+    rot: RotarySpec | None = None
+    softcap: float | None = None  # score bent to cap * tanh(score / cap)
+    v_mix_from: int | None = None  # values mixed with those of that layer (one weight, a tensor)
+
+    @property
+    def v_mix(self) -> bool:
+        return self.v_mix_from is not None
+
+
+@dataclass(frozen=True)
+class LatentSpec:
+    """Attention whose keys and values are images of one normed latent vector per position, beside a rotated
+    key part that all heads share; queries through a normed latent of their own."""
+
+    heads: int
+    dim: int                     # unrotated query / key size per head
+    rot_dim: int                 # rotated size
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rot: RotarySpec
+
+    @property
+    def pooled(self) -> tuple[int, int, int]:
+        """Storage of a position, as (kv heads, key size, value size): the latent up to a multiple of 32, then
+        the rotated part."""
+        return 1, -(-self.kv_rank // 32) * 32 + self.rot_dim, 0
 
 
 @dataclass(frozen=True)
@@ -83,13 +125,21 @@ class ParallelSpec:
     right: StateSpaceSpec
 
 
-MixerSpec = AttentionSpec | LinearAttentionSpec | StateSpaceSpec | ParallelSpec
+MixerSpec = AttentionSpec | LatentSpec | LinearAttentionSpec | StateSpaceSpec | ParallelSpec
 
 
 def attention_of(m: MixerSpec) -> AttentionSpec | None:
-    """The part of a mixer that keeps keys and values."""
+    """The part of a mixer that keeps keys and values per head."""
     m = m.left if isinstance(m, ParallelSpec) else m
     return m if isinstance(m, AttentionSpec) else None
+
+
+def pooled_shape(m: MixerSpec) -> tuple[int, int, int] | None:
+    """(kv heads, key size, value size) that a mixer keeps per position, if it keeps any of its own."""
+    if isinstance(m, LatentSpec):
+        return m.pooled
+    a = attention_of(m)
+    return None if a is None or a.kv_from is not None else (a.kv_heads, a.dim, a.vdim)
 
 
 def recurrence_of(m: MixerSpec) -> LinearAttentionSpec | StateSpaceSpec | None:
@@ -110,14 +160,26 @@ class GluSpec:
 
 
 @dataclass(frozen=True)
+class DenseSpec:
+    """down(act(up x)); ``act``: relu2 (square of relu) or gelu_tanh."""
+
+    ff: int
+    act: str
+
+
+@dataclass(frozen=True)
 class RouterSpec:
     """softmax over experts + identity outputs; the ``top`` largest of score + correction; weight
-    = score * scale.  An identity expert returns its input."""
+    = score * scale.  An identity expert returns its input.  ``renorm``: the largest logits instead, weights
+    = softmax over the chosen ones."""
 
     experts: int
     identity: int
     top: int
     scale: float
+    bias: bool = False           # on the logits
+    correction: bool = True
+    renorm: bool = False
 
     @property
     def outputs(self) -> int:
@@ -128,13 +190,14 @@ class RouterSpec:
 class MoeSpec:
     router: RouterSpec
     expert: GluSpec
-    shared: GluSpec | None = None  # for every token, times sigmoid of one number per token
+    shared: GluSpec | None = None  # for every token
+    shared_gate: bool = True     # ... times sigmoid of one number per token
 
 
 @dataclass(frozen=True)
 class LayerSpec:
     mixer: MixerSpec
-    mlp: MoeSpec | GluSpec | None
+    mlp: MoeSpec | GluSpec | DenseSpec | None
 
 
 @dataclass(frozen=True)
@@ -145,6 +208,9 @@ class NormSpec:
     pre: bool = False            # also on a sublayer's input (else only on its output)
     offset: float = 0.0          # gain = stored weight + offset
     mult: float = 1.0            # of a normed sublayer output in the residual sum
+    of_sum: bool = False         # of the sum keep * residual + output, which becomes the residual
+    keep: float = 1.0
+    center: bool = False         # the mean is taken off first (of_sum, and the last norm)
 
     def names(self, sublayer: int) -> tuple[str | None, str]:
         """Tensor names of the norms ahead of (None: none) and behind sublayer 1 or 2."""
@@ -159,12 +225,20 @@ class StackConfig:
     norm: NormSpec
     layers: tuple[LayerSpec, ...]
     raw: dict                    # config.json as read
+    embed_scale: float = 1.0
+    logit_scale: float = 1.0
+    tied: bool = False           # the head is the embedding table
+    side_dim: int | None = None  # a vector per token and layer, gated by the residual, joins it behind each layer
 
     def __post_init__(self):
         if min(self.vocab_size, self.hidden_size, len(self.layers)) <= 0:
             raise ValueError(f"{self.architecture}: vocab, width and the layer list must not be empty")
         for i, L in enumerate(self.layers):
             m, f, r = attention_of(L.mixer), L.mlp, recurrence_of(L.mixer)
+            if isinstance(L.mixer, LatentSpec):
+                c = L.mixer
+                if min(c.heads, c.dim, c.rot_dim, c.vdim, c.q_rank, c.kv_rank) <= 0 or c.rot_dim % 2 or c.rot.dims != c.rot_dim:
+                    raise ValueError(f"layer {i}: latent attention of sizes {c}")
             if r is not None:
                 h, g, d, e = r.core
                 if min(h, g, d, e) <= 0 or h % g:
@@ -183,6 +257,14 @@ class StackConfig:
                 raise ValueError(f"layer {i}: {m.heads} query heads over {m.kv_heads} key/value heads")
             if (m.window is not None and m.window <= 0) or m.keep_first < 0:
                 raise ValueError(f"layer {i}: window {m.window} with {m.keep_first} kept positions")
+            if m.rot is not None and (m.rot.dims <= 0 or m.rot.dims % 2 or m.rot.dims > m.dim):
+                raise ValueError(f"layer {i}: {m.rot.dims} rotated dimensions of {m.dim}")
+            if m.softcap is not None and m.softcap <= 0:
+                raise ValueError(f"layer {i}: softcap {m.softcap}")
+            if m.v_mix_from is not None:
+                src = attention_of(self.layers[m.v_mix_from].mixer) if 0 <= m.v_mix_from < i else None
+                if src is None or src.kv_heads * src.vdim != m.kv_heads * m.vdim:
+                    raise ValueError(f"layer {i}: its values do not fit those of layer {m.v_mix_from}")
             if m.kv_from is not None:
                 src = attention_of(self.layers[m.kv_from].mixer) if 0 <= m.kv_from < i else None
                 if src is None or src.kv_from is not None:
@@ -215,7 +297,9 @@ class StackConfig:
         if li is not None:
             return start_layer <= li < end_layer
         if key == "embed":
-            return start_layer == 0
+            return start_layer == 0 or (self.tied and end_layer == self.num_hidden_layers)
+        if key == "side.embed":
+            return self.side_dim is not None
         return key in ("head", "final.norm") and end_layer == self.num_hidden_layers
 
     def to_dict(self) -> dict:
@@ -307,7 +391,54 @@ def _novosun(d: dict) -> StackConfig:
     return StackConfig("Novosun", int(d["vocab"]), int(d["width"]), norm, tuple(layers), copy.deepcopy(d))
 
 
-READERS = {"Gekazen": _gekazen, "Novosun": _novosun}
+def _pimisun(d: dict) -> StackConfig:
+    """Pimisun: latent attention, and attention over a window (norms over the whole query and key projections,
+    rotary positions, bent scores, values mixed with those of the first such layer); dense feed-forwards with
+    the square of relu, or a mixture of silu-gated experts with a softmax over the chosen and a shared expert;
+    layer norms of the residual sums; a vector per token and layer beside them; a tied head."""
+
+    def rotary(m: dict) -> RotarySpec:
+        return RotarySpec(float(m["rot"]["base"]), int(m["rot"]["dims"]))
+
+    def silu(e: dict) -> GluSpec:
+        return GluSpec(ff=int(e["ff"]), limit=math.inf, alpha=1.0, shift=0.0)
+
+    layers, first = [], None
+    for i, L in enumerate(d["layers"]):
+        m, f = L["mixer"], L.get("mlp")
+        if L["type"] == "latent_attention":
+            rot = RotarySpec(float(m["rot"]["base"]), int(m["rot_dim"]))
+            mixer = LatentSpec(int(m["heads"]), int(m["dim"]), int(m["rot_dim"]), int(m["vdim"]), int(m["q_rank"]),
+                               int(m["kv_rank"]), float(m["scale"]), rot)
+        elif L["type"] == "attention":
+            mask, cap = m.get("mask") or {}, m.get("softcap")
+            mixer = AttentionSpec(
+                heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                scale=float(m["scale"]), window=None if mask.get("size") is None else int(mask["size"]), whole_norm=True,
+                rot=rotary(m) if m.get("rot") else None, softcap=None if cap is None else float(cap),
+                v_mix_from=first if m.get("v_mix") else None)
+            if m.get("v_mix") and first is None:
+                first = i
+        else:
+            raise ValueError(f"layer {i}: mixer type {L['type']!r} not supported (have 'latent_attention', 'attention')")
+        mlp = None
+        if f is not None and f["kind"] == "dense":
+            mlp = DenseSpec(ff=int(f["ff"]), act="relu2")
+        elif f is not None and f["kind"] == "moe":
+            r = f["router"]
+            mlp = MoeSpec(RouterSpec(int(r["experts"]), 0, int(r["top"]), 1.0, bias=True, correction=False, renorm=True),
+                          silu(f["expert"]), silu(f["shared"]) if f.get("shared") else None, shared_gate=False)
+        elif f is not None:
+            raise ValueError(f"layer {i}: feed-forward kind {f['kind']!r} not supported (have 'dense', 'moe')")
+        layers.append(LayerSpec(mixer, mlp))
+    norm = NormSpec(float(d["norm"]["eps"]), of_sum=True, keep=float(d.get("postln_alpha", 1.0)), center=True)
+    side = d.get("token_side")
+    return StackConfig("Pimisun", int(d["vocab"]), int(d["width"]), norm, tuple(layers), copy.deepcopy(d),
+                       embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)),
+                       logit_scale=float(d.get("logit_scale", 1.0)), tied=True, side_dim=int(side["dim"]) if side else None)
+
+
+READERS = {"Gekazen": _gekazen, "Novosun": _novosun, "Pimisun": _pimisun}
 
 
 def gekazen_dict(width: int, vocab: int, layers: int, *, heads: int, kv_heads: int, dim: int, vdim: int, experts: int,

@@ -15,7 +15,8 @@ import torch
 from . import dense_ops as D
 from .dense_ops import pad64, padded
 from .stack_config import (
-    AttentionSpec, GluSpec, LayerSpec, LinearAttentionSpec, MoeSpec, NormSpec, ParallelSpec, StateSpaceSpec,
+    AttentionSpec, DenseSpec, GluSpec, LatentSpec, LayerSpec, LinearAttentionSpec, MoeSpec, NormSpec, ParallelSpec, RotarySpec,
+    StateSpaceSpec,
 )
 
 
@@ -51,6 +52,10 @@ class Tensors:
         return None if name is None else (norm.offset + self.get(name, n).float()).contiguous()
 
 
+def turns(rot: RotarySpec | None, device) -> torch.Tensor | None:
+    return None if rot is None else torch.tensor(rot.turns(), dtype=torch.float64, device=device)
+
+
 class _Part:
     """A mixer, or one of the parts of one.  ``main`` / ``tail``: its rows of the layer's projection, in
     element-type and float32 columns; ``biases`` of ``main`` (or None); ``col`` / ``tcol``: where its
@@ -77,16 +82,22 @@ class AttentionPart(_Part):
             self.biases = [t.get(f"{n}.b", rows) for n, rows in outs]
             self.o_b = t.f32("o.b", H)
         self.slopes = None if m.slopes is None else torch.tensor(m.slopes, dtype=torch.float32, device=t.device)
-        self.q_gain = t.f32("q.norm", m.dim) if m.qk_gain else None
-        self.k_gain = t.f32("k.norm", m.dim) if m.qk_gain and m.kv_from is None else None
+        gained = m.qk_gain or m.whole_norm
+        self.q_gain = t.f32("q.norm", m.dim * (m.heads if m.whole_norm else 1)) if gained else None
+        self.k_gain = t.f32("k.norm", m.dim * (m.kv_heads if m.whole_norm else 1)) if gained and m.kv_from is None else None
+        self.freq = turns(m.rot, t.device)
+        self.v_weight = float(t.get("vmix").float()) if m.v_mix else 0.0
+        self.v_col = m.heads * m.dim + m.kv_heads * m.dim  # its values among its columns
 
     def bind(self, cache, kv_index: int, dtype, eps: float) -> D.PagedAttention:
-        return D.PagedAttention(self.spec, self.slopes, kv_index, cache, eps, self.q_gain, self.k_gain)
+        return D.PagedAttention(self.spec, self.slopes, kv_index, cache, eps, self.q_gain, self.k_gain, self.freq)
 
     def run(self, att: D.PagedAttention, bf, b, y, y2, eps: float) -> torch.Tensor:
         m, n, own = self.spec, b.rows, self.spec.kv_from is None
         qkv, out = y[:, self.col :], bf.mixed("attn", self.width)
         gate = y2[:, self.tcol :] if m.head_gate else None
+        if m.v_mix:
+            att.mix_values(bf.values[m.v_mix_from], self.v_weight)
         if b.decode:
             att.rows(qkv, out, b.slot, b.pos, n, b.keys, append=own, gate=gate)
             return out
@@ -96,6 +107,59 @@ class AttentionPart(_Part):
             att.prompt(qkv, out, *b.blocks[att.prompt_block(m)], gate=gate)
         if b.n_single:
             att.rows(qkv, out, b.slot, b.pos, b.n_single, b.keys, append=False, lst=b.single, gate=gate)
+        return out
+
+
+class LatentPart(_Part):
+    """Columns, all float32: the queries' latent, the keys' and values' latent, the shared rotated key part.
+    The queries' second matrix leaves a head's unrotated part at a multiple of 64 columns (operands of the
+    products per head), behind them the rotated parts at multiples of 8."""
+
+    def __init__(self, spec: LatentSpec, t: Tensors, H: int, norm: NormSpec):
+        self.spec = m = spec
+        h, d, r, e, c = m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank
+        self.main = []
+        self.tail = [t.get("dq", m.q_rank, H), t.get("dkv", c + r, H)]
+        self.q_gain, self.kv_gain = t.f32("dq.norm", m.q_rank), t.f32("dkv.norm", c)
+        self.freq = turns(m.rot, t.device)
+        self.nope_pad, self.d8, r8 = pad64(d), pad8(d), pad8(r)
+        self.rot_col = h * self.nope_pad
+        self.q_cols = self.rot_col + h * r8
+        uq = t.get("uq", h * (d + r), m.q_rank).view(h, d + r, m.q_rank)
+        rows = torch.zeros(self.q_cols, m.q_rank, dtype=uq.dtype, device=t.device)
+        rows[: self.rot_col].view(h, self.nope_pad, m.q_rank)[:, :d] = uq[:, :d]
+        rows[self.rot_col :].view(h, r8, m.q_rank)[:, :r] = uq[:, d:]
+        self.uq = padded(rows, t.dtype, t.device)
+        uk, uv = t.get("uk", h * d, c).view(h, d, c), t.get("uv", h * e, c)
+        self.uk = padded(uk.transpose(1, 2), t.dtype, t.device)       # [heads, latent, unrotated]
+        self.uv = padded(uv.view(h, e, c), t.dtype, t.device)         # [heads, values, latent]
+        self.uk_rows = self.uv_rows = None
+        if t.dtype == torch.bfloat16:  # (the 32-bit mode does not expand)
+            k = torch.zeros(h, self.d8, c, dtype=uk.dtype, device=t.device)
+            k[:, :d] = uk
+            self.uk_rows = padded(k.view(h * self.d8, c), t.dtype, t.device)
+            self.uv_rows = self.uv.view(h * e, -1)
+        self.width = h * e
+        self.o = t.mat(("o", H, self.width))
+
+    def bind(self, cache, kv_index: int, dtype, eps: float) -> D.LatentAttention:
+        return D.LatentAttention(self.spec, self, kv_index, cache, eps)
+
+    def run(self, att: D.LatentAttention, bf, b, y, y2, eps: float) -> torch.Tensor:
+        m, n = self.spec, b.rows
+        cols = y2[:, self.tcol :]
+        kv = cols[:, m.q_rank :]
+        q, out = bf.mixed("lat_q", self.q_cols), bf.mixed("attn", self.width)
+        ql, ol = (bf.mixed(s, m.heads * pad64(m.kv_rank)) for s in ("lat_ql", "lat_ol"))
+        D.norm_linear(cols, self.q_gain, eps, bf.mixed("lat_c", m.q_rank), self.uq, q, n)
+        if b.decode:
+            att.rows(q, kv, ql, ol, out, b.slot, b.pos, n, b.keys, append=True)
+            return out
+        att.prepare(q, kv, b.slot, b.pos, n)
+        if b.latent.n_blocks:
+            att.prompt(q, kv, out, b.slot, b.pos, *b.latent.lists)
+        if b.latent.n_rows:
+            att.rows(q, kv, ql, ol, out, b.slot, b.pos, b.latent.n_rows, b.keys, append=False, lst=b.latent.rows)
         return out
 
 
@@ -173,14 +237,24 @@ class StateSpacePart(_RecurrentPart):
 
 
 class DenseFF:
-    def __init__(self, spec: GluSpec, t: Tensors, H: int):
+    def __init__(self, spec: GluSpec | DenseSpec, t: Tensors, H: int):
         self.spec = spec
-        self.gate, self.up = t.mat(("gate", spec.ff, H)), t.mat(("up", spec.ff, H))
-        self.down = t.mat(("down", H, spec.ff))
+        self.gate = t.mat(("gate", spec.ff, H)) if isinstance(spec, GluSpec) else None
+        self.up, self.down = t.mat(("up", spec.ff, H)), t.mat(("down", H, spec.ff))
+        self.after = D.After(spec.act) if isinstance(spec, DenseSpec) else None
+
+
+class TokenSide:
+    """A vector per token, gated by the residual, on its way into it behind a layer: ``table`` is the layer's part
+    of all tokens' vectors."""
+
+    def __init__(self, dim: int, table: torch.Tensor, t: Tensors, H: int):
+        self.gate, self.proj, self.gain = t.mat(("gate", dim, H)), t.mat(("proj", H, dim)), t.f32("norm", H)
+        self.table = table
 
 
 class MoeFF:
-    """Experts stacked; the shared expert's gate is one more output of the router product."""
+    """Experts stacked; the shared expert's gate, if it has one, is one more output of the router product."""
 
     def __init__(self, spec: MoeSpec, t: Tensors, H: int):
         self.spec = f = spec
@@ -193,20 +267,26 @@ class MoeFF:
             return out
 
         self.gate, self.up, self.down = stack("gate", ff, H), stack("up", ff, H), stack("down", H, ff)
-        self.correction = t.f32("correction", r.outputs)
+        self.correction = t.f32("correction", r.outputs) if r.correction else torch.zeros(r.outputs, device=t.device)
+        self.gate_col = r.outputs if f.shared is not None and f.shared_gate else -1
         rows = [("router", r.outputs, H)]
         self.s_gate = self.s_up = self.s_down = None
         if f.shared is not None:
-            rows.append(("shared.sg", 1, H))
+            if f.shared_gate:
+                rows.append(("shared.sg", 1, H))
             self.s_gate, self.s_up = t.mat(("shared.gate", f.shared.ff, H)), t.mat(("shared.up", f.shared.ff, H))
             self.s_down = t.mat(("shared.down", H, f.shared.ff))
-        self.router = t.mat(*rows)
+        self.router, self.router_b = t.mat(*rows), None
+        if r.bias:
+            self.router_b = torch.zeros(self.router.shape[0], device=t.device)
+            self.router_b[: r.outputs] = t.f32("router.b", r.outputs)
 
 
 class Layer:
-    """One layer's tensors: the parts of its mixer behind one projection, its feed-forward, its norms."""
+    """One layer's tensors: the parts of its mixer behind one projection, its feed-forward, its norms, its token
+    input (``side``: size and the table of all layers' parts)."""
 
-    def __init__(self, spec: LayerSpec, w: dict, i: int, H: int, norm: NormSpec, dtype, device):
+    def __init__(self, spec: LayerSpec, w: dict, i: int, H: int, norm: NormSpec, dtype, device, side=None):
         self.index, self.spec = i, spec
         t = Tensors(w, f"l{i}.", dtype, device)
         self.pre1, self.norm1 = (t.gain(n, H, norm) for n in norm.names(1))
@@ -216,13 +296,18 @@ class Layer:
             self.parts = [AttentionPart(m.left, mix.at("left."), H, norm), StateSpacePart(m.right, mix.at("right."), H, norm)]
             self.gain_a, self.gain_b = mix.f32("left.out", H), mix.f32("right.out", H)
         else:
-            kinds = {AttentionSpec: AttentionPart, LinearAttentionSpec: LinearAttentionPart, StateSpaceSpec: StateSpacePart}
+            kinds = {AttentionSpec: AttentionPart, LatentSpec: LatentPart, LinearAttentionSpec: LinearAttentionPart,
+                     StateSpaceSpec: StateSpacePart}
             self.parts = [kinds[type(m)](m, mix, H, norm)]
         self._project(H, dtype, device)
         self.ff = self.pre2 = self.norm2 = None
         if spec.mlp is not None:
             self.ff = (MoeFF if isinstance(spec.mlp, MoeSpec) else DenseFF)(spec.mlp, t.at("mlp."), H)
             self.pre2, self.norm2 = (t.gain(n, H, norm) for n in norm.names(2))
+        self.side = None
+        if side is not None:
+            dim, table = side
+            self.side = TokenSide(dim, table[:, i * dim : (i + 1) * dim], t.at("side."), H)
 
     def _project(self, H: int, dtype, device) -> None:
         """The parts' rows one below the other, element-type columns first.  An attention part's q, k, v are
@@ -258,5 +343,6 @@ class Layer:
         self.proj_b = torch.cat(biases).float().contiguous() if any_bias else None
 
     def tensors(self) -> list[torch.Tensor]:
-        holders = [self, *self.parts] + ([self.ff] if self.ff is not None else [])
-        return [t for h in holders for t in vars(h).values() if isinstance(t, torch.Tensor)]
+        holders = [self, *self.parts] + [x for x in (self.ff, self.side) if x is not None]
+        found = [t for h in holders for t in vars(h).values() if isinstance(t, torch.Tensor)]
+        return list({t.data_ptr(): t for t in found}.values())  # (views of the same matrix once)

@@ -18,6 +18,8 @@ Launches of a layer (rows R of the step):
             also routes, weighted down-projections in one launch.  The norms of a sublayer's output,
             its residual sum and the norm of the next input run inside the next product (up to 4 rows)
             or as a launch of their own
+            Latent attention: the queries' second matrix, its products per head on both sides of the attention;
+            a token's vector behind a layer: its gate and its projection
   R > 16    the same with GEMMs, the experts grouped by expert, their weighted sum inside the
             norm + residual launch; portions of prompts take the tiled attention and the chunked
             recurrence, single tokens beside them the split attention and the step
@@ -32,9 +34,9 @@ from . import dense_ops as D
 from . import ops
 from .dense_ops import pad64, padded
 from .model import DecoderShard
-from .paged_cache import PagedKVCache
-from .stack_config import GluSpec, MoeSpec, StackConfig, StateSpaceSpec, attention_of, recurrence_of
-from .stack_layers import AttentionPart, Layer, pad8
+from .paged_cache import PAGE, PagedKVCache, pages_for
+from .stack_config import LatentSpec, MoeSpec, StackConfig, StateSpaceSpec, attention_of, pooled_shape, recurrence_of
+from .stack_layers import AttentionPart, LatentPart, Layer, pad8
 
 
 class _Buffers:
@@ -56,6 +58,7 @@ class _Buffers:
         self.branch = self._z(rows, H, dtype=torch.float32)  # a sublayer's output
         self.branch2 = self._z(rows, H, dtype=torch.float32) if model.two_branches else None
         self.experts: dict[tuple[int, int], D.ExpertRows] = {}
+        self.values: dict[int, torch.Tensor] = {}  # of layers whose values later layers mix in
         # outputs of a single-token step (last shard)
         self.logits = self.logits16 = None
         self.next_token = self._z(seqs, dtype=torch.int32)
@@ -105,19 +108,27 @@ class _Buffers:
         return self._get("shared_out", self.cap, self.model.cfg.hidden_size)
 
 
+class _LatentRows:
+    """A step's rows as latent attention takes them: portions over expanded keys (``pages`` to gather, ``blocks`` of
+    tokens), the other rows one by one (``rows``)."""
+
+    def __init__(self, pages, n_pages: int, blocks, n_blocks: int, rows, n_rows: int):
+        self.lists, self.n_blocks, self.rows, self.n_rows = (blocks, n_blocks, pages, n_pages), n_blocks, rows, n_rows
+
+
 class _Batch:
     """What the mixers need to know about the rows of a step, on the device."""
 
     def __init__(self, rows: int, slot, pos, keys: int, single=None, n_single: int | None = None, blocks=None,
                  want=None, n_want: int | None = None, chunks=None, n_chunks: int = 0, seqs=None, n_seqs: int = 0,
-                 alone=None, n_alone: int = 0):
+                 alone=None, n_alone: int = 0, latent: _LatentRows | None = None):
         self.rows, self.slot, self.pos, self.keys = rows, slot, pos, keys
         self.single, self.n_single = single, rows if n_single is None else n_single  # rows alone (None: all)
         self.blocks = blocks or {}                                                   # tokens -> (list, count)
         self.want, self.n_want = want, rows if n_want is None else n_want            # rows with logits
         # recurrences: portions of several tokens, cut into chunks; rows that are a portion by themselves
         self.chunks, self.n_chunks, self.seqs, self.n_seqs = chunks, n_chunks, seqs, n_seqs
-        self.alone, self.n_alone = alone, n_alone
+        self.alone, self.n_alone, self.latent = alone, n_alone, latent
 
     @property
     def decode(self) -> bool:
@@ -135,9 +146,19 @@ class StackModel(DecoderShard):
         self.end_layer = cfg.num_hidden_layers if end_layer is None else end_layer
         if not (0 <= self.start_layer < self.end_layer <= cfg.num_hidden_layers):
             raise ValueError(f"bad layer range [{start_layer},{end_layer}) of {cfg.num_hidden_layers}")
-        H = cfg.hidden_size
-        self.layers = [Layer(cfg.layers[i], weights, i, H, cfg.norm, dtype, self.device)
+        H, side = cfg.hidden_size, None
+        if cfg.side_dim is not None:
+            if not self.is_first:
+                raise ValueError(f"{cfg.architecture}: every layer reads the tokens, a shard must start at layer 0")
+            t = weights["side.embed"]
+            if tuple(t.shape) != (cfg.vocab_size, cfg.num_hidden_layers * cfg.side_dim):
+                raise ValueError(f"side.embed: shape {tuple(t.shape)}, config says {cfg.vocab_size} x {cfg.num_hidden_layers} parts of "
+                                 f"{cfg.side_dim}")
+            side = (cfg.side_dim, t.to(self.device, dtype).contiguous())
+        self.layers = [Layer(cfg.layers[i], weights, i, H, cfg.norm, dtype, self.device, side)
                        for i in range(self.start_layer, self.end_layer)]
+        self.mixed_from = {m.v_mix_from for m in (attention_of(L.spec.mixer) for L in self.layers) if m is not None and m.v_mix}
+        self.has_latent = any(isinstance(L.spec.mixer, LatentSpec) for L in self.layers)
         self.two_branches = any(len(L.parts) > 1 for L in self.layers)
         # layer -> index of the pool's layer that holds its keys and values, its recurrent state
         self.kv_index: dict[int, int] = {}
@@ -150,13 +171,18 @@ class StackModel(DecoderShard):
                 h, _, d, e = r.core
                 self.state_index[L.index] = len(self.state_shapes)
                 self.state_shapes.append((h, d, e, *((r.conv, r.channels) if isinstance(r, StateSpaceSpec) else (0, 0))))
-            m = attention_of(L.spec.mixer)
+            m, shape = attention_of(L.spec.mixer), pooled_shape(L.spec.mixer)
+            if shape is not None:
+                self.kv_index[L.index] = len(self.kv_shapes)
+                self.kv_shapes.append(shape)
             if m is None:
                 continue
+            if m.v_mix and m.v_mix_from < self.start_layer:
+                raise ValueError(f"layer {L.index} mixes in the values of layer {m.v_mix_from}, which is outside the shard "
+                                 f"[{self.start_layer},{self.end_layer})")
             if m.kv_from is None:
-                self.kv_index[L.index] = len(self.kv_shapes)
-                self.kv_shapes.append((m.kv_heads, m.dim, m.vdim))
-            elif m.kv_from not in self.kv_index:
+                continue
+            if m.kv_from not in self.kv_index:
                 raise ValueError(f"layer {L.index} uses the keys of layer {m.kv_from}, which is outside the shard "
                                  f"[{self.start_layer},{self.end_layer})")
             else:
@@ -165,8 +191,9 @@ class StackModel(DecoderShard):
         if self.is_first:
             self.embed = padded(weights["embed"].to(self.device), dtype, self.device)
         if self.is_last:
-            self.norm = (cfg.norm.offset + weights["final.norm"].to(self.device).float()).contiguous()
-            self.head = padded(weights["head"].to(self.device), dtype, self.device)
+            self.norm = ((cfg.norm.offset + weights["final.norm"].to(self.device).float()) * cfg.logit_scale).contiguous()
+            tied = self.embed if cfg.tied else None
+            self.head = tied if tied is not None else padded(weights["embed" if cfg.tied else "head"].to(self.device), dtype, self.device)
         self._bufs: dict[tuple, _Buffers] = {}
         self._graphs: dict[tuple, tuple] = {}
         self._bound: tuple | None = None  # (cache, per layer and part the argument blocks)
@@ -214,7 +241,7 @@ class StackModel(DecoderShard):
     def _mixers(self, cache: PagedKVCache) -> list[list]:
         """Per layer, the bound operator of each part of its mixer."""
         if self._bound is None or self._bound[0] is not cache:
-            self._bound = (cache, [[p.bind(cache, (self.kv_index if isinstance(p, AttentionPart) else self.state_index)[L.index],
+            self._bound = (cache, [[p.bind(cache, (self.kv_index if isinstance(p, (AttentionPart, LatentPart)) else self.state_index)[L.index],
                                            self.dtype, self.cfg.eps) for p in L.parts] for L in self.layers])
         return self._bound[1]
 
@@ -228,55 +255,72 @@ class StackModel(DecoderShard):
             D.norm_rows(bf.h, pre, self.cfg.eps, bf.xb, n)
 
     def _product(self, bf: _Buffers, n: int, due: D.Branches | None, pre, w, out, bias=None, tail=None, up=None, spec=None,
-                 keep_operand: bool = False) -> None:
+                 keep_operand: bool = False, after: D.After | None = None) -> None:
         """out <- operand @ w^T (or the gated pair), after the outstanding norms and sum;
         ``keep_operand``: bf.xb is read by later launches too"""
         if due is not None and len(bf.hs) > 1 and D.post_linear_fits(n, w, bf.xb, self.cfg.hidden_size, pre is not None):
             x = bf.h
             bf.cur ^= 1
-            D.post_linear(x, due, self.cfg.eps, bf.h, bf.xb if keep_operand else None, w, out, n, bias, tail, pre, up, spec)
+            D.post_linear(x, due, self.cfg.eps, bf.h, bf.xb if keep_operand else None, w, out, n, bias, tail, pre, up, spec, after)
             return
         self._settle(bf, n, due, pre)
         if up is not None:
             D.glu(bf.xb, w, up, out, n, spec)
         else:
-            D.linear(bf.xb, w, out, n, bias=bias, tail=tail)
+            D.linear(bf.xb, w, out, n, bias=bias, tail=tail, after=after)
 
     def _mixer(self, L: Layer, bound: list, bf: _Buffers, b: _Batch, due: D.Branches | None) -> D.Branches:
         """The mixer of the residual; returns its output on the way into the residual"""
         n, eps = b.rows, self.cfg.eps
-        y = bf.cols("proj", pad8(L.n_main))
-        y2 = bf.f32("proj_tail", L.n_tail) if L.n_tail else None
-        self._product(bf, n, due, L.pre1, L.proj, y, bias=L.proj_b, tail=(y2, L.n_tail) if L.n_tail else None)
+        p, mixed = L.parts[0], L.index in self.mixed_from
+        y2 = bf.f32("proj_tail", pad8(L.n_tail)) if L.n_tail else None
+        if L.n_main:  # (a layer whose values others mix in keeps its columns to itself)
+            y = bf.cols("proj_kept" if mixed else "proj", pad8(L.n_main))
+            self._product(bf, n, due, L.pre1, L.proj, y, bias=L.proj_b, tail=(y2, L.n_tail) if L.n_tail else None)
+        else:
+            y = None
+            self._product(bf, n, due, L.pre1, L.proj, y2, bias=L.proj_b)
+        if mixed:
+            bf.values[L.index] = y[:, p.col + p.v_col :]
         outs = [p.run(op, bf, b, y, y2, eps) for p, op in zip(L.parts, bound)]
-        p = L.parts[0]
         if len(L.parts) == 1:
             D.linear(outs[0], p.o, bf.branch, n, bias=p.o_b)
-            return D.Branches(bf.branch, L.norm1, self.cfg.norm.mult)
+            return D.Branches(bf.branch, L.norm1, self.cfg.norm.mult, norm=self.cfg.norm)
         D.linear_pair(outs[0], p.o, bf.branch, outs[1], L.parts[1].o, bf.branch2, n)
         return D.Branches(bf.branch, L.norm1, self.cfg.norm.mult, bf.branch2, L.gain_a, L.gain_b)
 
     def _dense(self, L: Layer, bf: _Buffers, n: int, due: D.Branches) -> D.Branches:
-        f: GluSpec = L.spec.mlp
+        f = L.spec.mlp
         act = bf.mixed("ff", f.ff)
-        self._product(bf, n, due, L.pre2, L.ff.gate, act, up=L.ff.up, spec=f)
+        if L.ff.gate is None:
+            self._product(bf, n, due, L.pre2, L.ff.up, act, after=L.ff.after)
+        else:
+            self._product(bf, n, due, L.pre2, L.ff.gate, act, up=L.ff.up, spec=f)
         D.linear(act, L.ff.down, bf.branch, n)
-        return D.Branches(bf.branch, L.norm2, self.cfg.norm.mult)
+        return D.Branches(bf.branch, L.norm2, self.cfg.norm.mult, norm=self.cfg.norm)
+
+    def _side(self, L: Layer, bf: _Buffers, n: int, due: D.Branches | None) -> D.Branches:
+        """The tokens' vectors, gated by the residual: gelu(gate x) * vector, projected; then normed and added"""
+        s = L.side
+        act = bf.mixed("side", self.cfg.side_dim)
+        self._product(bf, n, due, None, s.gate, act, after=D.After("gelu_tanh", s.table, bf.tokens))
+        D.linear(act, s.proj, bf.branch, n)
+        return D.Branches(bf.branch, s.gain)
 
     def _moe(self, L: Layer, bf: _Buffers, n: int, due: D.Branches) -> D.Branches | None:
         """The experts of the residual: bf.branch, or already normed and added (returns None)"""
         f, H, w = L.spec.mlp, self.cfg.hidden_size, L.ff
         r, mult = f.router, self.cfg.norm.mult
         logits, idx, wt = bf.router_logits(w.router.shape[0]), bf.idx(r.top), bf.wt(r.top)
-        self._product(bf, n, due, L.pre2, w.router, logits, keep_operand=True)
+        self._product(bf, n, due, L.pre2, w.router, logits, bias=w.router_b, keep_operand=True)
         if n <= D.GEMV_MAX_ROWS:
             key = (L.index, bf.cur)
             if key not in bf.experts:
                 bf.experts[key] = D.ExpertRows(f, w, bf, H, bf.h)
             bf.experts[key].glu(n)
             bf.experts[key].down(n)
-            return D.Branches(bf.branch, L.norm2, mult)
-        D.moe_route(logits, w.correction, r.scale, idx, wt, n)
+            return D.Branches(bf.branch, L.norm2, mult, norm=self.cfg.norm)
+        D.moe_route(logits, w.correction, r.scale, idx, wt, n, r.renorm)
         act, out = bf.act(r.top, f.expert.ff), bf.expert_out(r.top)
         ws = ops.moe_group(idx[:n], r.experts, check_indices=False)  # identity ids are past the end: left out
         D.grouped_gemm(bf.xb, w.gate, ws, act, n, r.top, up=w.up, spec=f.expert)
@@ -286,7 +330,8 @@ class StackModel(DecoderShard):
             sact, shared = bf.shared_act(f.shared.ff), bf.shared_out()
             D.glu_gemm(bf.xb, w.s_gate, w.s_up, sact, n, f.shared)
             D.linear(sact, w.s_down, shared, n)
-        D.moe_sum_post_norm(out, idx, wt, shared, logits, r.experts, r.outputs, L.norm2, self.cfg.eps, bf.h, bf.xb, n, mult)
+        D.moe_sum_post_norm(out, idx, wt, shared, logits, r.experts, w.gate_col, L.norm2, self.cfg.eps, bf.h, bf.xb, n, mult,
+                            self.cfg.norm)
         return None
 
     def _forward(self, cache: PagedKVCache, bf: _Buffers, b: _Batch, logits: bool) -> torch.Tensor:
@@ -295,7 +340,7 @@ class StackModel(DecoderShard):
         n, H, eps = b.rows, self.cfg.hidden_size, self.cfg.eps
         bf.cur = 0
         if self.is_first:
-            D.embed_rows(bf.tokens[:n], self.embed, bf.h, bf.xb, H)
+            D.embed_rows(bf.tokens[:n], self.embed, bf.h, bf.xb, H, self.cfg.embed_scale)
         else:
             bf.xb[:n, :H].copy_(bf.h[:n])
         due = None  # the latest sublayer's output, which still has to pass its norm
@@ -303,6 +348,8 @@ class StackModel(DecoderShard):
             due = self._mixer(L, bound, bf, b, due)
             if L.ff is not None:
                 due = (self._moe if isinstance(L.spec.mlp, MoeSpec) else self._dense)(L, bf, n, due)
+            if L.side is not None:
+                due = self._side(L, bf, n, due)
             if self.layer_hook is not None:
                 self._settle(bf, n, due, None)
                 due = None
@@ -313,7 +360,7 @@ class StackModel(DecoderShard):
                 bf.hs[0][:n].copy_(bf.h[:n])
                 bf.cur = 0
             return bf.h[:n]
-        D.norm_rows(bf.h, self.norm, eps, bf.xn, b.n_want, rows=b.want)
+        D.norm_rows(bf.h, self.norm, eps, bf.xn, b.n_want, rows=b.want, center=self.cfg.norm.center)
         if bf.logits is None or bf.logits.shape[0] != b.n_want:
             bf.logits = torch.empty(b.n_want, self.cfg.vocab_size, dtype=self.dtype, device=self.device)
             bf.logits16 = None
@@ -340,6 +387,7 @@ class StackModel(DecoderShard):
         sizes = {D.PagedAttention.prompt_block(m) for m in (attention_of(L.spec.mixer) for L in self.layers) if m is not None}
         blocks: dict[int, list] = {s: [] for s in sizes}
         chunks, seqs, alone = [], [], []
+        pages, lat_blocks, lat_rows = [], [], []  # latent attention
         C = D.recur_chunk() if self.state_shapes else 0
         at, keys = 0, 1
         tiled = self.dtype == torch.bfloat16  # the 32-bit mode runs every position by itself
@@ -353,13 +401,18 @@ class StackModel(DecoderShard):
             else:
                 for s in sizes:
                     blocks[s] += [(at + o, row, p0 + o, min(s, c - o)) for o in range(0, c, s)]
+            if self.has_latent and tiled and c >= D.LATENT_SHORT:
+                lat_blocks += [(at + o, len(pages) * PAGE, p0 + o, min(D.LATENT_BLOCK, c - o)) for o in range(0, c, D.LATENT_BLOCK)]
+                pages += [(row, i) for i in range(pages_for(p0 + c))]
+            elif self.has_latent:
+                lat_rows.extend(range(at, at + c))
             if C and c == 1:
                 alone.append(at)
             elif C:
                 seqs.append((len(chunks), -(-c // C), 0, 0))
                 chunks += [(at + o, row, p0 + o, min(C, c - o), p0, 0, 0, 0) for o in range(0, c, C)]
             at += c
-        parts = [slot, pos] + [np.asarray(x, np.int32).reshape(-1) for x in (single, want, chunks, seqs, alone)]
+        parts = [slot, pos] + [np.asarray(x, np.int32).reshape(-1) for x in (single, want, chunks, seqs, alone, pages, lat_blocks, lat_rows)]
         have = [s for s in sizes if blocks[s]]
         parts += [np.asarray(blocks[s], np.int32).reshape(-1) for s in have]
         starts, total = [], 0
@@ -371,11 +424,12 @@ class StackModel(DecoderShard):
             flat[s0 : s0 + p.size] = p
         dev = torch.from_numpy(flat).to(self.device)
         t = [dev[s0 : s0 + p.size] for s0, p in zip(starts, parts)]
+        latent = _LatentRows(t[7], len(pages), t[8], len(lat_blocks), t[9], len(lat_rows)) if self.has_latent else None
         one_each = all(c == 1 for _, c in counts)
         return _Batch(n, t[0], t[1], keys, single=None if one_each else t[2], n_single=len(single),
-                      blocks={s: (t[7 + i], len(blocks[s])) for i, s in enumerate(have)},
+                      blocks={s: (t[10 + i], len(blocks[s])) for i, s in enumerate(have)},
                       want=t[3], n_want=len(want), chunks=t[4], n_chunks=len(chunks), seqs=t[5], n_seqs=len(seqs),
-                      alone=t[6], n_alone=len(alone))
+                      alone=t[6], n_alone=len(alone), latent=latent)
 
     def step(self, cache: PagedKVCache, entries: list[tuple[int, list[int], list[int]]]) -> torch.Tensor | None:
         """One batch: ``entries`` are (cache row, its next tokens, places among them whose logits are

@@ -437,44 +437,52 @@ int exo_sample(const uint16_t* logits, const exo_sampler_params* params, int32_t
  * both).  Row strides (ld*) of matrix operands are multiples of 64 elements and the columns past
  * the logical size are zero. ---- */
 
-/* x[i] = xb[i] = table[ids[i]]: the float32 residual and its copy in the element type. */
+/* x[i] = xb[i] = scale * table[ids[i]]: the float32 residual and its copy in the element type. */
 int exo_embed_rows(const int32_t* ids, const void* table, float* x, void* xb, int n, int V, int H,
-                   int ldt, int ldx, int dtype, exo_stream_t stream);
-/* y[i] = x[rows[i]] / rms * gain (rows null: row i); x float32 [.., H]. */
+                   int ldt, int ldx, float scale, int dtype, exo_stream_t stream);
+/* y[i] = x[rows[i]] / rms * gain (rows null: row i), the mean taken off x first if center; x float32
+ * [.., ldx]. */
 int exo_norm_rows(const float* x, const int32_t* rows, const float* gain, void* y, int n, int H,
-                  int ldy, float eps, int dtype, exo_stream_t stream);
+                  int ldx, int ldy, float eps, int center, int dtype, exo_stream_t stream);
 /* Norm of a sublayer's output, then the residual sum: x_out = x + mult * gain * v / rms(v), where v
- * is the branch, or (branch2) half the sum of two branches normed each with a gain of its own; the
- * next product's operand is x_out, or (pre) x_out / rms(x_out) * pre.  Branches and x float32 [.., H]. */
+ * is the branch, or (branch2) half the sum of two branches normed each with a gain of its own; or
+ * (sum) norm of the residual sum: x_out = gain * norm(keep * x + v), norm being division by the RMS,
+ * after taking the mean off if center; the next product's operand is x_out, or (pre)
+ * x_out / rms(x_out) * pre.  x float32 [.., H], branches [.., ldb]. */
 typedef struct {
   const float *x, *branch, *branch2, *gain_a, *gain_b, *gain, *pre;
   float* x_out;
   void* operand; /* element type */
-  int H;
-  float eps, mult;
+  int H, ldb, sum, center;
+  float eps, mult, keep;
 } exo_post_norm;
 /* ... as a launch of its own, in place (x_out == x); operand [n][ldx]. */
-int exo_post_norm_add(const exo_post_norm* q, int ldb, int n, int ldx, int dtype,
-                      exo_stream_t stream);
+int exo_post_norm_add(const exo_post_norm* q, int n, int ldx, int dtype, exo_stream_t stream);
 /* The same with the branch formed from a token's experts: sum of wt * y over the chosen experts
- * (idx >= experts: the input x itself), plus sigmoid(logits[gate_col]) * shared. */
+ * (idx >= experts: the input x itself), plus sigmoid(logits[gate_col]) * shared (gate_col < 0: shared as
+ * it is). */
 int exo_moe_sum_post_norm(const void* y, const int32_t* idx, const float* wt, const void* shared,
                           const float* logits, int top, int experts, int ldy, int lds, int ldl,
                           int gate_col, const exo_post_norm* q, int n, int ldx, int dtype,
                           exo_stream_t stream);
-/* softmax over n logits; the `top` largest of score + correction; weight = score * scale. */
+/* softmax over n logits; the `top` largest of score + correction; weight = score * scale.  renorm: the
+ * largest of logit + correction, weights = softmax over the chosen logits alone, times scale. */
 int exo_moe_route(const float* logits, const float* correction, int32_t* idx, float* wt, int rows,
-                  int n, int ldl, int top, float scale, exo_stream_t stream);
+                  int n, int ldl, int top, float scale, int renorm, exo_stream_t stream);
 
 /* y[M,N] = x[M,K] @ w[N,K]^T (+ bias): columns below n1 to y (element type, or float32 if y_f32),
  * the rest to y2 (float32; n1 = N: none).  w_up non-null: the gated pair instead, with g = min(x @ w^T,
- * limit), u = clamp(x @ w_up^T, +-limit): y = g sigmoid(alpha g) (u + shift). */
+ * limit), u = clamp(x @ w_up^T, +-limit): y = g sigmoid(alpha g) (u + shift).  act (one plain output):
+ * 1 square of relu, 2 gelu (tanh form); mul non-null: then times mul[mul_rows[m]] (element type, row
+ * stride ldmul; mul_rows null: row m). */
 typedef struct {
   const void *x, *w, *w_up;
   const float* bias;
   void* y;
   float* y2;
-  int M, N, n1, ldx, ldw, ldy, ldy2, y_f32, dtype;
+  const void* mul;
+  const int32_t* mul_rows;
+  int M, N, n1, ldx, ldw, ldy, ldy2, y_f32, dtype, act, ldmul;
   float limit, alpha, shift;
 } exo_linear;
 /* up to 16 rows; b non-null: a second product over the same number of rows in the same launch */
@@ -482,7 +490,8 @@ int exo_linear_rows(const exo_linear* a, const exo_linear* b, exo_stream_t strea
 int exo_linear_gemm(const exo_linear* a, float* workspace, int64_t workspace_floats,
                     exo_stream_t stream);
 /* exo_post_norm_add and the product in one launch (few rows: exo_post_linear_fits): a->x is not
- * read, the residual goes to q->x_out (not q->x), the operand also to q->operand (may be null). */
+ * read, the residual goes to q->x_out (not q->x), the operand also to q->operand (may be null).  q->x and
+ * q->x_out null: the operand is the normed branch alone. */
 int exo_post_linear_fits(int M, int N, int H, int ldx, int dtype);
 int exo_post_linear(const exo_post_norm* q, const exo_linear* a, exo_stream_t stream);
 /* Experts of a prompt by (token, slot) pair through exo_moe_group's workspace; w_up null: the
@@ -494,7 +503,7 @@ int exo_dense_grouped_gemm(const void* x, const void* w, const void* w_up, const
 
 /* Experts of a decode step (up to 16 rows): gated products, then the weighted sum.  correction
  * non-null: the gated launch also routes (as exo_moe_route over `outputs` logits) and leaves idx
- * and wt; null: they are given. */
+ * and wt; null: they are given.  gate_col < 0: the shared expert has no gate. */
 typedef struct {
   const void *x, *gate, *up, *down, *shared_gate, *shared_up, *shared_down;
   void *act, *shared_act;
@@ -503,7 +512,7 @@ typedef struct {
   int32_t* idx;
   float* wt;
   const float *logits, *correction;
-  int rows, top, experts, ff, shared_ff, H, ldx, lda, ldsa, ldl, gate_col, outputs, dtype;
+  int rows, top, experts, ff, shared_ff, H, ldx, lda, ldsa, ldl, gate_col, outputs, renorm, dtype;
   float router_scale, limit, alpha, shift, shared_limit, shared_alpha, shared_shift;
 } exo_moe_rows;
 int exo_moe_glu_rows(const exo_moe_rows* args, exo_stream_t stream);
@@ -513,17 +522,26 @@ int exo_moe_down_rows(const exo_moe_rows* args, exo_stream_t stream);
  * [page][kv_heads][ldv][64]; table [slots][max_pages]; row i of qkv belongs to slot[i] at
  * position pos[i].  window 0: causal; else a key is seen if fewer than `window` positions back or
  * among the first keep_first positions.  slopes: per-head distance penalty, or null.  q_gain, k_gain
- * [dim]: gains of the query / key norm (unit_qk), or null.  gate [rows][ldg]: head h's output times
+ * [dim]: gains of the query / key norm (unit_qk), or null; whole_norm: RMS norms over the whole query and
+ * key projections instead, gains [heads * dim], [kv_heads * dim].  rot: so many leading dimensions of a head
+ * turned by position * freq[i] turns, pair (2i, 2i + 1).  softcap > 0: score to cap * tanh(score / cap).
+ * v_mix [rows][ldmix]: values (1 - mix) v + mix v_mix, or null.  prepared: queries went through
+ * exo_paged_prepare.  gate [rows][ldg]: head h's output times
  * sigmoid(gate[h]), or null. */
 typedef struct {
   const void* qkv;
   void *k_pool, *v_pool;
   const int32_t *table, *slot, *pos, *list;
   const float *slopes, *q_gain, *k_gain, *gate;
+  const double* freq;
+  const void* v_mix;
   void* out;
-  float scale, eps;
-  int n, heads, kv_heads, dim, vdim, ldq, ldk, ldv, ldo, ldg, max_pages, window, keep_first, unit_qk, dtype;
+  float scale, eps, softcap, mix;
+  int n, heads, kv_heads, dim, vdim, ldq, ldk, ldv, ldo, ldg, max_pages, window, keep_first, unit_qk, whole_norm, rot, ldmix,
+      prepared, dtype;
 } exo_paged_attn;
+/* whole_norm, rot, v_mix: queries of all n rows in place (qkv is written), keys and values into the pool */
+int exo_paged_prepare(const exo_paged_attn* args, exo_stream_t stream);
 /* keys (normalised if unit_qk) and values of all n rows into the pool */
 int exo_paged_append(const exo_paged_attn* args, exo_stream_t stream);
 /* one query position per row (list: the rows, null: all n); append: also stores the row's own key
@@ -536,6 +554,56 @@ int exo_paged_attn_rows(const exo_paged_attn* args, int nsplit, int append, void
  * at most exo_paged_prompt_block(heads, kv_heads) tokens of one sequence */
 int exo_paged_prompt_block(int heads, int kv_heads);
 int exo_paged_attn_prompt(const exo_paged_attn* args, exo_stream_t stream);
+
+/* Latent attention: a position's normed latent [rank] and a rotated key part [rot] that all heads share
+ * in pool [page][64][ldk], the latter at the latent size rounded up to 32.  kv float32 [rows][ldkv] holds
+ * both as projected; q [rows][ldq] the heads' rotated query parts at rot_col, each at a multiple of 8;
+ * q_latent [rows][ldql] the heads' queries through their key matrices, each at a multiple of 64.
+ * prepared: exo_latent_prepare has run. */
+typedef struct {
+  const void *q, *q_latent;
+  const float *kv, *gain;
+  const double* freq;
+  void* pool;
+  const int32_t *table, *slot, *pos, *list;
+  void* out;
+  float* parts;
+  int64_t parts_floats;
+  float scale, eps;
+  int n, heads, rank, rot, rot_col, ldq, ldql, ldkv, ldk, ldo, max_pages, prepared, nsplit, dtype;
+} exo_latent_attn;
+/* latents and shared key parts of all n rows into the pool, the rotated query parts in place */
+int exo_latent_prepare(const exo_latent_attn* args, exo_stream_t stream);
+/* one query position per row: weighted latents to out (nsplit 1; head h at a multiple of 64) or partials
+ * of nsplit key ranges to parts; append: also stores the row's own latent and key part */
+int64_t exo_latent_parts(int n, int heads, int rank, int nsplit); /* floats */
+int exo_latent_rows(const exo_latent_attn* args, int append, exo_stream_t stream);
+/* y[row][h] = w[h] x[row][h], w [heads][N][ldw], for n rows (list: which, or null); parts non-null: x is
+ * merged from the partials of exo_latent_rows (in the order of its rows) */
+typedef struct {
+  const void *x, *w;
+  const float* parts;
+  int64_t parts_floats;
+  void* y;
+  const int32_t* list;
+  int n, heads, N, K, ldx, x_head, ldw, ldy, y_head, nsplit, dtype;
+} exo_head_linear_args;
+int exo_head_linear(const exo_head_linear_args* args, exo_stream_t stream);
+/* bf16: pages [n_pages][2] = slot, page of its sequence -> latents c [64 n_pages][rank up to 64], shared
+ * key parts k [64 n_pages][rot up to 8] */
+int exo_latent_gather(const exo_latent_attn* args, const int32_t* pages, int n_pages, void* c, void* k,
+                      exo_stream_t stream);
+/* portions of prompts, bf16, over expanded keys [keys][ldk] (d8 per head), shared parts [keys][r8] and
+ * values [heads * vdim][ldv]: list holds n blocks {first row, first key row of the sequence, first
+ * position, tokens} of at most 128 tokens; queries prepared, head h's at h * q_head */
+typedef struct {
+  const void *q, *k, *k_rot, *v;
+  const int32_t* list;
+  void* out;
+  float scale;
+  int n, heads, vdim, d8, r8, ldq, q_head, rot_col, ldk, ldv, ldo;
+} exo_latent_prompt_args;
+int exo_latent_prompt(const exo_latent_prompt_args* args, exo_stream_t stream);
 
 /* Recurrent mixers.  Per head, from S = 0: S <- diag(a_t) S + k_t v_t^T, o_t = S^T (q_scale q_t), S
  * [dim][vdim] float32.  per_channel: a_t per key channel = sigmoid(z)^(inv_tau) with z = low @ decay_w +

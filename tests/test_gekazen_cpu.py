@@ -249,7 +249,7 @@ def test_new_entry_points_check_their_arguments():
     assert lib.exo_linear_rows(native.Linear(**dict(lin, n1=4)), None, None) == -1  # no second output
     assert lib.exo_linear_rows(native.Linear(**dict(lin, ldx=72, ldw=72)), None, None) == -1
     assert b"multiples of 64" in lib.exo_last_error()
-    assert lib.exo_moe_route(16, 16, 16, 16, 1, 600, 600, 2, 1.0, None) == -1
+    assert lib.exo_moe_route(16, 16, 16, 16, 1, 600, 600, 2, 1.0, 0, None) == -1
     a = native.PagedAttn(qkv=16, k_pool=16, v_pool=16, table=16, slot=16, pos=16, out=16, n=1, heads=3, kv_heads=2,
                          dim=64, vdim=64, ldk=64, ldv=64, ldq=999, ldo=999, max_pages=1)
     assert lib.exo_paged_attn_rows(a, 1, 0, None, 0, None) == -1

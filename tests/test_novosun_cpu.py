@@ -246,8 +246,8 @@ def test_new_entry_points_check_their_arguments():
         assert b"exo_recur_chunks" in lib.exo_last_error()
     assert lib.exo_gated_norm_rows(native.GatedNorm(y=16, gate=16, gain=16, out=16, width=10, groups=3, period=10, ldy=10, ldg=10,
                                                     ldo=10), None, 1, None) == -1
-    q = native.PostNorm(x=16, x_out=16, branch=16, gain=16, operand=16, H=64, branch2=16)
-    assert lib.exo_post_norm_add(q, 64, 1, 64, 0, None) == -1 and b"gain each" in lib.exo_last_error()
+    q = native.PostNorm(x=16, x_out=16, branch=16, gain=16, operand=16, H=64, ldb=64, branch2=16)
+    assert lib.exo_post_norm_add(q, 1, 64, 0, None) == -1 and b"gain each" in lib.exo_last_error()
     lin = native.Linear(x=16, w=16, w_up=16, y=16, M=1, N=8, n1=8, ldx=64, ldw=64, ldy=8)
     assert lib.exo_linear_rows(lin, lin, None) == -1 and b"gated pair" in lib.exo_last_error()
     assert lib.exo_post_linear(q, lin, None) == -1
