@@ -340,6 +340,11 @@ LATENT_BLOCK = 128  # tokens of a block of expanded prompt attention
 LATENT_SHORT = 32   # portions below this many tokens go through the absorbed rows
 
 
+def latent_expands(spec) -> bool:
+    """Whether a design's expanded keys and values fit the prompt kernel (else all rows are absorbed)."""
+    return -(-spec.dim // 8) + -(-spec.rot_dim // 8) <= 32 and spec.vdim <= 256
+
+
 class LatentAttention:
     """Latent attention of one layer over a paged pool.  ``spec``: LatentSpec; ``w``: the layer's tensors
     (``stack_layers.LatentPart``); ``li``: index of the pool's layer."""

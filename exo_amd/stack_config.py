@@ -474,3 +474,24 @@ def novosun_dict(width: int, vocab: int, kinds: str, *, heads: int, kv_heads: in
     mlp = None if ff is None else dict(kind="dense", ff=ff, limit=limit)
     layers = [dict(copy.deepcopy(linear if k == "g" else parallel), mlp=copy.deepcopy(mlp)) for k in kinds]
     return dict(architecture="Novosun", vocab=vocab, width=width, norm=dict(eps=eps), residual_mult=mult, layers=layers)
+
+
+def pimisun_dict(width: int, vocab: int, kinds: str, *, heads: int, kv_heads: int, dim: int, rot: int, window: int, lat_heads: int,
+                 lat_dim: int, lat_rot: int, lat_vdim: int, q_rank: int, kv_rank: int, ff: int, experts: int, top: int,
+                 expert_ff: int, shared_ff: int | None, side: int, dense: int = 1, softcap: float = 30.0, base: float = 5e5,
+                 alpha: float = 2.0, eps: float = 1e-6) -> dict:
+    """A ``config.json`` of the design (benchmarks); ``kinds``: a letter per layer, l for latent attention, a for
+    attention; the first ``dense`` layers have a dense feed-forward, the others experts."""
+    latent = dict(type="latent_attention", mixer=dict(
+        heads=lat_heads, dim=lat_dim, rot_dim=lat_rot, vdim=lat_vdim, q_rank=q_rank, kv_rank=kv_rank,
+        rot=dict(base=base, dims=lat_rot), scale=(lat_dim + lat_rot) ** -0.5))
+    attention = dict(type="attention", mixer=dict(
+        heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, mask=dict(size=window), rot=dict(base=base, dims=rot), scale=dim ** -0.5,
+        softcap=softcap, v_mix=True))
+    moe = dict(kind="moe", expert=dict(ff=expert_ff), router=dict(experts=experts, top=top))
+    if shared_ff:
+        moe["shared"] = dict(ff=shared_ff)
+    layers = [dict(copy.deepcopy(latent if k == "l" else attention), mlp=dict(kind="dense", ff=ff) if i < dense else copy.deepcopy(moe))
+              for i, k in enumerate(kinds)]
+    return dict(architecture="Pimisun", vocab=vocab, width=width, norm=dict(eps=eps), postln_alpha=alpha, embedding=dict(scale=1.0),
+                logit_scale=1.0, token_side=dict(dim=side), layers=layers)

@@ -158,7 +158,8 @@ class StackModel(DecoderShard):
         self.layers = [Layer(cfg.layers[i], weights, i, H, cfg.norm, dtype, self.device, side)
                        for i in range(self.start_layer, self.end_layer)]
         self.mixed_from = {m.v_mix_from for m in (attention_of(L.spec.mixer) for L in self.layers) if m is not None and m.v_mix}
-        self.has_latent = any(isinstance(L.spec.mixer, LatentSpec) for L in self.layers)
+        latents = [L.spec.mixer for L in self.layers if isinstance(L.spec.mixer, LatentSpec)]
+        self.has_latent, self.expands = bool(latents), all(map(D.latent_expands, latents))
         self.two_branches = any(len(L.parts) > 1 for L in self.layers)
         # layer -> index of the pool's layer that holds its keys and values, its recurrent state
         self.kv_index: dict[int, int] = {}
@@ -401,7 +402,7 @@ class StackModel(DecoderShard):
             else:
                 for s in sizes:
                     blocks[s] += [(at + o, row, p0 + o, min(s, c - o)) for o in range(0, c, s)]
-            if self.has_latent and tiled and c >= D.LATENT_SHORT:
+            if self.has_latent and self.expands and tiled and c >= D.LATENT_SHORT:
                 lat_blocks += [(at + o, len(pages) * PAGE, p0 + o, min(D.LATENT_BLOCK, c - o)) for o in range(0, c, D.LATENT_BLOCK)]
                 pages += [(row, i) for i in range(pages_for(p0 + c))]
             elif self.has_latent:
