@@ -41,6 +41,15 @@ NOVOSUN_SIZES = {
     "4k": ("gp" * 3, 8, 256, 512, 128, 64, 128, 8, 13824),
 }
 
+# Pimisun layers beside a Gekazen of that size (its attention and experts): kinds of the layers (l latent attention,
+# a attention), latent heads / unrotated / rotated / value size / latent of queries / of keys and values, ff of the
+# one dense layer, size of a token's vector
+PIMISUN_SIZES = {
+    "1k": ("la" * 12, 16, 64, 32, 64, 384, 256, 2560, 64),
+    "2k": ("la" * 8, 16, 128, 64, 128, 1024, 512, 6912, 64),
+    "4k": ("la" * 3, 64, 128, 64, 128, 1536, 512, 13824, 128),
+}
+
 
 def parse_args():
     ap = argparse.ArgumentParser()
@@ -60,12 +69,12 @@ def parse_args():
     ap.add_argument("--pmc-copy", action="store_true",
                     help="also launch one plain 256 MiB copy kernel: the known-size dispatch that "
                          "calibrates FETCH_SIZE / WRITE_SIZE in a rocprofv3 --pmc pass")
-    ap.add_argument("--workload", default="decode", choices=["decode", "qmatmul_sweep", "gekazen", "novosun"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "qmatmul_sweep", "gekazen", "novosun", "pimisun"],
                     help="decode (default, the headline), the quantised-matmul shape sweep, or a layer-list design "
                          "beside the closest other model of equal size, whole steps and launch by launch: Gekazen "
-                         "beside a Qwen3-MoE, Novosun beside a Gekazen")
+                         "beside a Qwen3-MoE, Novosun and Pimisun beside a Gekazen")
     ap.add_argument("--gekazen-size", "--size", dest="size", default="all", choices=["all"] + list(GEKAZEN_SIZES),
-                    help="sizes of the gekazen and novosun workloads")
+                    help="sizes of the gekazen, novosun and pimisun workloads")
     return ap.parse_args()
 
 
@@ -469,20 +478,14 @@ def qwen_model(torch, size):
     return ShardModel(cfg, synth_weights(cfg, seed=0, device="cuda:0"))
 
 
-def gekazen_launches(torch, m, B, ctx):
-    """Per-launch times of a step of B rows (B <= 16: single tokens at context ctx; else one prompt)."""
-    from exo_amd import dense_ops as D
-    from exo_amd import ops
-
-    c, prompt = m.cfg, B > 16
-    H, Ls = c.hidden_size, m.layers
-    cache = m.make_cache(1 if prompt else B, ctx + B + 64)
+def launch_setup(torch, m, B, ctx):
+    """Cache, buffers and batch of a step of B rows (B <= 16: single tokens at context ctx; else one prompt)."""
+    cache = m.make_cache(1 if B > 16 else B, ctx + B + 64)
     g = torch.Generator().manual_seed(7)
-    toks = lambda n: torch.randint(0, c.vocab_size, (n,), generator=g).tolist()  # noqa: E731
-    if prompt:
+    toks = lambda n: torch.randint(0, m.cfg.vocab_size, (n,), generator=g).tolist()  # noqa: E731
+    if B > 16:
         cache.reserve([0], B)
-        batch = m._batch(cache, [(0, B)], [])
-        bf = m._buffers(1, B)
+        batch, bf = m._batch(cache, [(0, B)], []), m._buffers(1, B)
         bf.tokens[:B].copy_(torch.tensor(toks(B), dtype=torch.int32))
     else:
         for r in range(B):
@@ -492,6 +495,67 @@ def gekazen_launches(torch, m, B, ctx):
         m.decode_step(cache, B, use_graph=False)
         from exo_amd.stack_model import _Batch
         batch = _Batch(B, torch.arange(B, dtype=torch.int32, device="cuda"), cache.pos[:B] - 1, m._keys_hint(cache, slice(0, B)))
+    return cache, bf, batch
+
+
+def expert_launches(torch, m, bf, B, Ls, picks, norm, add, rows, pre, product):
+    """The launches of a mixture of experts over the layers Ls, with the experts ``picks`` that each chose."""
+    from exo_amd import dense_ops as D
+    from exo_amd import ops
+
+    c, prompt, H = m.cfg, B > 16, m.cfg.hidden_size
+    f = Ls[0].spec.mlp
+    e, r = f.expert, f.router
+    real = [int((p < r.experts).sum()) for p in picks]
+    uniq = [len(set(p[p < r.experts].tolist())) for p in picks]
+    pairs, experts = sum(real) / len(real), sum(uniq) / len(uniq)
+    lg, idx, wt = bf.router_logits(Ls[0].ff.router.shape[0]), bf.idx(r.top), bf.wt(r.top)
+    n = Ls[0].ff.router.shape[0]
+    add(pre + "router", lambda L: product(L, L.ff.router, lg, L.ff.router_b, xb=bf.xb), 2 * n * H + 2 * B * (n + H), 2 * B * n * H)
+    if prompt:
+        add("routing", lambda L: D.moe_route(lg, L.ff.correction, r.scale, idx, wt, B, r.renorm), B * r.outputs * 4, 0)
+    per = 2 * e.ff * H
+    sh = f.shared.ff * H * 2
+    if not prompt:
+        for L in Ls:
+            if (L.index, bf.cur) not in bf.experts:
+                bf.experts[L.index, bf.cur] = D.ExpertRows(f, L.ff, bf, H, bf.h)
+        ex = [bf.experts[L.index, bf.cur] for L in Ls]
+        # every layer streams the experts it chose in the forward above
+        logits = [torch.full((B, lg.shape[1]), -30.0, device="cuda").scatter_(1, p.long().to("cuda"), 3.0) for p in picks]
+        set_logits = [(lambda t=t: lg[:B].copy_(t)) for t in logits]
+        chosen = [p.to("cuda") for p in picks]
+        set_idx = [(lambda t=t: idx[:B].copy_(t)) for t in chosen]
+        both = lambda a, b: (lambda: (a(), b()))  # noqa: E731
+        for name, pre_fns, fns, mats in (
+                ("routing, experts: gate, up (+ shared)", set_logits, [(lambda x=x: x.glu(B)) for x in ex], 2),
+                ("experts: down, weighted sum (+ shared)", set_idx, [(lambda x=x: x.down(B)) for x in ex], 1)):
+            us = time_launches(torch, [both(a, b) for a, b in zip(pre_fns, fns)]) - time_launches(torch, pre_fns)
+            rows.append(row_of(name, us, mats * (experts * per + sh), mats * 2 * (pairs * e.ff * H + B * f.shared.ff * H)))
+    else:
+        act, eo = bf.act(r.top, e.ff), bf.expert_out(r.top)
+        bf.idx(r.top)[:B].copy_(picks[0].to("cuda"))
+        ws = ops.moe_group(idx[:B], r.experts, check_indices=False)
+        add("group", lambda L: ops.moe_group(idx[:B], r.experts, check_indices=False), B * r.top * 8, 0)
+        add("experts: gate, up", lambda L: D.grouped_gemm(bf.xb, L.ff.gate, ws, act, B, r.top, up=L.ff.up, spec=e),
+            2 * experts * per + 2 * B * H + 2 * pairs * e.ff, 4 * pairs * e.ff * H)
+        add("experts: down", lambda L: D.grouped_gemm(act, L.ff.down, ws, eo, B, r.top, x_per_pair=True),
+            experts * per + 2 * pairs * (H + e.ff), 2 * pairs * e.ff * H)
+        sa, so = bf.shared_act(f.shared.ff), bf.shared_out()
+        add("shared: gate, up", lambda L: D.glu_gemm(bf.xb, L.ff.s_gate, L.ff.s_up, sa, B, f.shared),
+            2 * sh + 2 * B * (H + f.shared.ff), 4 * B * f.shared.ff * H)
+        add("shared: down", lambda L: D.linear(sa, L.ff.s_down, so, B), sh + 2 * B * (H + f.shared.ff), 2 * B * f.shared.ff * H)
+        add("expert sum, norm + residual", lambda L: D.moe_sum_post_norm(eo, idx, wt, so, lg, r.experts, L.ff.gate_col, L.norm2,
+                                                                     c.eps, bf.h, bf.xb, B, norm=norm), 2 * (pairs + B) * H + 10 * B * H, 0)
+
+
+def gekazen_launches(torch, m, B, ctx):
+    """Per-launch times of a step of B rows (B <= 16: single tokens at context ctx; else one prompt)."""
+    from exo_amd import dense_ops as D
+
+    c, prompt = m.cfg, B > 16
+    H, Ls = c.hidden_size, m.layers
+    cache, bf, batch = launch_setup(torch, m, B, ctx)
     picks = []
 
     def hook(i, h):
@@ -500,12 +564,8 @@ def gekazen_launches(torch, m, B, ctx):
     m.layer_hook = hook
     m._forward(cache, bf, batch, False)
     m.layer_hook = None
-    a, f = c.layers[0].mixer, c.layers[0].mlp
-    e, r = f.expert, f.router
+    a = c.layers[0].mixer
     att = [bound[0] for bound in m._mixers(cache)]
-    real = [int((p < r.experts).sum()) for p in picks]
-    uniq = [len(set(p[p < r.experts].tolist())) for p in picks]
-    pairs, experts = sum(real) / len(real), sum(uniq) / len(uniq)
     qkv, out = bf.cols("proj", -(-Ls[0].n_main // 8) * 8), bf.mixed("attn", a.heads * a.vdim)
     vis = [min(i + 1, (a.window or 1 << 30) + a.keep_first) for i in (range(B) if prompt else [ctx] * B)]
     kvb = 2 * a.kv_heads * (a.dim + a.vdim) * (B if prompt else sum(vis))
@@ -539,43 +599,7 @@ def gekazen_launches(torch, m, B, ctx):
     if not fused:
         add("norm + residual (twice a layer)" if not prompt else "norm + residual",
             lambda L: D.post_norm_add(D.Branches(bf.branch, L.norm1), c.eps, bf.h, bf.xb, B), B * H * 14, 0)
-    lg, idx, wt = bf.router_logits(Ls[0].ff.router.shape[0]), bf.idx(r.top), bf.wt(r.top)
-    add(pre + "router", lambda L: product(L, L.ff.router, lg, xb=bf.xb), *mm(Ls[0].ff.router.shape[0], H))
-    if prompt:
-        add("routing", lambda L: D.moe_route(lg, L.ff.correction, r.scale, idx, wt, B), B * r.outputs * 4, 0)
-    per = 2 * e.ff * H
-    sh = f.shared.ff * H * 2
-    if not prompt:
-        for L in Ls:
-            if (L.index, bf.cur) not in bf.experts:
-                bf.experts[L.index, bf.cur] = D.ExpertRows(f, L.ff, bf, H, bf.h)
-        ex = [bf.experts[L.index, bf.cur] for L in Ls]
-        # every layer streams the experts it chose in the forward above
-        logits = [torch.full((B, lg.shape[1]), -30.0, device="cuda").scatter_(1, p.long().to("cuda"), 3.0) for p in picks]
-        set_logits = [(lambda t=t: lg[:B].copy_(t)) for t in logits]
-        chosen = [p.to("cuda") for p in picks]
-        set_idx = [(lambda t=t: idx[:B].copy_(t)) for t in chosen]
-        both = lambda a, b: (lambda: (a(), b()))  # noqa: E731
-        for name, pre_fns, fns, mats in (
-                ("routing, experts: gate, up (+ shared)", set_logits, [(lambda x=x: x.glu(B)) for x in ex], 2),
-                ("experts: down, weighted sum (+ shared)", set_idx, [(lambda x=x: x.down(B)) for x in ex], 1)):
-            us = time_launches(torch, [both(a, b) for a, b in zip(pre_fns, fns)]) - time_launches(torch, pre_fns)
-            rows.append(row_of(name, us, mats * (experts * per + sh), mats * 2 * (pairs * e.ff * H + B * f.shared.ff * H)))
-    else:
-        act, eo = bf.act(r.top, e.ff), bf.expert_out(r.top)
-        bf.idx(r.top)[:B].copy_(picks[0].to("cuda"))
-        ws = ops.moe_group(idx[:B], r.experts, check_indices=False)
-        add("group", lambda L: ops.moe_group(idx[:B], r.experts, check_indices=False), B * r.top * 8, 0)
-        add("experts: gate, up", lambda L: D.grouped_gemm(bf.xb, L.ff.gate, ws, act, B, r.top, up=L.ff.up, spec=e),
-            2 * experts * per + 2 * B * H + 2 * pairs * e.ff, 4 * pairs * e.ff * H)
-        add("experts: down", lambda L: D.grouped_gemm(act, L.ff.down, ws, eo, B, r.top, x_per_pair=True),
-            experts * per + 2 * pairs * (H + e.ff), 2 * pairs * e.ff * H)
-        sa, so = bf.shared_act(f.shared.ff), bf.shared_out()
-        add("shared: gate, up", lambda L: D.glu_gemm(bf.xb, L.ff.s_gate, L.ff.s_up, sa, B, f.shared),
-            2 * sh + 2 * B * (H + f.shared.ff), 4 * B * f.shared.ff * H)
-        add("shared: down", lambda L: D.linear(sa, L.ff.s_down, so, B), sh + 2 * B * (H + f.shared.ff), 2 * B * f.shared.ff * H)
-        add("expert sum, norm + residual", lambda L: D.moe_sum_post_norm(eo, idx, wt, so, lg, r.experts, r.outputs, L.norm2,
-                                                                     c.eps, bf.h, bf.xb, B), 2 * (pairs + B) * H + 10 * B * H, 0)
+    expert_launches(torch, m, bf, B, Ls, picks, c.norm, add, rows, pre, product)
     return rows
 
 
@@ -699,24 +723,10 @@ def novosun_launches(torch, m, B, ctx):
     """Per-launch times of a step of B rows (B <= 16: single tokens at context ctx; else one prompt)."""
     from exo_amd import dense_ops as D
     from exo_amd.stack_layers import LinearAttentionPart
-    from exo_amd.stack_model import _Batch
 
     c, prompt = m.cfg, B > 16
     H, eps = c.hidden_size, c.eps
-    cache = m.make_cache(1 if prompt else B, ctx + B + 64)
-    g = torch.Generator().manual_seed(7)
-    toks = lambda n: torch.randint(0, c.vocab_size, (n,), generator=g).tolist()  # noqa: E731
-    if prompt:
-        cache.reserve([0], B)
-        batch, bf = m._batch(cache, [(0, B)], []), m._buffers(1, B)
-        bf.tokens[:B].copy_(torch.tensor(toks(B), dtype=torch.int32))
-    else:
-        for r in range(B):
-            m.step(cache, [(r, toks(ctx), [])])
-        bf = m._buffers(B, 1)
-        bf.tokens.copy_(torch.tensor(toks(B), dtype=torch.int32))
-        m.decode_step(cache, B, use_graph=False)
-        batch = _Batch(B, torch.arange(B, dtype=torch.int32, device="cuda"), cache.pos[:B] - 1, m._keys_hint(cache, slice(0, B)))
+    cache, bf, batch = launch_setup(torch, m, B, ctx)
     m._forward(cache, bf, batch, False)
     lin = [(L, o) for L, o in zip(m.layers, m._mixers(cache)) if isinstance(L.parts[0], LinearAttentionPart)]
     par = [(L, o) for L, o in zip(m.layers, m._mixers(cache)) if len(L.parts) > 1]
@@ -793,6 +803,134 @@ def novosun_launches(torch, m, B, ctx):
     return rows
 
 
+def pimisun_model(torch, size, pimi):
+    from exo_amd.stack_config import StackConfig, pimisun_dict
+    from exo_amd.stack_model import StackModel
+
+    H, _, hq, hkv, hd, E, ident, top, eff, V, _ = size
+    kinds, lh, ld, lr, lv, qr, kr, ff, side = pimi
+    E -= ident
+    cfg = StackConfig.from_dict(pimisun_dict(H, V, kinds, heads=hq, kv_heads=hkv, dim=hd, rot=hd // 2, window=4096, lat_heads=lh,
+                                             lat_dim=ld, lat_rot=lr, lat_vdim=lv, q_rank=qr, kv_rank=kr, ff=ff, experts=E, top=top,
+                                             expert_ff=eff, shared_ff=eff, side=side))
+    vectors = {"norm1": H, "norm2": H, "final.norm": H, "side.norm": H, "q.norm": hq * hd, "k.norm": hkv * hd, "dq.norm": qr,
+               "dkv.norm": kr, "router.b": E}
+    mats = {"side.embed": (V, len(kinds) * side), "side.gate": (side, H), "side.proj": (H, side), "embed": (V, H), "mix.q": (hq * hd, H),
+            "mix.k": (hkv * hd, H), "mix.v": (hkv * hd, H), "mix.dq": (qr, H), "mix.uq": (lh * (ld + lr), qr), "mix.dkv": (kr + lr, H),
+            "mix.uk": (lh * ld, kr), "mix.uv": (lh * lv, kr), "mlp.router": (E, H), "mlp.up": (ff, H), "mlp.down": (H, ff)}
+
+    def shape_of(key):
+        for name, n in vectors.items():
+            if key == name or key.endswith("." + name):
+                return (n,), 0.0 if name == "router.b" else 1.0, 0.1
+        if key.endswith("vmix"):
+            return (), 0.4, 0.1
+        if key.endswith("mix.o"):
+            i = int(key[1 : key.index(".")])
+            return (H, lh * lv if kinds[i] == "l" else hq * hd), 0.0, 0.02
+        for name, shape in mats.items():
+            if key == name or key.endswith("." + name):
+                return shape, 0.0, 0.02
+        return (H, eff) if key.endswith("down") else (eff, H), 0.0, 0.02  # an expert's
+
+    return StackModel(cfg, RandomTensors(torch, shape_of))
+
+
+def pimisun_launches(torch, m, B, ctx):
+    """Per-launch times of a step of B rows (B <= 16: single tokens at context ctx; else one prompt)."""
+    from exo_amd import dense_ops as D
+    from exo_amd.stack_config import LatentSpec, MoeSpec
+
+    c, prompt = m.cfg, B > 16
+    H, eps = c.hidden_size, c.eps
+    cache, bf, batch = launch_setup(torch, m, B, ctx)
+    picks = []
+
+    def hook(i, h):
+        if isinstance(c.layers[i].mlp, MoeSpec):
+            picks.append(bf.idx(c.layers[i].mlp.router.top)[:B].cpu())
+    m.layer_hook = hook
+    m._forward(cache, bf, batch, False)
+    m.layer_hook = None
+    op = [bound[0] for bound in m._mixers(cache)]
+    every = m.layers
+    lat, att = ([L for L in every if isinstance(L.spec.mixer, LatentSpec) == t] for t in (True, False))
+    moe, dense = ([L for L in every if isinstance(L.spec.mlp, MoeSpec) == t] for t in (True, False))
+    rows, fused = [], not prompt and D.post_linear_fits(B, every[0].proj, bf.xb, H)
+    other = torch.empty_like(bf.h)
+
+    def add(name, fn, nbytes, flops, which=moe):
+        fns = [(lambda L=L: fn(L)) for L in which]
+        rows.append(row_of(name, time_launches(torch, fns * -(-12 // len(fns))), nbytes, flops))
+
+    def mm(n, k, rows=B):
+        return 2 * n * k + 2 * rows * (n + k), 2 * rows * n * k
+
+    def product(L, w, out, bias=None, xb=None, after=None):
+        if fused:
+            D.post_linear(bf.h, D.Branches(bf.branch, L.norm1, norm=c.norm), eps, other, xb, w, out, B, bias, after=after)
+        else:
+            D.linear(bf.xb, w, out, B, bias=bias, after=after)
+    pre = "norm, residual, " if fused else ""
+    # attention
+    a, L0 = att[0].spec.mixer, att[0]
+    qkv, out = bf.cols("proj", -(-L0.n_main // 8) * 8), bf.mixed("attn", a.heads * a.vdim)
+    vis = [min(i + 1, a.window or 1 << 30) for i in (range(B) if prompt else [ctx] * B)]
+    kvb = 2 * a.kv_heads * (a.dim + a.vdim) * (B if prompt else sum(vis))
+    add(pre + "qkv", lambda L: product(L, L.proj, qkv), *mm(L0.n_main, H), att)
+    fl = 2 * sum(vis) * a.heads * (a.dim + a.vdim)
+    if prompt:
+        add("norm, turn queries; append keys, values", lambda L: op[L.index].append(qkv, batch.slot, batch.pos, B),
+            2 * kvb + 4 * B * a.heads * a.dim, 0, att)
+        add("attention", lambda L: op[L.index].prompt(qkv, out, *batch.blocks[op[L0.index].prompt_block(a)]),
+            kvb + 4 * B * a.heads * a.dim, fl, att)
+    else:
+        add("norm, append, attention", lambda L: op[L.index].rows(qkv, out, batch.slot, batch.pos, B, batch.keys, append=True), kvb, fl, att)
+    add("o", lambda L: D.linear(out, L.parts[0].o, bf.branch, B), *mm(H, a.heads * a.vdim), att)
+    # latent attention
+    s, L0 = lat[0].spec.mixer, lat[0]
+    p, n = L0.parts[0], s.heads
+    down = bf.f32("proj_tail", -(-L0.n_tail // 8) * 8)
+    q, lo = bf.mixed("lat_q", p.q_cols), bf.mixed("attn", p.width)
+    ql, ol, lc = *(bf.mixed(x, n * D.pad64(s.kv_rank)) for x in ("lat_ql", "lat_ol")), bf.mixed("lat_c", s.q_rank)
+    keys = [i + 1 for i in range(B)] if prompt else [ctx] * B
+    store = 2 * (s.kv_rank + s.rot_dim) * (B if prompt else sum(keys))
+    add(pre + "latent: down projections", lambda L: product(L, L.proj, down), *mm(L0.n_tail, H), lat)
+    kv = down[:, s.q_rank :]
+    add("latent: norm, queries", lambda L: D.norm_linear(down, L.parts[0].q_gain, eps, lc, L.parts[0].uq, q, B),
+        *mm(n * (s.dim + s.rot_dim), s.q_rank), lat)
+    if prompt:
+        add("latent: norm, turn, append", lambda L: op[L.index].prepare(q, kv, batch.slot, batch.pos, B),
+            B * (6 * (s.kv_rank + s.rot_dim) + 4 * n * s.rot_dim), 0, lat)
+        parts = {L.index: dict(op[L.index].prompt_launches(q, kv, lo, batch.slot, batch.pos, *batch.latent.lists)) for L in lat}
+        dk = s.dim + s.rot_dim
+        for name, nb, g in (("gather", 2 * store, 0), ("keys", *mm(n * s.dim, s.kv_rank)), ("values", *mm(n * s.vdim, s.kv_rank)),
+                            ("attention", 2 * B * n * 2 * (dk + s.vdim), 2 * sum(keys) * n * (dk + s.vdim))):
+            add(f"latent: {name}", lambda L: parts[L.index][name](), nb, g, lat)
+    else:
+        add("latent: keys into queries, attention, values", lambda L: op[L.index].rows(q, kv, ql, ol, lo, batch.slot, batch.pos, B, batch.keys,
+                                                                                      append=True),
+            store + 2 * n * s.kv_rank * (s.dim + s.vdim), 2 * sum(keys) * n * (2 * s.kv_rank + s.rot_dim), lat)
+        add("latent: - keys into queries", lambda L: D.head_linear(q, p.nope_pad, L.parts[0].uk, ql, D.pad64(s.kv_rank), B, s.dim),
+            *mm(n * s.kv_rank, s.dim), lat)
+        add("latent: - values (no merge)", lambda L: D.head_linear(ol, D.pad64(s.kv_rank), L.parts[0].uv, lo, s.vdim, B, s.kv_rank),
+            *mm(n * s.vdim, s.kv_rank), lat)
+    add("latent: o", lambda L: D.linear(lo, L.parts[0].o, bf.branch, B), *mm(H, p.width), lat)
+    # feed-forwards, the tokens' vectors
+    if not fused:
+        add("norm of the sum", lambda L: D.post_norm_add(D.Branches(bf.branch, L.norm1, norm=c.norm), eps, bf.h, bf.xb, B), B * H * 14, 0, every)
+    f = dense[0].spec.mlp
+    act = bf.mixed("ff", f.ff)
+    add(pre + "dense: up, square of relu", lambda L: product(L, L.ff.up, act, after=L.ff.after), *mm(f.ff, H), dense)
+    add("dense: down", lambda L: D.linear(act, L.ff.down, bf.branch, B), *mm(H, f.ff), dense)
+    expert_launches(torch, m, bf, B, moe, picks, c.norm, add, rows, pre, product)
+    sa = bf.mixed("side", c.side_dim)
+    add(pre + "token vector: gate", lambda L: product(L, L.side.gate, sa, after=D.After("gelu_tanh", L.side.table, bf.tokens)),
+        *mm(c.side_dim, H), every)
+    add("token vector: projection", lambda L: D.linear(sa, L.side.proj, bf.branch, B), *mm(H, c.side_dim), every)
+    return rows
+
+
 def step_rates(torch, m, args, tag) -> dict:
     """Whole steps: prompt and decode throughput at batch 1, 4, 8 and 16."""
     from exo_amd.generate import prefill
@@ -837,8 +975,9 @@ def stack_workload(args):
     torch.cuda.set_device(0)
     kinds = {"gekazen": (lambda size, name: gekazen_model(torch, size, 4096), gekazen_launches),
              "novosun": (lambda size, name: novosun_model(torch, size, NOVOSUN_SIZES[name]), novosun_launches),
+             "pimisun": (lambda size, name: pimisun_model(torch, size, PIMISUN_SIZES[name]), pimisun_launches),
              "qwen3_moe": (lambda size, name: qwen_model(torch, size), qwen_launches)}
-    pair = ("gekazen", "qwen3_moe") if args.workload == "gekazen" else ("novosun", "gekazen")
+    pair = (args.workload, "qwen3_moe" if args.workload == "gekazen" else "gekazen")
     report = {}
     for name in (GEKAZEN_SIZES if args.size == "all" else [args.size]):
         size, res = GEKAZEN_SIZES[name], {}
@@ -854,7 +993,8 @@ def stack_workload(args):
             torch.cuda.empty_cache()
         report[name] = res
     first = next(iter(report.values()))[pair[0]]
-    sizes = {k: GEKAZEN_SIZES[k] if args.workload == "gekazen" else GEKAZEN_SIZES[k] + NOVOSUN_SIZES[k] for k in report}
+    own = {"gekazen": {}, "novosun": NOVOSUN_SIZES, "pimisun": PIMISUN_SIZES}[args.workload]
+    sizes = {k: GEKAZEN_SIZES[k] + own.get(k, ()) for k in report}
     print(json.dumps({
         "metric": f"decode tok/s, {pair[0].capitalize()} design, batch 1", "value": first["decode_tok_s_b1"], "unit": "tok/s",
         "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "ms_per_step": first["us_per_step_b1"] * 1e-3,
@@ -873,7 +1013,7 @@ def main():
         sys.exit(2)
     if args.workload == "qmatmul_sweep":
         return qmatmul_sweep(args)
-    if args.workload in ("gekazen", "novosun"):
+    if args.workload in ("gekazen", "novosun", "pimisun"):
         return stack_workload(args)
     import torch
 

@@ -388,20 +388,27 @@ class LatentAttention:
     def prompt(self, q, kv, out, slot, pos, blocks, n_blocks: int, pages, n_pages: int) -> None:
         """Portions of prompts over expanded keys and values: ``pages`` int32 [n, 2] (cache row, page of its
         sequence), ``blocks`` int32 [n, 4] (first row, first gathered key row, first position, tokens)."""
+        for _, launch in self.prompt_launches(q, kv, out, slot, pos, blocks, n_blocks, pages, n_pages):
+            launch()
+
+    def prompt_launches(self, q, kv, out, slot, pos, blocks, n_blocks: int, pages, n_pages: int) -> list[tuple]:
+        """The launches of ``prompt``, by name."""
         s, w, lib, dev = self.spec, self.w, native.load(), q.device
         n, H, r8 = 64 * n_pages, s.heads, -(-s.rot_dim // 8) * 8
         new = lambda kind, *shape: latent_workspace(kind, shape[0] * shape[1], torch.bfloat16, dev).view(*shape)  # noqa: E731
         c, kr = new("latents", n, pad64(s.kv_rank)), new("rotated", n, r8)
         k, v = new("keys", n, H * w.d8), new("values", H * s.vdim, n)
         a = self._bind(q, kv, slot, pos, 1)
-        check(lib.exo_latent_gather(C.byref(a), pages.data_ptr(), n_pages, c.data_ptr(), kr.data_ptr(), _stream()), "latent_gather")
-        linear(c, w.uk_rows, k, n, force_gemm=True)
-        linear(w.uv_rows, c, v, H * s.vdim, force_gemm=True)
         p = native.LatentPrompt(
             q=q.data_ptr(), k=k.data_ptr(), k_rot=kr.data_ptr(), v=v.data_ptr(), list=blocks.data_ptr(), out=out.data_ptr(),
             scale=s.scale, n=n_blocks, heads=H, vdim=s.vdim, d8=w.d8, r8=r8, ldq=q.stride(0), q_head=w.nope_pad,
             rot_col=w.rot_col, ldk=k.stride(0), ldv=v.stride(0), ldo=out.stride(0))
-        check(lib.exo_latent_prompt(C.byref(p), _stream()), "latent_prompt")
+        return [
+            ("gather", lambda: check(lib.exo_latent_gather(C.byref(a), pages.data_ptr(), n_pages, c.data_ptr(), kr.data_ptr(),
+                                                           _stream()), "latent_gather")),
+            ("keys", lambda: linear(c, w.uk_rows, k, n, force_gemm=True)),
+            ("values", lambda: linear(w.uv_rows, c, v, H * s.vdim, force_gemm=True)),
+            ("attention", lambda: check(lib.exo_latent_prompt(C.byref(p), _stream()), "latent_prompt"))]
 
 
 def head_linear(x, x_head: int, w, y, y_head: int, n: int, K: int, lst=None, parts=None, nsplit: int = 1) -> None:
