@@ -75,6 +75,15 @@ __device__ __forceinline__ float clamped_glu(float g, float u, const GluConst& c
   return g / (1.f + expf(-c.alpha * g)) * (u + c.shift);
 }
 
+// ... for a result in the element type: bf16 takes the units' exponential and reciprocal
+template <typename T>
+__device__ __forceinline__ float gated(float g, float u, const GluConst& c) {
+  if (sizeof(T) == 4) return clamped_glu(g, u, c);
+  g = fminf(g, c.limit);
+  u = fminf(fmaxf(u, -c.limit), c.limit);
+  return g * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * c.alpha * g)) * (u + c.shift);
+}
+
 // What happens to a product's result ahead of its store: an activation, then a factor out of a table
 // (element type) whose row is given by an index list (null: the result's own row).
 struct Epilogue {
@@ -83,14 +92,18 @@ struct Epilogue {
   const int32_t* mul_rows;
   int ldmul;
 };
-template <typename T>
-__device__ __forceinline__ float finish(float v, size_t m, int n, const Epilogue& e) {
-  if (e.act == 1) {
+__device__ __forceinline__ float activated(float v, int act) {
+  if (act == 1) {
     v = fmaxf(v, 0.f);
     v *= v;
-  } else if (e.act == 2) {
+  } else if (act == 2) {
     v = 0.5f * v * (1.f + tanhf(0.79788456080286536f * (v + 0.044715f * v * v * v)));
   }
+  return v;
+}
+template <typename T>
+__device__ __forceinline__ float finish(float v, size_t m, int n, const Epilogue& e) {
+  v = activated(v, e.act);
   if (e.mul) v *= Elem<T>::load(reinterpret_cast<const T*>(e.mul)[(e.mul_rows ? (size_t)e.mul_rows[m] : m) * e.ldmul + n]);
   return v;
 }

@@ -432,36 +432,106 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const GemmParams p) 
   }
 
   // ---- epilogue: element e of tile (i, j): row wm + 32 i + 8 (e / 4) + 4 half + e % 4, column lane
+  // One plain output, or a partial one: every store at 32-bit offsets from the tile's first row, rows past
+  // the end dropped by the buffer's range, columns past N by an offset beyond it.  (The whole offset is in
+  // the vector register: the scalar one takes no part in the range check.)
+  if (!GROUPED && !PAIR && (p.ksplit > 1 || (p.n1 == p.N && !p.ep.mul))) {
+    const bool part = p.ksplit > 1, f32 = part || p.y_f32 || sizeof(T) == 4;
+    const uint32_t ld = part ? (uint32_t)p.N : (uint32_t)p.ldy, size = f32 ? 4 : 2;
+    char* base = part ? reinterpret_cast<char*>(p.part + ((size_t)blockIdx.z * p.M + m0) * p.N)
+                      : reinterpret_cast<char*>(p.y) + (size_t)m0 * ld * size;
+    const __amdgpu_buffer_rsrc_t ry = buf_of(base, (uint32_t)min(m_end - m0, BM) * ld * size);
+    uint32_t voff[NJ];
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+      const int n = n0 + wn + 32 * j + frow;
+      voff[j] = n < p.N ? ((uint32_t)(wm + 4 * half) * ld + n) * size : kPastEnd;
+      if (!part && p.bias) {
+        const float b = n < p.N ? p.bias[n] : 0.f;
+#pragma unroll
+        for (int i = 0; i < MI; ++i)
+#pragma unroll
+          for (int e = 0; e < 16; ++e) acc[i][j][e] += b;
+      }
+    }
+    if (!part && p.ep.act) {
+#pragma unroll
+      for (int i = 0; i < MI; ++i)
+#pragma unroll
+        for (int j = 0; j < NJ; ++j)
+#pragma unroll
+          for (int e = 0; e < 16; ++e) acc[i][j][e] = activated(acc[i][j][e], p.ep.act);
+    }
+    auto store = [&](auto put) __attribute__((always_inline)) {
+#pragma unroll
+      for (int i = 0; i < MI; ++i)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) {
+          const uint32_t roff = (uint32_t)(32 * i + 8 * (e >> 2) + (e & 3)) * ld * size;
+#pragma unroll
+          for (int j = 0; j < NJ; ++j) put(acc[i][j][e], voff[j] + roff);
+        }
+    };
+    if (f32)
+      store([&](float v, uint32_t at) { __builtin_amdgcn_raw_buffer_store_b32(__builtin_bit_cast(uint32_t, v), ry, at, 0, 0); });
+    else
+      store([&](float v, uint32_t at) { __builtin_amdgcn_raw_buffer_store_b16(f2bf(v), ry, at, 0, 0); });
+    return;
+  }
+  // Gated pairs and an expert's rows, in the element type: the same with a row's offset from the list of
+  // pairs (four consecutive tile rows at a time).
+  if (GROUPED || PAIR) {
+    const uint32_t ld = (uint32_t)p.ldy * sizeof(T);
+    char* base = reinterpret_cast<char*>(p.y) + (GROUPED ? 0 : (size_t)m0 * ld);
+    const __amdgpu_buffer_rsrc_t ry = buf_of(base, GROUPED ? kPastEnd : (uint32_t)min(m_end - m0, BM) * ld);
+    constexpr int JS = PAIR ? 2 : 1;  // accumulators per output
+    uint32_t coff[NJ / JS];
+#pragma unroll
+    for (int j = 0; j < NJ / JS; ++j) {
+      const int n = PAIR ? n0 + (wave & 1) * (16 * NJ) + j * 32 + frow : n0 + wn + 32 * j + frow;
+      coff[j] = n < p.N ? (uint32_t)n * sizeof(T) : kPastEnd;
+    }
+#pragma unroll
+    for (int i = 0; i < MI; ++i)
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const int t0 = wm + 32 * i + 8 * k + 4 * half;
+        int rows[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) rows[e] = GROUPED ? row_pair[t0 + e] : t0 + e;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const bool in = GROUPED ? t0 + e < m_end : true;  // (not grouped: by the range)
+#pragma unroll
+          for (int j = 0; j < NJ / JS; ++j) {
+            float v = acc[i][JS * j][4 * k + e];
+            if (PAIR) v = gated<T>(v, acc[i][JS * j + JS - 1][4 * k + e], p.glu);
+            const uint32_t off = in && coff[j] != kPastEnd ? (uint32_t)rows[e] * ld + coff[j] : kPastEnd;
+            if (sizeof(T) == 4)
+              __builtin_amdgcn_raw_buffer_store_b32(__builtin_bit_cast(uint32_t, v), ry, off, 0, 0);
+            else
+              __builtin_amdgcn_raw_buffer_store_b16(f2bf(v), ry, off, 0, 0);
+          }
+        }
+      }
+    return;
+  }
 #pragma unroll
   for (int i = 0; i < MI; ++i)
 #pragma unroll
     for (int e = 0; e < 16; ++e) {
       const int tr = wm + 32 * i + 8 * (e >> 2) + 4 * half + (e & 3);
       if (m0 + tr >= m_end) continue;
-      const size_t row = GROUPED ? (size_t)row_pair[tr] : (size_t)(m0 + tr);
-      if (PAIR) {
+      const size_t row = (size_t)(m0 + tr);
 #pragma unroll
-        for (int j = 0; j < NJ; j += 2) {
-          const int n = n0 + (wave & 1) * (16 * NJ) + (j >> 1) * 32 + frow;
-          if (n < p.N)
-            reinterpret_cast<T*>(p.y)[row * p.ldy + n] =
-                Elem<T>::make(clamped_glu(acc[i][j][e], acc[i][j + 1 < NJ ? j + 1 : j][e], p.glu));
-        }
-      } else {
-#pragma unroll
-        for (int j = 0; j < NJ; ++j) {
-          const int n = n0 + wn + 32 * j + frow;
-          if (n >= p.N) continue;
-          if (p.ksplit > 1) {
-            p.part[((size_t)blockIdx.z * p.M + row) * p.N + n] = acc[i][j][e];
-          } else {
-            const float v = acc[i][j][e] + (p.bias ? p.bias[n] : 0.f);
-            if (GROUPED || n < p.n1)
-              store_out<T>(p.y, row * p.ldy + n, finish<T>(v, row, n, p.ep), p.y_f32);
-            else
-              p.y2[row * p.ldy2 + n - p.n1] = v;
-          }
-        }
+      for (int j = 0; j < NJ; ++j) {
+        const int n = n0 + wn + 32 * j + frow;
+        if (n >= p.N) continue;
+        const float v = acc[i][j][e] + (p.bias ? p.bias[n] : 0.f);
+        if (n < p.n1)
+          store_out<T>(p.y, row * p.ldy + n, finish<T>(v, row, n, p.ep), p.y_f32);
+        else
+          p.y2[row * p.ldy2 + n - p.n1] = v;
       }
     }
 }
@@ -609,7 +679,7 @@ static int linear_check(const exo_linear* a, const char* what) {
               "%s: need M, N > 0 and equal row strides that are multiples of 64 (got M=%d N=%d %d/%d)", what, a->M, a->N,
               a->ldx, a->ldw);
   EXO_REQUIRE((((uintptr_t)a->x | (uintptr_t)a->w | (uintptr_t)a->w_up) & 15) == 0, "%s: operands must be 16-byte aligned", what);
-  EXO_REQUIRE((int64_t)a->ldw * 256 * 4 < (1ll << 31), "%s: row stride %d too large", what, a->ldw);
+  EXO_REQUIRE((int64_t)a->ldw * 256 * 4 < (1ll << 31) && (int64_t)a->ldy * 512 < (1ll << 31), "%s: row strides %d / %d too large", what, a->ldw, a->ldy);
   EXO_REQUIRE(a->n1 > 0 && a->n1 <= a->N && a->ldy >= a->n1 && (a->n1 == a->N || (a->y2 && a->ldy2 >= a->N - a->n1)),
               "%s: outputs do not hold %d columns (%d in the first: %d, %d)", what, a->N, a->n1, a->ldy, a->ldy2);
   EXO_REQUIRE(!a->w_up || (a->n1 == a->N && !a->bias), "%s: a gated pair has one output and no bias", what);
@@ -703,6 +773,7 @@ extern "C" int exo_dense_grouped_gemm(const void* x, const void* w, const void* 
               "exo_dense_grouped_gemm: bad arguments (T=%d topk=%d E=%d)", T, topk, E);
   EXO_REQUIRE((int64_t)T * (x_per_pair ? topk : 1) * ldx * (dtype ? 4 : 2) < (1ll << 32),
               "exo_dense_grouped_gemm: activations exceed 32-bit byte offsets");
+  EXO_REQUIRE((int64_t)T * topk * ldy * (dtype ? 4 : 2) < kPastEnd, "exo_dense_grouped_gemm: outputs exceed 31-bit byte offsets");
   const int64_t pairs = (int64_t)T * topk;
   const int tiles = (int)((pairs + 127) / 128) + E;  // exo_moe_group's list length
   EXO_REQUIRE(tiles <= 65535, "exo_dense_grouped_gemm: %d row tiles exceed the grid limit", tiles);
