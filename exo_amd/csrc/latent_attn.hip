@@ -14,8 +14,8 @@
 //
 // latent_rows_kernel: one query position and up to 16 heads per workgroup.  A tile of keys (64, or 32 in
 // the 32-bit mode) is staged in LDS once and read twice: as rows for the scores, and transposed on the way
-// out of LDS for the weighted sum - each wave scores 16 keys, then sums a quarter of the latent's columns
-// over all of them.  The next tile is in registers meanwhile.  Splits leave float32 partials that the
+// out of LDS for the weighted sum - four of the eight waves score 16 keys
+// each, then each wave sums an eighth of the latent's columns over all of them.  The next tile is in registers meanwhile.  Splits leave float32 partials that the
 // following product with the value matrices merges while it stages its operand.
 #include "../../include/exo_mi355x.h"
 #include "dense.h"
@@ -25,6 +25,7 @@ namespace {
 
 constexpr int kPage = 64;
 constexpr int kWaves = 4;
+constexpr int kRowWaves = 8, kRowThreads = 64 * kRowWaves;  // of latent_rows_kernel
 constexpr int kMaxRot = 128;
 constexpr float kLog2e = 1.4426950408889634f;
 constexpr int kPRow = 144;  // bytes of a head's weights of one tile in LDS
@@ -132,14 +133,15 @@ __device__ __forceinline__ uint4 transposed<float>(const char* tile, int stride,
 }
 
 template <typename T, int KMAX, bool FUSE>
-__global__ __launch_bounds__(64 * kWaves) void latent_rows_kernel(const Params p) {
+__global__ __launch_bounds__(kRowThreads) void latent_rows_kernel(const Params p) {
   constexpr int ES = (int)sizeof(T), KT = ES == 2 ? 64 : 32;     // keys per tile
   constexpr int KS = KMAX * ES / 64;                             // 64-byte steps over a key
-  constexpr int LOADS = KT * KMAX * ES / 16 / 256;
-  constexpr int OT = (KMAX < 512 ? KMAX : 512) / 64;             // 16-column tiles of the sum per wave
+  constexpr int LOADS = (KT * KMAX * ES / 16 + kRowThreads - 1) / kRowThreads;
+  constexpr int OT = ((KMAX < 512 ? KMAX : 512) / 16 + kRowWaves - 1) / kRowWaves;  // 16-column tiles of the sum per wave
   constexpr int PK = 64 / ES;                                    // keys per product of the second kind
   extern __shared__ __attribute__((aligned(16))) char lds[];
-  __shared__ float wm[kWaves][16], wl[kWaves][16];
+  constexpr int SW = KT / 16;                                    // waves that score
+  __shared__ float wm[SW][16], wl[SW][16];
   __shared__ float2 cs[kMaxRot / 2];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r = lane & 15, g = lane >> 4;
@@ -159,16 +161,16 @@ __global__ __launch_bounds__(64 * kWaves) void latent_rows_kernel(const Params p
     const char* src = reinterpret_cast<const char*>(pool_row<T>(p, table[key0 / kPage], key0 % kPage));
 #pragma unroll
     for (int i = 0; i < LOADS; ++i)
-      reg[i] = load16(src + (size_t)min(tid + 256 * i, nvec - 1) * 16);
+      reg[i] = load16(src + (size_t)min(tid + kRowThreads * i, nvec - 1) * 16);
   };
   int j = split;
   const bool early = j < nt && !(FUSE && j == nt - 1);  // (not the tile that the row's own key goes into)
   if (early) load_tile(j);
 
   // ---- queries: absorbed part, turned part, zeros; the row's own latent
-  for (int i = tid; 2 * i < p.rot; i += 256) cs[i] = turn_of(pos, p.freq[i]);
+  for (int i = tid; 2 * i < p.rot; i += kRowThreads) cs[i] = turn_of(pos, p.freq[i]);
   const int cvec = p.c32 * ES / 16;
-  for (int i = tid; i < 16 * vpr; i += 256) {
+  for (int i = tid; i < 16 * vpr; i += kRowThreads) {
     const int h = (i * magic) >> 20, c = i - h * vpr;
     uint4 v{0, 0, 0, 0};
     if (h < gs && c < cvec)
@@ -177,7 +179,7 @@ __global__ __launch_bounds__(64 * kWaves) void latent_rows_kernel(const Params p
   }
   __syncthreads();
   const int half = p.rot / 2;
-  for (int i = tid; i < gs * half; i += 256) {
+  for (int i = tid; i < gs * half; i += kRowThreads) {
     const int h = i / half, d = i - h * half;
     const T* src = reinterpret_cast<const T*>(p.q) + (size_t)row * p.ldq + p.rot_col + (h0 + h) * p.r8 + 2 * d;
     float2 x{Elem<T>::load(src[0]), Elem<T>::load(src[1])};
@@ -187,16 +189,18 @@ __global__ __launch_bounds__(64 * kWaves) void latent_rows_kernel(const Params p
   }
   if (FUSE && split == (nt - 1) % p.nsplit) {
     T* dst = pool_row<T>(p, table[pos / kPage], pos % kPage);
-    if (wave == kWaves - 1) put_latent<T>(p, row, dst, lane);
-    if (wave == kWaves - 2) put_rotated<T>(p, row, dst, cs, lane);
+    if (wave == kRowWaves - 1) put_latent<T>(p, row, dst, lane);
+    if (wave == kRowWaves - 2) put_rotated<T>(p, row, dst, cs, lane);
     wait_own_stores_done();
   }
   __syncthreads();
   if (!early && j < nt) load_tile(j);
   uint4 q[KS];
 #pragma unroll
-  for (int s = 0; s < KS; ++s)
-    if (s < ksteps) q[s] = *reinterpret_cast<const uint4*>(lds + r * stride + s * 64 + g * 16);
+  for (int s = 0; s < KS; ++s) {  // (steps past the key: zeros times its last step again, no branch in the loops)
+    q[s] = load16(lds + r * stride + min(s, ksteps - 1) * 64 + g * 16);
+    if (s >= ksteps) q[s] = uint4{0, 0, 0, 0};
+  }
   __syncthreads();
 
   const float sc = p.scale * kLog2e;
@@ -207,19 +211,19 @@ __global__ __launch_bounds__(64 * kWaves) void latent_rows_kernel(const Params p
   for (; j < nt; j += p.nsplit) {
 #pragma unroll
     for (int i = 0; i < LOADS; ++i) {
-      const uint32_t v = tid + 256 * i;
+      const uint32_t v = tid + kRowThreads * i;
       if ((int)v < nvec) *reinterpret_cast<uint4*>(lds + v * 16 + ((v * magic) >> 20) * 16) = reg[i];
     }
     if (j + p.nsplit < nt) load_tile(j + p.nsplit);
     __syncthreads();
     float x[4], mx = -INFINITY;
-    if (wave * 16 < KT) {
+    if (wave < SW) {
       floatx4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
       const char* kr = lds + (wave * 16 + r) * stride + g * 16;
 #pragma unroll
       for (int s = 0; s < KS; s += 2) {
-        if (s < ksteps) s0 = Elem<T>::mma16(*reinterpret_cast<const uint4*>(kr + s * 64), q[s], s0);
-        if (s + 1 < KS && s + 1 < ksteps) s1 = Elem<T>::mma16(*reinterpret_cast<const uint4*>(kr + s * 64 + 64), q[s + 1 < KS ? s + 1 : s], s1);
+        s0 = Elem<T>::mma16(load16(kr + min(s, ksteps - 1) * 64), q[s], s0);
+        if (s + 1 < KS) s1 = Elem<T>::mma16(load16(kr + min(s + 1, ksteps - 1) * 64), q[s + 1 < KS ? s + 1 : s], s1);
       }
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
@@ -229,15 +233,15 @@ __global__ __launch_bounds__(64 * kWaves) void latent_rows_kernel(const Params p
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
     }
-    if (g == 0) wm[wave][r] = mx;
+    if (wave < SW && g == 0) wm[wave][r] = mx;
     __syncthreads();
     float mn = m;
 #pragma unroll
-    for (int w = 0; w < kWaves; ++w) mn = fmaxf(mn, wm[w][r]);  // finite: a dealt tile holds a visible key
+    for (int w = 0; w < SW; ++w) mn = fmaxf(mn, wm[w][r]);  // finite: a dealt tile holds a visible key
     const float a = __builtin_amdgcn_exp2f(m - mn);
     m = mn;
     float sum = 0.f;
-    if (wave * 16 < KT) {
+    if (wave < SW) {
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         x[e] = __builtin_amdgcn_exp2f(x[e] - mn);
@@ -256,11 +260,11 @@ __global__ __launch_bounds__(64 * kWaves) void latent_rows_kernel(const Params p
         *reinterpret_cast<floatx4*>(dst) = floatx4{x[0], x[1], x[2], x[3]};
       }
     }
-    if (g == 0) wl[wave][r] = sum;
+    if (wave < SW && g == 0) wl[wave][r] = sum;
     __syncthreads();
     l *= a;
 #pragma unroll
-    for (int w = 0; w < kWaves; ++w) l += wl[w][r];
+    for (int w = 0; w < SW; ++w) l += wl[w][r];
 #pragma unroll
     for (int t = 0; t < OT; ++t)
 #pragma unroll
@@ -271,12 +275,9 @@ __global__ __launch_bounds__(64 * kWaves) void latent_rows_kernel(const Params p
       const uint4 lo = ES == 2 ? *reinterpret_cast<const uint4*>(pw + (16 + r) * kPRow + k * 64 + g * 16) : hi;
 #pragma unroll
       for (int t = 0; t < OT; ++t) {
-        const int dt = wave + kWaves * t;
-        if (dt < dtiles) {
-          const uint4 v = transposed<T>(lds, stride, k * PK, dt * 16, r, g);
-          o[t] = Elem<T>::mma16(v, hi, o[t]);
-          if (ES == 2) o[t] = Elem<T>::mma16(v, lo, o[t]);
-        }
+        const uint4 v = transposed<T>(lds, stride, k * PK, min(wave + kRowWaves * t, dtiles - 1) * 16, r, g);
+        o[t] = Elem<T>::mma16(v, hi, o[t]);
+        if (ES == 2) o[t] = Elem<T>::mma16(v, lo, o[t]);
       }
     }
     __syncthreads();  // the tile and its weights are no longer read
@@ -287,7 +288,7 @@ __global__ __launch_bounds__(64 * kWaves) void latent_rows_kernel(const Params p
     T* out = reinterpret_cast<T*>(p.out) + (size_t)row * p.ldo + (size_t)(h0 + r) * p.cp;
 #pragma unroll
     for (int t = 0; t < OT; ++t) {
-      const int d = (wave + kWaves * t) * 16 + 4 * g;
+      const int d = (wave + kRowWaves * t) * 16 + 4 * g;
       if (d < p.c32) {
 #pragma unroll
         for (int e = 0; e < 4; ++e) out[d + e] = Elem<T>::make(o[t][e] * inv);
@@ -298,7 +299,7 @@ __global__ __launch_bounds__(64 * kWaves) void latent_rows_kernel(const Params p
   float* part = p.parts + (((size_t)blockIdx.z * p.H + h0 + r) * p.nsplit + split) * (p.c32 + 4);
 #pragma unroll
   for (int t = 0; t < OT; ++t) {
-    const int d = (wave + kWaves * t) * 16 + 4 * g;
+    const int d = (wave + kRowWaves * t) * 16 + 4 * g;
     if (d < p.c32) *reinterpret_cast<floatx4*>(part + d) = o[t];
   }
   if (wave == 0 && g == 0) part[p.c32] = m, part[p.c32 + 1] = l;
@@ -438,7 +439,7 @@ int launch_rows(const Params& p, hipStream_t st) {
     }
     done = true;
   }
-  fn<<<dim3(p.nsplit, (p.H + p.gsz - 1) / p.gsz, p.n), 64 * kWaves, lds, st>>>(p);
+  fn<<<dim3(p.nsplit, (p.H + p.gsz - 1) / p.gsz, p.n), kRowThreads, lds, st>>>(p);
   return EXO_OK;
 }
 template <typename T, int KMAX>
@@ -447,7 +448,8 @@ int launch_rows_f(const Params& p, bool fuse, hipStream_t st) {
 }
 template <typename T>
 int launch_rows_k(const Params& p, bool fuse, hipStream_t st) {
-  return p.ldk <= 192 ? launch_rows_f<T, 192>(p, fuse, st) : p.ldk <= 320 ? launch_rows_f<T, 320>(p, fuse, st) : launch_rows_f<T, 640>(p, fuse, st);
+  return p.ldk <= 192 ? launch_rows_f<T, 192>(p, fuse, st) : p.ldk <= 320 ? launch_rows_f<T, 320>(p, fuse, st)
+         : p.ldk <= 576 ? launch_rows_f<T, 576>(p, fuse, st) : launch_rows_f<T, 640>(p, fuse, st);
 }
 
 }  // namespace

@@ -373,7 +373,7 @@ class LatentAttention:
         s, w, lib = self.spec, self.w, native.load()
         head_linear(q, w.nope_pad, w.uk, ql, pad64(s.kv_rank), n, s.dim, lst)
         tiles, wgs = -(-keys // 64), n * (-(-s.heads // 16))
-        nsplit = max(1, min(-(-tiles // 2), 256 // wgs, 32))
+        nsplit = max(1, min(tiles, 256 // wgs, max(16, 64 // n)))  # (more partials cost the merge what they gain here)
         a = self._bind(q, kv, slot, pos, n, lst, not append)
         a.q_latent, a.ldql, a.nsplit = ql.data_ptr(), ql.stride(0), nsplit
         parts = None
