@@ -108,6 +108,28 @@ __device__ __forceinline__ void unit_row(const T* __restrict__ src, T* dst, int 
   for (int d = lane; d < D; d += 64) dst[d] = Elem<T>::make(Elem<T>::load(src[d]) * inv * (gain ? gain[d] : 1.f));
 }
 
+// this thread's share (of `threads`) of the sum of squares of src[0..n); vec: in vectors
+template <typename T>
+__device__ __forceinline__ float square_sum(const T* src, int n, bool vec, int thread, int threads) {
+  constexpr int VEC = Elem<T>::kVec;
+  float ss = 0.f;
+  if (vec) {
+    for (int c = thread * VEC; c < n; c += threads * VEC) {
+      float f[VEC];
+      unpack_vec<T>(load16(src + c), f);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss += f[e] * f[e];
+    }
+  } else {
+    for (int c = thread; c < n; c += threads) ss += Elem<T>::load(src[c]) * Elem<T>::load(src[c]);
+  }
+  return ss;
+}
+// cap * tanh(x) as 1 - 2 / (e^2x + 1): an absolute error of some 1e-7 cap, for scores of bf16 operands
+__device__ __forceinline__ float bent(float x, float cap) {
+  return cap - 2.f * cap * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(x * (2.f * kLog2e)) + 1.f);
+}
+
 // one wave: the pairs of src[0..D) times inv and gain, the first `rot` entries turned -> dst (may be src)
 template <typename T>
 __device__ __forceinline__ void turn_row(const T* src, T* dst, int D, float inv, const float* __restrict__ gain,
@@ -272,23 +294,6 @@ __device__ __forceinline__ void prepare_run(T* src, T* dst, int ldd, int heads, 
   }
 }
 template <typename T>
-__device__ __forceinline__ float row_square_sum(const T* src, int n, bool vec, int lane) {
-  constexpr int VEC = Elem<T>::kVec;
-  float ss = 0.f;
-  if (vec) {
-    for (int c = lane * VEC; c < n; c += 64 * VEC) {
-      float f[VEC];
-      unpack_vec<T>(*reinterpret_cast<const uint4*>(src + c), f);
-#pragma unroll
-      for (int e = 0; e < VEC; ++e) ss += f[e] * f[e];
-    }
-  } else {
-    for (int c = lane; c < n; c += 64) ss += Elem<T>::load(src[c]) * Elem<T>::load(src[c]);
-  }
-  return wave_sum(ss);
-}
-
-template <typename T>
 __global__ __launch_bounds__(64 * kAppendRows) void paged_prepare_kernel(const Params p) {
   __shared__ float2 cs[kAppendRows][kMaxRot / 2];
   __shared__ int s_page[kAppendRows], s_pos[kAppendRows];
@@ -303,8 +308,8 @@ __global__ __launch_bounds__(64 * kAppendRows) void paged_prepare_kernel(const P
     T* q = const_cast<T*>(reinterpret_cast<const T*>(p.qkv)) + (size_t)row * p.ldq;
     T* k = q + p.H * p.D;
     const bool vec = p.D % VEC == 0 && p.ldq % VEC == 0;
-    const float iq = p.whole ? 1.f / sqrtf(row_square_sum<T>(q, p.H * p.D, vec, lane) / (p.H * p.D) + p.eps) : 1.f;
-    const float ik = p.whole ? 1.f / sqrtf(row_square_sum<T>(k, p.G * p.D, vec, lane) / (p.G * p.D) + p.eps) : 1.f;
+    const float iq = p.whole ? 1.f / sqrtf(wave_sum(square_sum<T>(q, p.H * p.D, vec, lane, 64)) / (p.H * p.D) + p.eps) : 1.f;
+    const float ik = p.whole ? 1.f / sqrtf(wave_sum(square_sum<T>(k, p.G * p.D, vec, lane, 64)) / (p.G * p.D) + p.eps) : 1.f;
     prepare_run<T>(q, q, p.D, p.H, p.D, iq, p.qgain, cs[wave], p.rot, vec, lane);
     T* dst = reinterpret_cast<T*>(p.kpool) + ((size_t)page * p.G * kPage + pos % kPage) * p.ldk;
     prepare_run<T>(k, dst, kPage * p.ldk, p.G, p.D, ik, p.kgain, cs[wave], p.rot, vec, lane);
@@ -448,11 +453,9 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
     const T* src = reinterpret_cast<const T*>(p.qkv) + (size_t)row * p.ldq;
     for (int i = threadIdx.x; 2 * i < p.rot; i += 64 * kRowWaves) cs[i] = turn_of(pos, p.freq[i]);
     if (p.whole) {
-      float sq = 0.f, sk = 0.f;
-      for (int c = threadIdx.x; c < p.H * p.D; c += 64 * kRowWaves) sq += Elem<T>::load(src[c]) * Elem<T>::load(src[c]);
-      if (FUSE)
-        for (int c = p.H * p.D + threadIdx.x; c < (p.H + p.G) * p.D; c += 64 * kRowWaves)
-          sk += Elem<T>::load(src[c]) * Elem<T>::load(src[c]);
+      const bool vec = p.D % Elem<T>::kVec == 0 && p.ldq % Elem<T>::kVec == 0;
+      float sq = square_sum<T>(src, p.H * p.D, vec, threadIdx.x, 64 * kRowWaves);
+      float sk = FUSE ? square_sum<T>(src + p.H * p.D, p.G * p.D, vec, threadIdx.x, 64 * kRowWaves) : 0.f;
       sq = wave_sum(sq), sk = wave_sum(sk);
       if (lane == 0) ms[wave][0] = sq, ms[wave][1] = sk;
     }
@@ -506,7 +509,10 @@ __global__ __launch_bounds__(64 * kRowWaves) void paged_rows_kernel(const Params
     for (int e = 0; e < 4; ++e) s0[e] *= sc, s1[e] *= sc;
     if (p.cap > 0.f) {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) s0[e] = cap2 * tanhf(s0[e]), s1[e] = cap2 * tanhf(s1[e]);
+      for (int e = 0; e < 4; ++e) {
+        s0[e] = sizeof(T) == 2 ? bent(s0[e], cap2) : cap2 * tanhf(s0[e]);
+        s1[e] = sizeof(T) == 2 ? bent(s1[e], cap2) : cap2 * tanhf(s1[e]);
+      }
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
@@ -752,7 +758,7 @@ __global__ __launch_bounds__(256, DK > 128 ? 1 : 2) void paged_prompt_kernel(con
   // lane half kq are keys 16s + 8kq .. + 8 (the B operand order of the second product)
   const int jr = n >> 3;
   const int key_of_row = 16 * (jr >> 1) + 8 * ((n >> 2) & 1) + 4 * (jr & 1) + (n & 3);
-  const float sc = p.scale * kLog2e, cap2 = p.cap * kLog2e, icap = p.cap > 0.f ? 2.f * kLog2e * p.scale / p.cap : 0.f;
+  const float sc = p.scale * kLog2e, cap2 = p.cap * kLog2e, icap = p.cap > 0.f ? p.scale / p.cap : 0.f;
   const float slope = p.slopes ? p.slopes[hq] * kLog2e : 0.f;
 
   floatx16 o[DT];
@@ -791,12 +797,12 @@ __global__ __launch_bounds__(256, DK > 128 ? 1 : 2) void paged_prompt_kernel(con
     const int rel = qpos - key0 - 8 * kq;  // distance to the lane's first key
     const float base = -slope * (float)rel;
     float mx = -INFINITY;
-    if (p.cap > 0.f) {  // tanh(y) = 1 - 2 / (e^2y + 1)
+    if (p.cap > 0.f) {
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks)
 #pragma unroll
         for (int e = 0; e < 16; ++e)
-          s[ks][e] = cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s[ks][e] * icap) + 1.f);
+          s[ks][e] = bent(s[ks][e] * icap, cap2);
     }
     const float scl = p.cap > 0.f ? 1.f : sc;
 #pragma unroll

@@ -179,7 +179,9 @@ def post_linear(x, br: Branches, eps: float, x_out, xb, w, out, n: int, bias=Non
 def norm_linear(x, gain, eps: float, operand, w, out, n: int) -> None:
     """out[:n] = (x / rms * gain) @ w^T, x float32 rows; ``operand``: scratch for the normed rows."""
     br = Branches(x, gain)
-    if post_linear_fits(n, w, operand, gain.numel()):
+    fits = n <= GEMV_MAX_ROWS and n * gain.numel() <= 4096 and native.load().exo_post_linear_fits(
+        n, w.shape[0], gain.numel(), operand.shape[1], _code(operand))  # (no residual: any rows of a GEMV)
+    if fits:
         post_linear(None, br, eps, None, None, w, out, n)
     else:
         norm_rows(x, gain, eps, operand, n)
