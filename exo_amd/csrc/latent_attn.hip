@@ -20,6 +20,7 @@
 #include "../../include/exo_mi355x.h"
 #include "dense.h"
 #include "rotary.h"
+#include "route.h"
 
 namespace {
 
@@ -306,8 +307,10 @@ __global__ __launch_bounds__(kRowThreads) void latent_rows_kernel(const Params p
 }
 
 // ------------------------------------------------------------------------------ a matrix per head
-// y[row][h] = w[h] x[row][h]: 64 outputs of one head and up to 16 rows per workgroup, a 16x16 tile per wave.
-// With partials of split attention x is formed from them on the way into LDS.
+// y[row][h] = w[h] x[row][h]: outputs of one head and up to 16 rows per workgroup, 16x16 tiles; short rows a
+// wave per tile (KW 1), long ones over four waves (KW 4: two tiles, eight waves).  With partials of split
+// attention x is formed from them on the way into LDS, with few rows in several groups of splits side by
+// side: what counts then is how many loads follow each other.
 struct HeadLinear {
   const void* x;        // T [R][ldx], head h at h * xh
   const float* parts;   // [n][H][nsplit][K32 + 4], or null
@@ -319,70 +322,115 @@ struct HeadLinear {
 constexpr int kHeadBatch = 8;
 constexpr int kMaxSplits = 64;
 
-template <typename T, bool PARTS>
-__global__ __launch_bounds__(64 * kWaves) void head_linear_kernel(const HeadLinear p) {
+template <typename T, bool PARTS, int KW>
+__global__ __launch_bounds__(KW == 1 ? 256 : 512) void head_linear_kernel(const HeadLinear p) {
+  constexpr int NW = KW == 1 ? 4 : 8, TH = 64 * NW;
+  __shared__ floatx4 red[KW == 1 ? 1 : NW][KW == 1 ? 1 : 64];
   extern __shared__ __attribute__((aligned(16))) char xs[];  // PARTS: [rows][ldw * sizeof(T) + 16]
+  __shared__ floatx4 sums[PARTS ? TH : 1];
   __shared__ float fac[PARTS ? 16 : 1][PARTS ? kMaxSplits : 1];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r = lane & 15, g = lane >> 4, h = blockIdx.y;
   const int i0 = blockIdx.z * 16, rows = min(16, p.n - i0);
-  const int n0 = (blockIdx.x * kWaves + wave) * 16;
+  const int n0 = (blockIdx.x * (NW / KW) + wave / KW) * 16;
   const int ri = i0 + min(r, rows - 1), row = p.list ? p.list[ri] : ri;
-  const int steps = p.ldw * (int)sizeof(T) / 64, lrow = p.ldw * (int)sizeof(T) + 16;
+  const int all = p.ldw * (int)sizeof(T) / 64, each = (all + KW - 1) / KW;
+  const int first = min(wave % KW * each, all), steps = min(all, first + each), lrow = p.ldw * (int)sizeof(T) + 16;
   const char* wp = reinterpret_cast<const char*>(reinterpret_cast<const T*>(p.w) + ((size_t)h * p.N + min(n0 + r, p.N - 1)) * p.ldw) + g * 16;
   const char* xp = reinterpret_cast<const char*>(reinterpret_cast<const T*>(p.x) + (size_t)row * p.ldx + (size_t)h * p.xh) + g * 16;
   uint4 wv[kHeadBatch];
   auto load_w = [&](int s) {
 #pragma unroll
-    for (int i = 0; i < kHeadBatch; ++i) wv[i] = *reinterpret_cast<const uint4*>(wp + min(s + i, steps - 1) * 64);
+    for (int i = 0; i < kHeadBatch; ++i) wv[i] = load16(wp + min(s + i, all - 1) * 64);
   };
-  load_w(0);
+  load_w(first);
   if (PARTS) {
-    const int ps = p.K32 + 4;
-    for (int i = wave; i < rows; i += kWaves) {
+    // a thread's first item and group of splits: requested ahead of the factors
+    constexpr int PB = 16;
+    const int ps = p.K32 + 4, quads = p.ldw / 4, items = rows * quads;
+    const int groups = min(max(TH / items, 1), p.nsplit), per = (p.nsplit + groups - 1) / groups;
+    const int k = groups > 1 ? tid / items : 0;
+    const int s0 = k * per, s1 = min(p.nsplit, s0 + per);  // (none: s1 <= s0)
+    auto source = [&](int i) {  // (past the latent: zeros from its padding's product, never used)
+      const int m = i / quads, c = min(i % quads * 4, p.K32 - 4);
+      return p.parts + ((size_t)(i0 + m) * p.H + h) * p.nsplit * ps + c;
+    };
+    const int item = groups > 1 ? tid - k * items : min(tid, items - 1);
+    floatx4 pre[PB];
+    {
+      const float* src = source(item);
+#pragma unroll
+      for (int s = 0; s < PB; ++s) pre[s] = *reinterpret_cast<const floatx4*>(src + (size_t)min(s0 + s, s1 - 1) * ps);
+    }
+    for (int i = wave; i < rows; i += NW) {
       const float* src = p.parts + ((size_t)(i0 + i) * p.H + h) * p.nsplit * ps + p.K32;
       const bool on = lane < p.nsplit;
       const float m1 = on ? src[(size_t)lane * ps] : -INFINITY, l1 = on ? src[(size_t)lane * ps + 1] : 0.f;
-      const float mm = wave_max(m1);
+      const float mm = wave_max_f32_uniform(m1);
       const float w1 = m1 == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m1 - mm);
-      const float inv = 1.f / wave_sum(l1 * w1);
+      const float inv = 1.f / wave_sum_uniform(l1 * w1);
       if (on) fac[i][lane] = w1 * inv;
     }
     __syncthreads();
-    const int quads = p.ldw / 4;
-    for (int i = tid; i < rows * quads; i += 64 * kWaves) {
-      const int m = i / quads, c = (i - m * quads) * 4;
-      floatx4 v = {0.f, 0.f, 0.f, 0.f};
-      if (c < p.K32) {
-        const float* src = p.parts + ((size_t)(i0 + m) * p.H + h) * p.nsplit * ps + c;
-        for (int s0 = 0; s0 < p.nsplit; s0 += 8) {
-          floatx4 u[8];
+    auto add = [&](floatx4& v, const floatx4& u, int m, int s) {
+      const float f = s < s1 ? fac[m][s] : 0.f;
 #pragma unroll
-          for (int s = 0; s < 8; ++s) u[s] = *reinterpret_cast<const floatx4*>(src + (size_t)min(s0 + s, p.nsplit - 1) * ps);
+      for (int e = 0; e < 4; ++e) v[e] = fmaf(f, u[e], v[e]);
+    };
+    auto rest = [&](floatx4& v, int i, int s) {  // splits from s on
+      const float* src = source(i);
+      for (; s < s1; s += 8) {
+        floatx4 u[8];
 #pragma unroll
-          for (int s = 0; s < 8; ++s) {
-            const float f = s0 + s < p.nsplit ? fac[m][min(s0 + s, kMaxSplits - 1)] : 0.f;
+        for (int e = 0; e < 8; ++e) u[e] = *reinterpret_cast<const floatx4*>(src + (size_t)min(s + e, s1 - 1) * ps);
 #pragma unroll
-            for (int e = 0; e < 4; ++e) v[e] = fmaf(f, u[s][e], v[e]);
-          }
-        }
+        for (int e = 0; e < 8; ++e) add(v, u[e], i / quads, min(s + e, kMaxSplits - 1));
       }
-      T* dst = reinterpret_cast<T*>(xs + m * lrow) + c;
+    };
+    auto leave = [&](int i, const floatx4& v) {
+      const int c = i % quads * 4;
+      T* dst = reinterpret_cast<T*>(xs + i / quads * lrow) + c;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) dst[e] = Elem<T>::make(v[e]);
+      for (int e = 0; e < 4; ++e) dst[e] = Elem<T>::make(c < p.K32 ? v[e] : 0.f);
+    };
+    floatx4 v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < PB; ++s) add(v, pre[s], item / quads, min(s0 + s, kMaxSplits - 1));
+    rest(v, item, s0 + PB);
+    if (groups > 1) {  // (then items <= TH / 2)
+      if (k < groups) sums[tid] = v;
+      __syncthreads();
+      if (tid < items) {
+        for (int o = 1; o < groups; ++o) v += sums[tid + o * items];
+        leave(tid, v);
+      }
+    } else {
+      if (tid < items) leave(tid, v);
+      for (int i = tid + TH; i < items; i += TH) {
+        floatx4 w = {0.f, 0.f, 0.f, 0.f};
+        rest(w, i, 0);
+        leave(i, w);
+      }
     }
     __syncthreads();
     xp = xs + min(r, rows - 1) * lrow + g * 16;
   }
   floatx4 acc = {0.f, 0.f, 0.f, 0.f};
-  for (int s = 0; s < steps; s += kHeadBatch) {
+  for (int s = first; s < steps; s += kHeadBatch) {
     uint4 xv[kHeadBatch];
 #pragma unroll
-    for (int i = 0; i < kHeadBatch; ++i) xv[i] = *reinterpret_cast<const uint4*>(xp + min(s + i, steps - 1) * 64);
+    for (int i = 0; i < kHeadBatch; ++i) xv[i] = load16(xp + min(s + i, all - 1) * 64);
 #pragma unroll
     for (int i = 0; i < kHeadBatch; ++i)
       if (s + i < steps) acc = Elem<T>::mma16(wv[i], xv[i], acc);
     if (s + kHeadBatch < steps) load_w(s + kHeadBatch);
+  }
+  if (KW > 1) {
+    red[wave][lane] = acc;
+    __syncthreads();
+    if (wave % KW) return;
+#pragma unroll
+    for (int k = 1; k < KW; ++k) acc += red[wave + k][lane];
   }
   if (r >= rows) return;
   T* y = reinterpret_cast<T*>(p.y) + (size_t)row * p.ldy + (size_t)h * p.yh;
@@ -501,19 +549,21 @@ extern "C" int exo_head_linear(const exo_head_linear_args* a, exo_stream_t strea
   HeadLinear p{};
   p.x = a->x, p.parts = a->parts, p.w = a->w, p.y = a->y, p.list = a->list, p.n = a->n, p.H = a->heads, p.N = a->N;
   p.K32 = (a->K + 31) / 32 * 32, p.ldx = a->ldx, p.xh = a->x_head, p.ldw = a->ldw, p.ldy = a->ldy, p.yh = a->y_head, p.nsplit = a->nsplit;
-  const dim3 grid(exo_ceil_div(p.N, 16 * kWaves), p.H, exo_ceil_div(p.n, 16));
+  const bool split = p.parts || p.ldw > 128;
+  const int threads = split ? 512 : 256;
+  const dim3 grid(exo_ceil_div(p.N, split ? 32 : 64), p.H, exo_ceil_div(p.n, 16));
   EXO_REQUIRE(grid.z <= 65535, "exo_head_linear: too many rows (%d)", p.n);
   const int lds = p.parts ? (p.n < 16 ? p.n : 16) * (p.ldw * (a->dtype == 0 ? 2 : 4) + 16) : 0;
   const hipStream_t st = (hipStream_t)stream;
   if (p.parts) {
     if (a->dtype == 0)
-      head_linear_kernel<bf16_t, true><<<grid, 64 * kWaves, lds, st>>>(p);
+      head_linear_kernel<bf16_t, true, 4><<<grid, threads, lds, st>>>(p);
     else
-      head_linear_kernel<float, true><<<grid, 64 * kWaves, lds, st>>>(p);
-  } else if (a->dtype == 0) {
-    head_linear_kernel<bf16_t, false><<<grid, 64 * kWaves, 0, st>>>(p);
+      head_linear_kernel<float, true, 4><<<grid, threads, lds, st>>>(p);
   } else {
-    head_linear_kernel<float, false><<<grid, 64 * kWaves, 0, st>>>(p);
+    const auto fn = a->dtype == 0 ? (split ? head_linear_kernel<bf16_t, false, 4> : head_linear_kernel<bf16_t, false, 1>)
+                                  : (split ? head_linear_kernel<float, false, 4> : head_linear_kernel<float, false, 1>);
+    fn<<<grid, threads, 0, st>>>(p);
   }
   EXO_CHECK_LAUNCH("exo_head_linear");
   return EXO_OK;
