@@ -307,10 +307,10 @@ __global__ __launch_bounds__(kRowThreads) void latent_rows_kernel(const Params p
 }
 
 // ------------------------------------------------------------------------------ a matrix per head
-// y[row][h] = w[h] x[row][h]: outputs of one head and up to 16 rows per workgroup, 16x16 tiles; short rows a
-// wave per tile (KW 1), long ones over four waves (KW 4: two tiles, eight waves).  With partials of split
-// attention x is formed from them on the way into LDS, with few rows in several groups of splits side by
-// side: what counts then is how many loads follow each other.
+// y[row][h] = w[h] x[row][h]: outputs of one head and up to 16 rows per workgroup, 16x16 tiles, a wave per
+// tile.  With partials of split attention x is formed from them on the way into LDS, with few rows in several
+// groups of splits side by side (what counts then is how many loads follow each other), and a tile's product
+// is dealt out over four waves.
 struct HeadLinear {
   const void* x;        // T [R][ldx], head h at h * xh
   const float* parts;   // [n][H][nsplit][K32 + 4], or null
@@ -322,9 +322,9 @@ struct HeadLinear {
 constexpr int kHeadBatch = 8;
 constexpr int kMaxSplits = 64;
 
-template <typename T, bool PARTS, int KW>
-__global__ __launch_bounds__(KW == 1 ? 256 : 512) void head_linear_kernel(const HeadLinear p) {
-  constexpr int NW = KW == 1 ? 4 : 8, TH = 64 * NW;
+template <typename T, bool PARTS>
+__global__ __launch_bounds__(PARTS ? 512 : 256) void head_linear_kernel(const HeadLinear p) {
+  constexpr int KW = PARTS ? 4 : 1, NW = PARTS ? 8 : 4, TH = 64 * NW;
   __shared__ floatx4 red[KW == 1 ? 1 : NW][KW == 1 ? 1 : 64];
   extern __shared__ __attribute__((aligned(16))) char xs[];  // PARTS: [rows][ldw * sizeof(T) + 16]
   __shared__ floatx4 sums[PARTS ? TH : 1];
@@ -549,21 +549,20 @@ extern "C" int exo_head_linear(const exo_head_linear_args* a, exo_stream_t strea
   HeadLinear p{};
   p.x = a->x, p.parts = a->parts, p.w = a->w, p.y = a->y, p.list = a->list, p.n = a->n, p.H = a->heads, p.N = a->N;
   p.K32 = (a->K + 31) / 32 * 32, p.ldx = a->ldx, p.xh = a->x_head, p.ldw = a->ldw, p.ldy = a->ldy, p.yh = a->y_head, p.nsplit = a->nsplit;
-  const bool split = p.parts || p.ldw > 128;
-  const int threads = split ? 512 : 256;
-  const dim3 grid(exo_ceil_div(p.N, split ? 32 : 64), p.H, exo_ceil_div(p.n, 16));
+  const int threads = p.parts ? 512 : 256;
+  const dim3 grid(exo_ceil_div(p.N, p.parts ? 32 : 64), p.H, exo_ceil_div(p.n, 16));
   EXO_REQUIRE(grid.z <= 65535, "exo_head_linear: too many rows (%d)", p.n);
   const int lds = p.parts ? (p.n < 16 ? p.n : 16) * (p.ldw * (a->dtype == 0 ? 2 : 4) + 16) : 0;
   const hipStream_t st = (hipStream_t)stream;
   if (p.parts) {
     if (a->dtype == 0)
-      head_linear_kernel<bf16_t, true, 4><<<grid, threads, lds, st>>>(p);
+      head_linear_kernel<bf16_t, true><<<grid, threads, lds, st>>>(p);
     else
-      head_linear_kernel<float, true, 4><<<grid, threads, lds, st>>>(p);
+      head_linear_kernel<float, true><<<grid, threads, lds, st>>>(p);
+  } else if (a->dtype == 0) {
+    head_linear_kernel<bf16_t, false><<<grid, threads, 0, st>>>(p);
   } else {
-    const auto fn = a->dtype == 0 ? (split ? head_linear_kernel<bf16_t, false, 4> : head_linear_kernel<bf16_t, false, 1>)
-                                  : (split ? head_linear_kernel<float, false, 4> : head_linear_kernel<float, false, 1>);
-    fn<<<grid, threads, 0, st>>>(p);
+    head_linear_kernel<float, false><<<grid, threads, 0, st>>>(p);
   }
   EXO_CHECK_LAUNCH("exo_head_linear");
   return EXO_OK;
