@@ -35,4 +35,8 @@ Pin status per function (what, other than the formula itself, checks it):
 * ``gekazen`` (a design the reference does not have)  pinned - attention with mask and distance
   penalty against ``torch.nn.functional.scaled_dot_product_attention``, norms, gated unit and
   routing on hand-worked values, causality.
+* ``novosun`` (the same)  pinned - recurrence against decayed attention pair by pair, convolution and
+  attention against ``torch``, the rest on hand-worked values, causality.
+* ``pimisun`` (the same)  pinned - rotation against complex products, attention and gelu against
+  ``torch``, latent attention against its absorbed form, the rest on hand-worked values, causality.
 """

@@ -48,8 +48,9 @@ def mixed_config():
     ], width=100)
 
 
-def weights(cfg: dict, seed: int = 0) -> dict[str, np.ndarray]:
-    """bf16-representable float32 arrays by tensor name."""
+def weights(cfg: dict, seed: int = 0, choosy: bool = True) -> dict[str, np.ndarray]:
+    """bf16-representable float32 arrays by tensor name.  ``choosy``: every expert is chosen by some token; else the
+    routers' logits lie apart from each other and few choices are close enough for bf16 rounding to turn them."""
     from oracle.affine import bf16_round
 
     r = np.random.default_rng(seed)
@@ -97,9 +98,8 @@ def weights(cfg: dict, seed: int = 0) -> dict[str, np.ndarray]:
                 put(p + "mlp.down", W, f["ff"])
             else:
                 n = f["router"]["experts"]
-                # logits apart from each other: few choices that bf16 rounding could turn
-                put(p + "mlp.router", n, W, std=0.5 / np.sqrt(W))
-                put(p + "mlp.router.b", n, std=0.0, mean=r.permutation(n) * 1.2)
+                put(p + "mlp.router", n, W, std=(3.0 if choosy else 0.4) / np.sqrt(W))
+                put(p + "mlp.router.b", n, std=0.0, mean=r.permutation(n) * (0.3 if choosy else 1.2))
                 for e in range(n):
                     glu(f"{p}mlp.e{e}.", f["expert"]["ff"])
                 if f.get("shared"):
@@ -108,3 +108,23 @@ def weights(cfg: dict, seed: int = 0) -> dict[str, np.ndarray]:
         put(p + "side.proj", W, S)
         norm(p + "side.norm", W)
     return out
+
+
+def forward_and_gaps(cfg: dict, w, tokens):
+    """Oracle logits, and per token the smallest gap over the layers between the last chosen and the first unchosen
+    router logit (a bf16 model may choose otherwise where it is tiny)."""
+    from oracle import pimisun as O
+
+    seen, orig = [], O.route
+
+    def spy(logits, top):
+        z = np.sort(logits)[::-1]
+        seen.append(z[top - 1] - z[top] if top < len(z) else np.inf)
+        return orig(logits, top)
+
+    O.route = spy
+    try:
+        lg = O.forward(cfg, w, tokens)
+    finally:
+        O.route = orig
+    return lg, np.min(np.asarray(seen).reshape(-1, len(tokens)), axis=0)

@@ -312,26 +312,28 @@ def test_product_per_head_over_listed_rows(device, dtype):
 
 @pytest.fixture(scope="module")
 def built():
-    """(config, float64 weights, {dtype: model}, tokens, oracle logits) of the mixed configuration."""
+    """The mixed configuration: config, tokens; by dtype float64 weights, model, oracle logits."""
     if not torch.cuda.is_available():
         pytest.skip("no GPU")
     cfg = U.mixed_config()
-    w = U.weights(cfg, 11)
-    models = {t: build_model(config_from_dict(cfg), torch_weights(w, "cuda"), dtype=t) for t in DTYPES}
+    w = {t: U.weights(cfg, 11, choosy=t == F32) for t in DTYPES}
+    models = {t: build_model(config_from_dict(cfg), torch_weights(w[t], "cuda"), dtype=t) for t in DTYPES}
     toks = {name: rng(s).integers(0, cfg["vocab"], n).tolist() for s, (name, n) in
             enumerate({"a": 300, "b": 141, "c": 64, "d": 23, "e": 1}.items())}
-    w64 = O.to_float64(w)
-    want = {k: O.forward(cfg, w64, t) for k, t in toks.items()}
-    return types.SimpleNamespace(cfg=cfg, w=w64, models=models, toks=toks, want=want)
+    w64 = {t: O.to_float64(x) for t, x in w.items()}
+    both = {t: {k: U.forward_and_gaps(cfg, w64[t], x) for k, x in toks.items()} for t in DTYPES}
+    want, gaps = ({t: {k: v[i] for k, v in x.items()} for t, x in both.items()} for i in (0, 1))
+    return types.SimpleNamespace(cfg=cfg, w=w64, models=models, toks=toks, want=want, gaps=gaps)
 
 
-LIMIT = {BF: 1e-1, F32: 1e-4}  # of the worst position (bf16: where a router's choice is close); a typical one: 2e-2
+LIMIT = {BF: 1e-1, F32: 1e-4}  # of nearly all positions (bf16: a router's close choice may turn); a typical one: 2e-2
 
 
 def check_rows(built, dtype, name, places, logits, what):
-    err = rel_rms(logits, built.want[name][places])
+    err = rel_rms(logits, built.want[dtype][name][places])
     say(what, f"worst {err.max():.1e}, median {np.median(err):.1e}")
     assert np.quantile(err, 0.95) < LIMIT[dtype], f"{what}: {np.quantile(err, 0.95):.2e}"
+    err = np.where(built.gaps[dtype][name][places] < (0.05 if dtype == BF else 0), 0, err)
     assert err.max() < LIMIT[dtype] * (5 if dtype == BF else 1), f"{what}: {err.max():.2e} at {places[int(err.argmax())]}"
     assert np.median(err) < LIMIT[dtype] / 2, f"{what}: median {np.median(err):.2e}"
 
@@ -348,7 +350,7 @@ def test_model_in_portions(built, dtype, portion):
 @pytest.mark.parametrize("portion", [64, 1])
 def test_model_layers(built, dtype, portion):
     m, outs, want = built.models[dtype], [], []
-    O.forward(built.cfg, built.w, built.toks["c"], want)
+    O.forward(built.cfg, built.w[dtype], built.toks["c"], want)
     m.layer_hook = lambda i, h: outs.append(host(h).copy())
     try:
         play(m, built.toks, [[("c", portion)]] * 64)
@@ -358,6 +360,7 @@ def test_model_layers(built, dtype, portion):
     for i, w in enumerate(want):
         err = rel_rms(np.concatenate(outs[i::n]), w)
         assert np.median(err) < (3e-2 if dtype == BF else 3e-5), f"layer {i}: {np.median(err):.2e}"
+        err = np.where(built.gaps[dtype]["c"] < (0.05 if dtype == BF else 0), 0, err)
         assert err.max() < (3e-1 if dtype == BF else 3e-5), f"layer {i}: {err.max():.2e}"
 
 
@@ -373,14 +376,14 @@ def test_rows_move_and_are_cut_back(built):
     c = m.make_cache(3, 320)
     m.step(c, [(0, t["a"][:77], []), (1, t["b"][:50], [])])
     c.release(0)
-    assert rel_rms(host(m.step(c, [(0, t["c"], [63])])), built.want["c"][63:]).max() < 1e-4
+    assert rel_rms(host(m.step(c, [(0, t["c"], [63])])), built.want[F32]["c"][63:]).max() < 1e-4
     c.copy_row(1, 2)
-    assert rel_rms(host(m.step(c, [(2, t["b"][50:60], [9])])), built.want["b"][59:60]).max() < 1e-4
+    assert rel_rms(host(m.step(c, [(2, t["b"][50:60], [9])])), built.want[F32]["b"][59:60]).max() < 1e-4
     c.swap_rows(0, 2)
     lg = host(m.step(c, [(1, t["d"][:1], [0]), (0, t["b"][60:61], [0])]))
-    assert rel_rms(lg, np.stack([built.want["d"][0], built.want["b"][60]])).max() < 1e-4
+    assert rel_rms(lg, np.stack([built.want[F32]["d"][0], built.want[F32]["b"][60]])).max() < 1e-4
     c.trim(30, rows=[0])
-    assert rel_rms(host(m.step(c, [(0, t["b"][31:90], [58])])), built.want["b"][89:90]).max() < 1e-4
+    assert rel_rms(host(m.step(c, [(0, t["b"][31:90], [58])])), built.want[F32]["b"][89:90]).max() < 1e-4
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -393,7 +396,7 @@ def test_model_graph_decode_matches_steps(built, dtype, B):
     n0, n1 = 30, 46
     m.step(cache, [(r, s[: n0 - r % 7], []) for r, s in enumerate(seqs)])
     pos = [n0 - r % 7 for r in range(B)]
-    wants, errs = [O.forward(built.cfg, built.w, s[:n1]) for s in seqs], []
+    wants, errs = [O.forward(built.cfg, built.w[dtype], s[:n1]) for s in seqs], []
     for k in range(n1 - n0):
         bf = m._buffers(B, 1)
         bf.tokens.copy_(torch.tensor([s[p] for s, p in zip(seqs, pos)], dtype=torch.int32))
@@ -406,7 +409,7 @@ def test_model_graph_decode_matches_steps(built, dtype, B):
 
 def test_model_long_decode(built):
     m, toks = built.models[F32], rng(77).integers(0, built.cfg["vocab"], 560).tolist()
-    want = O.forward(built.cfg, built.w, toks)
+    want = O.forward(built.cfg, built.w[F32], toks)
     cache = m.make_cache(1, 600)
     m.step(cache, [(0, toks[:150], [])])
     bf = m._buffers(1, 1)
@@ -425,23 +428,23 @@ def test_model_long_decode(built):
 def test_other_orders_and_sizes(device, dtype, layers):
     """... among them key sizes that are too large to expand."""
     cfg = U.config(layers, width=130, vocab=97, eps=3e-3, alpha=1.0, embed=1.0, logit=1.0, side=1)
-    w = U.weights(cfg, 5)
+    w = U.weights(cfg, 5, choosy=dtype == F32)
     m = build_model(config_from_dict(cfg), torch_weights(w, "cuda"), dtype=dtype)
     toks = {"a": rng(1).integers(0, 97, 140).tolist(), "b": rng(2).integers(0, 97, 9).tolist()}
     want = {k: O.forward(cfg, w, t) for k, t in toks.items()}
     for sched in ([[("a", 140)]], [[("a", 70), ("b", 1)], [("b", 2), ("a", 3)]] + [[("a", 1), ("b", 1)]] * 90):
         for k, lg in play(m, toks, sched, max_tokens=256).items():
             err = rel_rms(lg, want[k])
-            assert np.quantile(err, 0.95) < LIMIT[dtype] and err.max() < LIMIT[dtype] * (5 if dtype == BF else 1)
+            assert np.quantile(err, 0.95 if dtype == BF else 1) < LIMIT[dtype] and np.median(err) < LIMIT[dtype] / 2
 
 
 def test_shards(built):
     """Every layer reads the tokens: a shard starts at layer 0, and layers that mix values hold the first."""
-    w = torch_weights({k: np.asarray(v, np.float32) for k, v in built.w.items()}, "cuda")
+    w = torch_weights({k: np.asarray(v, np.float32) for k, v in built.w[F32].items()}, "cuda")
     c = config_from_dict(built.cfg)
     x = build_model(c, w, 0, 3, dtype=F32)
     want = []
-    O.forward(built.cfg, built.w, built.toks["c"], want)
+    O.forward(built.cfg, built.w[F32], built.toks["c"], want)
     got = x(torch.tensor([built.toks["c"]]), x.make_cache(1, 100))
     assert rel_rms(host(got)[0], want[2]).max() < 1e-4
     with pytest.raises(ValueError, match="start at layer 0"):
@@ -452,7 +455,7 @@ def test_shards(built):
 
 
 def greedy_agrees(built, prompt, got, dtype):
-    S.greedy_agrees(lambda toks: O.forward(built.cfg, built.w, toks), prompt, got, dtype)
+    S.greedy_agrees(lambda toks: O.forward(built.cfg, built.w[dtype], toks), prompt, got, dtype)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -516,7 +519,7 @@ def test_generate_greedy(built, dtype):
 
 
 def test_builder_serves_a_checkpoint(built, tmp_path):
-    write_checkpoint(tmp_path, built.cfg, {k: np.asarray(v, np.float32) for k, v in built.w.items()})
+    write_checkpoint(tmp_path, built.cfg, {k: np.asarray(v, np.float32) for k, v in built.w[BF].items()})
     n = len(built.cfg["layers"])
     b = Mi355xBuilder(model_id="m", max_seq=512)
     bound = BoundInstance(bound_shard=ShardMetadata(model_id="m", start_layer=0, end_layer=n, n_layers=n), model_path=str(tmp_path))
@@ -531,7 +534,7 @@ def test_builder_serves_a_checkpoint(built, tmp_path):
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_trace_program(built, tmp_path, dtype):
     root = Path(__file__).resolve().parent.parent
-    write_checkpoint(tmp_path / "m", built.cfg, {k: np.asarray(v, np.float32) for k, v in built.w.items()})
+    write_checkpoint(tmp_path / "m", built.cfg, {k: np.asarray(v, np.float32) for k, v in built.w[dtype].items()})
     (tmp_path / "o").mkdir()
     t = built.toks
     steps = [dict(entries=[dict(id="x", tokens=t["b"][:100], want=[99, 3]), dict(id="y", tokens=t["d"][:2], want=[1])], end=[]),
@@ -546,6 +549,6 @@ def test_trace_program(built, tmp_path, dtype):
     assert r.returncode == 0, r.stderr
     assert [ln for ln in r.stdout.splitlines() if ln.startswith("done")] == ["done 0", "done 1", "done 2", "done 3"]
     got = np.concatenate([np.fromfile(tmp_path / "o" / f"{i}.f32", "<f4").reshape(-1, built.cfg["vocab"]) for i in (0, 2, 3)])
-    want = np.stack([built.want["b"][99], built.want["b"][3], built.want["d"][1], built.want["d"][22],
-                     built.want["b"][102], built.want["b"][101], built.want["d"][22]])
+    want = np.stack([built.want[dtype]["b"][99], built.want[dtype]["b"][3], built.want[dtype]["d"][1], built.want[dtype]["d"][22],
+                     built.want[dtype]["b"][102], built.want[dtype]["b"][101], built.want[dtype]["d"][22]])
     assert rel_rms(got, want).max() < LIMIT[dtype] * (5 if dtype == BF else 1)
