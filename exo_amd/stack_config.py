@@ -478,7 +478,7 @@ def novosun_dict(width: int, vocab: int, kinds: str, *, heads: int, kv_heads: in
 
 def pimisun_dict(width: int, vocab: int, kinds: str, *, heads: int, kv_heads: int, dim: int, rot: int, window: int, lat_heads: int,
                  lat_dim: int, lat_rot: int, lat_vdim: int, q_rank: int, kv_rank: int, ff: int, experts: int, top: int,
-                 expert_ff: int, shared_ff: int | None, side: int, dense: int = 1, softcap: float = 30.0, base: float = 5e5,
+                 expert_ff: int, shared_ff: int | None, side: int, dense: int = 1, softcap: float = 50.0, base: float = 1e4,
                  alpha: float = 2.0, eps: float = 1e-6) -> dict:
     """A ``config.json`` of the design (benchmarks); ``kinds``: a letter per layer, l for latent attention, a for
     attention; the first ``dense`` layers have a dense feed-forward, the others experts."""
